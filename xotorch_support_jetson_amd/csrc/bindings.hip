@@ -527,7 +527,7 @@ void splitk_resid_rmsnorm(const at::Tensor& ws, int64_t splits, const c10::optio
 // big_bm = 128 / 256: gemm_big tiles (pre-shuffled weights), else the weight-streaming kernel
 void gemm_moe(const at::Tensor& x, const at::Tensor& w, at::Tensor& y, const at::Tensor& off,
               const c10::optional<at::Tensor>& gather, int64_t epi, int64_t max_rows, bool wshuf, int64_t splits,
-              int64_t big_bm) {
+              int64_t big_bm, double epi_arg) {
   CHECK_BF16(x);
   CHECK_BF16(w);
   CHECK_GPU(y);
@@ -538,10 +538,10 @@ void gemm_moe(const at::Tensor& x, const at::Tensor& w, at::Tensor& y, const at:
   const int64_t E = w.size(0), N = w.size(1), K = w.size(2);
   XCHECK(x.size(1) == K, "gemm_moe: K mismatch");
   XCHECK(off.numel() == E + 1, "gemm_moe: off must have E+1 entries");
-  XCHECK(epi == 0 || epi == 2, "gemm_moe: epilogue must be none or silu");
+  XCHECK(epi == 0 || epi == 2 || epi == 3, "gemm_moe: epilogue must be none, silu or clamp_glu");
   const bool f32 = y.scalar_type() == at::kFloat;
   XCHECK(f32 || y.scalar_type() == at::kBFloat16, "gemm_moe: y must be bf16 or fp32");
-  XCHECK(y.size(1) == (epi == 2 ? N / 2 : N), "gemm_moe: y width mismatch");
+  XCHECK(y.size(1) == (epi >= 2 ? N / 2 : N), "gemm_moe: y width mismatch");
   XCHECK(splits >= 1 && y.size(0) % splits == 0, "gemm_moe: y rows must be splits * slots");
   const int64_t slots = y.size(0) / splits;
   XCHECK(max_rows >= 0 && max_rows <= slots, "gemm_moe: max_rows must be <= slots");
@@ -559,11 +559,11 @@ void gemm_moe(const at::Tensor& x, const at::Tensor& w, at::Tensor& y, const at:
     XCHECK(wshuf, "gemm_moe: the big-tile path needs pre-shuffled expert weights");
     rc = xot::launch_gemm_moe_big(bf(x), (int)x.stride(0), bf(w), y.data_ptr(), (int)y.stride(0), f32, (int)epi,
                                   off.data_ptr<int>(), gp, (int)E, (int)max_rows, (int)N, (int)K, (int)splits,
-                                  (long)(slots * y.size(1)), (int)big_bm, cur_stream());
+                                  (long)(slots * y.size(1)), (int)big_bm, (float)epi_arg, cur_stream());
   } else {
     rc = xot::launch_gemm_moe(bf(x), (int)x.stride(0), bf(w), y.data_ptr(), (int)y.stride(0), f32, (int)epi,
                               off.data_ptr<int>(), gp, (int)E, (int)max_rows, (int)N, (int)K, wshuf, (int)splits,
-                              (long)(slots * y.size(1)), cur_stream());
+                              (long)(slots * y.size(1)), (float)epi_arg, cur_stream());
   }
   XCHECK(rc == 0, "gemm_moe: unsupported shape N=", N, " K=", K, " epi=", epi, " splits=", splits);
 }
@@ -1051,7 +1051,8 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
         py::arg("ws"), py::arg("epi"), py::arg("bn"), py::arg("splits"), py::arg("reduce") = true);
   m.def("splitk_resid_rmsnorm", &splitk_resid_rmsnorm);
   m.def("gemm_moe", &gemm_moe, py::arg("x"), py::arg("w"), py::arg("y"), py::arg("off"), py::arg("gather"),
-        py::arg("epi"), py::arg("max_rows"), py::arg("wshuf"), py::arg("splits") = 1, py::arg("big_bm") = 0);
+        py::arg("epi"), py::arg("max_rows"), py::arg("wshuf"), py::arg("splits") = 1, py::arg("big_bm") = 0,
+        py::arg("epi_arg") = 0.0);
   m.def("moe_route", &moe_route);
   m.def("moe_route_ds", &moe_route_ds);
   m.def("mla_prep", &mla_prep);

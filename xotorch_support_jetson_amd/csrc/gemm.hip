@@ -8,6 +8,7 @@
 //       EPI_NONE     Y = acc (+bias)
 //       EPI_RESID    Y = R + acc (+bias)          (o_proj / down_proj + residual stream)
 //       EPI_SILU     Y[:, j] = silu(acc_gate) * acc_up   (gate/up weights interleaved per 16 rows)
+//       EPI_CLAMP_GLU  the clamped gated form of the same pairs (grouped expert GEMMs; limit: epi_arg)
 //  * gemm_tiled: prefill-shaped M.  128x128x64 LDS tiles, 4 waves in 2x2, register-staged
 //    global->LDS copy of tile k+1 overlapped with the MFMAs of tile k (async-STAGE split),
 //    padded rows (144 B) so every 16-lane ds_read_b128 group hits 16 distinct bank quads.
@@ -215,7 +216,7 @@ __global__ __launch_bounds__(256, OCC) void gemm_stream_kernel(const uint16_t* _
                                                              const int* __restrict__ moe_gather,
                                                              int* __restrict__ tickets, long ysplit,
                                                              const float* __restrict__ wscale, long xbat,
-                                                             long ybat, NormPro np) {
+                                                             long ybat, NormPro np, float epi_arg) {
   constexpr int KC = 32 * KS;
   static_assert(!W8 || (WSHUF && (KS == 4 || KS == 8) && MOE == 0),
                 "FP8 weights: pre-shuffled 128- or 256-deep chunks, dense GEMM");
@@ -613,7 +614,7 @@ __global__ __launch_bounds__(256, OCC) void gemm_stream_kernel(const uint16_t* _
           const int m = wrow + 16 * i + 4 * g + r;
           if (m < M) slab[(size_t)m * N + n0 + 16 * j + c] = acc[i][j][r];
         }
-  } else if constexpr (EPI == EPI_SILU && NTW >= 2) {
+  } else if constexpr (epi_is_glu(EPI) && NTW >= 2) {
 #pragma unroll
     for (int p = 0; p < NTW / 2; ++p) {  // pair (gate tile 2p, up tile 2p+1) -> 16 output columns
       const int col = (n0 >> 1) + 16 * p + c;
@@ -628,7 +629,7 @@ __global__ __launch_bounds__(256, OCC) void gemm_stream_kernel(const uint16_t* _
         for (int r = 0; r < 4; ++r) {
           const int m = wrow + 16 * i + 4 * g + r;
           if (m < M) {
-            const float v = silu(acc[i][2 * p][r] + bg) * (acc[i][2 * p + 1][r] + bu);
+            const float v = glu_pair<EPI>(acc[i][2 * p][r] + bg, acc[i][2 * p + 1][r] + bu, epi_arg);
             if constexpr (OUT_F32)
               reinterpret_cast<float*>(Yv)[(size_t)m * ldy + col] = v;
             else
@@ -636,7 +637,7 @@ __global__ __launch_bounds__(256, OCC) void gemm_stream_kernel(const uint16_t* _
           }
         }
     }
-  } else if constexpr (EPI != EPI_SILU) {
+  } else if constexpr (!epi_is_glu(EPI)) {
 #pragma unroll
     for (int j = 0; j < NTW; ++j) {
       const int col = n0 + 16 * j + c;
@@ -678,7 +679,7 @@ static void stream_launch(const uint16_t* X, int ldx, const uint16_t* W, int ldw
       (void)attr;
     }
     kern<<<grid, 256, SMEM, st>>>(X, ldx, W, ldw, bias, R, ldr, Y, ldy, nullptr, M, N, kper, mblocks, nullptr, nullptr,
-                                  nullptr, 0L, wscale, 0L, 0L, NormPro{});
+                                  nullptr, 0L, wscale, 0L, 0L, NormPro{}, 0.f);
   } else {
     auto kern = gemm_stream_kernel<MT, NTW, KS, EPI, F32, true, WSH, OCC, 0, W8>;
     if constexpr (SMEM > 65536) {
@@ -687,7 +688,7 @@ static void stream_launch(const uint16_t* X, int ldx, const uint16_t* W, int ldw
       (void)attr;
     }
     kern<<<grid, 256, SMEM, st>>>(X, ldx, W, ldw, bias, R, ldr, Y, ldy, ws, M, N, kper, mblocks, nullptr, nullptr,
-                                  nullptr, 0L, wscale, 0L, 0L, NormPro{});
+                                  nullptr, 0L, wscale, 0L, 0L, NormPro{}, 0.f);
     if (!reduce) return;  // slabs left for the consumer
     const int ncol = EPI == EPI_SILU ? N / 2 : N;
     long chunks = (long)M * (ncol / 8);
@@ -750,7 +751,7 @@ static void batched_launch(const uint16_t* X, int ldx, long xbat, const uint16_t
   dim3 grid(N / (64 * NTW) * mblocks, 1, B);
   gemm_stream_kernel<MT, NTW, KS, EPI_NONE, F32, false, true, OCC, 3><<<grid, 256, SMEM, st>>>(
       X, ldx, W, K, nullptr, nullptr, 0, Y, ldy, nullptr, M, N, K, mblocks, nullptr, nullptr, nullptr, 0L, nullptr,
-      xbat, ybat, NormPro{});
+      xbat, ybat, NormPro{}, 0.f);
 }
 
 // B independent GEMMs Y_e[M, N] = X_e[M, K] . W_e[N, K]^T on pre-shuffled weights W [B][N][K]
@@ -778,7 +779,8 @@ int launch_gemm_batched(const uint16_t* X, int ldx, long xbat, const uint16_t* W
 // ------------------------------------------------------------------------------------ grouped (MoE)
 template <int MT, int EPI, bool F32, bool WSH, int MOE>
 static void moe_launch(const uint16_t* X, int ldx, const uint16_t* W, void* Y, int ldy, const int* off,
-                       const int* gather, int E, int max_rows, int N, int K, int S, long ysplit, hipStream_t st) {
+                       const int* gather, int E, int max_rows, int N, int K, int S, long ysplit, float epi_arg,
+                       hipStream_t st) {
   constexpr int NTW = 2, KS = 4;
   constexpr int OCC = (MT * NTW >= 32) ? 1 : 2;
   constexpr int SMEM = 2 * 16 * MT * 32 * KS * 2;
@@ -786,40 +788,41 @@ static void moe_launch(const uint16_t* X, int ldx, const uint16_t* W, void* Y, i
   dim3 grid(N / (64 * NTW) * mblocks, S, E);
   gemm_stream_kernel<MT, NTW, KS, EPI, F32, false, WSH, OCC, MOE><<<grid, 256, SMEM, st>>>(
       X, ldx, W, K, nullptr, nullptr, 0, Y, ldy, nullptr, max_rows, N, K / S, mblocks, off, gather, nullptr,
-      S > 1 ? ysplit : 0L, nullptr, 0L, 0L, NormPro{});
+      S > 1 ? ysplit : 0L, nullptr, 0L, 0L, NormPro{}, epi_arg);
 }
 
 template <int EPI, bool F32, bool WSH, int MOE>
 static void moe_mt(const uint16_t* X, int ldx, const uint16_t* W, void* Y, int ldy, const int* off,
-                   const int* gather, int E, int max_rows, int N, int K, int S, long ysplit, hipStream_t st) {
+                   const int* gather, int E, int max_rows, int N, int K, int S, long ysplit, float epi_arg, hipStream_t st) {
   if (max_rows <= 16)
-    moe_launch<1, EPI, F32, WSH, MOE>(X, ldx, W, Y, ldy, off, gather, E, max_rows, N, K, S, ysplit, st);
+    moe_launch<1, EPI, F32, WSH, MOE>(X, ldx, W, Y, ldy, off, gather, E, max_rows, N, K, S, ysplit, epi_arg, st);
   else if (max_rows <= 64)
-    moe_launch<4, EPI, F32, WSH, MOE>(X, ldx, W, Y, ldy, off, gather, E, max_rows, N, K, S, ysplit, st);
+    moe_launch<4, EPI, F32, WSH, MOE>(X, ldx, W, Y, ldy, off, gather, E, max_rows, N, K, S, ysplit, epi_arg, st);
   else
-    moe_launch<8, EPI, F32, WSH, MOE>(X, ldx, W, Y, ldy, off, gather, E, max_rows, N, K, S, ysplit, st);
+    moe_launch<8, EPI, F32, WSH, MOE>(X, ldx, W, Y, ldy, off, gather, E, max_rows, N, K, S, ysplit, epi_arg, st);
 }
 
 int launch_gemm_moe(const uint16_t* X, int ldx, const uint16_t* W, void* Y, int ldy, bool out_f32, int epi,
                     const int* off, const int* gather, int E, int max_rows, int N, int K, bool wshuf, int S,
-                    long ysplit, hipStream_t s) {
+                    long ysplit, float epi_arg, hipStream_t s) {
   if (max_rows <= 0) return 0;
   if (N % 128 != 0 || S < 1 || K % (128 * S) != 0) return -1;
-  if (epi != EPI_NONE && epi != EPI_SILU) return -1;
-  if (epi == EPI_SILU && out_f32) return -1;
+  if (epi != EPI_NONE && !epi_is_glu(epi)) return -1;
+  if (epi_is_glu(epi) && out_f32) return -1;
   if (S > 1 && (epi != EPI_NONE || !out_f32)) return -1;  // K slices write fp32 partial slabs
 #define XOT_MOE(EPIV, F32V)                                                                                     \
   do {                                                                                                          \
     if (wshuf) {                                                                                                \
-      if (gather) moe_mt<EPIV, F32V, true, 2>(X, ldx, W, Y, ldy, off, gather, E, max_rows, N, K, S, ysplit, s);  \
-      else moe_mt<EPIV, F32V, true, 1>(X, ldx, W, Y, ldy, off, gather, E, max_rows, N, K, S, ysplit, s);         \
+      if (gather) moe_mt<EPIV, F32V, true, 2>(X, ldx, W, Y, ldy, off, gather, E, max_rows, N, K, S, ysplit, epi_arg, s);  \
+      else moe_mt<EPIV, F32V, true, 1>(X, ldx, W, Y, ldy, off, gather, E, max_rows, N, K, S, ysplit, epi_arg, s);         \
     } else {                                                                                                    \
-      if (gather) moe_mt<EPIV, F32V, false, 2>(X, ldx, W, Y, ldy, off, gather, E, max_rows, N, K, S, ysplit, s); \
-      else moe_mt<EPIV, F32V, false, 1>(X, ldx, W, Y, ldy, off, gather, E, max_rows, N, K, S, ysplit, s);        \
+      if (gather) moe_mt<EPIV, F32V, false, 2>(X, ldx, W, Y, ldy, off, gather, E, max_rows, N, K, S, ysplit, epi_arg, s); \
+      else moe_mt<EPIV, F32V, false, 1>(X, ldx, W, Y, ldy, off, gather, E, max_rows, N, K, S, ysplit, epi_arg, s);        \
     }                                                                                                           \
     return 0;                                                                                                   \
   } while (0)
   if (epi == EPI_SILU) XOT_MOE(EPI_SILU, false);
+  if (epi == EPI_CLAMP_GLU) XOT_MOE(EPI_CLAMP_GLU, false);
   if (out_f32) XOT_MOE(EPI_NONE, true);
   XOT_MOE(EPI_NONE, false);
 #undef XOT_MOE
@@ -878,12 +881,12 @@ static void stream_norm_launch(const uint16_t* W, const uint16_t* bias, void* Y,
   if (S == 1) {
     gemm_stream_kernel<1, NTW, 4, EPI, false, false, true, 2, 0, false, PM><<<grid, 256, smem, st>>>(
         nullptr, 0, W, K, bias, nullptr, 0, Y, ldy, nullptr, 1, N, kper, 1, nullptr, nullptr, nullptr, 0L, nullptr,
-        0L, 0L, np);
+        0L, 0L, np, 0.f);
     return;
   }
   gemm_stream_kernel<1, NTW, 4, EPI, false, true, true, 2, 0, false, PM><<<grid, 256, smem, st>>>(
       nullptr, 0, W, K, bias, nullptr, 0, Y, ldy, ws, 1, N, kper, 1, nullptr, nullptr, nullptr, 0L, nullptr, 0L, 0L,
-      np);
+      np, 0.f);
   if (!reduce) return;
   const int ncol = EPI == EPI_SILU ? N / 2 : N;
   splitk_reduce_kernel<EPI, false><<<(ncol / 8 + 255) / 256, 256, 0, st>>>(ws, S, 1, N, bias, nullptr, 0, Y, ldy);
@@ -905,11 +908,11 @@ int launch_gemm_stream_merge(const uint16_t* W, float* ws, long ws_elems, int N,
   if (ntw == 1)
     gemm_stream_kernel<1, 1, 4, EPI_NONE, false, true, true, 2, 0, false, 0, true><<<grid, 256, smem, s>>>(
         nullptr, 0, W, K, nullptr, nullptr, 0, nullptr, N, ws, 1, N, kper, 1, nullptr, nullptr, nullptr, 0L, nullptr,
-        0L, 0L, np);
+        0L, 0L, np, 0.f);
   else
     gemm_stream_kernel<1, 2, 4, EPI_NONE, false, true, true, 2, 0, false, 0, true><<<grid, 256, smem, s>>>(
         nullptr, 0, W, K, nullptr, nullptr, 0, nullptr, N, ws, 1, N, kper, 1, nullptr, nullptr, nullptr, 0L, nullptr,
-        0L, 0L, np);
+        0L, 0L, np, 0.f);
   return 0;
 }
 

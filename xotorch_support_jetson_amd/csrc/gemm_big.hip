@@ -55,7 +55,7 @@ __global__ __launch_bounds__(512, 1) void gemm_big_kernel(const uint16_t* __rest
                                                           int M, int N, int K, int S,
                                                           const int* __restrict__ moe_off = nullptr,
                                                           const int* __restrict__ moe_gather = nullptr,
-                                                          long ysplit = 0, int group_m = 4) {
+                                                          long ysplit = 0, int group_m = 4, float epi_arg = 0.f) {
   static_assert(WM * WN == 8, "8 waves");
   static_assert(BK == 32 || BK == 64, "k stage of 32 or 64");
   static_assert(BM % (16 * WM) == 0 && BM >= 128 && BM <= 512, "row tile of 128 .. 512 rows");
@@ -65,7 +65,7 @@ __global__ __launch_bounds__(512, 1) void gemm_big_kernel(const uint16_t* __rest
   constexpr int MT = BM / (16 * WM), NT = BN / (16 * WN);
   // odd NT (BN = 224: 7 row groups per wave): the gate/up pair that straddles two waves of a row is
   // joined through LDS in the epilogue
-  static_assert(EPI != EPI_SILU || NT % 2 == 0 || (PP == 0 && MOE == 0), "SiLU epilogue pairs gate/up n-tiles");
+  static_assert(!epi_is_glu(EPI) || NT % 2 == 0 || (PP == 0 && MOE == 0), "SiLU epilogue pairs gate/up n-tiles");
   constexpr int KS = BK / 32;                          // MFMA k-steps (and 1 KB W blocks per row group) per stage
   constexpr int SPR = BK / 8;                          // 16-B slots per X row in LDS
   constexpr int A_ELEMS = BM * BK, B_ELEMS = BN * BK;  // bf16 elements per stage
@@ -398,7 +398,7 @@ __global__ __launch_bounds__(512, 1) void gemm_big_kernel(const uint16_t* __rest
             if (cbase + 16 * j < N) slab[(size_t)m * N + cbase + 16 * j + c] = acc[i][j][r];
         }
       }
-  } else if constexpr (EPI == EPI_SILU) {
+  } else if constexpr (epi_is_glu(EPI)) {
     // (gate group at column gcol, up group at gcol + 16) -> 16 output columns starting at gcol / 2
     auto store_pair = [&](int gcol, auto gate, auto up) {
       if (gcol >= N) return;
@@ -414,7 +414,7 @@ __global__ __launch_bounds__(512, 1) void gemm_big_kernel(const uint16_t* __rest
         for (int r = 0; r < 4; ++r) {
           const int m = rbase + 16 * i + 4 * g + r;
           if (m < Mv) {
-            const float v = silu(gate(i)[r] + bg) * (up(i)[r] + bu);
+            const float v = glu_pair<EPI>(gate(i)[r] + bg, up(i)[r] + bu, epi_arg);
             if constexpr (OUT_F32)
               reinterpret_cast<float*>(Yv)[(size_t)m * ldy + col] = v;
             else
@@ -520,14 +520,14 @@ static void big_launch(const uint16_t* X, int ldx, const uint16_t* W, const uint
                        hipSuccess;
     (void)attr;
     kern<<<nwg, 512, SMEM, st>>>(X, ldx, W, bias, R, ldr, Y, ldy, nullptr, M, N, K, 1, nullptr, nullptr, 0L,
-                                 big_group_m());
+                                 big_group_m(), 0.f);
   } else {
     auto kern = gemm_big_kernel<BM, BN, WM, WN, BK, NBUF, EPI, false, true, 0, 0, 3, PP>;
     static bool attr = hipFuncSetAttribute((const void*)kern, hipFuncAttributeMaxDynamicSharedMemorySize, SMEM) ==
                        hipSuccess;
     (void)attr;
     kern<<<nwg, 512, SMEM, st>>>(X, ldx, W, bias, R, ldr, Y, ldy, ws, M, N, K, S, nullptr, nullptr, 0L,
-                                 big_group_m());
+                                 big_group_m(), 0.f);
     if (!reduce) return;  // slabs left for the consumer (fused reduce + residual + RMSNorm)
     const int ncol = EPI == EPI_SILU ? N / 2 : N;
     const long chunks = (long)M * (ncol / 8);
@@ -616,14 +616,14 @@ int launch_gemm_kgroup(const uint16_t* X, int ldx, const uint16_t* W, uint16_t* 
                        hipSuccess;
     (void)attr;
     kern<<<grid, 512, SMEM, st>>>(X, ldx, W, nullptr, Y, ldy, Y, ldy, nullptr, M, N, K, 1, koff, nullptr, 0L,
-                                  big_group_m());
+                                  big_group_m(), 0.f);
   } else {
     auto kern = gemm_big_kernel<256, 256, 2, 4, 64, 2, EPI_NONE, false, false, 4, 0, 3, 2>;
     static bool attr = hipFuncSetAttribute((const void*)kern, hipFuncAttributeMaxDynamicSharedMemorySize, SMEM) ==
                        hipSuccess;
     (void)attr;
     kern<<<grid, 512, SMEM, st>>>(X, ldx, W, nullptr, nullptr, 0, Y, ldy, nullptr, M, N, K, 1, koff, nullptr, 0L,
-                                  big_group_m());
+                                  big_group_m(), 0.f);
   }
   return 0;
 }
@@ -640,7 +640,8 @@ void launch_splitk_silu(const float* ws, int S, int M, int N, uint16_t* y, hipSt
 // ------------------------------------------------------------------------------------ grouped (MoE)
 template <int BM, int EPI, bool F32, int MOE, int BK = 64, int NBUF = 2, int PP = 0>
 static void big_moe_launch(const uint16_t* X, int ldx, const uint16_t* W, void* Y, int ldy, const int* off,
-                           const int* gather, int E, int max_rows, int N, int K, int S, long ysplit, hipStream_t st) {
+                           const int* gather, int E, int max_rows, int N, int K, int S, long ysplit, float epi_arg,
+                           hipStream_t st) {
   constexpr int BN = 256, WM = 2, WN = 4;
   constexpr int SMEM = NBUF * (BM + BN) * BK * 2;
   static_assert(SMEM <= 160 * 1024, "LDS");
@@ -650,7 +651,7 @@ static void big_moe_launch(const uint16_t* X, int ldx, const uint16_t* W, void* 
   (void)attr;
   dim3 grid(((max_rows + BM - 1) / BM) * (N / BN) * S, E);
   kern<<<grid, 512, SMEM, st>>>(X, ldx, W, nullptr, nullptr, 0, Y, ldy, nullptr, max_rows, N, K, S, off, gather,
-                                S > 1 ? ysplit : 0L, 4);
+                                S > 1 ? ysplit : 0L, 4, epi_arg);
 }
 
 // bm = row tile (128 / 192 / 256) + 1000 x pipeline variant: 0 = two 64-deep LDS stages (one in flight under
@@ -658,14 +659,14 @@ static void big_moe_launch(const uint16_t* X, int ldx, const uint16_t* W, void* 
 // BM 192 / 256: four 32-deep stages, three in flight); 2 (BM 192 / 256) = the two-phase ping-pong schedule
 template <int EPI, bool F32>
 static void big_moe_bm(const uint16_t* X, int ldx, const uint16_t* W, void* Y, int ldy, const int* off,
-                       const int* gather, int E, int max_rows, int N, int K, int S, long ysplit, int bm,
+                       const int* gather, int E, int max_rows, int N, int K, int S, long ysplit, int bm, float epi_arg,
                        hipStream_t st) {
 #define XOT_MOE(BM_, ...)                                                                                          \
   do {                                                                                                            \
     if (gather)                                                                                                   \
-      big_moe_launch<BM_, EPI, F32, 2, ##__VA_ARGS__>(X, ldx, W, Y, ldy, off, gather, E, max_rows, N, K, S, ysplit, st); \
+      big_moe_launch<BM_, EPI, F32, 2, ##__VA_ARGS__>(X, ldx, W, Y, ldy, off, gather, E, max_rows, N, K, S, ysplit, epi_arg, st); \
     else                                                                                                          \
-      big_moe_launch<BM_, EPI, F32, 1, ##__VA_ARGS__>(X, ldx, W, Y, ldy, off, gather, E, max_rows, N, K, S, ysplit, st); \
+      big_moe_launch<BM_, EPI, F32, 1, ##__VA_ARGS__>(X, ldx, W, Y, ldy, off, gather, E, max_rows, N, K, S, ysplit, epi_arg, st); \
   } while (0)
   switch (bm) {
     case 128: XOT_MOE(128); break;
@@ -683,21 +684,23 @@ static void big_moe_bm(const uint16_t* X, int ldx, const uint16_t* W, void* Y, i
 
 int launch_gemm_moe_big(const uint16_t* X, int ldx, const uint16_t* W, void* Y, int ldy, bool out_f32, int epi,
                         const int* off, const int* gather, int E, int max_rows, int N, int K, int S, long ysplit,
-                        int bm, hipStream_t s) {
+                        int bm, float epi_arg, hipStream_t s) {
   if (max_rows <= 0) return 0;
   if ((bm % 1000 != 128 && bm % 1000 != 192 && bm % 1000 != 256) || (bm > 1256 && bm != 2256 && bm != 2192 && bm != 2128) || N % 256 != 0 ||
       K % 128 != 0 || S < 1 ||
       S > K / 64)
     return -1;
-  if (epi != EPI_NONE && epi != EPI_SILU) return -1;
-  if (epi == EPI_SILU && out_f32) return -1;
+  if (epi != EPI_NONE && !epi_is_glu(epi)) return -1;
+  if (epi_is_glu(epi) && out_f32) return -1;
   if (S > 1 && (epi != EPI_NONE || !out_f32)) return -1;  // K slices write fp32 partial slabs
   if (epi == EPI_SILU)
-    big_moe_bm<EPI_SILU, false>(X, ldx, W, Y, ldy, off, gather, E, max_rows, N, K, S, ysplit, bm, s);
+    big_moe_bm<EPI_SILU, false>(X, ldx, W, Y, ldy, off, gather, E, max_rows, N, K, S, ysplit, bm, epi_arg, s);
+  else if (epi == EPI_CLAMP_GLU)
+    big_moe_bm<EPI_CLAMP_GLU, false>(X, ldx, W, Y, ldy, off, gather, E, max_rows, N, K, S, ysplit, bm, epi_arg, s);
   else if (out_f32)
-    big_moe_bm<EPI_NONE, true>(X, ldx, W, Y, ldy, off, gather, E, max_rows, N, K, S, ysplit, bm, s);
+    big_moe_bm<EPI_NONE, true>(X, ldx, W, Y, ldy, off, gather, E, max_rows, N, K, S, ysplit, bm, epi_arg, s);
   else
-    big_moe_bm<EPI_NONE, false>(X, ldx, W, Y, ldy, off, gather, E, max_rows, N, K, S, ysplit, bm, s);
+    big_moe_bm<EPI_NONE, false>(X, ldx, W, Y, ldy, off, gather, E, max_rows, N, K, S, ysplit, bm, epi_arg, s);
   return 0;
 }
 

@@ -4,7 +4,22 @@
 
 namespace xot {
 
-enum { EPI_NONE = 0, EPI_RESID = 1, EPI_SILU = 2 };
+enum { EPI_NONE = 0, EPI_RESID = 1, EPI_SILU = 2, EPI_CLAMP_GLU = 3 };
+
+// epilogues that turn a (gate, up) column pair into one output column
+constexpr bool epi_is_glu(int epi) { return epi == EPI_SILU || epi == EPI_CLAMP_GLU; }
+
+// silu(g) u, or the clamped form: g' sigmoid(1.702 g') (u' + 1) with g' = min(g, limit), u' = clamp(u, -limit, limit)
+template <int EPI>
+__device__ __forceinline__ float glu_pair(float g, float u, float limit) {
+  if constexpr (EPI == EPI_CLAMP_GLU) {
+    g = fminf(g, limit);
+    u = fminf(fmaxf(u, -limit), limit);
+    return g / (1.0f + __expf(-1.702f * g)) * (u + 1.0f);
+  } else {
+    return silu(g) * u;
+  }
+}
 
 typedef __attribute__((address_space(3))) void* lds_ptr_t;
 typedef __attribute__((address_space(1))) void* glb_ptr_t;

@@ -2,7 +2,8 @@
 // Mamba-2 (SSD) mixer's element-wise stages, non-gated feed-forward activations and the routed experts' sum.
 //
 //   gated_postnorm      x <- rms_norm(alpha x + y * sigmoid(gate + b)) * w, and its copy in the GEMM operand dtype
-//   qk_norm_rope_store  q / k / v biases, partial rotate-half RoPE, per-head RMS division, paged write of k and v
+//   qk_norm_rope_store  q / k / v biases, weighted RMS norm over the whole q (k) projection, partial rotate-half RoPE,
+//                       per-head RMS division, paged write of k and v
 //   kv_pool_update      mean key / value of every block of `pool` tokens that the step completed -> pooled caches
 //   attn_window_pool    softmax attention over [window tokens | pooled blocks before the window | sink]: a workgroup per
 //                       (token, head) for any sizes and fp32; an MFMA kernel for bf16 prompt portions
@@ -49,14 +50,17 @@ __global__ void gated_postnorm_k(float* __restrict__ x, const float* __restrict_
   }
 }
 
-// ------------------------------------------------------------------ biases + RoPE + per-head RMS division + paged write
+// ------------------------------------------------------------------ biases + norms + RoPE + paged write
 // cos_sin [rows, R]: row p = [cos(p f_0 .. f_{R/2-1}) | sin(...)].  Pair (i, i + R/2), i < R/2; dims >= R pass.
+// q_norm [H d] / k_norm [G d]: all of a token's q (k) numbers are first divided by their common RMS and weighted.
 // A wave per q / k head (d <= 256: four dims a lane); the values are written by all threads afterwards.
 template <typename AT>
 __global__ __launch_bounds__(256) void qk_norm_rope_store_k(
     const float* __restrict__ P, int ldp, const float* __restrict__ bias, int q_off, int k_off, int v_off, int H, int G,
     int d, int dv, int R, const int* __restrict__ pos, const float* __restrict__ cos_sin, const int64_t* __restrict__ slots,
-    float eps, int qk_norm, AT* __restrict__ q_out, AT* __restrict__ k_cache, AT* __restrict__ v_cache, int Gv) {
+    float eps, int qk_norm, AT* __restrict__ q_out, AT* __restrict__ k_cache, AT* __restrict__ v_cache, int Gv,
+    const float* __restrict__ q_norm, const float* __restrict__ k_norm) {
+  __shared__ float red[8];
   const int t = blockIdx.x;
   const float* row = P + (int64_t)t * ldp;
   const float* cs = cos_sin + (int64_t)pos[t] * R;
@@ -64,10 +68,28 @@ __global__ __launch_bounds__(256) void qk_norm_rope_store_k(
   const int64_t slot = slots[t];
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, nw = blockDim.x >> 6;
   const int heads = H + (k_off >= 0 ? G : 0);
+  float rq = 1.0f, rk = 1.0f;  // 1 / RMS of the whole query / key projection
+  if (q_norm) {
+    auto inv_rms = [&](int off, int n) {
+      float ss = 0.0f;
+      for (int i = threadIdx.x; i < n; i += blockDim.x) {
+        const float a = row[off + i] + (bias ? bias[off + i] : 0.0f);
+        ss += a * a;
+      }
+      return 1.0f / sqrtf(block_sum(ss, red) / (float)n + eps);
+    };
+    rq = inv_rms(q_off, H * d);
+    if (k_off >= 0) rk = inv_rms(k_off, G * d);
+  }
   for (int head = wave; head < heads; head += nw) {
     const bool isq = head < H;
     const int c0 = isq ? q_off + head * d : k_off + (head - H) * d;
-    auto at = [&](int i) { return row[c0 + i] + (bias ? bias[c0 + i] : 0.0f); };
+    const float* wn = !q_norm ? nullptr : isq ? q_norm + head * d : k_norm + (head - H) * d;
+    const float rn = isq ? rq : rk;
+    auto at = [&](int i) {
+      const float a = row[c0 + i] + (bias ? bias[c0 + i] : 0.0f);
+      return wn ? a * rn * wn[i] : a;
+    };
     float v[4];
     float ss = 0.0f;
 #pragma unroll
@@ -147,18 +169,26 @@ __global__ void kv_pool_update_k(const AT* __restrict__ k_cache, const AT* __res
 // A query at position i sees the tokens j with 0 <= i - j < window (window 0: all j <= i) and the pooled blocks b with
 // b pool + pool - 1 <= i - window; the softmax's denominator also holds exp(sink[head]).
 //
+// chunk > 0: only tokens of the query's own block of `chunk` positions are seen.
+//
 // Workgroup per (token, REP query heads of one kv head) (any d, dv <= 256, bf16 or fp32), WATT_WAVES waves: the key
 // tiles are dealt to the waves in turn; a lane loads a key row once and scores it against the REP heads, and a V^T run
 // of 8 keys once for the REP weighted sums.  A wave's running maxima start at -inf (wave 0: at the sinks' logits with
 // denominators of one); at the end the waves' (maximum, denominator, sums) are merged through LDS.
 constexpr int WATT_WAVES = 8;
 
+// the first token a query at position pos sees
+__device__ __forceinline__ int first_key(int pos, int window, int chunk) {
+  const int lo = window > 0 ? max(0, pos - window + 1) : 0;
+  return chunk > 0 ? max(lo, pos - pos % chunk) : lo;
+}
+
 template <typename AT, typename OT, int REP>
 __global__ __launch_bounds__(64 * WATT_WAVES) void attn_window_pool_k(
     const AT* __restrict__ q, const AT* __restrict__ k_cache, const AT* __restrict__ v_cache, const AT* __restrict__ kp,
     const AT* __restrict__ vp, const int* __restrict__ block_tables, int width, const int* __restrict__ cu_q,
     const int* __restrict__ ctx_lens, int B, const float* __restrict__ sink, float scale, int window, int pool, int per,
-    OT* __restrict__ out, int ldo, int H, int G, int d, int dv, int Gv) {
+    OT* __restrict__ out, int ldo, int H, int G, int d, int dv, int Gv, int chunk) {
   constexpr int TILE = REP >= 8 ? 128 : 256;
   extern __shared__ float sm[];
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
@@ -183,7 +213,7 @@ __global__ __launch_bounds__(64 * WATT_WAVES) void attn_window_pool_k(
 #pragma unroll
     for (int c = 0; c < 4; ++c) acc[r][c] = 0.0f;
   }
-  const int lo = window > 0 ? max(0, pos - window + 1) : 0;
+  const int lo = first_key(pos, window, chunk);
   const int nbv = (pool > 0 && window > 0 && pos - window + 1 >= pool) ? (pos - window + 1) / pool : 0;
 
   auto score = [&](const AT* kr, float* s) {
@@ -333,7 +363,8 @@ __global__ __launch_bounds__(64 * WATT_WAVES) void attn_window_pool_k(
   }
 }
 
-// MFMA kernel (bf16 caches; key size 32 NK, value size 32 NV; output bf16 or fp32): a workgroup owns 128 consecutive queries of one (sequence, head), 32 per wave, and
+// MFMA kernel (bf16 caches; key size 32 NK, value size 32 NV -- RAG: key / value sizes d <= 32 NK, dv <= 32 NV that are
+// multiples of 8, the tiles filled up with zeros --; output bf16 or fp32): a workgroup owns 128 consecutive queries of one (sequence, head), 32 per wave, and
 // walks first the pooled blocks that its last query sees, then the tokens from its first query's window on, a tile of
 // KT keys at a time: the K rows and V^T runs of the tile are staged in LDS and shared by the four waves (pooled
 // entries are gathered row by row and their values transposed on the way in).  Scores are computed transposed,
@@ -342,17 +373,18 @@ __global__ __launch_bounds__(64 * WATT_WAVES) void attn_window_pool_k(
 // denominators), and the exponentials, rounded to bf16, are as they lie the B operand of O^T += V^T P^T, whose k slots
 // (g, j) are read as keys {4g .. 4g+3, 16+4g .. 16+4g+3} on both operands.  Scores, maxima and sums are fp32 (base-2
 // exponentials of scores scaled by log2 e); the sink's logit starts the running maximum with a denominator of one.
-template <int NK, int NV, typename OT>
+template <int NK, int NV, typename OT, bool RAG>
 __global__ __launch_bounds__(256) void attn_window_pool_mfma_k(
     const uint16_t* __restrict__ q, const uint16_t* __restrict__ k_cache, const uint16_t* __restrict__ v_cache,
     const uint16_t* __restrict__ kp, const uint16_t* __restrict__ vp, const int* __restrict__ block_tables, int width,
     const int* __restrict__ cu_q, const int* __restrict__ ctx_lens, const float* __restrict__ sink, float scale, int window,
-    int pool, int per, OT* __restrict__ out, int ldo, int H, int G, int Gv) {
-  // key size D = 32 NK, value size DV = 32 NV (pooled blocks: NK == NV); G / Gv neighbouring key heads share a value head
+    int pool, int per, OT* __restrict__ out, int ldo, int H, int G, int Gv, int chunk, int d_rt, int dv_rt) {
+  // key size D = 32 NK, value size DV = 32 NV (pooled blocks: NK == NV, not RAG); G / Gv neighbouring key heads share a value head
   constexpr int D = NK * 32, DV = NV * 32, ND = NV * 2, QT = 2;
   constexpr int KT = (D > 192 || DV > 192) ? 32 : 64;  // keys per tile (a page holds a whole number of tiles)
   constexpr int KP = D + 8, VP = KT + 8;
   constexpr float L2E = 1.4426950408889634f;
+  const int d = RAG ? d_rt : D, dv = RAG ? dv_rt : DV;
   __shared__ __attribute__((aligned(16))) uint16_t sK[KT][KP], sV[DV][VP];
   const int b = blockIdx.x, h = blockIdx.z;
   const int wave = threadIdx.x >> 6, l = threadIdx.x & 63, c = l & 15, g4 = l >> 4;
@@ -367,17 +399,19 @@ __global__ __launch_bounds__(256) void attn_window_pool_mfma_k(
   // pooled blocks a query at position p sees: those that end at or before p - window
   auto blocks_seen = [&](int p) { return (pool > 0 && p - window + 1 >= pool) ? (p - window + 1) / pool : 0; };
   s16x8 qf[QT][NK];
-  int qpos[QT], qnb[QT];
+  int qpos[QT], qlo[QT], qnb[QT];  // position, first token seen, pooled blocks seen
   float m[QT], lsum[QT];
 #pragma unroll
   for (int qt = 0; qt < QT; ++qt) {
     const int local = qt * 16 + c;
     const bool ok = local < nq;
     qpos[qt] = pos0 + local;
+    qlo[qt] = first_key(qpos[qt], window, chunk);
     qnb[qt] = blocks_seen(qpos[qt]);
-    const uint16_t* qp = q + ((int64_t)(t0 + q0 + local) * H + h) * D + 8 * g4;
+    const uint16_t* qp = q + ((int64_t)(t0 + q0 + local) * H + h) * d + 8 * g4;
 #pragma unroll
-    for (int ks = 0; ks < NK; ++ks) qf[qt][ks] = ok ? ld16(qp + ks * 32) : s16x8{0, 0, 0, 0, 0, 0, 0, 0};
+    for (int ks = 0; ks < NK; ++ks)
+      qf[qt][ks] = ok && (!RAG || ks * 32 + 8 * g4 < d) ? ld16(qp + ks * 32) : s16x8{0, 0, 0, 0, 0, 0, 0, 0};
     m[qt] = sink ? sink[h] * L2E : -INFINITY;
     lsum[qt] = (sink && g4 == 0) ? 1.0f : 0.0f;  // (partial denominators: one of the query's four lanes counts the sink)
   }
@@ -391,6 +425,8 @@ __global__ __launch_bounds__(256) void attn_window_pool_mfma_k(
   const int wlast = ctx - qlen + wq0 + min(128, qlen - wq0) - 1;  // the workgroup's last query
   const int wpos0 = ctx - qlen + wq0;
   const int last = active ? pos0 + nq - 1 : -1;                  // the wave's last query
+  // the first token that the wave's first / last query sees
+  const int k_first = first_key(pos0, window, chunk), k_last = active ? first_key(last, window, chunk) : 0;
   constexpr int NCHUNK = KT * (D / 8), NCH = (NCHUNK + 255) / 256;
   constexpr int NCHUNKV = KT * (DV / 8), NCHV = (NCHUNKV + 255) / 256;
   s16x8 rk[NCH], rv[NCHV];
@@ -405,9 +441,8 @@ __global__ __launch_bounds__(256) void attn_window_pool_mfma_k(
         if (!active || kb >= blocks_seen(last)) continue;  // (wave-uniform) none of these blocks is seen by this wave
         full = kb + 32 <= blocks_seen(pos0);
       } else {
-        const int k_lo = window > 0 ? max(0, pos0 - window + 1) : 0;
-        if (!active || kb > last || kb + 31 < k_lo) continue;
-        full = kb + 31 <= pos0 && (window <= 0 || kb > last - window);
+        if (!active || kb > last || kb + 31 < k_first) continue;
+        full = kb + 31 <= pos0 && kb >= k_last;
       }
       f32x4 s[2][QT];
 #pragma unroll
@@ -433,7 +468,7 @@ __global__ __launch_bounds__(256) void attn_window_pool_mfma_k(
             float t = s[kt][qt][r] * sc2;
             if (!full) {
               const int kpos = kb + kt * 16 + 4 * g4 + r;
-              const bool vis = pooled ? kpos < qnb[qt] : (kpos <= qpos[qt] && (window <= 0 || qpos[qt] - kpos < window));
+              const bool vis = pooled ? kpos < qnb[qt] : (kpos <= qpos[qt] && kpos >= qlo[qt]);
               t = vis ? t : -INFINITY;
             }
             s[kt][qt][r] = t;
@@ -474,7 +509,7 @@ __global__ __launch_bounds__(256) void attn_window_pool_mfma_k(
   };
 
   // ---- pooled blocks [0, nbw): rows gathered from the pages that hold them, values transposed into sV
-  const int nbw = NK == NV ? blocks_seen(wlast) : 0;
+  const int nbw = NK == NV && !RAG ? blocks_seen(wlast) : 0;
   for (int tb = 0; tb < nbw; tb += KT) {
     __syncthreads();  // the previous tile has been consumed
 #pragma unroll
@@ -495,7 +530,7 @@ __global__ __launch_bounds__(256) void attn_window_pool_mfma_k(
   }
 
   // ---- tokens from the first query's window on
-  const int t_lo = (window > 0 ? max(0, wpos0 - window + 1) : 0) & ~(KT - 1);
+  const int t_lo = first_key(wpos0, window, chunk) & ~(KT - 1);
   auto fetch = [&](int tb) {
     const int64_t pg = (int64_t)bt[tb >> 6] * G + gk, pgv = (int64_t)bt[tb >> 6] * Gv + gv;
     const int koff = tb & 63;
@@ -504,14 +539,14 @@ __global__ __launch_bounds__(256) void attn_window_pool_mfma_k(
       const int ch = threadIdx.x + 256 * j;
       if (NCHUNK % 256 != 0 && ch >= NCHUNK) break;
       const int row = ch / (D / 8), cc = ch - row * (D / 8);
-      rk[j] = ld16(k_cache + ((pg * PAGE_TOK) + koff + row) * D + cc * 8);
+      rk[j] = !RAG || cc * 8 < d ? ld16(k_cache + ((pg * PAGE_TOK) + koff + row) * d + cc * 8) : s16x8{0, 0, 0, 0, 0, 0, 0, 0};
     }
 #pragma unroll
     for (int j = 0; j < NCHV; ++j) {
       const int ch = threadIdx.x + 256 * j;
       if (NCHUNKV % 256 != 0 && ch >= NCHUNKV) break;
       const int vrow = ch / (KT / 8), vc = ch - vrow * (KT / 8);
-      rv[j] = ld16(v_cache + (pgv * DV + vrow) * PAGE_TOK + koff + vc * 8);
+      rv[j] = !RAG || vrow < dv ? ld16(v_cache + (pgv * dv + vrow) * PAGE_TOK + koff + vc * 8) : s16x8{0, 0, 0, 0, 0, 0, 0, 0};
     }
   };
   fetch(t_lo);
@@ -542,9 +577,10 @@ __global__ __launch_bounds__(256) void attn_window_pool_mfma_k(
     ls += __shfl_xor(ls, 32, 64);
     if (qt * 16 + c >= nq) continue;
     const float inv = ls > 0.0f ? 1.0f / ls : 0.0f;
-    OT* op = out + (int64_t)(t0 + q0 + qt * 16 + c) * ldo + h * DV + 4 * g4;
+    OT* op = out + (int64_t)(t0 + q0 + qt * 16 + c) * ldo + h * dv + 4 * g4;
 #pragma unroll
     for (int db = 0; db < ND; ++db) {
+      if (RAG && db * 16 + 4 * g4 >= dv) continue;
       if constexpr (sizeof(OT) == 4) {
         *reinterpret_cast<f32x4*>(op + db * 16) = f32x4{o[qt][db][0] * inv, o[qt][db][1] * inv, o[qt][db][2] * inv, o[qt][db][3] * inv};
       } else {
@@ -770,7 +806,8 @@ void check_kv(const at::Tensor& k_cache, const at::Tensor& v_cache, at::ScalarTy
 void qk_norm_rope_store(const at::Tensor& P, const c10::optional<at::Tensor>& bias, int64_t q_off, int64_t k_off,
                         int64_t v_off, int64_t H, int64_t G, int64_t d, int64_t dv, int64_t R, const at::Tensor& pos,
                         const at::Tensor& cos_sin, const at::Tensor& slots, double eps, bool qk_norm, at::Tensor& q_out,
-                        at::Tensor& k_cache, at::Tensor& v_cache) {
+                        at::Tensor& k_cache, at::Tensor& v_cache, const c10::optional<at::Tensor>& q_norm,
+                        const c10::optional<at::Tensor>& k_norm) {
   const int ldp = ld_of(P, "P");
   const int64_t T = P.size(0);
   int64_t Gv = G;
@@ -796,18 +833,30 @@ void qk_norm_rope_store(const at::Tensor& P, const c10::optional<at::Tensor>& bi
     bp = bias->data_ptr<float>();
   }
   MCHECK(q_out.is_cuda() && is_act(q_out) && q_out.is_contiguous() && q_out.numel() == T * H * d, "q_out must be [T, H, d]");
+  const float *qn = nullptr, *kn = nullptr;
+  if (q_norm.has_value()) {
+    f32c(*q_norm, "q_norm");
+    MCHECK(q_norm->numel() == H * d, "q_norm must weigh every query number");
+    qn = q_norm->data_ptr<float>();
+    if (k_off >= 0) {
+      MCHECK(k_norm.has_value(), "a norm over the queries comes with one over the keys");
+      f32c(*k_norm, "k_norm");
+      MCHECK(k_norm->numel() == G * d, "k_norm must weigh every key number");
+      kn = k_norm->data_ptr<float>();
+    }
+  }
   // positions and slots are checked on the host by their producer (the block manager hands out slots < pages * 64
   // and the runner bounds positions by the table's rows)
   if (q_out.scalar_type() == at::kBFloat16)
     qk_norm_rope_store_k<uint16_t><<<T, 256, 0, stream()>>>(
         P.data_ptr<float>(), ldp, bp, (int)q_off, (int)k_off, (int)v_off, (int)H, (int)G, (int)d, (int)dv, (int)R,
         pos.data_ptr<int>(), cos_sin.data_ptr<float>(), slots.data_ptr<int64_t>(), (float)eps, (int)qk_norm,
-        (uint16_t*)q_out.data_ptr(), (uint16_t*)k_cache.data_ptr(), (uint16_t*)v_cache.data_ptr(), (int)Gv);
+        (uint16_t*)q_out.data_ptr(), (uint16_t*)k_cache.data_ptr(), (uint16_t*)v_cache.data_ptr(), (int)Gv, qn, kn);
   else
     qk_norm_rope_store_k<float><<<T, 256, 0, stream()>>>(
         P.data_ptr<float>(), ldp, bp, (int)q_off, (int)k_off, (int)v_off, (int)H, (int)G, (int)d, (int)dv, (int)R,
         pos.data_ptr<int>(), cos_sin.data_ptr<float>(), slots.data_ptr<int64_t>(), (float)eps, (int)qk_norm,
-        q_out.data_ptr<float>(), k_cache.data_ptr<float>(), v_cache.data_ptr<float>(), (int)Gv);
+        q_out.data_ptr<float>(), k_cache.data_ptr<float>(), v_cache.data_ptr<float>(), (int)Gv, qn, kn);
 }
 
 void check_pools(const at::Tensor& k_cache, const at::Tensor& kp, const at::Tensor& vp, int64_t pool, int64_t G, int64_t d,
@@ -850,22 +899,24 @@ void kv_pool_update(const at::Tensor& k_cache, const at::Tensor& v_cache, at::Te
         per, (int)G, (int)d, (int)dv);
 }
 
-template <int NK, int NV, typename OT>
+template <int NK, int NV, typename OT, bool RAG>
 void launch_wattn_mfma(dim3 grid, const at::Tensor& q, const at::Tensor& k_cache, const at::Tensor& v_cache, const uint16_t* kp,
                        const uint16_t* vp, const at::Tensor& block_tables, const at::Tensor& cu_q, const at::Tensor& ctx_lens,
-                       const float* sink, float scale, int window, int pool, int per, at::Tensor& out, int ldo, int H, int G) {
-  attn_window_pool_mfma_k<NK, NV, OT><<<grid, 256, 0, stream()>>>(
+                       const float* sink, float scale, int window, int pool, int per, at::Tensor& out, int ldo, int H, int G,
+                       int chunk) {
+  attn_window_pool_mfma_k<NK, NV, OT, RAG><<<grid, 256, 0, stream()>>>(
       (const uint16_t*)q.data_ptr(), (const uint16_t*)k_cache.data_ptr(), (const uint16_t*)v_cache.data_ptr(), kp, vp,
       block_tables.data_ptr<int>(), (int)block_tables.size(1), cu_q.data_ptr<int>(), ctx_lens.data_ptr<int>(), sink, scale,
-      window, pool, per, (OT*)out.data_ptr(), ldo, H, G, (int)v_cache.size(1));
+      window, pool, per, (OT*)out.data_ptr(), ldo, H, G, (int)v_cache.size(1), chunk, (int)k_cache.size(3),
+      (int)v_cache.size(2));
 }
 
 // max_qlen: the longest run of new tokens of one sequence in this step (below 16: single decoded tokens and short
-// portions -> the wave-per-token kernel; the MFMA kernel takes bf16 with d == dv in {32, 64, 128}).
+// portions -> the wave-per-token kernel; the MFMA kernel takes bf16 with sizes up to 128 that are multiples of 8).
 void attn_window_pool(const at::Tensor& q, const at::Tensor& k_cache, const at::Tensor& v_cache,
                       const c10::optional<at::Tensor>& kp, const c10::optional<at::Tensor>& vp, const at::Tensor& block_tables,
                       const at::Tensor& cu_q, const at::Tensor& ctx_lens, const c10::optional<at::Tensor>& sink, double scale,
-                      int64_t window, int64_t pool, at::Tensor& out, int64_t max_qlen) {
+                      int64_t window, int64_t pool, at::Tensor& out, int64_t max_qlen, int64_t chunk) {
   MCHECK(q.is_cuda() && is_act(q) && q.is_contiguous() && q.dim() == 3, "q must be contiguous [T, H, d]");
   const int64_t T = q.size(0), H = q.size(1), d = q.size(2), B = ctx_lens.numel();
   if (T == 0 || B == 0) return;
@@ -873,7 +924,7 @@ void attn_window_pool(const at::Tensor& q, const at::Tensor& k_cache, const at::
   const int64_t G = k_cache.size(1), dv = v_cache.size(2);
   check_kv(k_cache, v_cache, q.scalar_type(), G, d, dv);
   MCHECK(G > 0 && H % G == 0 && d <= 256 && dv <= 256, "head counts / sizes (at most 256)");
-  MCHECK(window >= 0 && pool >= 0, "window / pool must not be negative");
+  MCHECK(window >= 0 && pool >= 0 && chunk >= 0 && (pool == 0 || chunk == 0), "window / pool / chunk must not be negative (and no pool beside a chunk)");
   int per = 0;
   const bool pooled = pool > 0 && window > 0;
   if (pooled) {
@@ -895,25 +946,34 @@ void attn_window_pool(const at::Tensor& q, const at::Tensor& k_cache, const at::
   MCHECK(!pooled || Gv == G, "pooled blocks need a value head per key head");
   const int ldo = act_ld(out, T, H * dv, "out");
   const bool o32 = out.scalar_type() == at::kFloat;
-  // the MFMA kernel: bf16 caches, runs of 16 tokens or more, value size = key size in {32, 64, 128} (bf16 or fp32 output)
-  // or twice the key size in {32, 64} with fp32 output (differential attention's maps); pooled blocks need equal sizes
-  const bool same = d == dv && (d == 32 || d == 64 || d == 128), twice = dv == 2 * d && (d == 32 || d == 64) && o32 && !pooled;
-  if (q.scalar_type() == at::kBFloat16 && max_qlen >= 16 && (same || twice) && ldo % 4 == 0 && WATT_MFMA) {
+  // the MFMA kernel: bf16 caches, runs of 16 tokens or more, value size = key size in {32, 64, 96, 128} (bf16 or fp32 output)
+  // or twice the key size in {32, 64} with fp32 output (differential attention's maps), or (bf16 output, no pooled blocks)
+  // any two sizes up to 128 that are multiples of 8
+  const bool same = d == dv && d % 32 == 0 && d <= 128 && (d != 96 || !o32);
+  const bool twice = dv == 2 * d && (d == 32 || d == 64) && o32 && !pooled;
+  const bool ragged = !same && !o32 && !pooled && d % 8 == 0 && dv % 8 == 0 && d <= 128 && dv <= 128;
+  if (q.scalar_type() == at::kBFloat16 && max_qlen >= 16 && (same || twice || ragged) && ldo % 4 == 0 && WATT_MFMA) {
     const dim3 grid((unsigned)B, (unsigned)((max_qlen + 127) / 128), (unsigned)H);
     const uint16_t* kpp = pooled ? (const uint16_t*)kp->data_ptr() : nullptr;
     const uint16_t* vpp = pooled ? (const uint16_t*)vp->data_ptr() : nullptr;
     const int pl = pooled ? (int)pool : 0;
-#define WATT_MFMA_GO(NK, NV, OT)                                                                                            \
-  launch_wattn_mfma<NK, NV, OT>(grid, q, k_cache, v_cache, kpp, vpp, block_tables, cu_q, ctx_lens, sp, (float)scale,       \
-                                (int)window, pl, per, out, ldo, (int)H, (int)G)
-    if (twice && d == 32) WATT_MFMA_GO(1, 2, float);
-    else if (twice) WATT_MFMA_GO(2, 4, float);
-    else if (d == 32 && o32) WATT_MFMA_GO(1, 1, float);
-    else if (d == 32) WATT_MFMA_GO(1, 1, uint16_t);
-    else if (d == 64 && o32) WATT_MFMA_GO(2, 2, float);
-    else if (d == 64) WATT_MFMA_GO(2, 2, uint16_t);
-    else if (o32) WATT_MFMA_GO(4, 4, float);
-    else WATT_MFMA_GO(4, 4, uint16_t);
+    const int64_t big = (std::max(d, dv) + 31) / 32;
+#define WATT_MFMA_GO(NK, NV, OT, ...)                                                                                       \
+  launch_wattn_mfma<NK, NV, OT, ##__VA_ARGS__>(grid, q, k_cache, v_cache, kpp, vpp, block_tables, cu_q, ctx_lens, sp, (float)scale,       \
+                                (int)window, pl, per, out, ldo, (int)H, (int)G, (int)chunk)
+    if (ragged && big == 1) WATT_MFMA_GO(1, 1, uint16_t, true);
+    else if (ragged && big == 2) WATT_MFMA_GO(2, 2, uint16_t, true);
+    else if (ragged && big == 3) WATT_MFMA_GO(3, 3, uint16_t, true);
+    else if (ragged) WATT_MFMA_GO(4, 4, uint16_t, true);
+    else if (twice && d == 32) WATT_MFMA_GO(1, 2, float, false);
+    else if (twice) WATT_MFMA_GO(2, 4, float, false);
+    else if (d == 32 && o32) WATT_MFMA_GO(1, 1, float, false);
+    else if (d == 32) WATT_MFMA_GO(1, 1, uint16_t, false);
+    else if (d == 64 && o32) WATT_MFMA_GO(2, 2, float, false);
+    else if (d == 64) WATT_MFMA_GO(2, 2, uint16_t, false);
+    else if (d == 96) WATT_MFMA_GO(3, 3, uint16_t, false);
+    else if (o32) WATT_MFMA_GO(4, 4, float, false);
+    else WATT_MFMA_GO(4, 4, uint16_t, false);
 #undef WATT_MFMA_GO
     return;
   }
@@ -933,7 +993,7 @@ void attn_window_pool(const at::Tensor& q, const at::Tensor& k_cache, const at::
       pooled ? (const AT*)kp->data_ptr() : nullptr, pooled ? (const AT*)vp->data_ptr() : nullptr,                          \
       block_tables.data_ptr<int>(), (int)block_tables.size(1), cu_q.data_ptr<int>(), ctx_lens.data_ptr<int>(), (int)B, sp, \
       (float)scale, (int)window, pooled ? (int)pool : 0, per, (OT*)out.data_ptr(), ldo, (int)H, (int)G, (int)d, (int)dv,  \
-      (int)Gv)
+      (int)Gv, (int)chunk)
 #define WATT_REP(AT, OT)                   \
   switch (rep) {                           \
     case 8: WATT_GO(AT, OT, 8); break;     \

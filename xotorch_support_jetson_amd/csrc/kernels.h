@@ -94,11 +94,11 @@ void launch_splitk_resid_rmsnorm(const float* ws, int S, const uint16_t* bias, u
 // grouped expert GEMM on gemm_big tiles (bm = 128 or 256 rows per tile; large per-expert row counts)
 int launch_gemm_moe_big(const uint16_t* X, int ldx, const uint16_t* W, void* Y, int ldy, bool out_f32, int epi,
                         const int* off, const int* gather, int E, int max_rows, int N, int K, int S, long ysplit,
-                        int bm, hipStream_t s);
+                        int bm, float epi_arg, hipStream_t s);
 // grouped GEMM over experts: rows of expert e are off[e]..off[e+1] (slot order), W is [E][N][K]
 int launch_gemm_moe(const uint16_t* X, int ldx, const uint16_t* W, void* Y, int ldy, bool out_f32, int epi,
                     const int* off, const int* gather, int E, int max_rows, int N, int K, bool wshuf, int S,
-                    long ysplit, hipStream_t s);
+                    long ysplit, float epi_arg, hipStream_t s);
 void launch_splitk_silu(const float* ws, int S, int M, int N, uint16_t* y, hipStream_t s);
 int launch_moe_combine_norm(const float* y, const int32_t* slot_of, const float* topw, uint16_t* h,
                             const uint16_t* lnw, uint16_t* out, int T, int k, int D, int S, long ysplit, float eps,

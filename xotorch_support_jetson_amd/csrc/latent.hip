@@ -30,17 +30,18 @@ constexpr float LOG2E_F = 1.4426950408889634f;
 // ------------------------------------------------------------------ residual add of a normed sublayer result + next norm
 // norm of one row held in global memory: v / rms(v) * w, or with a bias the layer norm (v - mean) / sqrt(var + eps) * w + b
 // (the variance as the mean of the squared deviations, in a pass of its own).  Returns (shift, scale).
-__device__ __forceinline__ void row_norm_stats(const float* v, int D, bool center, float eps, float* red, float* shift,
-                                               float* scale) {
+// add (or null): one number per column, added to v first.
+__device__ __forceinline__ void row_norm_stats(const float* v, const float* add, int D, bool center, float eps, float* red,
+                                               float* shift, float* scale) {
   float mean = 0.0f;
   if (center) {
     float s = 0.0f;
-    for (int i = threadIdx.x; i < D; i += blockDim.x) s += v[i];
+    for (int i = threadIdx.x; i < D; i += blockDim.x) s += v[i] + (add ? add[i] : 0.0f);
     mean = block_sum(s, red) / D;
   }
   float ss = 0.0f;
   for (int i = threadIdx.x; i < D; i += blockDim.x) {
-    const float c = v[i] - mean;
+    const float c = v[i] + (add ? add[i] : 0.0f) - mean;
     ss += c * c;
   }
   ss = block_sum(ss, red);
@@ -52,20 +53,24 @@ template <typename AT>
 __global__ __launch_bounds__(256) void sandwich_add_norm_k(float* __restrict__ x, const float* __restrict__ y, int ldy,
                                                            const float* __restrict__ wb, const float* __restrict__ bb,
                                                            const float* __restrict__ wn, const float* __restrict__ bn,
-                                                           float mult, float eps, AT* __restrict__ out, int ldo, int D) {
+                                                           const float* __restrict__ yb, float mult, float eps,
+                                                           AT* __restrict__ out, int ldo, int D) {
   __shared__ float red[8];
   const int64_t t = blockIdx.x;
   float* xr = x + t * D;
   if (y) {
     const float* yr = y + t * ldy;
     float mu, r;
-    row_norm_stats(yr, D, bb != nullptr, eps, red, &mu, &r);
-    for (int i = threadIdx.x; i < D; i += blockDim.x) xr[i] += mult * ((yr[i] - mu) * r * wb[i] + (bb ? bb[i] : 0.0f));
+    row_norm_stats(yr, yb, D, bb != nullptr, eps, red, &mu, &r);
+    for (int i = threadIdx.x; i < D; i += blockDim.x) 
+      xr[i] += mult * ((yr[i] + (yb ? yb[i] : 0.0f) - mu) * r * wb[i] + (bb ? bb[i] : 0.0f));
   }
   if (wn) {  // (a thread re-reads the elements it wrote itself)
     float mu, r;
-    row_norm_stats(xr, D, bn != nullptr, eps, red, &mu, &r);
+    row_norm_stats(xr, nullptr, D, bn != nullptr, eps, red, &mu, &r);
     for (int i = threadIdx.x; i < D; i += blockDim.x) stf(out + t * ldo + i, (xr[i] - mu) * r * wn[i] + (bn ? bn[i] : 0.0f));
+  } else if (out) {
+    for (int i = threadIdx.x; i < D; i += blockDim.x) stf(out + t * ldo + i, xr[i]);
   }
 }
 
@@ -566,7 +571,8 @@ template <typename AT, int R>
 __global__ __launch_bounds__(256) void sandwich_add_norm_reg_k(float* __restrict__ x, const float* __restrict__ y, int ldy,
                                                                const float* __restrict__ wb, const float* __restrict__ bb,
                                                                const float* __restrict__ wn, const float* __restrict__ bn,
-                                                               float mult, float eps, AT* __restrict__ out, int ldo, int D) {
+                                                               const float* __restrict__ yb, float mult, float eps,
+                                                               AT* __restrict__ out, int ldo, int D) {
   __shared__ float red[8];
   const int64_t t = blockIdx.x;
   float* xr = x + t * D;
@@ -601,7 +607,7 @@ __global__ __launch_bounds__(256) void sandwich_add_norm_reg_k(float* __restrict
 #pragma unroll
     for (int r = 0; r < R; ++r) {
       const int i = threadIdx.x + 256 * r;
-      yv[r] = i < D ? yr[i] : 0.0f;
+      yv[r] = i < D ? yr[i] + (yb ? yb[i] : 0.0f) : 0.0f;
     }
     float mu, rs;
     stats(yv, bb != nullptr, &mu, &rs);
@@ -622,6 +628,12 @@ __global__ __launch_bounds__(256) void sandwich_add_norm_reg_k(float* __restrict
       const int i = threadIdx.x + 256 * r;
       if (i < D) stf(out + t * ldo + i, (xv[r] - mu) * rs * wn[i] + (bn ? bn[i] : 0.0f));
     }
+  } else if (out) {  // the stream itself, in the operand dtype
+#pragma unroll
+    for (int r = 0; r < R; ++r) {
+      const int i = threadIdx.x + 256 * r;
+      if (i < D) stf(out + t * ldo + i, xv[r]);
+    }
   }
 }
 
@@ -631,12 +643,13 @@ const bool LATT_MFMA = []() { const char* e = getenv("XOT_LATT_MFMA"); return !(
 
 void sandwich_add_norm(at::Tensor& x, const c10::optional<at::Tensor>& y, const c10::optional<at::Tensor>& wb,
                        const c10::optional<at::Tensor>& wn, double eps, const c10::optional<at::Tensor>& out,
-                       const c10::optional<at::Tensor>& bb, const c10::optional<at::Tensor>& bn, double mult) {
+                       const c10::optional<at::Tensor>& bb, const c10::optional<at::Tensor>& bn, double mult,
+                       const c10::optional<at::Tensor>& yb) {
   f32c(x, "x");
   MCHECK(x.dim() == 2, "x must be [T, D]");
   const int64_t T = x.size(0), D = x.size(1);
   if (T == 0) return;
-  const float *yp = nullptr, *bp = nullptr, *np = nullptr, *bbp = nullptr, *bnp = nullptr;
+  const float *yp = nullptr, *bp = nullptr, *np = nullptr, *bbp = nullptr, *bnp = nullptr, *ybp = nullptr;
   int ldy = 0, ldo = 0;
   if (bb.has_value()) {
     f32c(*bb, "bb");
@@ -647,6 +660,11 @@ void sandwich_add_norm(at::Tensor& x, const c10::optional<at::Tensor>& y, const 
     f32c(*bn, "bn");
     MCHECK(bn->numel() == D && wn.has_value(), "the next norm's bias must hold D numbers");
     bnp = bn->data_ptr<float>();
+  }
+  if (yb.has_value()) {
+    f32c(*yb, "yb");
+    MCHECK(yb->numel() == D && y.has_value(), "the result's bias must hold D numbers");
+    ybp = yb->data_ptr<float>();
   }
   if (y.has_value()) {
     ldy = ld_of(*y, "y");
@@ -661,14 +679,16 @@ void sandwich_add_norm(at::Tensor& x, const c10::optional<at::Tensor>& y, const 
   if (wn.has_value()) {
     f32c(*wn, "wn");
     MCHECK(wn->numel() == D && out.has_value(), "the next norm needs D weights and an output");
-    ldo = act_ld_min(*out, T, D, "out");
     np = wn->data_ptr<float>();
+  }
+  if (out.has_value()) {
+    ldo = act_ld_min(*out, T, D, "out");
     op = out->data_ptr();
     bf = out->scalar_type() == at::kBFloat16;
   }
-  if (!yp && !np) return;
+  if (!yp && !op) return;
 #define SAN_GO(KERNEL, AT)                                                                                              \
-  KERNEL<<<T, 256, 0, stream()>>>(x.data_ptr<float>(), yp, ldy, bp, bbp, np, bnp, (float)mult, (float)eps, (AT*)op, ldo, \
+  KERNEL<<<T, 256, 0, stream()>>>(x.data_ptr<float>(), yp, ldy, bp, bbp, np, bnp, ybp, (float)mult, (float)eps, (AT*)op, ldo, \
                                   (int)D)
 #define SAN_PICK(AT)                                                     \
   if (D <= 1024) SAN_GO((sandwich_add_norm_reg_k<AT, 4>), AT);           \

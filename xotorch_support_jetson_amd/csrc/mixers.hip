@@ -2,6 +2,7 @@
 //
 //   resid_scale_norm   x += s1 * y1 (+ s2 * y2) on the fp32 residual stream, then RMS norm with one scalar gain
 //   gelu_mul           gelu_tanh(gate) * up out of a fused projection's columns
+//   gelu_gather_mul    gelu_tanh(gate) * the token's slice of a table (per-layer side inputs)
 //   rope_kv_store      partial rotate-half RoPE on q and k, paged write of the rotated key and of the value
 //                      (the value may be the un-rotated key)
 //   attn_gated_chunk   chunk-local attention with sigmoid(score + bias[head]) weights, no normalisation: an MFMA
@@ -58,6 +59,21 @@ __global__ void gelu_mul_k(const float* __restrict__ P, int ldp, int gate_off, i
   const float z = P[t * ldp + gate_off + i], u = P[t * ldp + up_off + i];
   const float g = 0.5f * z * (1.0f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z)));
   stf(out + t * ldo + i, g * u);
+}
+
+// gelu_tanh(gate) * the token's slice of a table: out[t, i] = gelu(P[t, off + i]) * table[ids[t], col0 + i]
+template <typename AT>
+__global__ void gelu_gather_mul_k(const float* __restrict__ P, int ldp, int off, const AT* __restrict__ table, int64_t ldt,
+                                  int V, const int* __restrict__ ids, int col0, int n, AT* __restrict__ out, int ldo,
+                                  int64_t total) {
+  const int64_t idx = (int64_t)blockIdx.x * blockDim.x + threadIdx.x;
+  if (idx >= total) return;
+  const int64_t t = idx / n;
+  const int i = (int)(idx - t * n);
+  const float z = P[t * ldp + off + i];
+  const float e = ldf(table + (int64_t)min(max(ids[t], 0), V - 1) * ldt + col0 + i);
+  const float g = 0.5f * z * (1.0f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z)));
+  stf(out + t * ldo + i, g * e);
 }
 
 // ------------------------------------------------------------------ RoPE + paged key / value write
@@ -799,6 +815,31 @@ void gelu_mul(const at::Tensor& P, int64_t gate_off, int64_t up_off, int64_t F, 
                                                     out.data_ptr<float>(), ldo, total);
 }
 
+void gelu_gather_mul(const at::Tensor& P, int64_t off, const at::Tensor& table, const at::Tensor& ids, int64_t col0, int64_t n,
+                     at::Tensor& out) {
+  const int ldp = ld_of(P, "P");
+  const int64_t T = P.size(0);
+  cols_ok(P, off, n, "gate");
+  i32c(ids, "ids");
+  MCHECK(ids.numel() == T, "ids must hold one table row per token");
+  const int ldo = act_ld_min(out, T, n, "out");
+  MCHECK(table.is_cuda() && table.scalar_type() == out.scalar_type() && table.is_contiguous() && table.dim() == 2 &&
+             table.size(0) >= 1 && col0 >= 0 && col0 + n <= table.size(1),
+         "the table must be [V, >= col0 + n] of the output's dtype");
+  const int64_t total = T * n;
+  if (total == 0) return;
+  const int blocks = (int)((total + 255) / 256);
+  if (out.scalar_type() == at::kBFloat16)
+    gelu_gather_mul_k<uint16_t><<<blocks, 256, 0, stream()>>>(P.data_ptr<float>(), ldp, (int)off,
+                                                              (const uint16_t*)table.data_ptr(), table.size(1),
+                                                              (int)table.size(0), ids.data_ptr<int>(), (int)col0, (int)n,
+                                                              (uint16_t*)out.data_ptr(), ldo, total);
+  else
+    gelu_gather_mul_k<float><<<blocks, 256, 0, stream()>>>(P.data_ptr<float>(), ldp, (int)off, table.data_ptr<float>(),
+                                                           table.size(1), (int)table.size(0), ids.data_ptr<int>(), (int)col0,
+                                                           (int)n, out.data_ptr<float>(), ldo, total);
+}
+
 void rope_kv_store(const at::Tensor& P, int64_t q_off, int64_t k_off, int64_t v_off, int64_t H, int64_t G, int64_t d,
                    int64_t R, const at::Tensor& pos, const at::Tensor& cos_sin, const at::Tensor& slots, at::Tensor& q_out,
                    at::Tensor& k_cache, at::Tensor& v_cache) {
@@ -1090,6 +1131,7 @@ void gated_rmsnorm(const at::Tensor& o, const at::Tensor& w, const at::Tensor& P
 void bind_mixers(pybind11::module& m) {
   m.def("resid_scale_norm", &resid_scale_norm);
   m.def("gelu_mul", &gelu_mul);
+  m.def("gelu_gather_mul", &gelu_gather_mul);
   m.def("rope_kv_store", &rope_kv_store);
   m.def("attn_gated_chunk", &attn_gated_chunk);
   m.def("delta_prep", &delta_prep);

@@ -89,7 +89,7 @@ __global__ __launch_bounds__(1024) void moe_route_kernel(const float* __restrict
 // exclusive scan of the counts -> expert offsets, slot per (token, j), and the counters reset to zero for
 // the next launch (so the graph-captured sequence needs no memset).
 constexpr int MOE_DS_MAX_E = 256;
-constexpr int MOE_DS_MAX_G = 16;
+constexpr int MOE_DS_MAX_G = 32;
 constexpr int MOE_DS_EPL = MOE_DS_MAX_E / 64;  // experts per lane
 
 __global__ __launch_bounds__(256) void moe_topk_ds_kernel(const float* __restrict__ logits,

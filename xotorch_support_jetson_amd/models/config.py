@@ -70,7 +70,10 @@ class WindowAttnSpec:
   frequency scaling rot_scaling = (factor, low, high, original); qk_norm divides q and k by their RMS per head after
   the rotation.  kv_from >= 0: no key / value projections, the layer reads that layer's caches with its own queries
   and its own window / pool.  gate "elem": the heads' outputs times sigmoid of a projection of the mixer's input, element
-  by element."""
+  by element.  chunk > 0: a query sees only tokens of its own block of `chunk` positions, counted from the sequence's
+  start.  proj_norm: one weighted RMS norm over the whole query projection (and one over the whole key projection) before
+  the rotation.  rot_interleaved: rotation pairs (2i, 2i + 1) instead of (i, i + rot_dims / 2).  sink_one: one is added to
+  the softmax's denominator (a sink whose logit is zero).  out_bias: the output projection has a bias."""
   heads: int
   kv_heads: int
   dim: int
@@ -86,6 +89,11 @@ class WindowAttnSpec:
   sink: bool = True
   kv_from: int = -1
   gate: str = "none"  # none | elem
+  chunk: int = 0
+  proj_norm: bool = False
+  rot_interleaved: bool = False
+  sink_one: bool = False
+  out_bias: bool = False
 
 
 @dataclass(frozen=True)
@@ -137,13 +145,17 @@ class FeedForwardSpec:
   Gated kinds, W_down (a(W_gate h) * b(W_up h)): "clamped_glu": g = min(gate, limit), u = clamp(up, -limit, limit),
   g sigmoid(1.702 g) (u + 1); "silu_moe": `experts` SiLU-gated experts, scores = softmax of the router logits over
   all experts, the `top` largest chosen and weighted by their scores as they are (no renormalisation), plus
-  (shared_ff > 0) one ungated shared expert of the same form."""
-  kind: str  # polynorm | relu2_moe | clamped_glu | silu_moe
+  (shared_ff > 0) one ungated shared expert of the same form; "clamped_moe": experts of the clamped_glu form with `limit`
+  (the shared expert: `shared_limit`), softmax scores, the choice among the experts of the `keep` best of `groups` equal
+  groups of neighbours (a group's value: its largest score), weights as they are.
+  "relu2": act(z) = relu(z)^2."""
+  kind: str  # polynorm | relu2_moe | clamped_glu | silu_moe | clamped_moe | relu2
   ff: int
   experts: int = 0
   top: int = 0
   shared_ff: int = 0
-  limit: float = 0.0  # clamped_glu
+  limit: float = 0.0  # clamped_glu, clamped_moe
+  shared_limit: float = 0.0  # clamped_moe
   # relu2_moe routing.  "softmax_top": the rule above.  "sigmoid_groups": scores = sigmoid(logits); the choice is made on
   # scores + a learned correction, among the experts of the `keep` best of `groups` equal groups of neighbours (a
   # group's value: the sum of its two largest corrected scores); weights = the chosen experts' uncorrected scores over
@@ -199,6 +211,7 @@ class MixedLayerSpec:
   ffn: Optional[FeedForwardSpec] = None
   lattn: Optional[LatentAttnSpec] = None  # sandwich blocks
   dattn: Optional[DiffAttnSpec] = None  # sandwich blocks; a "parallel" layer there is wattn beside rec
+  side: int = 0  # size of the layer's per-token side input (a slice of a second embedding table), 0: none
 
   @property
   def kv_dims(self) -> Optional[tuple]:
@@ -231,7 +244,7 @@ class MixedLayerSpec:
 
 @dataclass(frozen=True)
 class ModelConfig:
-  model_type: str  # llama | qwen2 | mistral | mixtral | ... | tarepel | mogelix | nenizen
+  model_type: str  # llama | qwen2 | mistral | mixtral | ... | tarepel | mogelix | nenizen | kopalorn | torinex
   vocab_size: int
   hidden_size: int
   intermediate_size: int
@@ -295,6 +308,19 @@ class ModelConfig:
   norm_kind: str = "rms"  # rms | layer
   residual_mult: float = 1.0
   loop_input: str = "linear"  # linear | add
+  # sandwich blocks without the norms in front (Torinex): the sublayers read the stream itself, x += norm_b(sublayer(x))
+  input_norm: bool = True
+
+  @property
+  def side_dim(self) -> int:
+    """Columns per layer of the side-input table (0: the model has none)."""
+    return max([s.side for s in self.layer_specs] + [0]) if self.layer_specs else 0
+
+  @property
+  def hidden_width(self) -> int:
+    """Columns of the hidden state that travels between shards: the stream, and one more with the token's id when
+    later layers look it up again (side inputs)."""
+    return self.hidden_size + (1 if self.side_dim else 0)
 
   def layer_runs(self, layers=None) -> list:
     """[(layer, pass or -1)] in execution order for the given layers (default: all): a looped layer appears once per
@@ -391,7 +417,7 @@ class ModelConfig:
 
   def num_params(self) -> int:
     emb = self.vocab_size * self.hidden_size
-    layers = sum(self.params_per_layer(i) for i in range(self.num_layers))
+    layers = sum(self.params_per_layer(i) for i in range(self.num_layers)) + self.vocab_size * self.side_dim * self.num_layers
     return layers + emb * (1 if self.tie_word_embeddings else 2) + self.hidden_size
 
   def to_dict(self) -> dict:
@@ -424,7 +450,20 @@ def _ln_sandwich_params(D: int, s: MixedLayerSpec) -> int:
   return n
 
 
+def _outnorm_params(D: int, s: MixedLayerSpec) -> int:
+  """Layers whose sublayers read the stream itself and are normed behind (biased window attention, side input)."""
+  a, f = s.wattn, s.ffn
+  n = (D + 2) * a.heads * a.dim + (a.heads * a.vdim + 1) * D + D
+  if a.kv_from < 0:
+    n += a.kv_heads * ((D + 2) * a.dim + (D + 1) * a.vdim)
+  if f is not None:
+    n += D + (2 * D * f.ff if f.kind == "relu2" else f.experts * (3 * D * f.ff + D) + 3 * D * f.shared_ff)
+  return n + (2 * D * s.side + D if s.side else 0)
+
+
 def mixed_layer_params(D: int, s: MixedLayerSpec) -> int:
+  if s.wattn is not None and s.wattn.proj_norm:
+    return _outnorm_params(D, s)
   if s.dattn is not None or (s.rec is not None and s.rec.rule in ("lightning", "mlstm")):
     return _ln_sandwich_params(D, s)
   if s.lattn is not None:
@@ -708,7 +747,65 @@ def _kopalorn_config(cfg: dict) -> ModelConfig:
     norm_kind="layer", residual_mult=float(cfg.get("residual_mult", 1.0)), loop_input="add")
 
 
+def _torinex_config(cfg: dict) -> ModelConfig:
+  """Torinex config.json: {"architecture", "vocab", "width", "norm": {"eps"}, "token_side": {"dim"} | null, "layers":
+  [{"type": "attention", "mixer": {"heads", "kv_heads", "dim", "vdim", "mask": {"size"}, "rot": {"base", "dims"}, "scale",
+  "kv_from"}, "mlp": {"kind": "dense", "ff"} | {"kind": "moe", "expert": {"ff", "limit"}, "router": {"experts", "top",
+  "groups": {"count", "keep"}}, "shared": {"ff", "limit"}} | null}]}.  Without "mask" every earlier token is seen, without
+  "rot" nothing is rotated; "kv_from": j borrows layer j's keys and values."""
+  specs = []
+  side = int((cfg.get("token_side") or {}).get("dim", 0))
+  for i, L in enumerate(cfg["layers"]):
+    m, mlp = L["mixer"], L.get("mlp")
+    if L["type"] != "attention":
+      raise ValueError(f"layer {i}: unknown layer type {L['type']!r}")
+    ffn = None
+    if mlp is not None:
+      kind = mlp.get("kind", "dense")
+      if kind == "dense":
+        ffn = FeedForwardSpec("relu2", int(mlp["ff"]))
+      elif kind == "moe":
+        r, sh = mlp["router"], mlp.get("shared")
+        gr = r.get("groups") or {}
+        cnt = int(gr.get("count", 1))
+        ffn = FeedForwardSpec("clamped_moe", int(mlp["expert"]["ff"]), int(r["experts"]), int(r["top"]),
+                              int(sh["ff"]) if sh else 0, limit=float(mlp["expert"]["limit"]),
+                              shared_limit=float(sh["limit"]) if sh else 0.0, route="softmax_groups", groups=cnt,
+                              keep=int(gr.get("keep", cnt)))
+        if not 1 <= ffn.top <= ffn.experts or ffn.experts % ffn.groups or not 1 <= ffn.keep <= ffn.groups or \
+           ffn.keep * (ffn.experts // ffn.groups) < ffn.top:
+          raise ValueError(f"layer {i}: top {ffn.top} of {ffn.experts} experts in {ffn.groups} groups, {ffn.keep} kept")
+      else:
+        raise ValueError(f"layer {i}: unsupported feed-forward kind {kind!r}")
+    rot, src = m.get("rot") or {}, m.get("kv_from")
+    a = WindowAttnSpec(int(m["heads"]), int(m["kv_heads"]), int(m["dim"]), int(m["vdim"]), 0, 0, int(rot.get("dims", 0)),
+                       float(rot.get("base", 10000.0)), None, float(m["scale"]), qk_norm=False, bias=True, sink=False,
+                       kv_from=-1 if src is None else int(src), chunk=int((m.get("mask") or {}).get("size", 0)),
+                       proj_norm=True, rot_interleaved=True, sink_one=True, out_bias=True)
+    if a.heads % a.kv_heads or a.rot_dims % 2 or a.rot_dims > a.dim:
+      raise ValueError(f"layer {i}: heads {a.heads} / kv_heads {a.kv_heads} / rotary dims {a.rot_dims} do not fit")
+    if a.kv_from >= 0:
+      b = specs[a.kv_from].wattn if a.kv_from < i else None
+      if b is None or b.kv_from >= 0 or (b.kv_heads, b.dim, b.vdim, b.rot_dims, b.rot_base) != \
+         (a.kv_heads, a.dim, a.vdim, a.rot_dims, a.rot_base):
+        raise ValueError(f"layer {i}: kv_from {a.kv_from} must name an earlier layer with projections of its own, the same "
+                         "key / value heads and the same rotation")
+    specs.append(MixedLayerSpec("attention", wattn=a, ffn=ffn, side=side))
+  if side and int(cfg["vocab"]) > 1 << 24:
+    raise ValueError("token ids travel between shards as fp32 numbers: at most 2^24 of them")
+  first = specs[0].wattn
+  return ModelConfig(
+    model_type="torinex", vocab_size=int(cfg["vocab"]), hidden_size=int(cfg["width"]),
+    intermediate_size=max([s.ffn.ff for s in specs if s.ffn is not None] + [0]), num_layers=len(specs),
+    num_heads=first.heads, num_kv_heads=first.kv_heads, head_dim=first.dim, rms_norm_eps=float(cfg["norm"]["eps"]),
+    rope_theta=first.rot_base, max_position_embeddings=int(cfg.get("max_positions", 1 << 20)), tie_word_embeddings=True,
+    bos_token_id=int(cfg.get("bos_token_id", 0)), eos_token_ids=tuple(cfg.get("eos_token_ids", ())),
+    layer_specs=tuple(specs), block="sandwich", input_norm=False)
+
+
 def from_hf_config(cfg: dict) -> ModelConfig:
+  if cfg.get("architecture") == "Torinex":
+    return _torinex_config(cfg)
   if cfg.get("architecture") == "Kopalorn":
     return _kopalorn_config(cfg)
   if cfg.get("architecture") == "Nenizen":
@@ -1003,6 +1100,21 @@ TINY_KOPALORN = {
                "rot": {"base": 1000.0, "dims": 32}}},
   ]}
 PRESETS["tiny-kopalorn"] = _kopalorn_config(TINY_KOPALORN)
+_TINY_CMOE = {"kind": "moe", "expert": {"ff": 40, "limit": 1.2}, "shared": {"ff": 56, "limit": 2.0},
+              "router": {"experts": 6, "top": 2, "groups": {"count": 3, "keep": 2}}}
+_TINY_CHUNK = {"heads": 4, "kv_heads": 2, "dim": 24, "vdim": 16, "mask": {"size": 37}, "rot": {"base": 10000.0, "dims": 16},
+               "scale": 0.3}
+TINY_TORINEX = {
+  "architecture": "Torinex", "vocab": 312, "width": 104, "norm": {"eps": 1e-5}, "token_side": {"dim": 12},
+  "layers": [
+    {"type": "attention", "mlp": {"kind": "dense", "ff": 152}, "mixer": _TINY_CHUNK},
+    {"type": "attention", "mlp": _TINY_CMOE,
+     "mixer": {"heads": 6, "kv_heads": 2, "dim": 16, "vdim": 16, "mask": {"size": 70}, "rot": {"base": 500.0, "dims": 16},
+               "scale": 0.25}},
+    {"type": "attention", "mlp": None, "mixer": dict(_TINY_CHUNK, kv_from=0, mask={"size": 20}, scale=0.2)},
+    {"type": "attention", "mlp": _TINY_CMOE, "mixer": dict(_TINY_CHUNK, kv_from=0)},
+  ]}
+PRESETS["tiny-torinex"] = _torinex_config(TINY_TORINEX)
 # aliases of the reference's model cards that share an architecture
 for _alias, _base in {"llama-3.1-70b-bf16": "llama-3.1-70b", "nemotron-70b": "llama-3.1-70b",
                       "deepseek-r1-distill-llama-70b": "llama-3.1-70b", "deepseek-r1-distill-llama-8b": "llama-3.1-8b",

@@ -491,10 +491,15 @@ class ShardModel:
     c, w = self.c, self.w
     if c.has_state and (self.state is None or inp.state_slots is None):
       raise RuntimeError("a model with recurrent layers needs a state pool and the step's state slots")
+    ids = None  # (token ids, for layers with side inputs: shards after the first find them in the hidden state's last column)
     if self.shard.is_first_layer():
-      h = w.embed.index_select(0, x.view(-1).long().clamp(0, w.embed.shape[0] - 1))
+      ids = x.view(-1).long().clamp(0, w.embed.shape[0] - 1)
+      h = w.embed.index_select(0, ids)
+      ids = ids.to(torch.int32)
     else:
-      h = x.to(torch.float32).contiguous().clone()
+      if c.side_dim:
+        ids = x[:, c.hidden_size].to(torch.int32)
+      h = x[:, :c.hidden_size].to(torch.float32).contiguous().clone()
     T, D = h.shape
     n = len(self.layer_ids)
     last = self.shard.is_last_layer()
@@ -502,7 +507,7 @@ class ShardModel:
     if c.block == "postln":
       return self._forward_postln(h, inp, adt)
     if c.block == "sandwich":
-      return self._forward_sandwich(h, inp, adt)
+      return self._forward_sandwich(h, inp, adt, ids)
     bufs = {}
 
     def rows(name: str, live: int, padded: int) -> torch.Tensor:
@@ -543,8 +548,8 @@ class ShardModel:
 
   # ------------------------------------------------------------------ post-norm blocks (window attention / SSD, MoE)
   def _window_attn(self, P: torch.Tensor, lw, j: int, inp: StepInputs, mix: torch.Tensor) -> None:
-    """Softmax attention over a sliding window, pooled blocks before it and a sink: biases + RoPE + per-head RMS
-    division + paged write, the pooled caches' update for blocks that this step completed, then the attention."""
+    """Softmax attention over a sliding window or the query's chunk, pooled blocks and a sink: biases + norms + RoPE + paged
+    write, the pooled caches' update for blocks that this step completed, then the attention."""
     a = lw.spec.wattn
     q = torch.empty(P.shape[0], a.heads, a.dim, dtype=mix.dtype, device=P.device)
     tab = self.rope_tabs.get((a.rot_dims, a.rot_base, a.rot_scaling))
@@ -552,14 +557,15 @@ class ShardModel:
     K.qk_norm_rope_store(P, lw.in_b, lw.cols["q"][0], lw.cols["k"][0] if own else -1, lw.cols["v"][0] if own else -1,
                          a.heads, a.kv_heads, a.dim, a.vdim, a.rot_dims if tab is not None else 0, inp.positions,
                          tab if tab is not None else torch.zeros(1, 0, device=P.device), inp.slots, self.c.rms_norm_eps,
-                         a.qk_norm, q, self.kv.k[j], self.kv.v[j])
+                         a.qk_norm, q, self.kv.k[j], self.kv.v[j], lw.q_norm if a.proj_norm else None,
+                         lw.k_norm if a.proj_norm else None)
     if self.kv.pool_owner[j]:
       K.kv_pool_update(self.kv.k[j], self.kv.v[j], self.kv.kp[j], self.kv.vp[j], inp.block_tables, inp.cu_q, inp.ctx_lens,
                        a.pool, inp.max_qlen)
     pool = a.pool if self.kv.kp[j] is not None else 0
     o = mix[:, :a.heads * a.vdim]
     K.attn_window_pool(q, self.kv.k[j], self.kv.v[j], self.kv.kp[j], self.kv.vp[j], inp.block_tables, inp.cu_q,
-                       inp.ctx_lens, lw.sink, a.scale, a.window, pool, o, max_qlen=inp.max_qlen)
+                       inp.ctx_lens, lw.sink, a.scale, a.window, pool, o, max_qlen=inp.max_qlen, chunk=a.chunk)
     if a.gate != "none":  # one sigmoid gate per element, from the mixer's input, applied in place
       K.sigmoid_gate_mul(o, P, lw.cols["gate"][0], mix)
 
@@ -776,23 +782,25 @@ class ShardModel:
       return torch.bmm(x, w)
     return torch.bmm(x.float(), w.float()).to(x.dtype)
 
-  def _silu_moe(self, hn: torch.Tensor, P: torch.Tensor, lw, rows) -> torch.Tensor:
-    """SiLU-gated experts chosen by the softmax scores' top-k (weights: the scores as they are) + the ungated shared
-    expert -> fp32 [T, D].  Routing on the framework's grouped top-k kernel, experts on the grouped GEMMs (bf16) or per
-    expert on the vendor SGEMM (fp32)."""
+  def _glu_moe(self, hn: torch.Tensor, P: torch.Tensor, lw, rows) -> torch.Tensor:
+    """Gated experts (SiLU, or the clamped form) chosen by the softmax scores' top-k, maybe among the best groups (weights:
+    the scores as they are) + the ungated shared expert -> fp32 [T, D].  Routing on the framework's grouped top-k kernel,
+    experts on the grouped GEMMs (bf16) or per expert on the vendor SGEMM (fp32)."""
     f, dev = lw.spec.ffn, P.device
     T, D = hn.shape[0], self.c.hidden_size
     E, k = f.experts, f.top
+    clamped = f.kind == "clamped_moe"
     r0 = lw.ff_cols["router"][0]
     logits = P[:, r0:r0 + E].contiguous()
     Fp, Dq, S = lw.ex_down_w.shape[2], lw.ex_down_w.shape[1], 1
+    method = 1 if f.groups > 1 else 0  # (a group's value: its largest score)
     if P.is_cuda:
       topw = torch.empty(T * k, dtype=torch.float32, device=dev)
       topi, slot_of, sorted_tok = (torch.empty(T * k, dtype=torch.int32, device=dev) for _ in range(3))
       off = torch.empty(E + 1, dtype=torch.int32, device=dev)
-      K.moe_route_ds(logits, None, k, 1, 1, 0, False, False, 1.0, outs=(topw, topi, slot_of, sorted_tok, off))
+      K.moe_route_ds(logits, None, k, f.groups, f.keep, method, False, False, 1.0, outs=(topw, topi, slot_of, sorted_tok, off))
     else:
-      topw, idx = torch.topk(torch.softmax(logits.float(), -1), k, dim=-1)
+      topw, idx = K.moe_route_ds(logits, None, k, f.groups, f.keep, method, False, False, 1.0)
       topw, topi = topw.reshape(-1), idx.reshape(-1).int()
       order = torch.argsort(topi, stable=True)
       slot_of = torch.empty_like(order)
@@ -810,8 +818,8 @@ class ShardModel:
       S = S_dn if big else (4 if T * k <= 64 else 2)
       if Fp % (256 * S):
         S = 1
-      act = torch.empty(T * k, Fp, dtype=torch.bfloat16, device=dev)  # silu(gate) * up in the GEMM's epilogue
-      C.gemm_moe(hn, lw.ex_up_w, act, off, sorted_tok, K.EPI["silu"], T, sh_up, 1, bm)
+      act = torch.empty(T * k, Fp, dtype=torch.bfloat16, device=dev)  # the gated activation in the GEMM's epilogue
+      C.gemm_moe(hn, lw.ex_up_w, act, off, sorted_tok, K.EPI["clamp_glu" if clamped else "silu"], T, sh_up, 1, bm, f.limit)
       y = torch.empty(S * T * k, Dq, dtype=torch.float32, device=dev)
       C.gemm_moe(act, lw.ex_down_w, y, off, None, K.EPI["none"], T, sh_dn, S, bm_dn)
     else:
@@ -822,18 +830,28 @@ class ShardModel:
         if offs[e + 1] > offs[e]:
           xe = hn.index_select(0, sorted_tok[offs[e]:offs[e + 1]].long()).float()
           gu = (xe @ lw.ex_up_w[e].float().t()).reshape(xe.shape[0], Fp // 16, 2, 16)  # (gate | up tiles of 16)
-          act = (torch.nn.functional.silu(gu[:, :, 0]) * gu[:, :, 1]).reshape(xe.shape[0], Fp)
+          gu = torch.cat([gu[:, :, 0].reshape(-1, Fp), gu[:, :, 1].reshape(-1, Fp)], 1)
+          act = torch.empty(xe.shape[0], Fp, dtype=torch.float32, device=dev)
+          K.glu_act(gu, 0, Fp, Fp, clamped, f.limit, act)
           y[offs[e]:offs[e + 1]] = act @ lw.ex_down_w[e].float().t()
     sh_y = None
     if f.shared_ff:
       act = rows("sh_act", f.shared_ff, lw.down_w.shape[1])
-      K.glu_act(P, lw.ff_cols["sh_gate"][0], lw.ff_cols["sh_up"][0], f.shared_ff, False, 0.0, act)
+      K.glu_act(P, lw.ff_cols["sh_gate"][0], lw.ff_cols["sh_up"][0], f.shared_ff, clamped, f.shared_limit, act)
       sh_y = self._proj(act, lw.down_w)
     out = torch.empty(T, D, dtype=torch.float32, device=dev)
     K.moe_weighted_sum(y, slot_of, topw, k, sh_y, None, 0, out, splits=S)
     return out
 
-  def _forward_sandwich(self, h: torch.Tensor, inp: StepInputs, adt) -> torch.Tensor:
+  def _side_input(self, hn: torch.Tensor, lw, j: int, ids: torch.Tensor, rows) -> torch.Tensor:
+    """The layer's slice of the side-input table at each token, gated by the stream (gelu_tanh of a projection) and
+    projected to the width -> fp32 rows, not normed yet."""
+    n = lw.spec.side
+    act = rows("side", n, lw.side_proj_w.shape[1])
+    K.gelu_gather_mul(self._proj(hn, lw.side_gate_w), 0, self.w.side_embed, ids, (j - self.layer_ids[0]) * n, n, act)
+    return self._proj(act, lw.side_proj_w)
+
+  def _forward_sandwich(self, h: torch.Tensor, inp: StepInputs, adt, ids: Optional[torch.Tensor] = None) -> torch.Tensor:
     """Layer runs (a looped layer once per pass, each pass with caches and states of its own) of sandwich blocks on the
     fp32 stream h (hn: the normed sublayer input in the GEMMs' operand dtype):
       pass start:  h <- [h | embedding output] @ loop_in^T + step[pass]       (loop_input "linear")
@@ -843,9 +861,11 @@ class ShardModel:
       P = hn @ ff_w^T                    gate | up, or router | shared expert's projections
       h += mult * norm2b(ff(P));  hn = the next run's norm1(h)
     The norms are RMS norms with a weight, or (norm_kind "layer") layer norms with weight and bias.  Mixers: latent
-    attention; differential attention; mlstm; gated attention beside lightning attention, each projected to the width,
-    RMS-normed with its own weight and averaged.
-    Returns h (non-last shard) or softcap(head(final_norm(h rows inp.last_idx)))."""
+    attention; differential attention; window / chunk attention; mlstm; gated attention beside lightning attention, each
+    projected to the width, RMS-normed with its own weight and averaged.
+    Without input norms (input_norm False) hn is the stream itself in the operand dtype.  A layer with a side input ends
+    with h += norm(proj(gelu_tanh(hn @ gate^T) * its slice of the token's side-input row)).
+    Returns h (non-last shard; with the token ids as one more column when the model has side inputs) or softcap(head(final_norm(h rows inp.last_idx)))."""
     c, w = self.c, self.w
     T, D = h.shape
     Dp = -(-D // 128) * 128
@@ -878,7 +898,7 @@ class ShardModel:
           h += x0
         h += w.loop_step[t]
         fresh = True
-      if fresh:
+      if fresh:  # (no norm weight: the op copies the stream)
         K.sandwich_add_norm(h, None, None, lw.norm1, eps, hn, bn=lw.norm1_b)
       P = self._proj(hn, lw.in_w)
       mix = rows("mix", lw.mix_cols["mix"][1], lw.out_w.shape[1])
@@ -901,23 +921,32 @@ class ShardModel:
       # the norm that follows this run: the next run's input norm unless a pass starts there
       nl = w.layers[runs[j + 1][0]] if j + 1 < len(runs) and runs[j + 1][1] < 0 else None
       nxt, nxt_b = (nl.norm1, nl.norm1_b) if nl is not None else (None, None)
+      hn_nxt = hn if nl is not None else None
+      after = (lw.side_norm is not None, f is not None)  # what still reads hn in this layer: the side input, the feed-forward
       if f is None:
-        K.sandwich_add_norm(h, y, lw.norm1b, nxt, eps, hn, bb=lw.norm1b_b, bn=nxt_b, mult=mult)
+        K.sandwich_add_norm(h, y, lw.norm1b, nxt, eps, hn if after[0] else hn_nxt, bb=lw.norm1b_b, bn=nxt_b, mult=mult,
+                            yb=lw.out_b)
       else:
-        K.sandwich_add_norm(h, y, lw.norm1b, lw.norm2, eps, hn, bb=lw.norm1b_b, bn=lw.norm2_b, mult=mult)
+        K.sandwich_add_norm(h, y, lw.norm1b, lw.norm2, eps, hn, bb=lw.norm1b_b, bn=lw.norm2_b, mult=mult, yb=lw.out_b)
         P = self._proj(hn, lw.ff_w)
         if f.kind == "clamped_glu":
           act = rows("act", f.ff, lw.down_w.shape[1])
           K.glu_act(P, lw.ff_cols["gate"][0], lw.ff_cols["up"][0], f.ff, True, f.limit, act)
           y = self._proj(act, lw.down_w)
+        elif f.kind == "relu2":
+          act = rows("act", f.ff, lw.down_w.shape[1])
+          K.relu2(P, lw.ff_cols["up"][0], f.ff, act)
+          y = self._proj(act, lw.down_w)
         elif f.kind == "relu2_moe":
           y = self._relu2_moe(hn, P, lw, rows)
         else:
-          y = self._silu_moe(hn, P, lw, rows)
-        K.sandwich_add_norm(h, y, lw.norm2b, nxt, eps, hn, bb=lw.norm2b_b, bn=nxt_b, mult=mult)
-      fresh = nxt is None
+          y = self._glu_moe(hn, P, lw, rows)
+        K.sandwich_add_norm(h, y, lw.norm2b, nxt, eps, hn if after[0] else hn_nxt, bb=lw.norm2b_b, bn=nxt_b, mult=mult)
+      if after[0]:
+        K.sandwich_add_norm(h, self._side_input(hn, lw, li, ids, rows), lw.side_norm, nxt, eps, hn_nxt, bn=nxt_b)
+      fresh = nl is None
     if not self.shard.is_last_layer():
-      return h
+      return torch.cat([h, ids.to(torch.float32)[:, None]], 1) if c.side_dim else h
     hl = h.index_select(0, inp.last_idx)
     xn = torch.zeros(hl.shape[0], Dp, dtype=adt, device=h.device)
     K.sandwich_add_norm(hl, None, None, w.norm, eps, xn, bn=w.norm_b)

@@ -82,6 +82,7 @@ class ShardWeights:
   # at the start of each pass [times, D] fp32
   loop_in: Optional[torch.Tensor] = None
   loop_step: Optional[torch.Tensor] = None
+  side_embed: Optional[torch.Tensor] = None  # [V, this shard's layers x side_dim]: the layers' per-token side inputs
 
   def nbytes(self) -> int:
     seen, total = set(), 0
@@ -94,7 +95,7 @@ class ShardWeights:
   def all_tensors(self) -> Iterable[torch.Tensor]:
     for lw in self.layers.values():
       yield from lw.tensors().values()
-    for t in (self.embed, self.norm, self.norm_b, self.lm_head, self.loop_in, self.loop_step):
+    for t in (self.embed, self.norm, self.norm_b, self.lm_head, self.loop_in, self.loop_step, self.side_embed):
       if t is not None:
         yield t
     if self.vision:
@@ -345,6 +346,7 @@ def prepare_for_decode(sw: "ShardWeights", keep_rowmajor: Iterable[str] = (), fp
       if lw.in_w.dtype == torch.bfloat16:
         lw.in_w, lw.out_w, lw.down_w, lw.ff_w = wide(lw.in_w), wide(lw.out_w), wide(lw.down_w), wide(lw.ff_w)
         lw.uq_w, lw.out2_w = wide(lw.uq_w), wide(lw.out2_w)
+        lw.side_gate_w, lw.side_proj_w = wide(lw.side_gate_w), wide(lw.side_proj_w)
         lw.ex_up_w, lw.ex_down_w = conv(lw.ex_up_w), conv(lw.ex_down_w)  # experts: shuffled per expert
     if sw.lm_head is not None and sw.lm_head.dtype == torch.bfloat16:
       sw.lm_head = wide(sw.lm_head)
@@ -747,6 +749,14 @@ class MixedLayerWeights:
   decay: Optional[torch.Tensor] = None
   gate_b: Optional[torch.Tensor] = None
   lam: float = 0.0
+  # sandwich blocks without input norms: norm1b / norm2b only (the checkpoint's norm1 / norm2); q_norm [H dim] / k_norm
+  # [G dim] weigh the norms over the whole projections (rotary dims in pair order like the projections' rows); the side
+  # input's gate and output projections and the weight of the norm over its result
+  k_norm: Optional[torch.Tensor] = None
+  out_b: Optional[torch.Tensor] = None  # [D] fp32: bias of the output projection
+  side_gate_w: Optional[torch.Tensor] = None  # [side padded, Dp]
+  side_proj_w: Optional[torch.Tensor] = None  # [Dn, side padded]
+  side_norm: Optional[torch.Tensor] = None  # [D] fp32
 
   def tensors(self) -> Dict[str, torch.Tensor]:
     return {k: v for k, v in self.__dict__.items() if isinstance(v, torch.Tensor)}
@@ -906,22 +916,111 @@ def build_sandwich_layer(spec, get, p: str, D: int, device, dtype) -> MixedLayer
     fb = [("gate", get(q + "gate")), ("up", get(q + "up"))]
     down = get(q + "down")
   else:
-    fb = [("router", get(q + "router"))]
-    down = None
-    if f.shared_ff:
-      fb += [("sh_gate", get(q + "shared.gate")), ("sh_up", get(q + "shared.up"))]
-      down = get(q + "shared.down")
-    Fp, Dp = _up(f.ff, 128), _up(D, 128)
-    # gate and up rows interleaved in tiles of 16 (the grouped GEMM's SiLU epilogue pairs them)
-    lw.ex_up_w = dev(torch.stack([interleave_gate_up(_pad2(get(q + f"e{e}.gate"), Fp, Dp), _pad2(get(q + f"e{e}.up"), Fp, Dp))
-                                  for e in range(f.experts)]), dtype)
-    lw.ex_down_w = dev(torch.stack([_pad2(get(q + f"e{e}.down"), Dp, Fp) for e in range(f.experts)]), dtype)
+    fb, down = _gated_moe_weights(lw, f, get, q, D, dev, dtype)
   ff_w, lw.ff_cols = _fused_rows(fb, D)
   lw.ff_w = dev(ff_w, dtype)
   if down is not None:
     lw.down_w = dev(_pad2(down, _up(D, 64), _up(down.shape[1], 128)), dtype)
   lw.norm2, lw.norm2b = dev(get(p + "norm2")), dev(get(p + "norm2b"))
   return lw
+
+
+def _gated_moe_weights(lw: MixedLayerWeights, f, get, q: str, D: int, dev, dtype):
+  """Gated experts (SiLU or clamped) stacked and padded; -> the fused blocks [router | shared gate | shared up] and the
+  shared expert's down projection (None: no shared expert)."""
+  fb, down = [("router", get(q + "router"))], None
+  if f.shared_ff:
+    fb += [("sh_gate", get(q + "shared.gate")), ("sh_up", get(q + "shared.up"))]
+    down = get(q + "shared.down")
+  Fp, Dp = _up(f.ff, 128), _up(D, 128)
+  # gate and up rows interleaved in tiles of 16 (the grouped GEMM's gated epilogues pair them)
+  lw.ex_up_w = dev(torch.stack([interleave_gate_up(_pad2(get(q + f"e{e}.gate"), Fp, Dp), _pad2(get(q + f"e{e}.up"), Fp, Dp))
+                                for e in range(f.experts)]), dtype)
+  lw.ex_down_w = dev(torch.stack([_pad2(get(q + f"e{e}.down"), Dp, Fp) for e in range(f.experts)]), dtype)
+  return fb, down
+
+
+def build_outnorm_layer(spec, get, p: str, D: int, device, dtype) -> MixedLayerWeights:
+  """One layer whose sublayers read the stream itself (window attention with biases and norms over the whole query and
+  key projections; relu^2 or clamped-expert feed-forward; side input) from `get(name)`."""
+  def dev(t, dt=torch.float32):
+    return t.to(device=device, dtype=dt).contiguous()
+  m = p + "mix."
+  a, f = spec.wattn, spec.ffn
+
+  def heads_in_pair_order(t, n):  # rows (or entries) of n heads, rotation pairs (2i, 2i + 1) -> (i, i + R / 2)
+    order = _pair_order(a.dim, a.rot_dims) if a.rot_interleaved else torch.arange(a.dim)
+    return t.reshape(n, a.dim, *t.shape[1:])[:, order].reshape(t.shape)
+  own = a.kv_from < 0
+  parts = [("q", a.heads)] + ([("k", a.kv_heads), ("v", 0)] if own else [])
+  blocks = [(n, heads_in_pair_order(get(m + n), h) if h else get(m + n)) for n, h in parts]
+  in_w, cols = _fused_rows(blocks, D)
+  b = torch.zeros(in_w.shape[0])
+  for n, h in parts:
+    t = get(m + n + ".b")
+    b[cols[n][0]:cols[n][0] + cols[n][1]] = heads_in_pair_order(t, h) if h else t
+  out = get(m + "o")
+  lw = MixedLayerWeights(spec, dev(in_w, dtype), cols, dev(_pad2(out, _up(D, 64), _up(out.shape[1], 128)), dtype),
+                         {"mix": (0, out.shape[1])})
+  lw.in_b, lw.out_b = dev(b), dev(get(m + "o.b"))
+  lw.q_norm = dev(heads_in_pair_order(get(m + "q.norm"), a.heads))
+  if own:
+    lw.k_norm = dev(heads_in_pair_order(get(m + "k.norm"), a.kv_heads))
+  if a.sink_one:
+    lw.sink = torch.zeros(a.heads, device=device)
+  lw.norm1b = dev(get(p + "norm1"))
+  if f is not None:
+    q = p + "mlp."
+    if f.kind == "relu2":
+      fb, down = [("up", get(q + "up"))], get(q + "down")
+    else:
+      fb, down = _gated_moe_weights(lw, f, get, q, D, dev, dtype)
+    # (a dense feed-forward's rows are padded like the down projection's columns: its activation is the GEMM's output)
+    ff_w, lw.ff_cols = _fused_rows(fb, D, 128 if f.kind == "relu2" else 64)
+    lw.ff_w = dev(ff_w, dtype)
+    if down is not None:
+      lw.down_w = dev(_pad2(down, _up(D, 64), _up(down.shape[1], 128)), dtype)
+    lw.norm2b = dev(get(p + "norm2"))
+  if spec.side:
+    s = p + "side."
+    lw.side_gate_w = dev(_pad2(get(s + "gate"), _up(spec.side, 64), _up(D, 128)), dtype)
+    lw.side_proj_w = dev(_pad2(get(s + "proj"), _up(D, 64), _up(spec.side, 128)), dtype)
+    lw.side_norm = dev(get(s + "norm"))
+  return lw
+
+
+def outnorm_tensor_shapes(c: ModelConfig) -> Dict[str, tuple]:
+  """Name -> shape of every tensor of a checkpoint whose blocks norm the sublayers' results only (Torinex); the LM head is
+  the embedding table."""
+  D, out = c.hidden_size, {}
+  out["embed"] = (c.vocab_size, D)
+  if c.side_dim:
+    out["side.embed"] = (c.vocab_size, c.num_layers * c.side_dim)
+  for i, s in enumerate(c.layer_specs):
+    p, m, a, f = f"l{i}.", f"l{i}.mix.", s.wattn, s.ffn
+    out[p + "norm1"] = (D,)
+    proj = [("q", a.heads * a.dim)] + ([("k", a.kv_heads * a.dim), ("v", a.kv_heads * a.vdim)] if a.kv_from < 0 else [])
+    for n, rows in proj:
+      out[m + n], out[m + n + ".b"] = (rows, D), (rows,)
+      if n != "v":
+        out[m + n + ".norm"] = (rows,)
+    out[m + "o"], out[m + "o.b"] = (D, a.heads * a.vdim), (D,)
+    if f is not None:
+      q = p + "mlp."
+      out[p + "norm2"] = (D,)
+      if f.kind == "relu2":
+        out[q + "up"], out[q + "down"] = (f.ff, D), (D, f.ff)
+      else:
+        for e in range(f.experts):
+          out[q + f"e{e}.gate"], out[q + f"e{e}.up"], out[q + f"e{e}.down"] = (f.ff, D), (f.ff, D), (D, f.ff)
+        out[q + "router"] = (f.experts, D)
+        if f.shared_ff:
+          out[q + "shared.gate"], out[q + "shared.up"], out[q + "shared.down"] = (f.shared_ff, D), (f.shared_ff, D), \
+            (D, f.shared_ff)
+    if s.side:
+      out[p + "side.gate"], out[p + "side.proj"], out[p + "side.norm"] = (s.side, D), (D, s.side), (D,)
+  out["final.norm"] = (D,)
+  return out
 
 
 def _pair_order(d: int, R: int) -> torch.Tensor:
@@ -1122,6 +1221,8 @@ def mixed_tensor_shapes(c: ModelConfig) -> Dict[str, tuple]:
   """Name -> shape of every tensor of a mixed-layer checkpoint (random init, checkpoint validation)."""
   if c.block == "postln":
     return postln_tensor_shapes(c)
+  if c.block == "sandwich" and not c.input_norm:
+    return outnorm_tensor_shapes(c)
   if c.block == "sandwich":
     return ln_sandwich_tensor_shapes(c) if c.norm_kind == "layer" else sandwich_tensor_shapes(c)
   D, out = c.hidden_size, {}
@@ -1169,7 +1270,7 @@ def random_mixed_tensors(c: ModelConfig, seed: int = 0) -> Dict[str, torch.Tenso
            "out": 1.0 + 0.1 * torch.randn(shape, generator=g)}.get(leaf)
       if t is None:
         t = torch.randn(shape, generator=g) * 0.4
-    elif leaf in ("sink", "D", "act") or (leaf == "b" and c.block == "postln"):
+    elif leaf in ("sink", "D", "act") or (leaf == "b" and (c.block == "postln" or not c.input_norm)):
       t = torch.randn(shape, generator=g) * (0.5 if leaf == "b" else 1.0)
     elif leaf in ("norm1", "norm2", "norm1b", "norm2b") or name == "final.norm":
       t = 1.0 + 0.1 * torch.randn(shape, generator=g)
@@ -1187,6 +1288,8 @@ def random_mixed_tensors(c: ModelConfig, seed: int = 0) -> Dict[str, torch.Tenso
       t = torch.randn(shape, generator=g) * 0.3
     elif name == "embed":
       t = torch.randn(shape, generator=g) * (0.25 if c.block == "sandwich" else 1.0)
+    elif name == "side.embed":
+      t = torch.randn(shape, generator=g)
     else:
       t = torch.randn(shape, generator=g) / shape[-1] ** 0.5
     out[name] = t.to(torch.bfloat16).float()
@@ -1200,11 +1303,16 @@ def mixed_weights(c: ModelConfig, shard: Shard, get, device, dtype) -> ShardWeig
   build = {"postln": build_postln_layer, "sandwich": build_sandwich_layer}.get(c.block, build_mixed_layer)
   if c.block == "sandwich" and c.norm_kind == "layer":
     build = build_ln_sandwich_layer
+  elif c.block == "sandwich" and not c.input_norm:
+    build = build_outnorm_layer
   for i in shard.layers():
     sw.layers[i] = build(c.layer_specs[i], get, f"l{i}.", D, device, dtype)
   if shard.is_first_layer():
     # gathered into the fp32 residual; a model that scales its embedding output gathers from the scaled table
     sw.embed = (get("embed") * c.embed_scale).to(device=device, dtype=torch.float32).contiguous()
+  if c.side_dim and len(sw.layers):
+    n, first = c.side_dim, min(sw.layers)
+    sw.side_embed = get("side.embed")[:, first * n:(max(sw.layers) + 1) * n].to(device=device, dtype=dtype).contiguous()
   if c.loop and c.loop_input == "add" and any(c.loop[0] <= i < c.loop[1] for i in shard.layers()):
     sw.loop_step = get("loop.step").to(device=device, dtype=torch.float32).contiguous()
   elif c.loop and any(c.loop[0] <= i < c.loop[1] for i in shard.layers()):
@@ -1225,7 +1333,7 @@ def mixed_weights(c: ModelConfig, shard: Shard, get, device, dtype) -> ShardWeig
 
 
 def load_mixed_weights(model_dir: Path, c: ModelConfig, shard: Shard, device, dtype) -> ShardWeights:
-  """Tarepel / Mogelix / Nenizen checkpoint (flat names: embed, l<i>.norm1, l<i>.mix.*, l<i>.mlp.*, l<i>.ls1 / ls2 or l<i>.rg1 /
+  """Checkpoint of a mixed-layer design (flat names: embed, l<i>.norm1, l<i>.mix.*, l<i>.mlp.*, l<i>.ls1 / ls2 or l<i>.rg1 /
   rg2, final.norm, head).  The decay rank of a gated-linear-attention layer is the a1 tensor's row count."""
   from safetensors import safe_open
   wm = _weight_map(Path(model_dir))
@@ -1240,7 +1348,7 @@ def load_mixed_weights(model_dir: Path, c: ModelConfig, shard: Shard, device, dt
     return handles[f].get_tensor(name).float()
   want = mixed_tensor_shapes(c)
   for name, shape in want.items():
-    if name.split(".")[0] in ("embed", "final", "head", "loop") or int(name.split(".")[0][1:]) in shard.layers():
+    if name.split(".")[0] in ("embed", "final", "head", "loop", "side") or int(name.split(".")[0][1:]) in shard.layers():
       got = tuple(get(name).shape) if not name.endswith((".a1", ".a2")) else None
       if name == "loop.step" and got is not None and got[1:] == tuple(shape)[1:] and got[0] >= shape[0]:
         continue

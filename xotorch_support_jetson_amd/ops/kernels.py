@@ -14,7 +14,7 @@ import torch
 from . import reference as ref
 from ._ext import require
 
-EPI = {"none": 0, "resid": 1, "silu": 2}
+EPI = {"none": 0, "resid": 1, "silu": 2, "clamp_glu": 3}
 PAGE = 64
 
 
@@ -513,13 +513,14 @@ def gated_postnorm(x, y, P, g_off: int, gate_b, alpha: float, w, eps: float, out
 
 
 def qk_norm_rope_store(P, bias, q_off: int, k_off: int, v_off: int, H: int, G: int, d: int, dv: int, R: int, pos, cos_sin,
-                       slots, eps: float, qk_norm: bool, q_out, k_cache, v_cache) -> None:
-  """q / k / v = P's columns (+ bias, one fp32 number per column of P); rotate-half RoPE on the first R dims of every
-  q / k head, then (qk_norm) each head divided by its RMS; q -> q_out [T, H, d], k -> k_cache [pages, G, 64, d],
+                       slots, eps: float, qk_norm: bool, q_out, k_cache, v_cache, q_norm=None, k_norm=None) -> None:
+  """q / k / v = P's columns (+ bias, one fp32 number per column of P); with q_norm [H d] (and k_norm [G d] for the keys)
+  all of a token's q numbers together are divided by their RMS and weighted (the keys likewise); rotate-half RoPE on the
+  first R dims of every q / k head, then (qk_norm) each head divided by its RMS; q -> q_out [T, H, d], k -> k_cache [pages, G, 64, d],
   v -> v_cache [pages, Gv, dv, 64] at `slots` (Gv = v_cache's heads: G, or fewer when neighbouring key heads share a
   value head).  k_off < 0: the layer has no keys and values of its own."""
   _mix("qk_norm_rope_store", _gpu(P))(P, bias, int(q_off), int(k_off), int(v_off), int(H), int(G), int(d), int(dv), int(R),
-                                      pos, cos_sin, slots, float(eps), bool(qk_norm), q_out, k_cache, v_cache)
+                                      pos, cos_sin, slots, float(eps), bool(qk_norm), q_out, k_cache, v_cache, q_norm, k_norm)
 
 
 def kv_pool_update(k_cache, v_cache, kp, vp, block_tables, cu_q, ctx_lens, pool: int, max_qlen: int) -> None:
@@ -530,12 +531,12 @@ def kv_pool_update(k_cache, v_cache, kp, vp, block_tables, cu_q, ctx_lens, pool:
 
 
 def attn_window_pool(q, k_cache, v_cache, kp, vp, block_tables, cu_q, ctx_lens, sink, scale: float, window: int,
-                     pool: int, out, max_qlen: int = 0) -> None:
+                     pool: int, out, max_qlen: int = 0, chunk: int = 0) -> None:
   """out [T, H dv] = softmax attention of each new token over the tokens at most window - 1 places back (window 0:
-  all), the pooled blocks that end at or before position - window (pool 0: none), and the per-head sink logit.  Key
+  all) and, with chunk > 0, in its own block of `chunk` positions (counted from the sequence's start), the pooled blocks that end at or before position - window (pool 0: none), and the per-head sink logit.  Key
   head g reads value head g / (G / Gv) (the caches' head counts); out may be fp32 beside bf16 caches."""
   _mix("attn_window_pool", _gpu(q))(q, k_cache, v_cache, kp, vp, block_tables, cu_q, ctx_lens, sink, float(scale),
-                                    int(window), int(pool), out, int(max_qlen) or int(q.shape[0]))
+                                    int(window), int(pool), out, int(max_qlen) or int(q.shape[0]), int(chunk))
 
 
 def ssd_prep(P, x_off: int, dt_off: int, conv_w, conv_b, conv_state, state_slots, cu_q, A_log, dt_bias, H: int, dv: int,
@@ -569,11 +570,12 @@ def moe_weighted_sum(y, slot_of, topw, k: int, sh_y, P, shg_off: int, out, split
 
 
 # ------------------------------------------------------------------ sandwich blocks (csrc/latent.hip)
-def sandwich_add_norm(x, y, wb, wn, eps: float, out=None, bb=None, bn=None, mult: float = 1.0) -> None:
-  """fp32 stream rows x [T, D] += mult * norm(y) * wb in place (y None: nothing is added); with wn, out[:, :D] =
-  norm(x) * wn in out's dtype (the next GEMM's operand).  norm = division by the RMS, or, with the biases bb / bn, the
+def sandwich_add_norm(x, y, wb, wn, eps: float, out=None, bb=None, bn=None, mult: float = 1.0, yb=None) -> None:
+  """fp32 stream rows x [T, D] += mult * norm(y + yb) * wb in place (y None: nothing is added; yb: one fp32 number per
+  column, or None); with wn, out[:, :D] = norm(x) * wn in out's dtype (the next GEMM's operand), with out alone out[:, :D] =
+  x.  norm = division by the RMS, or, with the biases bb / bn, the
   layer norm (v - mean) / sqrt(var + eps) * w + b."""
-  _mix("sandwich_add_norm", _gpu(x))(x, y, wb, wn, float(eps), out, bb, bn, float(mult))
+  _mix("sandwich_add_norm", _gpu(x))(x, y, wb, wn, float(eps), out, bb, bn, float(mult), yb)
 
 
 def latent_kv_store(P, ckv_off: int, R: int, dr: int, kv_norm, q_off: int, q_rank: int, q_norm, eps: float, rot_dims: int,
@@ -614,6 +616,12 @@ def glu_act(P, gate_off: int, up_off: int, F: int, clamped: bool, limit: float, 
   """out[:, :F] = silu(g) * u, or (clamped) g' sigmoid(1.702 g') (u' + 1) with g' = min(g, limit), u' = clamp(u,
   -limit, limit); g = P[:, gate_off : +F], u = P[:, up_off : +F]."""
   _mix("glu_act", _gpu(P))(P, int(gate_off), int(up_off), int(F), bool(clamped), float(limit), out)
+
+
+def gelu_gather_mul(P, off: int, table, ids, col0: int, n: int, out) -> None:
+  """out[:, :n] = gelu_tanh(P[:, off : +n]) * table[ids, col0 : +n]; table [V, cols] in out's dtype, ids [T] int32 (rows of
+  the table; ids outside it are clamped)."""
+  _mix("gelu_gather_mul", _gpu(P))(P, int(off), table, ids, int(col0), int(n), out)
 
 
 # ------------------------------------------------------------------ layer-norm sandwich blocks (csrc/recurrent_gates.hip)

@@ -382,13 +382,16 @@ def pool_dims(pool: int) -> int:
 
 
 def qk_norm_rope_store(P, bias, q_off, k_off, v_off, H, G, d, dv, R, pos, cos_sin, slots, eps, qk_norm, q_out, k_cache,
-                       v_cache):
+                       v_cache, q_norm=None, k_norm=None):
   T = P.shape[0]
   Gv = v_cache.shape[1] if k_off >= 0 else G  # value heads (fewer than key heads when key heads share values)
   Pb = P.float() if bias is None else P.float() + bias.float()
   half = R // 2
 
-  def prep(x):
+  def prep(x, w):
+    if w is not None:  # one norm over the token's whole projection
+      y = x.reshape(T, -1)
+      x = (y / torch.sqrt(y.pow(2).mean(-1, keepdim=True) + eps) * w.float()).reshape(x.shape)
     if R:
       cs = cos_sin[pos.long()]
       c, s = cs[:, None, :half], cs[:, None, half:]
@@ -397,12 +400,12 @@ def qk_norm_rope_store(P, bias, q_off, k_off, v_off, H, G, d, dv, R, pos, cos_si
     if qk_norm:
       x = x / torch.sqrt(x.pow(2).mean(-1, keepdim=True) + eps)
     return x
-  q_out.copy_(prep(Pb[:, q_off:q_off + H * d].reshape(T, H, d)).to(q_out.dtype))
+  q_out.copy_(prep(Pb[:, q_off:q_off + H * d].reshape(T, H, d), q_norm).to(q_out.dtype))
   if k_off < 0:
     return
   ok = slots >= 0
   s = slots[ok].long()
-  k_cache[s // PAGE, :, s % PAGE] = prep(Pb[:, k_off:k_off + G * d].reshape(T, G, d))[ok].to(k_cache.dtype)
+  k_cache[s // PAGE, :, s % PAGE] = prep(Pb[:, k_off:k_off + G * d].reshape(T, G, d), k_norm)[ok].to(k_cache.dtype)
   v_cache[s // PAGE, :, :, s % PAGE] = Pb[:, v_off:v_off + Gv * dv].reshape(T, Gv, dv)[ok].to(v_cache.dtype)
 
 
@@ -428,7 +431,8 @@ def kv_pool_update(k_cache, v_cache, kp, vp, block_tables, cu_q, ctx_lens, pool,
       vp[dst, :, e] = v_cache[pages, :, :, toks % PAGE].float().mean(0).to(vp.dtype)
 
 
-def attn_window_pool(q, k_cache, v_cache, kp, vp, block_tables, cu_q, ctx_lens, sink, scale, window, pool, out, max_qlen=0):
+def attn_window_pool(q, k_cache, v_cache, kp, vp, block_tables, cu_q, ctx_lens, sink, scale, window, pool, out, max_qlen=0,
+                     chunk=0):
   T, H, d = q.shape
   G, dv = k_cache.shape[1], v_cache.shape[2]
   rep = H // G
@@ -452,6 +456,8 @@ def attn_window_pool(q, k_cache, v_cache, kp, vp, block_tables, cu_q, ctx_lens, 
     vis = kpos <= qpos
     if window:
       vis = vis & (qpos - kpos < window)
+    if chunk:
+      vis = vis & (qpos // chunk == kpos // chunk)
     if nb:
       last = torch.arange(nb)[None, :] * pool + pool - 1
       vis = torch.cat([vis, last <= qpos - window], 1)
@@ -516,8 +522,8 @@ def moe_weighted_sum(y, slot_of, topw, k, sh_y, P, shg_off, out, splits=1):
 
 # ------------------------------------------------------------------ sandwich blocks: latent attention, gated feed-forwards
 # Torch twins of csrc/latent.hip.
-def sandwich_add_norm(x, y, wb, wn, eps, out, bb=None, bn=None, mult=1.0):
-  """x += mult * norm(y) in place (y None: nothing is added); with wn, out[:, :D] = norm(x).  norm(v) = v / rms(v) * w,
+def sandwich_add_norm(x, y, wb, wn, eps, out, bb=None, bn=None, mult=1.0, yb=None):
+  """x += mult * norm(y + yb) in place (y None: nothing is added); with wn, out[:, :D] = norm(x), with out alone = x.  norm(v) = v / rms(v) * w,
   or with a bias (bb / bn) the layer norm (v - mean) / sqrt(var + eps) * w + b."""
   D = x.shape[1]
 
@@ -527,9 +533,15 @@ def sandwich_add_norm(x, y, wb, wn, eps, out, bb=None, bn=None, mult=1.0):
     c = v - v.mean(-1, keepdim=True)
     return c / torch.sqrt(c.pow(2).mean(-1, keepdim=True) + eps) * w.float() + b.float()
   if y is not None:
-    x += mult * norm(y[:, :D].float(), wb, bb)
-  if wn is not None:
-    out[:, :D] = norm(x, wn, bn).to(out.dtype)
+    x += mult * norm(y[:, :D].float() + (yb.float() if yb is not None else 0.0), wb, bb)
+  if out is not None:
+    out[:, :D] = (norm(x, wn, bn) if wn is not None else x).to(out.dtype)
+
+
+def gelu_gather_mul(P, off, table, ids, col0, n, out):
+  """out[:, :n] = gelu_tanh(P[:, off : +n]) * table[ids, col0 : +n]."""
+  e = table[ids.long().clamp(0, table.shape[0] - 1), col0:col0 + n].float()
+  out[:, :n] = (F.gelu(P[:, off:off + n].float(), approximate="tanh") * e).to(out.dtype)
 
 
 def _rope_pairs(x, cs, R, interleaved):

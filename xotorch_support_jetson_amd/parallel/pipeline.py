@@ -63,7 +63,7 @@ class RingStage:
     self.top_k = top_k
     dev = runner.device
     self.seed_off = torch.tensor([seed, 0], dtype=torch.int64, device=dev)
-    self.D = runner.config.hidden_size
+    self.D = runner.config.hidden_width
     V = runner.config.vocab_size
     # rows of the last stage's share (GEMM-tile aligned).  XOT_HEAD_SPLIT: its fraction of the vocab -- the first
     # stage also runs the embedding, the candidate copy and the sampler over its columns, so a share above one

@@ -165,7 +165,7 @@ class RingServer:
     self.r, self.rank, self.world = runner, rank, world
     self.first, self.last = runner.shard.is_first_layer(), runner.shard.is_last_layer()
     self.prev, self.next = (rank - 1) % world, (rank + 1) % world
-    self.D = runner.config.hidden_size
+    self.D = runner.config.hidden_width
     self.dev = runner.device
     self._make_stage(runner, rank, world)
     self.lanes = max(1, world) * self.lanes_per_rank

@@ -385,7 +385,7 @@ class ShardRunner:
     if self.shard.is_first_layer():
       g["x"] = torch.zeros(Bp, dtype=torch.int32, device=dev)
     else:
-      g["x"] = torch.zeros(Bp, c.hidden_size, dtype=self.hidden_dtype, device=dev)
+      g["x"] = torch.zeros(Bp, c.hidden_width, dtype=self.hidden_dtype, device=dev)
     inp = StepInputs(g["pos"], g["slots"], g["tables"], g["ctx"], g["cu"], g["last"], 1, True)
     if self.sm is not None:
       # warm-up and capture run on padding rows only (state slot -1, no KV slot): no request's state is touched
