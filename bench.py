@@ -213,6 +213,30 @@ def memory_configs(name: str):
   return memory, hybrid_configs(name)[0]
 
 
+def chunk_configs(name: str):
+  """(Torinex-design config, the closest existing model: a Mixtral-style stack -- grouped-query softmax attention, SwiGLU
+  and every second layer 8 SiLU experts, 2 chosen, plus a shared expert -- of equal width, depth, heads, feed-forward and
+  expert sizes).  Torinex layers: attention inside chunks (the size's chunk) with norms over the whole projections, relu^2
+  feed-forward and clamped experts (4 groups, 2 kept) in turn, a side input of 256 per layer; the last layer borrows the
+  keys and values of the one before it."""
+  from xotorch_support_jetson_amd.models.config import ModelConfig, from_hf_config
+  z = MIXER_SIZES[name]
+  H, G, d, chunk, rot = z["attn"]
+  W, L = z["width"], z["layers"]
+  fe = (z["ff"] // 2 + 127) // 128 * 128
+  mix = {"heads": H, "kv_heads": G, "dim": d, "vdim": d, "scale": d ** -0.5, "mask": {"size": chunk}, "rot": {"base": 5e5, "dims": d}}
+  moe = {"kind": "moe", "expert": {"ff": fe, "limit": 7.0}, "router": {"experts": 8, "top": 2, "groups": {"count": 4, "keep": 2}},
+         "shared": {"ff": fe, "limit": 7.0}}
+  layers = [{"type": "attention", "mlp": moe if i % 2 == 0 else {"kind": "dense", "ff": z["ff"]},
+             "mixer": dict(mix, kv_from=i - 1) if i == L - 1 else mix} for i in range(L)]
+  chunked = from_hf_config({"architecture": "Torinex", "vocab": 32000, "width": W, "norm": {"eps": 1e-5}, "token_side": {"dim": 256},
+                            "layers": layers})
+  mixtral = ModelConfig("mixtral", 32000, W, z["ff"], L, H, G, d, 1e-5, 5e5, None, 32768, True, num_experts=8,
+                        num_experts_per_tok=2, bos_token_id=1, eos_token_ids=(2,), moe_intermediate_size=fe,
+                        n_shared_experts=1, moe_layer_freq=2)
+  return chunked, mixtral
+
+
 def bench_mixers(args, sizes=None, kinds=("tarepel", "llama"), configs=mixer_configs,
                  what="Tarepel-design layers beside a Llama-style stack of equal size"):
   """Prefill and decode throughput of mixed-layer designs at sizes like a real model's (random weights), beside
@@ -298,7 +322,11 @@ def main():
                   help="instead of the headline: Kopalorn-design layers (differential window attention, mlstm, gated "
                        "attention beside lightning attention, relu^2 experts with grouped sigmoid routing) beside the "
                        "Mogelix-design stack at the named sizes; one GPU")
-  ap.add_argument("--mixer-batch", type=int, default=16, help="--mixers / --hybrid / --latent / --memory: sequences per step")
+  ap.add_argument("--chunked", default=None, metavar="SIZES",
+                  help="instead of the headline: Torinex-design layers (chunk-local attention with projection norms, relu^2 "
+                       "and clamped-expert feed-forwards, side inputs) beside a Mixtral-style stack at the named sizes; one GPU")
+  ap.add_argument("--mixer-batch", type=int, default=16,
+                  help="--mixers / --hybrid / --latent / --memory / --chunked: sequences per step")
   args = ap.parse_args()
   os.environ["XOT_WEIGHT_DTYPE"] = args.weight_dtype
   if args.mixers:
@@ -314,6 +342,10 @@ def main():
   if args.memory:
     return bench_mixers(args, args.memory, ("kopalorn", "mogelix"), memory_configs,
                         "Kopalorn-design layers beside a Mogelix-design stack of equal size")
+
+  if args.chunked:
+    return bench_mixers(args, args.chunked, ("torinex", "mixtral"), chunk_configs,
+                        "Torinex-design layers beside a Mixtral-style stack of equal size")
 
   from xotorch_support_jetson_amd.models.config import preset
   from xotorch_support_jetson_amd.parallel.comm import P2PTransport, init_distributed

@@ -19,6 +19,12 @@
 #include "mixer_util.h"
 
 namespace xot {
+
+// csrc/window_attention.hip
+bool window_attention(const at::Tensor& q, const at::Tensor& k_cache, const at::Tensor& v_cache, const at::Tensor& block_tables,
+                      const at::Tensor& cu_q, const at::Tensor& ctx_lens, const float* sink, double scale, int64_t window,
+                      int64_t chunk, at::Tensor& out, int64_t ldo, int64_t max_qlen);
+
 namespace {
 using namespace mix;
 
@@ -946,6 +952,9 @@ void attn_window_pool(const at::Tensor& q, const at::Tensor& k_cache, const at::
   MCHECK(!pooled || Gv == G, "pooled blocks need a value head per key head");
   const int ldo = act_ld(out, T, H * dv, "out");
   const bool o32 = out.scalar_type() == at::kFloat;
+  if (q.scalar_type() == at::kBFloat16 && !pooled && WATT_MFMA &&
+      window_attention(q, k_cache, v_cache, block_tables, cu_q, ctx_lens, sp, scale, window, chunk, out, ldo, max_qlen))
+    return;
   // the MFMA kernel: bf16 caches, runs of 16 tokens or more, value size = key size in {32, 64, 96, 128} (bf16 or fp32 output)
   // or twice the key size in {32, 64} with fp32 output (differential attention's maps), or (bf16 output, no pooled blocks)
   // any two sizes up to 128 that are multiples of 8
