@@ -210,3 +210,88 @@ def test_grouped_gemm_with_the_clamped_epilogue(T, E, k, F, D, bm, shuffled):
     want = oracle.clamped_expert(x[tok[lo:hi].long()].double(), dict(t, gate=g[e].double(), up=u[e].double()), "", lim)
     if hi > lo:
       close(act[lo:hi], want, 1e-2, f"expert {e}")
+
+
+@pytest.mark.gpu
+@pytest.mark.parametrize("M", [1, 5, 40, 130, 300, 520, 2100])
+@pytest.mark.parametrize("N,D", [(256, 128), (512, 384), (768, 256)])
+def test_gemm_with_the_feed_forward_epilogues(M, N, D):
+  """relu^2 and the clamped gate in the epilogue of the dense projections, every kernel configuration the policy would try."""
+  from xotorch_support_jetson_amd.ops import linear as L
+  lim = 0.9
+  x = rnd(M, D, seed=1).bfloat16()
+  w = rnd(N, D, seed=2, scale=D ** -0.5 * 2).bfloat16()
+  up = torch.relu(x.double() @ w.double().T) ** 2
+  g, u = w[:N // 2], w[N // 2:]
+  glu = oracle.clamped_expert(x.double(), {"gate": g.double(), "up": u.double(), "down": torch.eye(N // 2, dtype=F64)}, "", lim)
+  for epi, wt, want in (("relu2", w, up), ("clamp_glu", interleave_gate_up(g, u), glu)):
+    ws = L.to_stream_layout(wt.contiguous().cuda())
+    xd = x.cuda()
+    close(L.linear(xd, ws, epi=epi, epi_arg=lim), want, 1.5e-2, f"{epi} as chosen")
+    cands = [("stream",) + c for c in L.policy._stream_cands(M, N, D, epi)] if M <= 512 else []
+    if M >= 65:
+      cands += [c for c in L.policy._big_cands(M, N, D) if c[1] in (2256, 128, 4256)]
+    for cfg in cands:
+      out = torch.full((M, want.shape[1]), 7.0, dtype=torch.bfloat16, device="cuda")
+      L._shuffled_call(xd, ws, None, None, epi, out, cfg, lim)
+      close(out, want, 1.5e-2, f"{epi} {cfg}")
+
+
+@pytest.mark.gpu
+@pytest.mark.parametrize("M", [1, 30])
+def test_split_projection_read_as_slabs(M):
+  """A split-K projection left unreduced: the consumers' sums equal the reduced product's results."""
+  from xotorch_support_jetson_amd.ops import linear as L
+  D, N, n = 1024, 256, 200
+  x, w = rnd(M, D, seed=1).bfloat16().cuda(), L.to_stream_layout(rnd(N, D, seed=2, scale=D ** -0.5).bfloat16().cuda())
+  key = ("sh", L._m_bucket(M), N, D, "none", False, str(torch.float32))
+  keep = L.policy.table.get(key)
+  try:
+    L.policy.table[key] = ("stream", 1, 4)
+    full = L.linear(x, w, out_dtype=torch.float32).clone()
+    res = {}
+    for name, P in (("slabs", L.linear_slabs(x, w)), ("reduced", full)):
+      assert (P.dim() == 3) == (name == "slabs")
+      h, o = rnd(M, n, seed=3).cuda(), torch.zeros(M, n, dtype=torch.bfloat16, device="cuda")
+      K.sandwich_add_norm(h, P, rnd(n, seed=4).cuda(), None, 1e-5, o, yb=rnd(n, seed=5).cuda())
+      e = torch.zeros(M, 64, dtype=torch.bfloat16, device="cuda")
+      K.gelu_gather_mul(P, 100, rnd(9, 64, seed=6).bfloat16().cuda(), torch.arange(M, dtype=torch.int32, device="cuda") % 9, 3, 60, e)
+      q = torch.empty(M, 4, 24, dtype=torch.bfloat16, device="cuda")
+      kc, vc = (torch.zeros(1, 2, *s, dtype=torch.bfloat16, device="cuda") for s in ((64, 24), (20, 64)))
+      K.qk_norm_rope_store(P, rnd(N, seed=7).cuda(), 0, 96, 144, 4, 2, 24, 20, 16, torch.arange(M, dtype=torch.int32, device="cuda"),
+                           build_cos_sin(16, 64, 100.0, None, torch.device("cuda")), torch.arange(M, device="cuda"), 1e-5, False, q,
+                           kc, vc, rnd(96, seed=8).cuda(), rnd(48, seed=9).cuda())
+      res[name] = [t.double().cpu() for t in (h, o, e, q, kc, vc)]
+    for a, b in zip(res["slabs"], res["reduced"]):
+      close(a, b, 8e-3)
+  finally:
+    if keep is None:
+      L.policy.table.pop(key, None)
+    else:
+      L.policy.table[key] = keep
+
+
+@pytest.mark.gpu
+@pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
+def test_values_of_many_tokens_are_stored_through_tiles(dtype):
+  """300 tokens of several sequences at scrambled slots (some without one): keys and values as one by one."""
+  T, H, G, d, dv = 300, 6, 3, 8, 40
+  P = rnd(T, H * d + G * (d + dv), seed=1).cuda()
+  slots = torch.randperm(384, generator=torch.Generator().manual_seed(2))[:T].cuda()
+  slots[::17] = -1
+  pos, tab = torch.arange(T, dtype=torch.int32, device="cuda") % 100, build_cos_sin(8, 100, 100.0, None, torch.device("cuda"))
+  res = []
+  for step in (T, 50):  # (50 tokens at a time: written by the rotation kernel itself)
+    q = torch.empty(T, H, d, dtype=dtype, device="cuda")
+    kc, vc = torch.full((6, G, 64, d), 5.0, dtype=dtype, device="cuda"), torch.full((6, G, dv, 64), 5.0, dtype=dtype, device="cuda")
+    for lo in range(0, T, step):
+      s = slice(lo, lo + step)
+      K.qk_norm_rope_store(P[s], None, 0, H * d, (H + G) * d, H, G, d, dv, 8, pos[s], tab, slots[s].contiguous(), 1e-5, False, q[s], kc, vc,
+                           torch.ones(H * d, device="cuda"), torch.ones(G * d, device="cuda"))
+    res.append((q, kc, vc))
+  for a, b in zip(*res):
+    assert torch.equal(a, b)
+  ok = (slots >= 0).cpu()
+  s = slots.cpu()[ok]
+  want = P[:, (H + G) * d:].cpu()[ok].reshape(-1, G, dv).to(dtype)
+  assert torch.equal(res[0][2].cpu()[s // 64, :, :, s % 64], want)

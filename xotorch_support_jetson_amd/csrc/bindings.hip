@@ -240,7 +240,7 @@ void gemm(const at::Tensor& x, const at::Tensor& w, at::Tensor& y, const c10::op
 // an fp32 workspace of >= splits*M*N floats).  ntw: 16-row n-tiles per wave (1 or 2).
 void gemm_stream(const at::Tensor& x, const at::Tensor& w, at::Tensor& y, const c10::optional<at::Tensor>& bias,
                  const c10::optional<at::Tensor>& res, const c10::optional<at::Tensor>& ws, int64_t epi, int64_t ntw,
-                 int64_t splits, bool wshuf, bool reduce) {
+                 int64_t splits, bool wshuf, bool reduce, double epi_arg) {
   CHECK_BF16(x);
   CHECK_BF16(w);
   CHECK_GPU(y);
@@ -251,7 +251,7 @@ void gemm_stream(const at::Tensor& x, const at::Tensor& w, at::Tensor& y, const 
   XCHECK(w.size(1) == K, "gemm_stream: K mismatch");
   const bool f32 = y.scalar_type() == at::kFloat;
   XCHECK(f32 || y.scalar_type() == at::kBFloat16, "gemm_stream: y must be bf16 or fp32");
-  XCHECK(y.size(0) == M && y.size(1) == (epi == 2 ? N / 2 : N), "gemm_stream: y shape mismatch");
+  XCHECK(y.size(0) == M && y.size(1) == (epi == 2 || epi == 3 ? N / 2 : N), "gemm_stream: y shape mismatch");
   XCHECK(M <= 65536, "gemm_stream: M must be <= 65536");
   if (bias.has_value()) {
     CHECK_BF16((*bias));
@@ -277,7 +277,7 @@ void gemm_stream(const at::Tensor& x, const at::Tensor& w, at::Tensor& y, const 
   const int rc = xot::launch_gemm_stream(bf(x), (int)x.stride(0), bf(w), (int)K, bf_opt(bias),
                                          epi == 1 ? bf(*res) : nullptr, (int)ldr, y.data_ptr(), (int)y.stride(0), f32,
                                          (int)epi, wsp, ws_elems, (int)M, (int)N, (int)K, (int)ntw, (int)splits,
-                                         wshuf, reduce, cur_stream());
+                                         wshuf, reduce, (float)epi_arg, cur_stream());
   XCHECK(rc == 0, "gemm_stream: unsupported shape M=", M, " N=", N, " K=", K, " epi=", epi, " ntw=", ntw,
          " splits=", splits);
 }
@@ -380,7 +380,7 @@ void gemm_stream8(const at::Tensor& x, const at::Tensor& w8, const at::Tensor& w
 // bn: 256 or 128 output columns per workgroup; splits > 1 needs an fp32 workspace of splits*M*N.
 void gemm_big(const at::Tensor& x, const at::Tensor& w, at::Tensor& y, const c10::optional<at::Tensor>& bias,
               const c10::optional<at::Tensor>& res, const c10::optional<at::Tensor>& ws, int64_t epi, int64_t bn,
-              int64_t splits, bool reduce) {
+              int64_t splits, bool reduce, double epi_arg) {
   CHECK_BF16(x);
   CHECK_BF16(w);
   CHECK_GPU(y);
@@ -391,7 +391,7 @@ void gemm_big(const at::Tensor& x, const at::Tensor& w, at::Tensor& y, const c10
   XCHECK(w.size(1) == K, "gemm_big: K mismatch");
   const bool f32 = y.scalar_type() == at::kFloat;
   XCHECK(f32 || y.scalar_type() == at::kBFloat16, "gemm_big: y must be bf16 or fp32");
-  XCHECK(y.size(0) == M && y.size(1) == (epi == 2 ? N / 2 : N), "gemm_big: y shape mismatch");
+  XCHECK(y.size(0) == M && y.size(1) == (epi == 2 || epi == 3 ? N / 2 : N), "gemm_big: y shape mismatch");
   XCHECK(M <= (1 << 24), "gemm_big: M too large");
   if (bias.has_value()) {
     CHECK_BF16((*bias));
@@ -415,7 +415,7 @@ void gemm_big(const at::Tensor& x, const at::Tensor& w, at::Tensor& y, const c10
   }
   const int rc = xot::launch_gemm_big(bf(x), (int)x.stride(0), bf(w), bf_opt(bias), epi == 1 ? bf(*res) : nullptr,
                                       (int)ldr, y.data_ptr(), (int)y.stride(0), f32, (int)epi, wsp, ws_elems, (int)M,
-                                      (int)N, (int)K, (int)bn, (int)splits, reduce, cur_stream());
+                                      (int)N, (int)K, (int)bn, (int)splits, reduce, (float)epi_arg, cur_stream());
   XCHECK(rc == 0, "gemm_big: unsupported shape M=", M, " N=", N, " K=", K, " epi=", epi, " bn=", bn,
          " splits=", splits);
 }
@@ -1036,7 +1036,7 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("gemm", &gemm);
   m.def("gemm_stream", &gemm_stream, py::arg("x"), py::arg("w"), py::arg("y"), py::arg("bias"), py::arg("res"),
         py::arg("ws"), py::arg("epi"), py::arg("ntw"), py::arg("splits"), py::arg("wshuf"),
-        py::arg("reduce") = true);
+        py::arg("reduce") = true, py::arg("epi_arg") = 0.0);
   m.def("gemm_stream_norm", &gemm_stream_norm, py::arg("w"), py::arg("y"), py::arg("bias"), py::arg("ws"),
         py::arg("epi"), py::arg("ntw"), py::arg("splits"), py::arg("reduce"), py::arg("h"), py::arg("ws_in"),
         py::arg("s_in"), py::arg("bias_in"), py::arg("lnw"), py::arg("hout"), py::arg("eps"));
@@ -1048,7 +1048,8 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("gemm_batched", &gemm_batched, py::arg("x"), py::arg("xbat"), py::arg("K"), py::arg("w"), py::arg("y"),
         py::arg("ybat"), py::arg("ldy"), py::arg("M"));
   m.def("gemm_big", &gemm_big, py::arg("x"), py::arg("w"), py::arg("y"), py::arg("bias"), py::arg("res"),
-        py::arg("ws"), py::arg("epi"), py::arg("bn"), py::arg("splits"), py::arg("reduce") = true);
+        py::arg("ws"), py::arg("epi"), py::arg("bn"), py::arg("splits"), py::arg("reduce") = true,
+        py::arg("epi_arg") = 0.0);
   m.def("splitk_resid_rmsnorm", &splitk_resid_rmsnorm);
   m.def("gemm_moe", &gemm_moe, py::arg("x"), py::arg("w"), py::arg("y"), py::arg("off"), py::arg("gather"),
         py::arg("epi"), py::arg("max_rows"), py::arg("wshuf"), py::arg("splits") = 1, py::arg("big_bm") = 0,

@@ -8,7 +8,8 @@
 //       EPI_NONE     Y = acc (+bias)
 //       EPI_RESID    Y = R + acc (+bias)          (o_proj / down_proj + residual stream)
 //       EPI_SILU     Y[:, j] = silu(acc_gate) * acc_up   (gate/up weights interleaved per 16 rows)
-//       EPI_CLAMP_GLU  the clamped gated form of the same pairs (grouped expert GEMMs; limit: epi_arg)
+//       EPI_CLAMP_GLU  the clamped gated form of the same pairs (limit: epi_arg; pre-shuffled weights)
+//       EPI_RELU2    Y = relu(acc (+bias))^2                           (pre-shuffled weights)
 //  * gemm_tiled: prefill-shaped M.  128x128x64 LDS tiles, 4 waves in 2x2, register-staged
 //    global->LDS copy of tile k+1 overlapped with the MFMAs of tile k (async-STAGE split),
 //    padded rows (144 B) so every 16-lane ds_read_b128 group hits 16 distinct bank quads.
@@ -650,6 +651,7 @@ __global__ __launch_bounds__(256, OCC) void gemm_stream_kernel(const uint16_t* _
           if (m < M) {
             float v = acc[i][j][r] + b;
             if constexpr (EPI == EPI_RESID) v += bf2f(R[(size_t)m * ldr + col]);
+            v = epi_elem<EPI>(v);
             if constexpr (OUT_F32)
               reinterpret_cast<float*>(Yv)[(size_t)m * ldy + col] = v;
             else
@@ -663,7 +665,7 @@ __global__ __launch_bounds__(256, OCC) void gemm_stream_kernel(const uint16_t* _
 template <int MT, int NTW, int KS, int EPI, bool F32, bool WSH, bool W8 = false>
 static void stream_launch(const uint16_t* X, int ldx, const uint16_t* W, int ldw, const uint16_t* bias,
                           const uint16_t* R, int ldr, void* Y, int ldy, float* ws, int M, int N, int K, int S,
-                          bool reduce, hipStream_t st, const float* wscale = nullptr) {
+                          bool reduce, hipStream_t st, const float* wscale = nullptr, float epi_arg = 0.f) {
   // occupancy request: 2 workgroups/CU while the register budget allows it (FP8 weights need a few more
   // registers for the widened fragments)
   constexpr int OCC = (MT * NTW >= (W8 ? 16 : 32)) ? 1 : 2;
@@ -679,7 +681,7 @@ static void stream_launch(const uint16_t* X, int ldx, const uint16_t* W, int ldw
       (void)attr;
     }
     kern<<<grid, 256, SMEM, st>>>(X, ldx, W, ldw, bias, R, ldr, Y, ldy, nullptr, M, N, kper, mblocks, nullptr, nullptr,
-                                  nullptr, 0L, wscale, 0L, 0L, NormPro{}, 0.f);
+                                  nullptr, 0L, wscale, 0L, 0L, NormPro{}, epi_arg);
   } else {
     auto kern = gemm_stream_kernel<MT, NTW, KS, EPI, F32, true, WSH, OCC, 0, W8>;
     if constexpr (SMEM > 65536) {
@@ -688,21 +690,21 @@ static void stream_launch(const uint16_t* X, int ldx, const uint16_t* W, int ldw
       (void)attr;
     }
     kern<<<grid, 256, SMEM, st>>>(X, ldx, W, ldw, bias, R, ldr, Y, ldy, ws, M, N, kper, mblocks, nullptr, nullptr,
-                                  nullptr, 0L, wscale, 0L, 0L, NormPro{}, 0.f);
+                                  nullptr, 0L, wscale, 0L, 0L, NormPro{}, epi_arg);
     if (!reduce) return;  // slabs left for the consumer
-    const int ncol = EPI == EPI_SILU ? N / 2 : N;
+    const int ncol = epi_is_glu(EPI) ? N / 2 : N;
     long chunks = (long)M * (ncol / 8);
     int blocks = (int)((chunks + 255) / 256);
     if (blocks > 2048) blocks = 2048;
-    splitk_reduce_kernel<EPI, F32><<<blocks, 256, 0, st>>>(ws, S, M, N, bias, R, ldr, Y, ldy);
+    splitk_reduce_kernel<EPI, F32><<<blocks, 256, 0, st>>>(ws, S, M, N, bias, R, ldr, Y, ldy, epi_arg);
   }
 }
 
 template <int EPI, bool F32>
 static int stream_dispatch(const uint16_t* X, int ldx, const uint16_t* W, int ldw, const uint16_t* bias,
                            const uint16_t* R, int ldr, void* Y, int ldy, float* ws, long ws_elems, int M, int N,
-                           int K, int ntw, int S, bool wshuf, bool reduce, hipStream_t st) {
-  if (EPI == EPI_SILU && ntw == 1) ntw = 2;
+                           int K, int ntw, int S, bool wshuf, bool reduce, hipStream_t st, float epi_arg = 0.f) {
+  if (epi_is_glu(EPI) && ntw == 1) ntw = 2;
   if (ntw != 1 && ntw != 2 && ntw != 4) return -1;
   const int mt = (M + 15) / 16;
   if (ntw == 4 && mt <= 2) ntw = 2;
@@ -710,22 +712,27 @@ static int stream_dispatch(const uint16_t* X, int ldx, const uint16_t* W, int ld
   const int KS = 4;
   if (K % (S * 32 * KS) != 0) return -1;  // whole 128-deep k-chunks per workgroup (odd counts: single tail)
   if (S > 1 && (ws == nullptr || ws_elems < (long)S * M * N)) return -1;
-  if (EPI == EPI_SILU && N % 32 != 0) return -1;
+  if (epi_is_glu(EPI) && N % 32 != 0) return -1;
+  constexpr bool SHUF_ONLY = EPI == EPI_CLAMP_GLU || EPI == EPI_RELU2;  // (built for pre-shuffled weights only)
+  if (SHUF_ONLY && !wshuf) return -1;
   if (wshuf && (KS != 4 || K % 128 != 0)) return -1;
 #define XOT_ST2(MTV, KSV, WSH)                                                                              \
   do {                                                                                                      \
-    if (ntw == 1 && EPI != EPI_SILU)                                                                        \
-      stream_launch<MTV, 1, KSV, EPI, F32, WSH>(X, ldx, W, ldw, bias, R, ldr, Y, ldy, ws, M, N, K, S, reduce, st);  \
+    if (ntw == 1 && !epi_is_glu(EPI))                                                                       \
+      stream_launch<MTV, 1, KSV, EPI, F32, WSH>(X, ldx, W, ldw, bias, R, ldr, Y, ldy, ws, M, N, K, S, reduce, st, nullptr, epi_arg);  \
     else if (ntw == 4 && MTV >= 4 && MTV <= 8)                                                                    \
-      stream_launch<MTV, 4, KSV, EPI, F32, WSH>(X, ldx, W, ldw, bias, R, ldr, Y, ldy, ws, M, N, K, S, reduce, st);  \
+      stream_launch<MTV, 4, KSV, EPI, F32, WSH>(X, ldx, W, ldw, bias, R, ldr, Y, ldy, ws, M, N, K, S, reduce, st, nullptr, epi_arg);  \
     else                                                                                                    \
-      stream_launch<MTV, 2, KSV, EPI, F32, WSH>(X, ldx, W, ldw, bias, R, ldr, Y, ldy, ws, M, N, K, S, reduce, st);  \
+      stream_launch<MTV, 2, KSV, EPI, F32, WSH>(X, ldx, W, ldw, bias, R, ldr, Y, ldy, ws, M, N, K, S, reduce, st, nullptr, epi_arg);  \
     return 0;                                                                                               \
   } while (0)
 #define XOT_ST(MTV, KSV)                  \
   do {                                    \
-    if (wshuf) XOT_ST2(MTV, KSV, true);   \
-    XOT_ST2(MTV, KSV, false);             \
+    if constexpr (SHUF_ONLY) XOT_ST2(MTV, KSV, true); \
+    else {                                \
+      if (wshuf) XOT_ST2(MTV, KSV, true); \
+      XOT_ST2(MTV, KSV, false);           \
+    }                                     \
   } while (0)
   if (mt <= 1) XOT_ST(1, 4);
   if (mt <= 2) XOT_ST(2, 4);
@@ -949,8 +956,12 @@ int launch_gemm_stream_norm(const uint16_t* W, const uint16_t* bias, void* Y, in
 int launch_gemm_stream(const uint16_t* X, int ldx, const uint16_t* W, int ldw, const uint16_t* bias,
                        const uint16_t* R, int ldr, void* Y, int ldy, bool out_f32, int epi, float* ws, long ws_elems,
                        int M, int N, int K, int ntw, int S, bool wshuf, bool reduce,
-                       hipStream_t s) {
+                       float epi_arg, hipStream_t s) {
   if (M <= 0) return 0;
+  if (epi == EPI_CLAMP_GLU)
+    return out_f32 ? -1 : stream_dispatch<EPI_CLAMP_GLU, false>(X, ldx, W, ldw, bias, R, ldr, Y, ldy, ws, ws_elems, M, N, K, ntw, S, wshuf, reduce, s, epi_arg);
+  if (epi == EPI_RELU2)
+    return out_f32 ? -1 : stream_dispatch<EPI_RELU2, false>(X, ldx, W, ldw, bias, R, ldr, Y, ldy, ws, ws_elems, M, N, K, ntw, S, wshuf, reduce, s);
   if (epi == EPI_SILU)
     return out_f32 ? stream_dispatch<EPI_SILU, true>(X, ldx, W, ldw, bias, R, ldr, Y, ldy, ws, ws_elems, M, N, K, ntw, S, wshuf, reduce, s)
                    : stream_dispatch<EPI_SILU, false>(X, ldx, W, ldw, bias, R, ldr, Y, ldy, ws, ws_elems, M, N, K, ntw, S, wshuf, reduce, s);

@@ -480,6 +480,7 @@ __global__ __launch_bounds__(512, 1) void gemm_big_kernel(const uint16_t* __rest
           if (m < Mv) {
             float v = acc[i0 + i][j][r] + bv;
             if constexpr (EPI == EPI_RESID) v += rv[i][r];
+            v = epi_elem<EPI>(v);
             if constexpr (OUT_F32)
               reinterpret_cast<float*>(Yv)[(size_t)m * ldy + col] = v;
             else
@@ -510,7 +511,7 @@ int gemm_big_group_m() {
 template <int BM, int BN, int WM, int WN, int BK, int NBUF, int EPI, bool F32, int PP = 0>
 static void big_launch(const uint16_t* X, int ldx, const uint16_t* W, const uint16_t* bias, const uint16_t* R,
                        int ldr, void* Y, int ldy, float* ws, int M, int N, int K, int S, bool reduce,
-                       hipStream_t st) {
+                       hipStream_t st, float epi_arg) {
   constexpr int SMEM = big_smem<BM, BN, BK, NBUF>();
   static_assert(SMEM <= 160 * 1024, "LDS");
   const int nwg = ((M + BM - 1) / BM) * ((N + BN - 1) / BN) * S;
@@ -520,45 +521,51 @@ static void big_launch(const uint16_t* X, int ldx, const uint16_t* W, const uint
                        hipSuccess;
     (void)attr;
     kern<<<nwg, 512, SMEM, st>>>(X, ldx, W, bias, R, ldr, Y, ldy, nullptr, M, N, K, 1, nullptr, nullptr, 0L,
-                                 big_group_m(), 0.f);
+                                 big_group_m(), epi_arg);
   } else {
     auto kern = gemm_big_kernel<BM, BN, WM, WN, BK, NBUF, EPI, false, true, 0, 0, 3, PP>;
     static bool attr = hipFuncSetAttribute((const void*)kern, hipFuncAttributeMaxDynamicSharedMemorySize, SMEM) ==
                        hipSuccess;
     (void)attr;
     kern<<<nwg, 512, SMEM, st>>>(X, ldx, W, bias, R, ldr, Y, ldy, ws, M, N, K, S, nullptr, nullptr, 0L,
-                                 big_group_m(), 0.f);
+                                 big_group_m(), epi_arg);
     if (!reduce) return;  // slabs left for the consumer (fused reduce + residual + RMSNorm)
-    const int ncol = EPI == EPI_SILU ? N / 2 : N;
+    const int ncol = epi_is_glu(EPI) ? N / 2 : N;
     const long chunks = (long)M * (ncol / 8);
     int blocks = (int)((chunks + 255) / 256);
     if (blocks > 2048) blocks = 2048;
-    splitk_reduce_kernel<EPI, F32><<<blocks, 256, 0, st>>>(ws, S, M, N, bias, R, ldr, Y, ldy);
+    splitk_reduce_kernel<EPI, F32><<<blocks, 256, 0, st>>>(ws, S, M, N, bias, R, ldr, Y, ldy, epi_arg);
   }
 }
 
 template <int EPI, bool F32>
 static int big_dispatch(const uint16_t* X, int ldx, const uint16_t* W, const uint16_t* bias, const uint16_t* R,
                         int ldr, void* Y, int ldy, float* ws, long ws_elems, int M, int N, int K, int bn, int S,
-                        bool reduce, hipStream_t st) {
+                        bool reduce, hipStream_t st, float epi_arg = 0.f) {
   // bn = tile code: BN (256 / 128 / 224), 1256 / 2256 (256 x 256 on the four- / two-phase ping-pong), plus
   // 10000 x BM for row tiles below 256 (160 / 192 / 224: M = 320 / 384 / 448 in two tiles without padding rows;
   // 2256 only with 192)
   const int bm = bn / 10000 ? bn / 10000 : 256, code = bn % 10000;
   if (code == 4256 && bm == 256) {  // four-wave 256 x 256 tile (gemm_w4.hip)
-    const int rc = launch_gemm_w4(X, ldx, W, bias, R, ldr, Y, ldy, F32, EPI, ws, M, N, K, S, big_group_m(), st);
+    const int rc = launch_gemm_w4(X, ldx, W, bias, R, ldr, Y, ldy, F32, EPI, ws, M, N, K, S, big_group_m(), epi_arg, st);
     if (rc != 0 || S == 1 || !reduce) return rc;
-    const int ncol = EPI == EPI_SILU ? N / 2 : N;
+    const int ncol = epi_is_glu(EPI) ? N / 2 : N;
     const long chunks = (long)M * (ncol / 8);
     int blocks = (int)((chunks + 255) / 256);
     if (blocks > 2048) blocks = 2048;
-    splitk_reduce_kernel<EPI, F32><<<blocks, 256, 0, st>>>(ws, S, M, N, bias, R, ldr, Y, ldy);
+    splitk_reduce_kernel<EPI, F32><<<blocks, 256, 0, st>>>(ws, S, M, N, bias, R, ldr, Y, ldy, epi_arg);
     return 0;
   }
 #define XOT_BIG(BM_, BN_, WM_, NBUF_, ...)                                                                        \
   big_launch<BM_, BN_, WM_, 8 / WM_, 64, NBUF_, EPI, F32, ##__VA_ARGS__>(X, ldx, W, bias, R, ldr, Y, ldy, ws, M, N, K, \
-                                                                         S, reduce, st)
-  if (bm == 256) {
+                                                                         S, reduce, st, epi_arg)
+  if constexpr (EPI == EPI_CLAMP_GLU || EPI == EPI_RELU2) {  // (built for the tiles that win: two-phase 256, 128 columns)
+    if (bm != 256) return -1;
+    if (code == 2256) XOT_BIG(256, 256, 2, 2, 2);
+    else if (code == 128) XOT_BIG(256, 128, 4, 3);
+    else return -1;
+    return 0;
+  } else if (bm == 256) {
     if (code == 256) XOT_BIG(256, 256, 2, 2);
     else if (code == 1256) XOT_BIG(256, 256, 2, 2, 1);  // ping-pong schedule of the 256 x 256 tile
     else if (code == 2256) XOT_BIG(256, 256, 2, 2, 2);  // the same in two phases per stage (4 barriers, not 8)
@@ -587,11 +594,15 @@ static int big_dispatch(const uint16_t* X, int ldx, const uint16_t* W, const uin
 
 int launch_gemm_big(const uint16_t* X, int ldx, const uint16_t* W, const uint16_t* bias, const uint16_t* R, int ldr,
                     void* Y, int ldy, bool out_f32, int epi, float* ws, long ws_elems, int M, int N, int K, int bn,
-                    int S, bool reduce, hipStream_t s) {
+                    int S, bool reduce, float epi_arg, hipStream_t s) {
   if (M <= 0) return 0;
   if (N % 16 != 0 || K % 128 != 0 || S < 1 || S > K / 64) return -1;  // tile codes: big_dispatch
   if (S > 1 && (ws == nullptr || ws_elems < (long)S * M * N)) return -1;
-  if (epi == EPI_SILU && N % 32 != 0) return -1;
+  if (epi_is_glu(epi) && N % 32 != 0) return -1;
+  if (epi == EPI_CLAMP_GLU)
+    return out_f32 ? -1 : big_dispatch<EPI_CLAMP_GLU, false>(X, ldx, W, bias, R, ldr, Y, ldy, ws, ws_elems, M, N, K, bn, S, reduce, s, epi_arg);
+  if (epi == EPI_RELU2)
+    return out_f32 ? -1 : big_dispatch<EPI_RELU2, false>(X, ldx, W, bias, R, ldr, Y, ldy, ws, ws_elems, M, N, K, bn, S, reduce, s);
   if (epi == EPI_SILU)
     return out_f32 ? big_dispatch<EPI_SILU, true>(X, ldx, W, bias, R, ldr, Y, ldy, ws, ws_elems, M, N, K, bn, S, reduce, s)
                    : big_dispatch<EPI_SILU, false>(X, ldx, W, bias, R, ldr, Y, ldy, ws, ws_elems, M, N, K, bn, S, reduce, s);

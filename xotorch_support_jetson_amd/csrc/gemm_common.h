@@ -4,7 +4,7 @@
 
 namespace xot {
 
-enum { EPI_NONE = 0, EPI_RESID = 1, EPI_SILU = 2, EPI_CLAMP_GLU = 3 };
+enum { EPI_NONE = 0, EPI_RESID = 1, EPI_SILU = 2, EPI_CLAMP_GLU = 3, EPI_RELU2 = 4 };
 
 // epilogues that turn a (gate, up) column pair into one output column
 constexpr bool epi_is_glu(int epi) { return epi == EPI_SILU || epi == EPI_CLAMP_GLU; }
@@ -47,14 +47,24 @@ __device__ __forceinline__ void wait_vm_upto(int n) {
   }
 }
 
+// element-wise epilogues: relu(v)^2, or v as it is
+template <int EPI>
+__device__ __forceinline__ float epi_elem(float v) {
+  if constexpr (EPI == EPI_RELU2) {
+    v = fmaxf(v, 0.f);
+    return v * v;
+  }
+  return v;
+}
+
 // Sum the S fp32 slabs of one output row at 8 output columns [o, o+8) and apply the epilogue.
 // wsrow = slab 0 of this row (slabs are sstride floats apart); rrow / yrow = this row of R / Y.
 template <int EPI, bool OUT_F32>
 __device__ __forceinline__ void splitk_out8(const float* __restrict__ wsrow, size_t sstride, int S, int o,
                                             const uint16_t* __restrict__ bias, const uint16_t* __restrict__ rrow,
-                                            void* __restrict__ yrow) {
+                                            void* __restrict__ yrow, float epi_arg = 0.f) {
   float v[8];
-  if constexpr (EPI == EPI_SILU) {
+  if constexpr (epi_is_glu(EPI)) {
     const int j = o >> 4, w = o & 15;
     float gs[8], us[8];
 #pragma unroll
@@ -76,7 +86,7 @@ __device__ __forceinline__ void splitk_out8(const float* __restrict__ wsrow, siz
 #pragma unroll
     for (int e = 0; e < 8; ++e) {
       const float bg = bias ? bf2f(bias[32 * j + w + e]) : 0.f, bu = bias ? bf2f(bias[32 * j + 16 + w + e]) : 0.f;
-      v[e] = silu(gs[e] + bg) * (us[e] + bu);
+      v[e] = glu_pair<EPI>(gs[e] + bg, us[e] + bu, epi_arg);
     }
   } else {
 #pragma unroll
@@ -100,6 +110,8 @@ __device__ __forceinline__ void splitk_out8(const float* __restrict__ wsrow, siz
 #pragma unroll
       for (int e = 0; e < 8; ++e) v[e] += bf2f(rr[e]);
     }
+#pragma unroll
+    for (int e = 0; e < 8; ++e) v[e] = epi_elem<EPI>(v[e]);
   }
   if constexpr (OUT_F32) {
     float* y = reinterpret_cast<float*>(yrow) + o;
@@ -118,8 +130,8 @@ template <int EPI, bool OUT_F32>
 __global__ __launch_bounds__(256) void splitk_reduce_kernel(const float* __restrict__ ws, int S, int M, int N,
                                                             const uint16_t* __restrict__ bias,
                                                             const uint16_t* __restrict__ R, int ldr,
-                                                            void* __restrict__ Yv, int ldy) {
-  const int ncol = EPI == EPI_SILU ? N / 2 : N;
+                                                            void* __restrict__ Yv, int ldy, float epi_arg = 0.f) {
+  const int ncol = epi_is_glu(EPI) ? N / 2 : N;
   const long total = (long)M * (ncol / 8);
   for (long t = blockIdx.x * 256L + threadIdx.x; t < total; t += (long)gridDim.x * 256) {
     const int m = (int)(t / (ncol / 8));
@@ -127,7 +139,7 @@ __global__ __launch_bounds__(256) void splitk_reduce_kernel(const float* __restr
     void* yrow = OUT_F32 ? (void*)(reinterpret_cast<float*>(Yv) + (size_t)m * ldy)
                          : (void*)(reinterpret_cast<uint16_t*>(Yv) + (size_t)m * ldy);
     splitk_out8<EPI, OUT_F32>(ws + (size_t)m * N, (size_t)M * N, S, o, bias,
-                              EPI == EPI_RESID ? R + (size_t)m * ldr : nullptr, yrow);
+                              EPI == EPI_RESID ? R + (size_t)m * ldr : nullptr, yrow, epi_arg);
   }
 }
 

@@ -111,10 +111,11 @@ __global__ __launch_bounds__(256, 1) void gemm_w4_kernel(const uint16_t* __restr
                                                          const uint16_t* __restrict__ bias,
                                                          const uint16_t* __restrict__ R, int ldr,
                                                          void* __restrict__ Yv, int ldy, float* __restrict__ ws,
-                                                         int M, int N, int K, int S, int group_m, int ldw) {
+                                                         int M, int N, int K, int S, int group_m, int ldw,
+                                                         float epi_arg) {
   using namespace w4;
-  static_assert(!TN || (!SPLIT && EPI != EPI_SILU), "TN: weight gradients (plain or residual epilogue)");
-  constexpr bool PERM = EPI != EPI_SILU && !TN;
+  static_assert(!TN || (!SPLIT && !epi_is_glu(EPI)), "TN: weight gradients (plain or residual epilogue)");
+  constexpr bool PERM = !epi_is_glu(EPI) && !TN;
   constexpr bool ASMRD = W4_ASMRD && !TN;
   extern __shared__ __attribute__((aligned(16))) uint16_t smem[];
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
@@ -537,6 +538,8 @@ __global__ __launch_bounds__(256, 1) void gemm_w4_kernel(const uint16_t* __restr
 #pragma unroll
               for (int e = 0; e < 8; ++e) v[e] += bf2f(rv[J][e]);
             }
+#pragma unroll
+            for (int e = 0; e < 8; ++e) v[e] = epi_elem<EPI>(v[e]);
             if constexpr (OUT_F32) {
               float* p = reinterpret_cast<float*>(Yv) + (size_t)m * ldy + col;
               *reinterpret_cast<f32x4*>(p) = f32x4{v[0], v[1], v[2], v[3]};
@@ -568,7 +571,7 @@ __global__ __launch_bounds__(256, 1) void gemm_w4_kernel(const uint16_t* __restr
             gv += bf2f(bias[gcol + r]);
             uv += bf2f(bias[gcol + 16 + r]);
           }
-          o4[r] = silu(gv) * uv;
+          o4[r] = glu_pair<EPI>(gv, uv, epi_arg);
         }
         const int col = obase + 16 * J + 4 * g;
         if constexpr (OUT_F32) {
@@ -588,13 +591,14 @@ __global__ __launch_bounds__(256, 1) void gemm_w4_kernel(const uint16_t* __restr
 
 template <int EPI, bool F32, bool SPLIT>
 static void w4_launch(const uint16_t* X, int ldx, const uint16_t* W, const uint16_t* bias, const uint16_t* R, int ldr,
-                      void* Y, int ldy, float* ws, int M, int N, int K, int S, int group_m, hipStream_t st) {
+                      void* Y, int ldy, float* ws, int M, int N, int K, int S, int group_m, hipStream_t st,
+                      float epi_arg = 0.f) {
   auto kern = gemm_w4_kernel<EPI, F32, SPLIT>;
   static bool attr =
       hipFuncSetAttribute((const void*)kern, hipFuncAttributeMaxDynamicSharedMemorySize, w4::SMEM) == hipSuccess;
   (void)attr;
   const int nwg = ((M + 255) / 256) * (N / 256) * S;
-  kern<<<nwg, 256, w4::SMEM, st>>>(X, ldx, W, bias, R, ldr, Y, ldy, ws, M, N, K, S, group_m, 0);
+  kern<<<nwg, 256, w4::SMEM, st>>>(X, ldx, W, bias, R, ldr, Y, ldy, ws, M, N, K, S, group_m, 0, epi_arg);
 }
 
 template <int EPI, bool F32>
@@ -605,7 +609,7 @@ static void w4_tn_launch(const uint16_t* Xt, int ldx, const uint16_t* Wt, int ld
       hipFuncSetAttribute((const void*)kern, hipFuncAttributeMaxDynamicSharedMemorySize, w4::SMEM) == hipSuccess;
   (void)attr;
   kern<<<(M / 256) * (N / 256), 256, w4::SMEM, st>>>(Xt, ldx, Wt, nullptr, R, ldr, Y, ldy, nullptr, M, N, K, 1,
-                                                       group_m, ldw);
+                                                       group_m, ldw, 0.f);
 }
 
 // Weight gradients on the token-major operands: Y [M, N] (+)= Xt^T . Wt, Xt [K, M] (ldx), Wt [K, N] (ldw); M, N
@@ -630,17 +634,21 @@ int launch_gemm_w4_tn(const uint16_t* Xt, int ldx, const uint16_t* Wt, int ldw, 
 // Tile code 4256 of launch_gemm_big.  S > 1 writes fp32 slabs (reduced by the caller's reduce kernel).
 int launch_gemm_w4(const uint16_t* X, int ldx, const uint16_t* W, const uint16_t* bias, const uint16_t* R, int ldr,
                    void* Y, int ldy, bool out_f32, int epi, float* ws, int M, int N, int K, int S, int group_m,
-                   hipStream_t st) {
+                   float epi_arg, hipStream_t st) {
   if (M <= 0) return 0;
   if (N % 256 != 0 || K % 128 != 0 || S < 1 || S > K / 64) return -1;
   if ((size_t)M * ldx * 2 >= (1ull << 32)) return -1;  // 32-bit byte offsets of the LDS-DMA buffer loads
   if (S > 1) {
     if (ws == nullptr) return -1;
-    if (epi == EPI_SILU) w4_launch<EPI_SILU, true, true>(X, ldx, W, bias, R, ldr, Y, ldy, ws, M, N, K, S, group_m, st);
+    if (epi_is_glu(epi)) w4_launch<EPI_SILU, true, true>(X, ldx, W, bias, R, ldr, Y, ldy, ws, M, N, K, S, group_m, st);
     else w4_launch<EPI_NONE, true, true>(X, ldx, W, bias, R, ldr, Y, ldy, ws, M, N, K, S, group_m, st);
     return 0;
   }
-  if (epi == EPI_SILU) {
+  if (epi == EPI_CLAMP_GLU || epi == EPI_RELU2) {
+    if (out_f32) return -1;
+    if (epi == EPI_RELU2) w4_launch<EPI_RELU2, false, false>(X, ldx, W, bias, R, ldr, Y, ldy, ws, M, N, K, 1, group_m, st);
+    else w4_launch<EPI_CLAMP_GLU, false, false>(X, ldx, W, bias, R, ldr, Y, ldy, ws, M, N, K, 1, group_m, st, epi_arg);
+  } else if (epi == EPI_SILU) {
     if (out_f32) w4_launch<EPI_SILU, true, false>(X, ldx, W, bias, R, ldr, Y, ldy, ws, M, N, K, 1, group_m, st);
     else w4_launch<EPI_SILU, false, false>(X, ldx, W, bias, R, ldr, Y, ldy, ws, M, N, K, 1, group_m, st);
   } else if (epi == EPI_RESID) {

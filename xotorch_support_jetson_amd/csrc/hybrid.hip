@@ -65,7 +65,7 @@ __global__ __launch_bounds__(256) void qk_norm_rope_store_k(
     const float* __restrict__ P, int ldp, const float* __restrict__ bias, int q_off, int k_off, int v_off, int H, int G,
     int d, int dv, int R, const int* __restrict__ pos, const float* __restrict__ cos_sin, const int64_t* __restrict__ slots,
     float eps, int qk_norm, AT* __restrict__ q_out, AT* __restrict__ k_cache, AT* __restrict__ v_cache, int Gv,
-    const float* __restrict__ q_norm, const float* __restrict__ k_norm) {
+    const float* __restrict__ q_norm, const float* __restrict__ k_norm, int S, int64_t ss_) {
   __shared__ float red[8];
   const int t = blockIdx.x;
   const float* row = P + (int64_t)t * ldp;
@@ -79,7 +79,7 @@ __global__ __launch_bounds__(256) void qk_norm_rope_store_k(
     auto inv_rms = [&](int off, int n) {
       float ss = 0.0f;
       for (int i = threadIdx.x; i < n; i += blockDim.x) {
-        const float a = row[off + i] + (bias ? bias[off + i] : 0.0f);
+        const float a = slab1(row + off + i, S, ss_) + (bias ? bias[off + i] : 0.0f);
         ss += a * a;
       }
       return 1.0f / sqrtf(block_sum(ss, red) / (float)n + eps);
@@ -93,7 +93,7 @@ __global__ __launch_bounds__(256) void qk_norm_rope_store_k(
     const float* wn = !q_norm ? nullptr : isq ? q_norm + head * d : k_norm + (head - H) * d;
     const float rn = isq ? rq : rk;
     auto at = [&](int i) {
-      const float a = row[c0 + i] + (bias ? bias[c0 + i] : 0.0f);
+      const float a = slab1(row + c0 + i, S, ss_) + (bias ? bias[c0 + i] : 0.0f);
       return wn ? a * rn * wn[i] : a;
     };
     float v[4];
@@ -131,9 +131,163 @@ __global__ __launch_bounds__(256) void qk_norm_rope_store_k(
     for (int e = threadIdx.x; e < Gv * dv; e += blockDim.x) {  // (Gv value heads: G, or fewer when key heads share values)
       const int g = e / dv, i = e - g * dv;
       const int64_t pg = (slot / PAGE_TOK) * Gv + g;
-      stf(v_cache + (pg * dv + i) * PAGE_TOK + (slot % PAGE_TOK), row[v_off + e] + (bias ? bias[v_off + e] : 0.0f));
+      stf(v_cache + (pg * dv + i) * PAGE_TOK + (slot % PAGE_TOK), slab1(row + v_off + e, S, ss_) + (bias ? bias[v_off + e] : 0.0f));
     }
   }
+}
+
+// The same without per-head division, WPT waves per token and four columns at a time: a lane takes rotation pairs of four
+// (dims 4u .. and R/2 + 4u .., or four unrotated dims) of any q / k head and keeps all NU of them in registers between the
+// sums over the whole projections and the writes.  Needs d, R / 2 and the column offsets to be multiples of four.  WPT 1
+// (many tokens): the values are left to v_store_tiled_k.  WPT 8 (few tokens, P maybe as split-K slabs): every load of a
+// step of four slabs is in flight together, the norms' weights and the angles under them.
+template <typename AT, int NU, int WPT, bool SLABS>
+__global__ __launch_bounds__(WPT == 1 ? 256 : 64 * WPT) void qk_norm_rope_vec_k(
+    const float* __restrict__ P, int ldp, int S, int64_t ss, const float* __restrict__ bias, int q_off, int k_off, int v_off,
+    int H, int G, int d, int dv, int R, const int* __restrict__ pos, const float* __restrict__ cos_sin,
+    const int64_t* __restrict__ slots, float eps, AT* __restrict__ q_out, AT* __restrict__ k_cache, AT* __restrict__ v_cache,
+    int Gv, const float* __restrict__ q_norm, const float* __restrict__ k_norm, int v_here, int T) {
+  constexpr int NL = 64 * WPT;  // lanes per token
+  __shared__ float red[2][WPT];
+  const int lane = WPT == 1 ? threadIdx.x & 63 : threadIdx.x;
+  const int t = WPT == 1 ? blockIdx.x * (blockDim.x >> 6) + (threadIdx.x >> 6) : blockIdx.x;
+  if (t >= T) return;  // (WPT 1: wave-uniform and no workgroup barrier below; else never)
+  const float* row = P + (int64_t)t * ldp;
+  const float* cs = cos_sin + (int64_t)pos[t] * R;
+  const int half = R >> 1, upr = half >> 2, uph = upr + ((d - R) >> 2);  // rotated units, units per head
+  const int units = (H + (k_off >= 0 ? G : 0)) * uph, nq = H * uph;
+  const float inv_uph = 1.0f / (float)uph;
+  const int64_t slot = slots[t];
+  const f32x4 zero = {0.f, 0.f, 0.f, 0.f};
+  auto ld = [](const float* p) { return *reinterpret_cast<const f32x4*>(p); };
+  auto head_of = [&](int w) { return (int)(((float)w + 0.5f) * inv_uph); };  // w / uph (w below 2^12: exact)
+  // a unit's first dim and head; lanes past the last unit repeat it (their loads and sums are not used)
+  auto unit = [&](int i, int* hd) {
+    const int w = min(lane + NL * i, units - 1);
+    *hd = head_of(w);
+    const int u = w - *hd * uph;
+    return u < upr ? 4 * u : R + 4 * (u - upr);
+  };
+  f32x4 a[NU], b[NU];
+  int col[NU], sec[NU];  // columns of the unit's two quarters (unrotated units: the same one twice)
+#pragma unroll
+  for (int i = 0; i < NU; ++i) {
+    int hd;
+    const int i0 = unit(i, &hd);
+    col[i] = (hd < H ? q_off + hd * d : k_off + (hd - H) * d) + i0;
+    sec[i] = i0 < half ? col[i] + half : col[i];
+    a[i] = ld(row + col[i]);
+    b[i] = ld(row + sec[i]);
+  }
+  if constexpr (SLABS) {
+    for (int s0 = 1; s0 < S; s0 += 4) {
+      f32x4 ta[4][NU], tb[4][NU];
+#pragma unroll
+      for (int k = 0; k < 4; ++k) {
+        const float* rs = row + min(s0 + k, S - 1) * ss;
+#pragma unroll
+        for (int i = 0; i < NU; ++i) {
+          ta[k][i] = ld(rs + col[i]);
+          tb[k][i] = ld(rs + sec[i]);
+        }
+      }
+#pragma unroll
+      for (int k = 0; k < 4; ++k) {
+        const float f = s0 + k < S ? 1.0f : 0.0f;
+#pragma unroll
+        for (int i = 0; i < NU; ++i) {
+          a[i] += f * ta[k][i];
+          b[i] += f * tb[k][i];
+        }
+      }
+    }
+  }
+  if (bias) {
+#pragma unroll
+    for (int i = 0; i < NU; ++i) {
+      a[i] += ld(bias + col[i]);
+      b[i] += ld(bias + sec[i]);
+    }
+  }
+  float rq = 1.f, rk = 1.f;
+  if (q_norm) {
+    float sq = 0.f, sk = 0.f;
+#pragma unroll
+    for (int i = 0; i < NU; ++i) {
+      const int w = lane + NL * i;
+      float s = 0.f;
+#pragma unroll
+      for (int e = 0; e < 4; ++e) s += a[i][e] * a[i][e] + (sec[i] != col[i] ? b[i][e] * b[i][e] : 0.0f);
+      sq += w < nq ? s : 0.f;
+      sk += w >= nq && w < units ? s : 0.f;
+    }
+    sq = wave_sum(sq);
+    sk = wave_sum(sk);
+    if constexpr (WPT > 1) {
+      if ((lane & 63) == 0) {
+        red[0][lane >> 6] = sq;
+        red[1][lane >> 6] = sk;
+      }
+      __syncthreads();
+      sq = sk = 0.f;
+#pragma unroll
+      for (int w = 0; w < WPT; ++w) {
+        sq += red[0][w];
+        sk += red[1][w];
+      }
+    }
+    rq = 1.0f / sqrtf(sq / (float)(H * d) + eps);
+    rk = 1.0f / sqrtf(sk / (float)(G * d) + eps);
+  }
+#pragma unroll
+  for (int i = 0; i < NU; ++i) {
+    int hd;
+    const int i0 = unit(i, &hd);
+    const bool isq = hd < H, rot = i0 < half;
+    f32x4 x = a[i], y = b[i];
+    if (q_norm) {
+      const float* wn = isq ? q_norm + hd * d + i0 : k_norm + (hd - H) * d + i0;
+      const float r = isq ? rq : rk;
+      x *= ld(wn) * r;
+      y *= ld(rot ? wn + half : wn) * r;
+    }
+    const f32x4 c = rot ? ld(cs + i0) : zero, s = rot ? ld(cs + half + i0) : zero;
+    if (lane + NL * i >= units || (!isq && slot < 0)) continue;
+    AT* dst = isq ? q_out + ((int64_t)t * H + hd) * d
+                  : k_cache + (((slot / PAGE_TOK) * G + (hd - H)) * PAGE_TOK + slot % PAGE_TOK) * d;
+    if (rot) {
+      st4(dst + i0, x * c - y * s);
+      st4(dst + half + i0, y * c + x * s);
+    } else {
+      st4(dst + i0, x);
+    }
+  }
+  if (v_here && k_off >= 0 && slot >= 0) {
+    AT* page = v_cache + (slot / PAGE_TOK) * Gv * dv * PAGE_TOK + slot % PAGE_TOK;
+    for (int e = lane; e < Gv * dv; e += NL)
+      stf(page + (int64_t)e * PAGE_TOK, slab1(row + v_off + e, S, ss) + (bias ? bias[v_off + e] : 0.0f));
+  }
+}
+
+// Values of many tokens -> the transposed cache [pages, Gv, dv, 64]: a workgroup takes 64 consecutive tokens and 64 columns
+// through LDS, so that a wave's store covers the 64 tokens of one column (128 bytes where their slots are neighbours).
+template <typename AT>
+__global__ __launch_bounds__(256) void v_store_tiled_k(const float* __restrict__ P, int ldp, int S, int64_t ss,
+                                                       const float* __restrict__ bias, int v_off, int n, int dv, int T,
+                                                       const int64_t* __restrict__ slots, AT* __restrict__ v_cache, int Gv) {
+  __shared__ float tile[64][65];
+  const int t0 = blockIdx.x * 64, c0 = blockIdx.y * 64;
+  for (int w = threadIdx.x; w < 64 * 64; w += 256) {
+    const int tt = w >> 6, c = w & 63;
+    if (t0 + tt < T && c0 + c < n)
+      tile[tt][c] = slab1(P + (int64_t)(t0 + tt) * ldp + v_off + c0 + c, S, ss) + (bias ? bias[v_off + c0 + c] : 0.0f);
+  }
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+  const int64_t slot = t0 + lane < T ? slots[t0 + lane] : -1;
+  __syncthreads();
+  if (slot < 0) return;
+  AT* page = v_cache + (slot / PAGE_TOK) * Gv * dv * PAGE_TOK + slot % PAGE_TOK;
+  for (int c = wave; c < 64 && c0 + c < n; c += 4) stf(page + (int64_t)(c0 + c) * PAGE_TOK, tile[lane][c]);
 }
 
 // ------------------------------------------------------------------ pooled keys and values
@@ -741,22 +895,54 @@ __global__ void relu2_k(const float* __restrict__ P, int ldp, int off, int F, AT
 
 // ------------------------------------------------------------------ routed experts' weighted sum + gated shared expert
 // y [splits * slots, >= D]: the down projection's K slices (summed here in a fixed order)
-__global__ void moe_weighted_sum_k(const float* __restrict__ y, int ldy, const int* __restrict__ slot_of,
-                                   const float* __restrict__ topw, int k, int splits, int64_t slots,
-                                   const float* __restrict__ sh, int lds, const float* __restrict__ P, int ldp, int shg_off,
-                                   float* __restrict__ out, int D) {
+// The k * splits terms' rows and weights are laid out in LDS once per token; W columns per thread.
+constexpr int MWS_TERMS = 512;
+
+template <int W>
+__global__ __launch_bounds__(256) void moe_weighted_sum_k(const float* __restrict__ y, int ldy, const int* __restrict__ slot_of,
+                                                          const float* __restrict__ topw, int k, int splits, int64_t slots,
+                                                          const float* __restrict__ sh, int lds, int shS, int64_t shss,
+                                                          const float* __restrict__ P, int ldp, int shg_off,
+                                                          float* __restrict__ out, int D) {
+  __shared__ int64_t trow[MWS_TERMS];
+  __shared__ float tw[MWS_TERMS];
   const int64_t t = blockIdx.x;
+  const int n = k * splits;
+  for (int q = threadIdx.x; q < n; q += blockDim.x) {
+    const int j = q / splits;
+    trow[q] = ((int64_t)(q - j * splits) * slots + slot_of[t * k + j]) * ldy;
+    tw[q] = topw[t * k + j];
+  }
+  __syncthreads();
   const float sg = !sh ? 0.0f : (P ? sigmoidf_(P[t * ldp + shg_off]) : 1.0f);  // (no gate: the shared expert is added as it is)
-  for (int i = threadIdx.x; i < D; i += blockDim.x) {
-    float acc = 0.0f;
-    for (int j = 0; j < k; ++j) {
-      const int64_t r = slot_of[t * k + j];
-      float ys = 0.0f;
-      for (int sp = 0; sp < splits; ++sp) ys += y[(sp * slots + r) * ldy + i];
-      acc += topw[t * k + j] * ys;
+  for (int i = W * threadIdx.x; i < D; i += W * blockDim.x) {
+    float acc[W];
+#pragma unroll
+    for (int c = 0; c < W; ++c) acc[c] = 0.0f;
+    auto add = [&](float f, const float* v) {
+#pragma unroll
+      for (int c = 0; c < W; ++c) acc[c] += f * v[c];
+    };
+    for (int q0 = 0; q0 < n; q0 += 4) {  // (four terms in flight; terms past the last repeat it with weight zero)
+      float v[4][W];
+#pragma unroll
+      for (int q = 0; q < 4; ++q) {
+        const float* p = y + trow[min(q0 + q, n - 1)] + i;
+        if constexpr (W == 4) *reinterpret_cast<f32x4*>(v[q]) = *reinterpret_cast<const f32x4*>(p);
+        else v[q][0] = *p;
+      }
+#pragma unroll
+      for (int q = 0; q < 4; ++q)
+        if (q0 + q < n) add(tw[q0 + q], v[q]);
     }
-    if (sh) acc += sg * sh[t * lds + i];
-    out[t * D + i] = acc;
+    if (sh) {
+      float v[W];
+      if constexpr (W == 4) *reinterpret_cast<f32x4*>(v) = slab4(sh + t * lds + i, shS, shss);
+      else v[0] = slab1(sh + t * lds + i, shS, shss);
+      add(sg, v);
+    }
+    if constexpr (W == 4) *reinterpret_cast<f32x4*>(out + t * D + i) = f32x4{acc[0], acc[1], acc[2], acc[3]};
+    else out[t * D + i] = acc[0];
   }
 }
 
@@ -814,8 +1000,8 @@ void qk_norm_rope_store(const at::Tensor& P, const c10::optional<at::Tensor>& bi
                         const at::Tensor& cos_sin, const at::Tensor& slots, double eps, bool qk_norm, at::Tensor& q_out,
                         at::Tensor& k_cache, at::Tensor& v_cache, const c10::optional<at::Tensor>& q_norm,
                         const c10::optional<at::Tensor>& k_norm) {
-  const int ldp = ld_of(P, "P");
-  const int64_t T = P.size(0);
+  const Slabs p = slabs_of(P, "P");
+  const int64_t T = p.T;
   int64_t Gv = G;
   if (T == 0) return;
   i32c(pos, "pos");
@@ -824,13 +1010,13 @@ void qk_norm_rope_store(const at::Tensor& P, const c10::optional<at::Tensor>& bi
          "pos / slots must hold one entry per token");
   MCHECK(R % 2 == 0 && R >= 0 && R <= d && (R == 0 || (cos_sin.dim() == 2 && cos_sin.size(1) == R)), "bad rotary dims");
   MCHECK(H > 0 && G > 0 && H % G == 0 && d > 0 && d <= 256 && dv > 0 && dv <= 256, "head counts / sizes (at most 256)");
-  cols_ok(P, q_off, H * d, "q");
+  cols_ok(p, q_off, H * d, "q");
   if (k_off >= 0) {
     MCHECK(v_off >= 0, "keys without values");
-    cols_ok(P, k_off, G * d, "k");
+    cols_ok(p, k_off, G * d, "k");
     check_kv(k_cache, v_cache, q_out.scalar_type(), G, d, dv);
     Gv = v_cache.size(1);
-    cols_ok(P, v_off, Gv * dv, "v");
+    cols_ok(p, v_off, Gv * dv, "v");
   }
   const float* bp = nullptr;
   if (bias.has_value()) {
@@ -853,16 +1039,50 @@ void qk_norm_rope_store(const at::Tensor& P, const c10::optional<at::Tensor>& bi
   }
   // positions and slots are checked on the host by their producer (the block manager hands out slots < pages * 64
   // and the runner bounds positions by the table's rows)
+  auto al16 = [](const float* x) { return (reinterpret_cast<uintptr_t>(x) & 15) == 0; };
+  const int64_t units = (H + (k_off >= 0 ? G : 0)) * (R / 8 + (d - R) / 4);
+  if (!qk_norm && p.vec && d % 4 == 0 && R % 8 == 0 && q_off % 4 == 0 && (k_off < 0 || k_off % 4 == 0) && al16(bp) && al16(qn) &&
+      al16(kn) && (R == 0 || al16(cos_sin.data_ptr<float>())) && units <= 64 * 20) {
+    const bool tiled = k_off >= 0 && T >= 256;
+    const dim3 vgrid((unsigned)((T + 63) / 64), (unsigned)((Gv * dv + 63) / 64));
+#define QK_VEC(AT, NU, WPT, SL)                                                                                           \
+  qk_norm_rope_vec_k<AT, NU, WPT, SL><<<WPT == 1 ? (T + 3) / 4 : T, WPT == 1 ? 256 : 64 * WPT, 0, stream()>>>(            \
+      p.p, p.ld, p.S, p.ss, bp, (int)q_off, (int)k_off, (int)v_off, (int)H, (int)G, (int)d, (int)dv, (int)R,             \
+      pos.data_ptr<int>(), cos_sin.data_ptr<float>(), slots.data_ptr<int64_t>(), (float)eps, (AT*)q_out.data_ptr(),       \
+      (AT*)k_cache.data_ptr(), (AT*)v_cache.data_ptr(), (int)Gv, qn, kn, tiled ? 0 : 1, (int)T)
+#define QK_NU(AT)                                                                                                         \
+  if (!many && p.S > 1 && units <= 512) QK_VEC(AT, 1, 8, true);                                                           \
+  else if (!many && p.S > 1) QK_VEC(AT, 3, 8, true);                                                                      \
+  else if (!many && units <= 512) QK_VEC(AT, 1, 8, false);                                                                \
+  else if (!many) QK_VEC(AT, 3, 8, false);                                                                                \
+  else if (units <= 128) QK_VEC(AT, 2, 1, false);                                                                         \
+  else if (units <= 320) QK_VEC(AT, 5, 1, false);                                                                         \
+  else if (units <= 640) QK_VEC(AT, 10, 1, false);                                                                        \
+  else QK_VEC(AT, 20, 1, false);                                                                                          \
+  if (tiled)                                                                                                              \
+    v_store_tiled_k<AT><<<vgrid, 256, 0, stream()>>>(p.p, p.ld, p.S, p.ss, bp, (int)v_off, (int)(Gv * dv), (int)dv,      \
+                                                     (int)T, slots.data_ptr<int64_t>(), (AT*)v_cache.data_ptr(), (int)Gv)
+    // (slabs of many tokens: three units per lane of eight waves)
+    const bool many = T >= 256 && p.S == 1;
+    if (q_out.scalar_type() == at::kBFloat16) {
+      QK_NU(uint16_t);
+    } else {
+      QK_NU(float);
+    }
+#undef QK_NU
+#undef QK_VEC
+    return;
+  }
   if (q_out.scalar_type() == at::kBFloat16)
     qk_norm_rope_store_k<uint16_t><<<T, 256, 0, stream()>>>(
-        P.data_ptr<float>(), ldp, bp, (int)q_off, (int)k_off, (int)v_off, (int)H, (int)G, (int)d, (int)dv, (int)R,
+        p.p, p.ld, bp, (int)q_off, (int)k_off, (int)v_off, (int)H, (int)G, (int)d, (int)dv, (int)R,
         pos.data_ptr<int>(), cos_sin.data_ptr<float>(), slots.data_ptr<int64_t>(), (float)eps, (int)qk_norm,
-        (uint16_t*)q_out.data_ptr(), (uint16_t*)k_cache.data_ptr(), (uint16_t*)v_cache.data_ptr(), (int)Gv, qn, kn);
+        (uint16_t*)q_out.data_ptr(), (uint16_t*)k_cache.data_ptr(), (uint16_t*)v_cache.data_ptr(), (int)Gv, qn, kn, p.S, p.ss);
   else
     qk_norm_rope_store_k<float><<<T, 256, 0, stream()>>>(
-        P.data_ptr<float>(), ldp, bp, (int)q_off, (int)k_off, (int)v_off, (int)H, (int)G, (int)d, (int)dv, (int)R,
+        p.p, p.ld, bp, (int)q_off, (int)k_off, (int)v_off, (int)H, (int)G, (int)d, (int)dv, (int)R,
         pos.data_ptr<int>(), cos_sin.data_ptr<float>(), slots.data_ptr<int64_t>(), (float)eps, (int)qk_norm,
-        q_out.data_ptr<float>(), k_cache.data_ptr<float>(), v_cache.data_ptr<float>(), (int)Gv, qn, kn);
+        q_out.data_ptr<float>(), k_cache.data_ptr<float>(), v_cache.data_ptr<float>(), (int)Gv, qn, kn, p.S, p.ss);
 }
 
 void check_pools(const at::Tensor& k_cache, const at::Tensor& kp, const at::Tensor& vp, int64_t pool, int64_t G, int64_t d,
@@ -1135,11 +1355,15 @@ void moe_weighted_sum(const at::Tensor& y, const at::Tensor& slot_of, const at::
              y.size(1) >= D,
          "moe_weighted_sum: shape mismatch");
   const float *sp = nullptr, *pp = nullptr;
-  int lds = 0, ldp = 0;
+  int lds = 0, ldp = 0, shS = 1;
+  int64_t shss = 0;
   if (sh_y.has_value()) {
-    lds = ld_of(*sh_y, "sh_y");
-    MCHECK(sh_y->size(0) == T && sh_y->size(1) >= D, "a shared expert needs its result [T, >= D]");
-    sp = sh_y->data_ptr<float>();
+    const Slabs sh = slabs_of(*sh_y, "sh_y");
+    MCHECK(sh.T == T && sh.n >= D, "a shared expert needs its result [T, >= D]");
+    lds = sh.ld;
+    shS = sh.S;
+    shss = sh.ss;
+    sp = sh.p;
     if (P.has_value()) {
       ldp = ld_of(*P, "P");
       MCHECK(P->size(0) == T, "P must have T rows");
@@ -1147,10 +1371,17 @@ void moe_weighted_sum(const at::Tensor& y, const at::Tensor& slot_of, const at::
       pp = P->data_ptr<float>();
     }
   }
+  MCHECK(k * splits <= MWS_TERMS, "moe_weighted_sum: at most ", MWS_TERMS, " chosen experts times K slices");
+  const bool vec = D % 4 == 0 && ldy % 4 == 0 && lds % 4 == 0 && shss % 4 == 0 && (reinterpret_cast<uintptr_t>(y.data_ptr()) & 15) == 0 &&
+                   (reinterpret_cast<uintptr_t>(sp) & 15) == 0 && (reinterpret_cast<uintptr_t>(out.data_ptr()) & 15) == 0;
   // (slot_of comes from the routing kernel: every entry is a row of y)
-  moe_weighted_sum_k<<<T, 256, 0, stream()>>>(y.data_ptr<float>(), ldy, slot_of.data_ptr<int>(), topw.data_ptr<float>(), (int)k,
-                                              (int)splits, (int64_t)(T * k), sp, lds, pp, ldp, (int)shg_off,
-                                              out.data_ptr<float>(), (int)D);
+#define MWS_GO(W)                                                                                                          \
+  moe_weighted_sum_k<W><<<T, 256, 0, stream()>>>(y.data_ptr<float>(), ldy, slot_of.data_ptr<int>(), topw.data_ptr<float>(), \
+                                                 (int)k, (int)splits, (int64_t)(T * k), sp, lds, shS, shss, pp, ldp,       \
+                                                 (int)shg_off, out.data_ptr<float>(), (int)D)
+  if (vec) MWS_GO(4);
+  else MWS_GO(1);
+#undef MWS_GO
 }
 
 }  // namespace

@@ -32,7 +32,7 @@ int launch_gemm_skinny(const uint16_t* X, int ldx, const uint16_t* W, int ldw, c
                        int nt, hipStream_t s);
 int launch_gemm_stream(const uint16_t* X, int ldx, const uint16_t* W, int ldw, const uint16_t* bias,
                        const uint16_t* R, int ldr, void* Y, int ldy, bool out_f32, int epi, float* ws, long ws_elems,
-                       int M, int N, int K, int ntw, int S, bool wshuf, bool reduce, hipStream_t s);
+                       int M, int N, int K, int ntw, int S, bool wshuf, bool reduce, float epi_arg, hipStream_t s);
 // Batch-1 decode GEMM whose input row is the RMSNorm of a residual projection's pending split-K sum:
 // x = rmsnorm(bf16(h + bias + sum_s ws[s])) * lnw, recomputed by every workgroup from the slabs (no separate
 // reduce + norm launch); workgroup (0, 0) stores the summed residual row to hout (never h itself: the other
@@ -71,14 +71,14 @@ int launch_gemm_stream8(const uint16_t* X, int ldx, const uint8_t* W, const floa
 // four-wave 256 x 256 tile (gemm_w4.hip; tile code 4256 of launch_gemm_big): N % 256 == 0, K % 128 == 0
 int launch_gemm_w4(const uint16_t* X, int ldx, const uint16_t* W, const uint16_t* bias, const uint16_t* R, int ldr,
                    void* Y, int ldy, bool out_f32, int epi, float* ws, int M, int N, int K, int S, int group_m,
-                   hipStream_t st);
+                   float epi_arg, hipStream_t st);
 // the same tile on token-major operands (weight gradients): Y [M, N] (+)= Xt^T . Wt, Xt [K, M], Wt [K, N]
 int launch_gemm_w4_tn(const uint16_t* Xt, int ldx, const uint16_t* Wt, int ldw, const uint16_t* R, int ldr, void* Y,
                       int ldy, bool out_f32, int epi, int M, int N, int K, int group_m, hipStream_t st);
 int gemm_big_group_m();  // grouped raster width of tall grids (XOT_GEMM_GROUP_M)
 int launch_gemm_big(const uint16_t* X, int ldx, const uint16_t* W, const uint16_t* bias, const uint16_t* R, int ldr,
                     void* Y, int ldy, bool out_f32, int epi, float* ws, long ws_elems, int M, int N, int K, int bn,
-                    int S, bool reduce, hipStream_t s);
+                    int S, bool reduce, float epi_arg, hipStream_t s);
 // B independent GEMMs Y_e = X_e . W_e^T (pre-shuffled W [B][N][K]; X_e = X + e*xbat, Y_e = Y + e*ybat)
 // training-GEMM layouts (csrc/layout.hip): src [R, C] row-major with row stride ld
 int launch_shuffle(const uint16_t* src, long ld, uint16_t* dst, int R, int C, hipStream_t s);

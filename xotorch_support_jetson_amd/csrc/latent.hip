@@ -31,17 +31,18 @@ constexpr float LOG2E_F = 1.4426950408889634f;
 // norm of one row held in global memory: v / rms(v) * w, or with a bias the layer norm (v - mean) / sqrt(var + eps) * w + b
 // (the variance as the mean of the squared deviations, in a pass of its own).  Returns (shift, scale).
 // add (or null): one number per column, added to v first.
-__device__ __forceinline__ void row_norm_stats(const float* v, const float* add, int D, bool center, float eps, float* red,
-                                               float* shift, float* scale) {
+// v may be S split-K slabs, ss floats apart.
+__device__ __forceinline__ void row_norm_stats(const float* v, int S, int64_t sstr, const float* add, int D, bool center,
+                                               float eps, float* red, float* shift, float* scale) {
   float mean = 0.0f;
   if (center) {
     float s = 0.0f;
-    for (int i = threadIdx.x; i < D; i += blockDim.x) s += v[i] + (add ? add[i] : 0.0f);
+    for (int i = threadIdx.x; i < D; i += blockDim.x) s += slab1(v + i, S, sstr) + (add ? add[i] : 0.0f);
     mean = block_sum(s, red) / D;
   }
   float ss = 0.0f;
   for (int i = threadIdx.x; i < D; i += blockDim.x) {
-    const float c = v[i] + (add ? add[i] : 0.0f) - mean;
+    const float c = slab1(v + i, S, sstr) + (add ? add[i] : 0.0f) - mean;
     ss += c * c;
   }
   ss = block_sum(ss, red);
@@ -54,20 +55,20 @@ __global__ __launch_bounds__(256) void sandwich_add_norm_k(float* __restrict__ x
                                                            const float* __restrict__ wb, const float* __restrict__ bb,
                                                            const float* __restrict__ wn, const float* __restrict__ bn,
                                                            const float* __restrict__ yb, float mult, float eps,
-                                                           AT* __restrict__ out, int ldo, int D) {
+                                                           AT* __restrict__ out, int ldo, int D, int S, int64_t ss) {
   __shared__ float red[8];
   const int64_t t = blockIdx.x;
   float* xr = x + t * D;
   if (y) {
     const float* yr = y + t * ldy;
     float mu, r;
-    row_norm_stats(yr, yb, D, bb != nullptr, eps, red, &mu, &r);
+    row_norm_stats(yr, S, ss, yb, D, bb != nullptr, eps, red, &mu, &r);
     for (int i = threadIdx.x; i < D; i += blockDim.x) 
-      xr[i] += mult * ((yr[i] + (yb ? yb[i] : 0.0f) - mu) * r * wb[i] + (bb ? bb[i] : 0.0f));
+      xr[i] += mult * ((slab1(yr + i, S, ss) + (yb ? yb[i] : 0.0f) - mu) * r * wb[i] + (bb ? bb[i] : 0.0f));
   }
   if (wn) {  // (a thread re-reads the elements it wrote itself)
     float mu, r;
-    row_norm_stats(xr, nullptr, D, bn != nullptr, eps, red, &mu, &r);
+    row_norm_stats(xr, 1, 0, nullptr, D, bn != nullptr, eps, red, &mu, &r);
     for (int i = threadIdx.x; i < D; i += blockDim.x) stf(out + t * ldo + i, (xr[i] - mu) * r * wn[i] + (bn ? bn[i] : 0.0f));
   } else if (out) {
     for (int i = threadIdx.x; i < D; i += blockDim.x) stf(out + t * ldo + i, xr[i]);
@@ -565,37 +566,44 @@ __global__ __launch_bounds__(256) void latent_attn_merge_k(const float* __restri
   }
 }
 
-// The same for rows of at most 256 R numbers: a thread keeps its R values of y and of x in registers, so each row is
-// read once (the sums run over registers; the variance still after the mean, as the mean of the squared deviations).
+// The same for rows of at most 1024 R numbers (a multiple of four): a thread keeps R groups of four values of y and of x in
+// registers, so each row is read once (the sums run over registers; the variance still after the mean, as the mean of the
+// squared deviations).  y may be S split-K slabs.
 template <typename AT, int R>
 __global__ __launch_bounds__(256) void sandwich_add_norm_reg_k(float* __restrict__ x, const float* __restrict__ y, int ldy,
                                                                const float* __restrict__ wb, const float* __restrict__ bb,
                                                                const float* __restrict__ wn, const float* __restrict__ bn,
                                                                const float* __restrict__ yb, float mult, float eps,
-                                                               AT* __restrict__ out, int ldo, int D) {
+                                                               AT* __restrict__ out, int ldo, int D, int S, int64_t ss_) {
   __shared__ float red[8];
   const int64_t t = blockIdx.x;
   float* xr = x + t * D;
-  float xv[R];
+  const f32x4 zero = {0.f, 0.f, 0.f, 0.f};
+  auto ld = [](const float* p) { return *reinterpret_cast<const f32x4*>(p); };
+  f32x4 xv[R];
 #pragma unroll
   for (int r = 0; r < R; ++r) {
-    const int i = threadIdx.x + 256 * r;
-    xv[r] = i < D ? xr[i] : 0.0f;
+    const int i = 4 * (threadIdx.x + 256 * r);
+    xv[r] = i < D ? ld(xr + i) : zero;
   }
   // (shift, scale) of a row held in registers
-  auto stats = [&](const float* v, bool center, float* mu, float* rs) {
+  auto stats = [&](const f32x4* v, bool center, float* mu, float* rs) {
     float mean = 0.0f;
     if (center) {
       float s = 0.0f;
 #pragma unroll
-      for (int r = 0; r < R; ++r) s += v[r];  // (entries past D are zero)
+      for (int r = 0; r < R; ++r) s += v[r][0] + v[r][1] + v[r][2] + v[r][3];  // (entries past D are zero)
       mean = block_sum(s, red) / D;
     }
     float ss = 0.0f;
 #pragma unroll
     for (int r = 0; r < R; ++r) {
-      const float c = threadIdx.x + 256 * r < D ? v[r] - mean : 0.0f;
-      ss += c * c;
+      if (4 * (threadIdx.x + 256 * r) >= D) continue;
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        const float c = v[r][e] - mean;
+        ss += c * c;
+      }
     }
     ss = block_sum(ss, red);
     *mu = mean;
@@ -603,20 +611,26 @@ __global__ __launch_bounds__(256) void sandwich_add_norm_reg_k(float* __restrict
   };
   if (y) {
     const float* yr = y + t * ldy;
-    float yv[R];
+    f32x4 yv[R];
 #pragma unroll
     for (int r = 0; r < R; ++r) {
-      const int i = threadIdx.x + 256 * r;
-      yv[r] = i < D ? yr[i] + (yb ? yb[i] : 0.0f) : 0.0f;
+      const int i = 4 * (threadIdx.x + 256 * r);
+      yv[r] = zero;
+      if (i < D) {
+        yv[r] = slab4(yr + i, S, ss_);
+        if (yb) yv[r] += ld(yb + i);
+      }
     }
     float mu, rs;
     stats(yv, bb != nullptr, &mu, &rs);
 #pragma unroll
     for (int r = 0; r < R; ++r) {
-      const int i = threadIdx.x + 256 * r;
+      const int i = 4 * (threadIdx.x + 256 * r);
       if (i < D) {
-        xv[r] += mult * ((yv[r] - mu) * rs * wb[i] + (bb ? bb[i] : 0.0f));
-        xr[i] = xv[r];
+        f32x4 a = (yv[r] - mu) * rs * ld(wb + i);
+        if (bb) a += ld(bb + i);
+        xv[r] += mult * a;
+        *reinterpret_cast<f32x4*>(xr + i) = xv[r];
       }
     }
   }
@@ -625,14 +639,18 @@ __global__ __launch_bounds__(256) void sandwich_add_norm_reg_k(float* __restrict
     stats(xv, bn != nullptr, &mu, &rs);
 #pragma unroll
     for (int r = 0; r < R; ++r) {
-      const int i = threadIdx.x + 256 * r;
-      if (i < D) stf(out + t * ldo + i, (xv[r] - mu) * rs * wn[i] + (bn ? bn[i] : 0.0f));
+      const int i = 4 * (threadIdx.x + 256 * r);
+      if (i < D) {
+        f32x4 a = (xv[r] - mu) * rs * ld(wn + i);
+        if (bn) a += ld(bn + i);
+        st4(out + t * ldo + i, a);
+      }
     }
   } else if (out) {  // the stream itself, in the operand dtype
 #pragma unroll
     for (int r = 0; r < R; ++r) {
-      const int i = threadIdx.x + 256 * r;
-      if (i < D) stf(out + t * ldo + i, xv[r]);
+      const int i = 4 * (threadIdx.x + 256 * r);
+      if (i < D) st4(out + t * ldo + i, xv[r]);
     }
   }
 }
@@ -650,7 +668,10 @@ void sandwich_add_norm(at::Tensor& x, const c10::optional<at::Tensor>& y, const 
   const int64_t T = x.size(0), D = x.size(1);
   if (T == 0) return;
   const float *yp = nullptr, *bp = nullptr, *np = nullptr, *bbp = nullptr, *bnp = nullptr, *ybp = nullptr;
-  int ldy = 0, ldo = 0;
+  int ldy = 0, ldo = 0, S = 1;
+  int64_t ss = 0;
+  bool vec = D % 4 == 0;
+  auto al = [&](const float* p) { vec = vec && (reinterpret_cast<uintptr_t>(p) & 15) == 0; };
   if (bb.has_value()) {
     f32c(*bb, "bb");
     MCHECK(bb->numel() == D && y.has_value(), "the result norm's bias must hold D numbers");
@@ -667,8 +688,12 @@ void sandwich_add_norm(at::Tensor& x, const c10::optional<at::Tensor>& y, const 
     ybp = yb->data_ptr<float>();
   }
   if (y.has_value()) {
-    ldy = ld_of(*y, "y");
-    MCHECK(y->size(0) == T && y->size(1) >= D && wb.has_value(), "the sublayer's result must be fp32 [T, >= D] rows with a norm weight");
+    const Slabs ys = slabs_of(*y, "y");
+    ldy = ys.ld;
+    S = ys.S;
+    ss = ys.ss;
+    vec = vec && ys.vec;
+    MCHECK(ys.T == T && ys.n >= D && wb.has_value(), "the sublayer's result must be fp32 [T, >= D] rows with a norm weight");
     f32c(*wb, "wb");
     MCHECK(wb->numel() == D, "the norm weight must hold D numbers");
     yp = y->data_ptr<float>();
@@ -683,17 +708,20 @@ void sandwich_add_norm(at::Tensor& x, const c10::optional<at::Tensor>& y, const 
   }
   if (out.has_value()) {
     ldo = act_ld_min(*out, T, D, "out");
+    vec = vec && ldo % 4 == 0;
     op = out->data_ptr();
     bf = out->scalar_type() == at::kBFloat16;
   }
   if (!yp && !op) return;
+  for (const float* p : {(const float*)x.data_ptr<float>(), bp, np, bbp, bnp, ybp, (const float*)op}) al(p);
 #define SAN_GO(KERNEL, AT)                                                                                              \
   KERNEL<<<T, 256, 0, stream()>>>(x.data_ptr<float>(), yp, ldy, bp, bbp, np, bnp, ybp, (float)mult, (float)eps, (AT*)op, ldo, \
-                                  (int)D)
+                                  (int)D, S, ss)
 #define SAN_PICK(AT)                                                     \
-  if (D <= 1024) SAN_GO((sandwich_add_norm_reg_k<AT, 4>), AT);           \
-  else if (D <= 2048) SAN_GO((sandwich_add_norm_reg_k<AT, 8>), AT);      \
-  else if (D <= 4096) SAN_GO((sandwich_add_norm_reg_k<AT, 16>), AT);     \
+  if (vec && D <= 1024) SAN_GO((sandwich_add_norm_reg_k<AT, 1>), AT);      \
+  else if (vec && D <= 2048) SAN_GO((sandwich_add_norm_reg_k<AT, 2>), AT); \
+  else if (vec && D <= 4096) SAN_GO((sandwich_add_norm_reg_k<AT, 4>), AT); \
+  else if (vec && D <= 8192) SAN_GO((sandwich_add_norm_reg_k<AT, 8>), AT); \
   else SAN_GO(sandwich_add_norm_k<AT>, AT)
   if (bf) {
     SAN_PICK(uint16_t);

@@ -51,6 +51,36 @@ __device__ __forceinline__ void ld8(const uint16_t* p, float* o) {
   for (int i = 0; i < 8; ++i) o[i] = bf2f(a[i]);
 }
 
+__device__ __forceinline__ void st4(float* p, f32x4 v) { *reinterpret_cast<f32x4*>(p) = v; }
+__device__ __forceinline__ void st4(uint16_t* p, f32x4 v) {
+  *reinterpret_cast<s16x4*>(p) = s16x4{(short)f2bf(v[0]), (short)f2bf(v[1]), (short)f2bf(v[2]), (short)f2bf(v[3])};
+}
+
+// element / four elements of a GEMM result that may still be S split-K slabs, ss floats apart (S = 1: a plain result)
+__device__ __forceinline__ float slab1(const float* p, int S, int64_t ss) {
+  float v = p[0];
+  for (int s0 = 1; s0 < S; s0 += 4) {  // (four loads in flight, without branches: slabs past the last repeat it, unused)
+    float a[4];
+#pragma unroll
+    for (int i = 0; i < 4; ++i) a[i] = p[min(s0 + i, S - 1) * ss];
+#pragma unroll
+    for (int i = 0; i < 4; ++i) v += s0 + i < S ? a[i] : 0.0f;
+  }
+  return v;
+}
+__device__ __forceinline__ f32x4 slab4(const float* p, int S, int64_t ss) {
+  f32x4 v = *reinterpret_cast<const f32x4*>(p);
+  for (int s0 = 1; s0 < S; s0 += 4) {
+    f32x4 a[4];
+#pragma unroll
+    for (int i = 0; i < 4; ++i) a[i] = *reinterpret_cast<const f32x4*>(p + min(s0 + i, S - 1) * ss);
+#pragma unroll
+    for (int i = 0; i < 4; ++i)
+      if (s0 + i < S) v += a[i];
+  }
+  return v;
+}
+
 // ------------------------------------------------------------------ host side
 #define MCHECK(cond, ...) TORCH_CHECK(cond, "xot mixers: ", __VA_ARGS__)
 
@@ -66,6 +96,30 @@ inline void i32c(const at::Tensor& t, const char* name) {
 inline int ld_of(const at::Tensor& P, const char* name) {
   MCHECK(P.is_cuda() && P.scalar_type() == at::kFloat && P.dim() == 2 && P.stride(1) == 1, name, " must be fp32 [T, n] rows");
   return (int)P.stride(0);
+}
+// fused projection output, plain [T, n] rows or unreduced split-K slabs [S, T, n]
+struct Slabs {
+  const float* p;
+  int64_t T, n;
+  int ld, S;
+  int64_t ss;
+  bool vec;  // rows and slabs start on 16-byte boundaries
+};
+inline Slabs slabs_of(const at::Tensor& P, const char* name) {
+  MCHECK(P.is_cuda() && P.scalar_type() == at::kFloat && (P.dim() == 2 || P.dim() == 3) && P.stride(-1) == 1, name,
+         " must be fp32 [T, n] rows or [slabs, T, n]");
+  Slabs r;
+  r.p = P.data_ptr<float>();
+  r.T = P.size(-2);
+  r.n = P.size(-1);
+  r.ld = (int)P.stride(-2);
+  r.S = P.dim() == 3 ? (int)P.size(0) : 1;
+  r.ss = P.dim() == 3 ? P.stride(0) : 0;
+  r.vec = r.ld % 4 == 0 && r.ss % 4 == 0 && (reinterpret_cast<uintptr_t>(r.p) & 15) == 0;
+  return r;
+}
+inline void cols_ok(const Slabs& P, int64_t off, int64_t n, const char* what) {
+  MCHECK(off >= 0 && n >= 0 && off + n <= P.n, what, ": columns [", off, ", ", off + n, ") outside the projection");
 }
 inline void cols_ok(const at::Tensor& P, int64_t off, int64_t n, const char* what) {
   MCHECK(off >= 0 && n >= 0 && off + n <= P.size(1), what, ": columns [", off, ", ", off + n, ") outside the projection");

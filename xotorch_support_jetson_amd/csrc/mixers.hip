@@ -61,19 +61,33 @@ __global__ void gelu_mul_k(const float* __restrict__ P, int ldp, int gate_off, i
   stf(out + t * ldo + i, g * u);
 }
 
-// gelu_tanh(gate) * the token's slice of a table: out[t, i] = gelu(P[t, off + i]) * table[ids[t], col0 + i]
-template <typename AT>
-__global__ void gelu_gather_mul_k(const float* __restrict__ P, int ldp, int off, const AT* __restrict__ table, int64_t ldt,
-                                  int V, const int* __restrict__ ids, int col0, int n, AT* __restrict__ out, int ldo,
-                                  int64_t total) {
+// gelu_tanh(gate) * the token's slice of a table: out[t, i] = gelu(P[t, off + i]) * table[ids[t], col0 + i]; W columns per
+// thread; P may be S split-K slabs
+template <typename AT, int W>
+__global__ __launch_bounds__(256) void gelu_gather_mul_k(const float* __restrict__ P, int ldp, int S, int64_t ss, int off,
+                                                         const AT* __restrict__ table, int64_t ldt, int V,
+                                                         const int* __restrict__ ids, int col0, int n, AT* __restrict__ out,
+                                                         int ldo, int64_t total) {
   const int64_t idx = (int64_t)blockIdx.x * blockDim.x + threadIdx.x;
   if (idx >= total) return;
-  const int64_t t = idx / n;
-  const int i = (int)(idx - t * n);
-  const float z = P[t * ldp + off + i];
-  const float e = ldf(table + (int64_t)min(max(ids[t], 0), V - 1) * ldt + col0 + i);
-  const float g = 0.5f * z * (1.0f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z)));
-  stf(out + t * ldo + i, g * e);
+  const int nw = n / W;
+  const int64_t t = idx / nw;
+  const int i = (int)(idx - t * nw) * W;
+  const float* pr = P + t * ldp + off + i;
+  const AT* e = table + (int64_t)min(max(ids[t], 0), V - 1) * ldt + col0 + i;
+  float z[W], y[W];
+  if constexpr (W == 4) {
+    const f32x4 v = slab4(pr, S, ss);
+#pragma unroll
+    for (int k = 0; k < 4; ++k) z[k] = v[k];
+  } else {
+    z[0] = slab1(pr, S, ss);
+  }
+#pragma unroll
+  for (int k = 0; k < W; ++k)
+    y[k] = 0.5f * z[k] * (1.0f + tanhf(0.7978845608028654f * (z[k] + 0.044715f * z[k] * z[k] * z[k]))) * ldf(e + k);
+  if constexpr (W == 4) st4(out + t * ldo + i, f32x4{y[0], y[1], y[2], y[3]});
+  else stf(out + t * ldo + i, y[0]);
 }
 
 // ------------------------------------------------------------------ RoPE + paged key / value write
@@ -817,27 +831,29 @@ void gelu_mul(const at::Tensor& P, int64_t gate_off, int64_t up_off, int64_t F, 
 
 void gelu_gather_mul(const at::Tensor& P, int64_t off, const at::Tensor& table, const at::Tensor& ids, int64_t col0, int64_t n,
                      at::Tensor& out) {
-  const int ldp = ld_of(P, "P");
-  const int64_t T = P.size(0);
-  cols_ok(P, off, n, "gate");
+  const Slabs p = slabs_of(P, "P");
+  const int64_t T = p.T;
+  cols_ok(p, off, n, "gate");
   i32c(ids, "ids");
   MCHECK(ids.numel() == T, "ids must hold one table row per token");
   const int ldo = act_ld_min(out, T, n, "out");
   MCHECK(table.is_cuda() && table.scalar_type() == out.scalar_type() && table.is_contiguous() && table.dim() == 2 &&
              table.size(0) >= 1 && col0 >= 0 && col0 + n <= table.size(1),
          "the table must be [V, >= col0 + n] of the output's dtype");
-  const int64_t total = T * n;
-  if (total == 0) return;
+  if (T * n == 0) return;
+  const bool vec = p.vec && off % 4 == 0 && n % 4 == 0 && ldo % 4 == 0 && (reinterpret_cast<uintptr_t>(out.data_ptr()) & 15) == 0;
+  const int64_t total = T * n / (vec ? 4 : 1);
   const int blocks = (int)((total + 255) / 256);
-  if (out.scalar_type() == at::kBFloat16)
-    gelu_gather_mul_k<uint16_t><<<blocks, 256, 0, stream()>>>(P.data_ptr<float>(), ldp, (int)off,
-                                                              (const uint16_t*)table.data_ptr(), table.size(1),
-                                                              (int)table.size(0), ids.data_ptr<int>(), (int)col0, (int)n,
-                                                              (uint16_t*)out.data_ptr(), ldo, total);
-  else
-    gelu_gather_mul_k<float><<<blocks, 256, 0, stream()>>>(P.data_ptr<float>(), ldp, (int)off, table.data_ptr<float>(),
-                                                           table.size(1), (int)table.size(0), ids.data_ptr<int>(), (int)col0,
-                                                           (int)n, out.data_ptr<float>(), ldo, total);
+#define GGM_GO(AT, W)                                                                                                     \
+  gelu_gather_mul_k<AT, W><<<blocks, 256, 0, stream()>>>(p.p, p.ld, p.S, p.ss, (int)off, (const AT*)table.data_ptr(),     \
+                                                         table.size(1), (int)table.size(0), ids.data_ptr<int>(),          \
+                                                         (int)col0, (int)n, (AT*)out.data_ptr(), ldo, total)
+  if (out.scalar_type() == at::kBFloat16) {
+    if (vec) GGM_GO(uint16_t, 4); else GGM_GO(uint16_t, 1);
+  } else {
+    if (vec) GGM_GO(float, 4); else GGM_GO(float, 1);
+  }
+#undef GGM_GO
 }
 
 void rope_kv_store(const at::Tensor& P, int64_t q_off, int64_t k_off, int64_t v_off, int64_t H, int64_t G, int64_t d,

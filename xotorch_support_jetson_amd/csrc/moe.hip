@@ -6,6 +6,7 @@
 // grouped GEMM treats rows independently and the combine sums each token's k slots in j order, so
 // results do not depend on it.  Everything stays on the device (graph-capturable).
 // moe_combine: h[t] += sum_j w[t, j] * y[slot_of[t, j]] with the expert outputs y in fp32.
+#include <algorithm>
 #include "common.h"
 #include "kernels.h"
 
@@ -85,9 +86,9 @@ __global__ __launch_bounds__(1024) void moe_route_kernel(const float* __restrict
 //   group_limited_greedy) or the sum of their two best choices (V3 noaux_tc); top-k experts by choice among
 //   the kept groups; weight = score (not choice), optionally renormalised, times routed_scaling_factor.
 // Kernel 1: one wave per token (lane l holds experts l, l+64, ..); group statistics from an LDS copy of the
-// token's choices; k rounds of a wave argmax; per-expert counts by global atomics.  Kernel 2 (one workgroup):
-// exclusive scan of the counts -> expert offsets, slot per (token, j), and the counters reset to zero for
-// the next launch (so the graph-captured sequence needs no memset).
+// token's choices; k rounds of a wave argmax; per-expert counts in LDS, added to the global counters once per workgroup
+// (which walks over many tokens).  Kernel 2 (one workgroup): exclusive scan of the counts -> expert offsets, slot per
+// (token, j), and the counters reset to zero for the next launch (so the graph-captured sequence needs no memset).
 constexpr int MOE_DS_MAX_E = 256;
 constexpr int MOE_DS_MAX_G = 32;
 constexpr int MOE_DS_EPL = MOE_DS_MAX_E / 64;  // experts per lane
@@ -98,64 +99,95 @@ __global__ __launch_bounds__(256) void moe_topk_ds_kernel(const float* __restric
                                                           int norm, float scale, float* __restrict__ topw,
                                                           int32_t* __restrict__ topi, int* __restrict__ cnt) {
   __shared__ float ch_lds[4][MOE_DS_MAX_E];
-  __shared__ unsigned keep_lds[4];
+  __shared__ int cnt_lds[MOE_DS_MAX_E];
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
-  const int t = blockIdx.x * 4 + wave;
-  if (t >= T) return;  // wave-uniform; no workgroup barrier below
-  const float* lg = logits + (size_t)t * E;
-  float sc[MOE_DS_EPL], chv[MOE_DS_EPL];
-  float mx = -INFINITY;
-#pragma unroll
-  for (int i = 0; i < MOE_DS_EPL; ++i) {
-    const int e = lane + 64 * i;
-    sc[i] = e < E ? lg[e] : -INFINITY;
-    mx = fmaxf(mx, sc[i]);
-  }
-  if (!sigmoid) {
-    mx = wave_max(mx);
-    float den = 0.f;
+  for (int e = threadIdx.x; e < E; e += 256) cnt_lds[e] = 0;
+  __syncthreads();
+  for (int t = blockIdx.x * 4 + wave; t < T; t += gridDim.x * 4) {  // wave-uniform; no workgroup barrier inside
+    const float* lg = logits + (size_t)t * E;
+    float sc[MOE_DS_EPL], chv[MOE_DS_EPL];
+    float mx = -INFINITY;
 #pragma unroll
     for (int i = 0; i < MOE_DS_EPL; ++i) {
-      sc[i] = lane + 64 * i < E ? __expf(sc[i] - mx) : 0.f;
-      den += sc[i];
+      const int e = lane + 64 * i;
+      sc[i] = e < E ? lg[e] : -INFINITY;
+      mx = fmaxf(mx, sc[i]);
     }
-    den = wave_sum(den);
+    if (!sigmoid) {
+      mx = wave_max(mx);
+      float den = 0.f;
 #pragma unroll
-    for (int i = 0; i < MOE_DS_EPL; ++i) sc[i] /= den;
-  } else {
+      for (int i = 0; i < MOE_DS_EPL; ++i) {
+        sc[i] = lane + 64 * i < E ? __expf(sc[i] - mx) : 0.f;
+        den += sc[i];
+      }
+      den = wave_sum(den);
 #pragma unroll
-    for (int i = 0; i < MOE_DS_EPL; ++i) sc[i] = lane + 64 * i < E ? 1.f / (1.f + expf(-sc[i])) : 0.f;
-  }
+      for (int i = 0; i < MOE_DS_EPL; ++i) sc[i] /= den;
+    } else {
 #pragma unroll
-  for (int i = 0; i < MOE_DS_EPL; ++i) {
-    const int e = lane + 64 * i;
-    chv[i] = e < E ? sc[i] + (bias != nullptr ? bias[e] : 0.f) : -INFINITY;
-    if (e < E) ch_lds[wave][e] = chv[i];
-  }
-  const int per = E / n_group;
-  unsigned keep = 0xffffffffu;
-  if (n_group > 1 && topk_group < n_group) {
-    __builtin_amdgcn_wave_barrier();
-    __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
-    // lane g < n_group: its group's best (V2) or best-two sum (V3) over the LDS copy
-    float gsc = -INFINITY;
-    if (lane < n_group) {
-      float a = -INFINITY, b2 = -INFINITY;
-      for (int e = lane * per; e < (lane + 1) * per; ++e) {
-        const float v = ch_lds[wave][e];
-        if (v > a) {
-          b2 = a;
-          a = v;
-        } else if (v > b2) {
-          b2 = v;
+      for (int i = 0; i < MOE_DS_EPL; ++i) sc[i] = lane + 64 * i < E ? 1.f / (1.f + expf(-sc[i])) : 0.f;
+    }
+#pragma unroll
+    for (int i = 0; i < MOE_DS_EPL; ++i) {
+      const int e = lane + 64 * i;
+      chv[i] = e < E ? sc[i] + (bias != nullptr ? bias[e] : 0.f) : -INFINITY;
+      if (e < E) ch_lds[wave][e] = chv[i];
+    }
+    const int per = E / n_group;
+    unsigned keep = 0xffffffffu;
+    if (n_group > 1 && topk_group < n_group) {
+      __builtin_amdgcn_wave_barrier();
+      __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+      // lane g < n_group: its group's best (V2) or best-two sum (V3) over the LDS copy
+      float gsc = -INFINITY;
+      if (lane < n_group) {
+        float a = -INFINITY, b2 = -INFINITY;
+        for (int e = lane * per; e < (lane + 1) * per; ++e) {
+          const float v = ch_lds[wave][e];
+          if (v > a) {
+            b2 = a;
+            a = v;
+          } else if (v > b2) {
+            b2 = v;
+          }
+        }
+        gsc = (method == 2 && per > 1) ? a + b2 : a;  // (a group of one expert has no second best)
+      }
+      keep = 0;
+      for (int j = 0; j < topk_group; ++j) {  // wave argmax over the groups (ties: lower group id)
+        float v = (lane < n_group && !(keep >> lane & 1u)) ? gsc : -INFINITY;
+        int id = lane;
+#pragma unroll
+        for (int o = 32; o > 0; o >>= 1) {
+          const float ov = __shfl_xor(v, o, 64);
+          const int oi = __shfl_xor(id, o, 64);
+          if (ov > v || (ov == v && oi < id)) {
+            v = ov;
+            id = oi;
+          }
+        }
+        keep |= 1u << id;
+      }
+    }
+#pragma unroll
+    for (int i = 0; i < MOE_DS_EPL; ++i) {
+      const int e = lane + 64 * i;
+      if (e >= E || !(keep >> (e / per) & 1u)) chv[i] = -INFINITY;
+    }
+    float wsum = 0.f, wj_mine = 0.f;
+    int ej_mine = 0;
+    for (int j = 0; j < k; ++j) {  // k rounds of a wave argmax over the kept experts (ties: lower expert id)
+      float v = -INFINITY;
+      int id = 0x7fffffff;
+#pragma unroll
+      for (int i = 0; i < MOE_DS_EPL; ++i) {
+        const int e = lane + 64 * i;
+        if (chv[i] > v) {
+          v = chv[i];
+          id = e;
         }
       }
-      gsc = (method == 2 && per > 1) ? a + b2 : a;  // (a group of one expert has no second best)
-    }
-    keep = 0;
-    for (int j = 0; j < topk_group; ++j) {  // wave argmax over the groups (ties: lower group id)
-      float v = (lane < n_group && !(keep >> lane & 1u)) ? gsc : -INFINITY;
-      int id = lane;
 #pragma unroll
       for (int o = 32; o > 0; o >>= 1) {
         const float ov = __shfl_xor(v, o, 64);
@@ -165,60 +197,34 @@ __global__ __launch_bounds__(256) void moe_topk_ds_kernel(const float* __restric
           id = oi;
         }
       }
-      keep |= 1u << id;
-    }
-  }
+      // (scores that are not numbers -- rows of a padded batch may hold anything -- leave no winner: take expert j,
+      // so that every index written below is an expert)
+      if (id >= E) id = j;
+      // the owner lane retires the winner and contributes its score
+      float wv = 0.f;
 #pragma unroll
-  for (int i = 0; i < MOE_DS_EPL; ++i) {
-    const int e = lane + 64 * i;
-    if (e >= E || !(keep >> (e / per) & 1u)) chv[i] = -INFINITY;
-  }
-  float wsum = 0.f, wj_mine = 0.f;
-  int ej_mine = 0;
-  for (int j = 0; j < k; ++j) {  // k rounds of a wave argmax over the kept experts (ties: lower expert id)
-    float v = -INFINITY;
-    int id = 0x7fffffff;
-#pragma unroll
-    for (int i = 0; i < MOE_DS_EPL; ++i) {
-      const int e = lane + 64 * i;
-      if (chv[i] > v) {
-        v = chv[i];
-        id = e;
+      for (int i = 0; i < MOE_DS_EPL; ++i)
+        if (lane + 64 * i == id) {
+          chv[i] = -INFINITY;
+          wv = sc[i];
+        }
+      wv = wave_sum(wv);
+      wsum += wv;
+      if (lane == j) {
+        wj_mine = wv;
+        ej_mine = id;
       }
     }
-#pragma unroll
-    for (int o = 32; o > 0; o >>= 1) {
-      const float ov = __shfl_xor(v, o, 64);
-      const int oi = __shfl_xor(id, o, 64);
-      if (ov > v || (ov == v && oi < id)) {
-        v = ov;
-        id = oi;
-      }
-    }
-    // (scores that are not numbers -- rows of a padded batch may hold anything -- leave no winner: take expert j,
-    // so that every index written below is an expert)
-    if (id >= E) id = j;
-    // the owner lane retires the winner and contributes its score
-    float wv = 0.f;
-#pragma unroll
-    for (int i = 0; i < MOE_DS_EPL; ++i)
-      if (lane + 64 * i == id) {
-        chv[i] = -INFINITY;
-        wv = sc[i];
-      }
-    wv = wave_sum(wv);
-    wsum += wv;
-    if (lane == j) {
-      wj_mine = wv;
-      ej_mine = id;
+    const float f = norm ? scale / (wsum + 1e-20f) : scale;
+    if (lane < k) {
+      topw[(size_t)t * k + lane] = wj_mine * f;
+      topi[(size_t)t * k + lane] = ej_mine;
+      atomicAdd(cnt_lds + ej_mine, 1);
     }
   }
-  const float f = norm ? scale / (wsum + 1e-20f) : scale;
-  if (lane < k) {
-    topw[(size_t)t * k + lane] = wj_mine * f;
-    topi[(size_t)t * k + lane] = ej_mine;
-    atomicAdd(cnt + ej_mine, 1);
-  }
+  __syncthreads();
+  for (int e = threadIdx.x; e < E; e += 256)
+    if (cnt_lds[e] > 0) atomicAdd(cnt + e, cnt_lds[e]);
 }
 
 __global__ __launch_bounds__(1024) void moe_slots_kernel(const int32_t* __restrict__ topi, int T, int E, int k,
@@ -254,7 +260,7 @@ int launch_moe_route_ds(const float* logits, const float* bias, int T, int E, in
       topk_group < 1 || topk_group > n_group || k > (E / n_group) * topk_group)
     return -1;
   if (T <= 0) return 0;
-  moe_topk_ds_kernel<<<(T + 3) / 4, 256, 0, s>>>(logits, bias, T, E, k, n_group, topk_group, method, sigmoid ? 1 : 0,
+  moe_topk_ds_kernel<<<std::min((T + 3) / 4, 512), 256, 0, s>>>(logits, bias, T, E, k, n_group, topk_group, method, sigmoid ? 1 : 0,
                                                  norm ? 1 : 0, scale, topw, topi, cnt);
   moe_slots_kernel<<<1, 1024, 0, s>>>(topi, T, E, k, cnt, slot_of, sorted_tok, off);
   return 0;

@@ -28,7 +28,8 @@ import torch
 from ..inference.shard import Shard
 from ..ops import kernels as K
 from ..ops._ext import require
-from ..ops.linear import FUSE_MERGE, FUSE_NORM, PendingNorm, layout_of, linear, linear_resid_norm, linear_rope_kv, scratch
+from ..ops.linear import (FUSE_MERGE, FUSE_NORM, PendingNorm, layout_of, linear, linear_resid_norm, linear_rope_kv,
+                          linear_slabs, scratch)
 from ..ops.rope import longrope_window, rope_shift, rope_table
 from .config import ModelConfig
 from .weights import ShardWeights, expert
@@ -442,6 +443,37 @@ class ShardModel:
       return torch.matmul(x, w.t())
     return linear(x, w, out_dtype=torch.float32)
 
+  @staticmethod
+  def _proj_slabs(x: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
+    """The same for a consumer that sums unreduced split-K slabs itself (and runs before the next GEMM): [T, n] or [S, T, n]."""
+    if x.dtype == torch.float32 or not x.is_cuda:
+      return ShardModel._proj(x, w)
+    return linear_slabs(x, w)
+
+  @staticmethod
+  def _fused_act(x: torch.Tensor, w: torch.Tensor, epi: str, limit: float = 0.0) -> Optional[torch.Tensor]:
+    """act(x @ w^T) in the GEMM's epilogue (bf16, pre-shuffled weights), or None where that is not built."""
+    if x.dtype != torch.bfloat16 or not x.is_cuda or layout_of(w) != "stream":
+      return None
+    return linear(x, w, epi=epi, epi_arg=limit)
+
+  @staticmethod
+  def _glu_tiles(gu: torch.Tensor, clamped: bool, limit: float, out: torch.Tensor) -> torch.Tensor:
+    """The gated activation of a product whose gate / up columns alternate in tiles of 16 -> out [rows, columns / 2]."""
+    n = gu.shape[1] // 2
+    t = gu.reshape(-1, n // 16, 2, 16)
+    K.glu_act(torch.cat([t[:, :, 0].reshape(-1, n), t[:, :, 1].reshape(-1, n)], 1), 0, n, n, clamped, limit, out)
+    return out
+
+  def _router(self, hn: torch.Tensor, w: torch.Tensor, E: int) -> torch.Tensor:
+    """fp32 router logits [T, E] of a projection whose first E rows are the router."""
+    if hn.is_cuda and hn.dtype == torch.bfloat16 and layout_of(w) == "rowmajor" and (
+        E in (4, 8, 16) or (E in (32, 64, 128, 160, 256) and hn.shape[1] % 512 == 0)):
+      out = torch.empty(hn.shape[0], E, dtype=torch.float32, device=hn.device)
+      require().router_logits(hn, w[:E], out)
+      return out
+    return self._proj(hn, w)[:, :E].contiguous()
+
   def _gated_attn(self, P: torch.Tensor, lw, j: int, inp: StepInputs, mix: torch.Tensor) -> None:
     """Chunk-local sigmoid attention: RoPE + paged write of (rotated key, key as projected), then the gated sum
     over the query's chunk, scaled into the mixers' output row."""
@@ -551,7 +583,7 @@ class ShardModel:
     """Softmax attention over a sliding window or the query's chunk, pooled blocks and a sink: biases + norms + RoPE + paged
     write, the pooled caches' update for blocks that this step completed, then the attention."""
     a = lw.spec.wattn
-    q = torch.empty(P.shape[0], a.heads, a.dim, dtype=mix.dtype, device=P.device)
+    q = torch.empty(mix.shape[0], a.heads, a.dim, dtype=mix.dtype, device=P.device)
     tab = self.rope_tabs.get((a.rot_dims, a.rot_base, a.rot_scaling))
     own = a.kv_from < 0
     K.qk_norm_rope_store(P, lw.in_b, lw.cols["q"][0], lw.cols["k"][0] if own else -1, lw.cols["v"][0] if own else -1,
@@ -782,19 +814,19 @@ class ShardModel:
       return torch.bmm(x, w)
     return torch.bmm(x.float(), w.float()).to(x.dtype)
 
-  def _glu_moe(self, hn: torch.Tensor, P: torch.Tensor, lw, rows) -> torch.Tensor:
+  def _glu_moe(self, hn: torch.Tensor, lw) -> torch.Tensor:
     """Gated experts (SiLU, or the clamped form) chosen by the softmax scores' top-k, maybe among the best groups (weights:
     the scores as they are) + the ungated shared expert -> fp32 [T, D].  Routing on the framework's grouped top-k kernel,
     experts on the grouped GEMMs (bf16) or per expert on the vendor SGEMM (fp32)."""
-    f, dev = lw.spec.ffn, P.device
+    f, dev = lw.spec.ffn, hn.device
     T, D = hn.shape[0], self.c.hidden_size
     E, k = f.experts, f.top
     clamped = f.kind == "clamped_moe"
-    r0 = lw.ff_cols["router"][0]
-    logits = P[:, r0:r0 + E].contiguous()
+    epi = "clamp_glu" if clamped else "silu"
+    logits = self._router(hn, lw.ff_w, E)
     Fp, Dq, S = lw.ex_down_w.shape[2], lw.ex_down_w.shape[1], 1
     method = 1 if f.groups > 1 else 0  # (a group's value: its largest score)
-    if P.is_cuda:
+    if hn.is_cuda:
       topw = torch.empty(T * k, dtype=torch.float32, device=dev)
       topi, slot_of, sorted_tok = (torch.empty(T * k, dtype=torch.int32, device=dev) for _ in range(3))
       off = torch.empty(E + 1, dtype=torch.int32, device=dev)
@@ -819,7 +851,7 @@ class ShardModel:
       if Fp % (256 * S):
         S = 1
       act = torch.empty(T * k, Fp, dtype=torch.bfloat16, device=dev)  # the gated activation in the GEMM's epilogue
-      C.gemm_moe(hn, lw.ex_up_w, act, off, sorted_tok, K.EPI["clamp_glu" if clamped else "silu"], T, sh_up, 1, bm, f.limit)
+      C.gemm_moe(hn, lw.ex_up_w, act, off, sorted_tok, K.EPI[epi], T, sh_up, 1, bm, f.limit)
       y = torch.empty(S * T * k, Dq, dtype=torch.float32, device=dev)
       C.gemm_moe(act, lw.ex_down_w, y, off, None, K.EPI["none"], T, sh_dn, S, bm_dn)
     else:
@@ -829,16 +861,16 @@ class ShardModel:
       for e in range(E):
         if offs[e + 1] > offs[e]:
           xe = hn.index_select(0, sorted_tok[offs[e]:offs[e + 1]].long()).float()
-          gu = (xe @ lw.ex_up_w[e].float().t()).reshape(xe.shape[0], Fp // 16, 2, 16)  # (gate | up tiles of 16)
-          gu = torch.cat([gu[:, :, 0].reshape(-1, Fp), gu[:, :, 1].reshape(-1, Fp)], 1)
           act = torch.empty(xe.shape[0], Fp, dtype=torch.float32, device=dev)
-          K.glu_act(gu, 0, Fp, Fp, clamped, f.limit, act)
+          self._glu_tiles(xe @ lw.ex_up_w[e].float().t(), clamped, f.limit, act)
           y[offs[e]:offs[e + 1]] = act @ lw.ex_down_w[e].float().t()
     sh_y = None
     if f.shared_ff:
-      act = rows("sh_act", f.shared_ff, lw.down_w.shape[1])
-      K.glu_act(P, lw.ff_cols["sh_gate"][0], lw.ff_cols["sh_up"][0], f.shared_ff, clamped, f.shared_limit, act)
-      sh_y = self._proj(act, lw.down_w)
+      act = self._fused_act(hn, lw.sh_gu_w, epi, f.shared_limit)
+      if act is None:
+        act = self._glu_tiles(self._proj(hn, lw.sh_gu_w), clamped, f.shared_limit,
+                              torch.empty(T, lw.sh_gu_w.shape[0] // 2, dtype=hn.dtype, device=dev))
+      sh_y = self._proj_slabs(act, lw.down_w)
     out = torch.empty(T, D, dtype=torch.float32, device=dev)
     K.moe_weighted_sum(y, slot_of, topw, k, sh_y, None, 0, out, splits=S)
     return out
@@ -848,15 +880,15 @@ class ShardModel:
     projected to the width -> fp32 rows, not normed yet."""
     n = lw.spec.side
     act = rows("side", n, lw.side_proj_w.shape[1])
-    K.gelu_gather_mul(self._proj(hn, lw.side_gate_w), 0, self.w.side_embed, ids, (j - self.layer_ids[0]) * n, n, act)
-    return self._proj(act, lw.side_proj_w)
+    K.gelu_gather_mul(self._proj_slabs(hn, lw.side_gate_w), 0, self.w.side_embed, ids, (j - self.layer_ids[0]) * n, n, act)
+    return self._proj_slabs(act, lw.side_proj_w)
 
   def _forward_sandwich(self, h: torch.Tensor, inp: StepInputs, adt, ids: Optional[torch.Tensor] = None) -> torch.Tensor:
     """Layer runs (a looped layer once per pass, each pass with caches and states of its own) of sandwich blocks on the
     fp32 stream h (hn: the normed sublayer input in the GEMMs' operand dtype):
       pass start:  h <- [h | embedding output] @ loop_in^T + step[pass]       (loop_input "linear")
                    h <- h + embedding output (passes after the first) + step[pass]       ("add")
-      P = hn @ in_w^T                    every projection that reads the mixer's input
+      P = hn @ in_w^T                    every projection that reads the mixer's input (split-K slabs where one kernel reads it)
       h += mult * norm1b(mixer(P) @ out_w^T);  hn = norm2(h)
       P = hn @ ff_w^T                    gate | up, or router | shared expert's projections
       h += mult * norm2b(ff(P));  hn = the next run's norm1(h)
@@ -900,7 +932,8 @@ class ShardModel:
         fresh = True
       if fresh:  # (no norm weight: the op copies the stream)
         K.sandwich_add_norm(h, None, None, lw.norm1, eps, hn, bn=lw.norm1_b)
-      P = self._proj(hn, lw.in_w)
+      # (window attention alone: the store kernel is the projection's only reader)
+      P = (self._proj_slabs if s.wattn is not None and s.wattn.gate == "none" and s.rec is None else self._proj)(hn, lw.in_w)
       mix = rows("mix", lw.mix_cols["mix"][1], lw.out_w.shape[1])
       if s.lattn is not None:
         self._latent_attn(P, lw, j, inp, mix, rows)
@@ -910,7 +943,7 @@ class ShardModel:
         self._window_attn(P, lw, j, inp, mix)
       else:
         self._mlstm(P, lw, j, inp, mix)
-      y = self._proj(mix, lw.out_w)
+      y = (self._proj if s.wattn is not None and s.rec is not None else self._proj_slabs)(mix, lw.out_w)
       if s.wattn is not None and s.rec is not None:  # the second mixer of a parallel layer, then the mean of the normed pair
         mix2 = rows("mix2", lw.mix_cols["mix2"][1], lw.out2_w.shape[1])
         self._lightning(P, lw, j, inp, mix2)
@@ -928,19 +961,20 @@ class ShardModel:
                             yb=lw.out_b)
       else:
         K.sandwich_add_norm(h, y, lw.norm1b, lw.norm2, eps, hn, bb=lw.norm1b_b, bn=lw.norm2_b, mult=mult, yb=lw.out_b)
-        P = self._proj(hn, lw.ff_w)
         if f.kind == "clamped_glu":
           act = rows("act", f.ff, lw.down_w.shape[1])
-          K.glu_act(P, lw.ff_cols["gate"][0], lw.ff_cols["up"][0], f.ff, True, f.limit, act)
-          y = self._proj(act, lw.down_w)
+          K.glu_act(self._proj(hn, lw.ff_w), lw.ff_cols["gate"][0], lw.ff_cols["up"][0], f.ff, True, f.limit, act)
+          y = self._proj_slabs(act, lw.down_w)
         elif f.kind == "relu2":
-          act = rows("act", f.ff, lw.down_w.shape[1])
-          K.relu2(P, lw.ff_cols["up"][0], f.ff, act)
-          y = self._proj(act, lw.down_w)
+          act = self._fused_act(hn, lw.ff_w, "relu2")
+          if act is None:
+            act = rows("act", f.ff, lw.down_w.shape[1])
+            K.relu2(self._proj(hn, lw.ff_w), lw.ff_cols["up"][0], f.ff, act)
+          y = self._proj_slabs(act, lw.down_w)
         elif f.kind == "relu2_moe":
-          y = self._relu2_moe(hn, P, lw, rows)
+          y = self._relu2_moe(hn, self._proj(hn, lw.ff_w), lw, rows)
         else:
-          y = self._glu_moe(hn, P, lw, rows)
+          y = self._glu_moe(hn, lw)
         K.sandwich_add_norm(h, y, lw.norm2b, nxt, eps, hn if after[0] else hn_nxt, bb=lw.norm2b_b, bn=nxt_b, mult=mult)
       if after[0]:
         K.sandwich_add_norm(h, self._side_input(hn, lw, li, ids, rows), lw.side_norm, nxt, eps, hn_nxt, bn=nxt_b)

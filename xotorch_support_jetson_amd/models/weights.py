@@ -346,7 +346,7 @@ def prepare_for_decode(sw: "ShardWeights", keep_rowmajor: Iterable[str] = (), fp
       if lw.in_w.dtype == torch.bfloat16:
         lw.in_w, lw.out_w, lw.down_w, lw.ff_w = wide(lw.in_w), wide(lw.out_w), wide(lw.down_w), wide(lw.ff_w)
         lw.uq_w, lw.out2_w = wide(lw.uq_w), wide(lw.out2_w)
-        lw.side_gate_w, lw.side_proj_w = wide(lw.side_gate_w), wide(lw.side_proj_w)
+        lw.side_gate_w, lw.side_proj_w, lw.sh_gu_w = wide(lw.side_gate_w), wide(lw.side_proj_w), wide(lw.sh_gu_w)
         lw.ex_up_w, lw.ex_down_w = conv(lw.ex_up_w), conv(lw.ex_down_w)  # experts: shuffled per expert
     if sw.lm_head is not None and sw.lm_head.dtype == torch.bfloat16:
       sw.lm_head = wide(sw.lm_head)
@@ -757,6 +757,7 @@ class MixedLayerWeights:
   side_gate_w: Optional[torch.Tensor] = None  # [side padded, Dp]
   side_proj_w: Optional[torch.Tensor] = None  # [Dn, side padded]
   side_norm: Optional[torch.Tensor] = None  # [D] fp32
+  sh_gu_w: Optional[torch.Tensor] = None  # shared gated expert: gate / up rows interleaved by 16 [2 Fs, Dp]
 
   def tensors(self) -> Dict[str, torch.Tensor]:
     return {k: v for k, v in self.__dict__.items() if isinstance(v, torch.Tensor)}
@@ -926,14 +927,15 @@ def build_sandwich_layer(spec, get, p: str, D: int, device, dtype) -> MixedLayer
 
 
 def _gated_moe_weights(lw: MixedLayerWeights, f, get, q: str, D: int, dev, dtype):
-  """Gated experts (SiLU or clamped) stacked and padded; -> the fused blocks [router | shared gate | shared up] and the
+  """Gated experts (SiLU or clamped) stacked and padded, the shared expert likewise; -> the blocks [router] and the
   shared expert's down projection (None: no shared expert)."""
   fb, down = [("router", get(q + "router"))], None
-  if f.shared_ff:
-    fb += [("sh_gate", get(q + "shared.gate")), ("sh_up", get(q + "shared.up"))]
-    down = get(q + "shared.down")
   Fp, Dp = _up(f.ff, 128), _up(D, 128)
-  # gate and up rows interleaved in tiles of 16 (the grouped GEMM's gated epilogues pair them)
+  # gate and up rows interleaved in tiles of 16 (the GEMMs' gated epilogues pair them)
+  if f.shared_ff:
+    Fs = _up(f.shared_ff, 128)
+    lw.sh_gu_w = dev(interleave_gate_up(_pad2(get(q + "shared.gate"), Fs, Dp), _pad2(get(q + "shared.up"), Fs, Dp)), dtype)
+    down = get(q + "shared.down")
   lw.ex_up_w = dev(torch.stack([interleave_gate_up(_pad2(get(q + f"e{e}.gate"), Fp, Dp), _pad2(get(q + f"e{e}.up"), Fp, Dp))
                                 for e in range(f.experts)]), dtype)
   lw.ex_down_w = dev(torch.stack([_pad2(get(q + f"e{e}.down"), Dp, Fp) for e in range(f.experts)]), dtype)

@@ -14,7 +14,8 @@ import torch
 from . import reference as ref
 from ._ext import require
 
-EPI = {"none": 0, "resid": 1, "silu": 2, "clamp_glu": 3}
+EPI = {"none": 0, "resid": 1, "silu": 2, "clamp_glu": 3, "relu2": 4}
+GLU_EPI = ("silu", "clamp_glu")  # epilogues that turn interleaved (gate, up) columns into half as many
 PAGE = 64
 
 

@@ -325,7 +325,7 @@ class GemmPolicy:
   @staticmethod
   def _stream_cands(M, N, Kd, epi):
     cands = []
-    for ntw in ((2, 4) if epi == "silu" else (1, 2, 4)):
+    for ntw in ((2, 4) if epi in K.GLU_EPI else (1, 2, 4)):
       if N % (64 * ntw) or (ntw == 4 and M <= 32):
         continue
       for S in (1, 2, 4, 8):
@@ -366,9 +366,9 @@ class GemmPolicy:
     got = self._lookup(key)
     if got is not None:
       return got
-    if (TALL_FIXED and W4 and M >= W4_PREF_M and N % 256 == 0 and Kd % 128 == 0
+    if (TALL_FIXED and W4 and M >= W4_PREF_M and N % 256 == 0 and Kd % 128 == 0 and (N > 256 or -(-M // 256) >= 256)
         and not (epi == "resid" and out_dtype == torch.float32) and M * x.stride(0) * 2 < (1 << 32)):
-      # (the last term: the tile's LDS-DMA loads take 32-bit byte offsets into X; taller / wider X take the
+      # (one column of tiles that leaves CUs idle is tuned like the small shapes; the last term: the tile's LDS-DMA loads take 32-bit byte offsets into X; taller / wider X take the
       # tuned candidates below)
       # tall GEMMs (prefill chunks, training): the four-wave tile at S = 1 won every tuned tall shape this round
       # (profiles/r5/headline/bench_r5o_tunelog.log), so it is taken without the cold-timing pass, which cost
@@ -380,13 +380,14 @@ class GemmPolicy:
     if M <= STREAM_MAX_M:
       cands += [("stream",) + c for c in self._stream_cands(M, N, Kd, epi)]
     if M >= BIG_MIN_M and Kd % 128 == 0:
-      cands += self._big_cands(M, N, Kd)
+      big = self._big_cands(M, N, Kd)
+      cands += [c for c in big if c[1] in (2256, 128, 4256)] if epi in ("clamp_glu", "relu2") else big  # (the tiles built with them)
     if not cands:
       raise RuntimeError(f"no GEMM configuration for pre-shuffled N={N} K={Kd} M={M}")
     if self._no_tuning():
       return self._heuristic(M, N, cands)
     scratch.splitk(x.device, max(_ws_elems(c, M, N) for c in cands))
-    y = torch.empty(M, N // 2 if epi == "silu" else N, dtype=out_dtype, device=x.device)
+    y = torch.empty(M, N // 2 if epi in K.GLU_EPI else N, dtype=out_dtype, device=x.device)
     times = {}
     for cfg in cands:
       try:
@@ -472,11 +473,11 @@ def _slab_read_ms(cfg, M, N) -> float:
 policy = GemmPolicy()
 
 
-def _stream_call(x, w, bias, residual, epi, out, cfg, shuffled: bool = True):
+def _stream_call(x, w, bias, residual, epi, out, cfg, shuffled: bool = True, epi_arg: float = 0.0):
   ntw, S = cfg
   M, N = x.shape[0], w.shape[0]
   ws = scratch.splitk(x.device, S * M * N) if S > 1 else None
-  require().gemm_stream(x, w, out, bias, residual, ws, K.EPI[epi], ntw, S, shuffled)
+  require().gemm_stream(x, w, out, bias, residual, ws, K.EPI[epi], ntw, S, shuffled, True, epi_arg)
   return out
 
 
@@ -505,13 +506,13 @@ def _linear8(x, w, bias, residual, epi, out, dt):
   return _stream8_call(x, w, bias, residual, epi, out, policy.stream8_cfg(x, w, bias, residual, epi, dt))
 
 
-def _shuffled_call(x, w, bias, residual, epi, out, cfg):
+def _shuffled_call(x, w, bias, residual, epi, out, cfg, epi_arg: float = 0.0):
   if cfg[0] == "stream":
-    return _stream_call(x, w, bias, residual, epi, out, cfg[1:])
+    return _stream_call(x, w, bias, residual, epi, out, cfg[1:], epi_arg=epi_arg)
   _, bn, S = cfg
   M, N = x.shape[0], w.shape[0]
   ws = scratch.splitk(x.device, S * M * N) if S > 1 else None
-  require().gemm_big(x, w, out, bias, residual, ws, K.EPI[epi], bn, S)
+  require().gemm_big(x, w, out, bias, residual, ws, K.EPI[epi], bn, S, True, epi_arg)
   return out
 
 
@@ -615,7 +616,9 @@ def _pending_cfg(p: PendingNorm, w: torch.Tensor, bias, epi: str):
 
 
 def linear(x: torch.Tensor, w: torch.Tensor, bias: torch.Tensor | None = None, residual: torch.Tensor | None = None,
-           epi: str = "none", out: torch.Tensor | None = None, out_dtype: torch.dtype | None = None) -> torch.Tensor:
+           epi: str = "none", out: torch.Tensor | None = None, out_dtype: torch.dtype | None = None,
+           epi_arg: float = 0.0) -> torch.Tensor:
+  """epi "clamp_glu" (limit: epi_arg) and "relu2" run on pre-shuffled GPU weights with bf16 output only."""
   if isinstance(x, PendingNorm):
     cfg = None if (residual is not None or (out_dtype not in (None, torch.bfloat16))
                    or (out is not None and out.dtype != torch.bfloat16)) else _pending_cfg(x, w, bias, epi)
@@ -637,12 +640,32 @@ def linear(x: torch.Tensor, w: torch.Tensor, bias: torch.Tensor | None = None, r
     impl = policy.choose(x, w, bias, residual, epi, dt)
     return _run_rowmajor(impl, x, w, bias, residual, epi, out, out_dtype)
   if out is None:
-    out = torch.empty(M, N // 2 if epi == "silu" else N, dtype=dt, device=x.device)
+    out = torch.empty(M, N // 2 if epi in K.GLU_EPI else N, dtype=dt, device=x.device)
   if x.stride(1) != 1 or x.stride(0) % 8:
     x = x.contiguous()
   cfg = policy.shuffled_cfg(x, w, bias, residual, epi, dt)
-  _shuffled_call(x, w, bias, residual, epi, out, cfg)
+  _shuffled_call(x, w, bias, residual, epi, out, cfg, epi_arg)
   return out
+
+
+def linear_slabs(x: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
+  """fp32 x @ w.T for a consumer that sums split-K slabs itself: [M, N], or [S, M, N] when the projection runs split over K
+  (a view of the shared scratch: valid until the next split-K GEMM)."""
+  if x.is_cuda and layout_of(w) == "stream":
+    if x.stride(1) != 1 or x.stride(0) % 8:
+      x = x.contiguous()
+    M, N = x.shape[0], w.shape[0]
+    cfg = policy.shuffled_cfg(x, w, None, None, "none", torch.float32)
+    S = cfg[2]
+    if S > 1:
+      ws = scratch.splitk(x.device, S * M * N)
+      y = torch.empty(M, N, dtype=torch.float32, device=x.device)  # shape carrier only: the slabs are not reduced
+      if cfg[0] == "stream":
+        require().gemm_stream(x, w, y, None, None, ws, K.EPI["none"], cfg[1], S, True, False)
+      else:
+        require().gemm_big(x, w, y, None, None, ws, K.EPI["none"], cfg[1], S, False)
+      return ws[:S * M * N].view(S, M, N)
+  return linear(x, w, out_dtype=torch.float32)
 
 
 
