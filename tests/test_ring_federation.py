@@ -72,6 +72,10 @@ async def _scenario_steps(eng, shard_dict):
   return await _steps(eng, Shard.from_dict(shard_dict))
 
 
+async def _scenario_prompt_steps(eng, shard_dict, prompt):
+  return await _steps(eng, Shard.from_dict(shard_dict), prompt=prompt)
+
+
 async def _scenario_protocol(eng, shard_dict, ckdir):
   """Prefix reuse with two concurrent requests, a failing rank, training, evaluation, checkpoint save / load."""
   from xotorch_support_jetson_amd.train.checkpoint import checkpoint_path
@@ -103,7 +107,7 @@ async def _scenario_protocol(eng, shard_dict, ckdir):
   return res
 
 
-SCENARIOS = {"steps": _scenario_steps, "protocol": _scenario_protocol}
+SCENARIOS = {"steps": _scenario_steps, "prompt_steps": _scenario_prompt_steps, "protocol": _scenario_protocol}
 
 
 def _worker(rank, world, port, q, scenario, args):
@@ -202,6 +206,17 @@ def test_federated_ring_matches_one_engine(world, lo, hi):
     res = _spawn(_worker_hidden, world, shard.to_dict(), h)
     want, _ = asyncio.run(cpu_engine().infer_tensor("h", shard, h, {}))
     assert np.allclose(res[0][0].float().numpy(), torch.as_tensor(want).float().numpy(), atol=2e-2, rtol=2e-2)
+
+
+def test_federated_ring_of_a_model_with_side_inputs():
+  """The hidden states between the ranks keep the fp32 stream and the token ids beside it (later layers look side inputs
+  up by them): two ranks give what one engine gives."""
+  shard = Shard("tiny-torinex", 0, 3, 4)
+  prompt = np.array([[3, 17, 301, 5, 299, 7, 11, 257, 31, 8]], dtype=np.int64)
+  ref = asyncio.run(_steps(cpu_engine(), shard, prompt=prompt))
+  got = _spawn(_worker, 2, "prompt_steps", (shard.to_dict(), prompt))[0][0]
+  for a, b in zip(got, ref):
+    assert np.allclose(a, b, atol=1e-4, rtol=1e-4), np.abs(a - b).max()
 
 
 def _worker_hidden(rank, world, port, q, shard_dict, h):

@@ -1108,11 +1108,13 @@ TINY_TORINEX = {
   "architecture": "Torinex", "vocab": 312, "width": 104, "norm": {"eps": 1e-5}, "token_side": {"dim": 12},
   "layers": [
     {"type": "attention", "mlp": {"kind": "dense", "ff": 152}, "mixer": _TINY_CHUNK},
+    {"type": "attention", "mlp": _TINY_CMOE, "mixer": dict(_TINY_CHUNK, kv_from=0, mask={"size": 20}, scale=0.2)},
     {"type": "attention", "mlp": _TINY_CMOE,
      "mixer": {"heads": 6, "kv_heads": 2, "dim": 16, "vdim": 16, "mask": {"size": 70}, "rot": {"base": 500.0, "dims": 16},
                "scale": 0.25}},
-    {"type": "attention", "mlp": None, "mixer": dict(_TINY_CHUNK, kv_from=0, mask={"size": 20}, scale=0.2)},
-    {"type": "attention", "mlp": _TINY_CMOE, "mixer": dict(_TINY_CHUNK, kv_from=0)},
+    {"type": "attention", "mlp": None,
+     "mixer": {"heads": 4, "kv_heads": 2, "dim": 16, "vdim": 16, "kv_from": 2, "mask": {"size": 33},
+               "rot": {"base": 500.0, "dims": 16}, "scale": 0.3}},
   ]}
 PRESETS["tiny-torinex"] = _torinex_config(TINY_TORINEX)
 # aliases of the reference's model cards that share an architecture

@@ -156,6 +156,11 @@ def _as_tensor(x) -> torch.Tensor:
   return x.detach() if isinstance(x, torch.Tensor) else torch.from_numpy(np.ascontiguousarray(np.asarray(x)))
 
 
+def _hidden_dtype(engine) -> torch.dtype:
+  """dtype of the hidden states between the ranks: what the engine's runner carries (mixed-layer models an fp32 stream)."""
+  return getattr(getattr(engine, "runner", None), "hidden_dtype", torch.bfloat16)
+
+
 # ------------------------------------------------------------------ one rank's part of a training step
 def _tied_shape(tr) -> Optional[list]:
   """[V, D] when the box holds both ends of a tied-embedding model (rank 0's embed, the last rank's head copy)."""
@@ -421,7 +426,7 @@ class RingFederatedEngine(InferenceEngine):
       # KV page operations every rank must mirror: those of rank 0's own first-layer cache, or the upstream's
       ops.append((st or {}).get("pc") if subs[0].is_first_layer() else st_in.get("pc"))
     payload = {"rids": [it[0] for it, _ in good], "qlens": qlens, "subs": [s.to_dict() for s in subs], "pc": ops}
-    x = torch.cat(rows).to(self.device, torch.bfloat16)
+    x = torch.cat(rows).to(self.device, _hidden_dtype(self.local))
     self.stats["batches"] += 1
     self.stats["requests"] += len(good)
     loop = asyncio.get_running_loop()
@@ -618,7 +623,7 @@ async def _follow_infer(local, wire: Wire, rank: int, subs: List[Shard], p: dict
       if sub.is_last_layer():
         y = torch.cat([_as_tensor(o[0]).reshape(1, -1).to(device, torch.float32) for o in outs])
       else:
-        y = torch.cat([_as_tensor(o[0]).reshape(-1, x.shape[-1]) for o in outs]).to(device, torch.bfloat16)
+        y = torch.cat([_as_tensor(o[0]).reshape(-1, x.shape[-1]) for o in outs]).to(device, _hidden_dtype(local))
     except Exception as e:  # noqa: BLE001 - the error word travels on to rank 0
       err = _err(rank, e)
   await on_io(wire.put, None if err else y, nxt, err)
