@@ -241,7 +241,7 @@ def bench_mixers(args, sizes=None, kinds=("tarepel", "llama"), configs=mixer_con
                  what="Tarepel-design layers beside a Llama-style stack of equal size"):
   """Prefill and decode throughput of mixed-layer designs at sizes like a real model's (random weights), beside
   the closest existing model (--mixers: Tarepel beside a Llama-style stack of equal width, depth, heads and
-  feed-forward; --hybrid: Mogelix beside Tarepel) on the same runner: one prefill step of --mixer-batch prompts of
+  feed-forward; --hybrid, --latent, --memory, --chunked: see their *_configs) on the same runner: one prefill step of --mixer-batch prompts of
   --prompt-len tokens, then HIP-graph decode steps at that context.  One JSON line; not the headline metric."""
   from xotorch_support_jetson_amd.inference.shard import Shard
   from xotorch_support_jetson_amd.runtime.runner import ShardRunner
