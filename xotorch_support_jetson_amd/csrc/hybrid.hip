@@ -23,7 +23,7 @@ namespace xot {
 // csrc/window_attention.hip
 bool window_attention(const at::Tensor& q, const at::Tensor& k_cache, const at::Tensor& v_cache, const at::Tensor& block_tables,
                       const at::Tensor& cu_q, const at::Tensor& ctx_lens, const float* sink, double scale, int64_t window,
-                      int64_t chunk, at::Tensor& out, int64_t ldo, int64_t max_qlen);
+                      int64_t chunk, int64_t keep, double softcap, at::Tensor& out, int64_t ldo, int64_t max_qlen);
 
 namespace {
 using namespace mix;
@@ -329,7 +329,8 @@ __global__ void kv_pool_update_k(const AT* __restrict__ k_cache, const AT* __res
 // A query at position i sees the tokens j with 0 <= i - j < window (window 0: all j <= i) and the pooled blocks b with
 // b pool + pool - 1 <= i - window; the softmax's denominator also holds exp(sink[head]).
 //
-// chunk > 0: only tokens of the query's own block of `chunk` positions are seen.
+// chunk > 0: only tokens of the query's own block of `chunk` positions are seen.  The sequence's first `keep` tokens are seen
+// wherever the query is.  softcap > 0: scores are softcap * tanh(score / softcap).
 //
 // Workgroup per (token, REP query heads of one kv head) (any d, dv <= 256, bf16 or fp32), WATT_WAVES waves: the key
 // tiles are dealt to the waves in turn; a lane loads a key row once and scores it against the REP heads, and a V^T run
@@ -348,7 +349,7 @@ __global__ __launch_bounds__(64 * WATT_WAVES) void attn_window_pool_k(
     const AT* __restrict__ q, const AT* __restrict__ k_cache, const AT* __restrict__ v_cache, const AT* __restrict__ kp,
     const AT* __restrict__ vp, const int* __restrict__ block_tables, int width, const int* __restrict__ cu_q,
     const int* __restrict__ ctx_lens, int B, const float* __restrict__ sink, float scale, int window, int pool, int per,
-    OT* __restrict__ out, int ldo, int H, int G, int d, int dv, int Gv, int chunk) {
+    OT* __restrict__ out, int ldo, int H, int G, int d, int dv, int Gv, int chunk, int keep, float softcap) {
   constexpr int TILE = REP >= 8 ? 128 : 256;
   extern __shared__ float sm[];
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
@@ -397,6 +398,10 @@ __global__ __launch_bounds__(64 * WATT_WAVES) void attn_window_pool_k(
     }
 #pragma unroll
     for (int r = 0; r < REP; ++r) s[r] *= scale;
+    if (softcap > 0.0f) {
+#pragma unroll
+      for (int r = 0; r < REP; ++r) s[r] = softcap * tanhf(s[r] / softcap);
+    }
   };
   // one tile of this wave: scores of the keys a0 + [0, n) (those outside [p0, p1) weigh nothing) -> softmax weights in
   // ws, the running maxima / denominators / accumulators rescaled.  ws is the wave's own: its lanes' LDS accesses
@@ -464,32 +469,36 @@ __global__ __launch_bounds__(64 * WATT_WAVES) void attn_window_pool_k(
       }
     }
   }
-  // tokens [lo, pos], tiles aligned to 8 keys
-  for (int a0 = lo & ~7; a0 <= pos; a0 += TILE, ++tile) {
-    if (tile % WATT_WAVES != wave) continue;
-    const int a1 = min(a0 + TILE, (pos + 8) & ~7);
-    weigh(a0, a1 - a0, lo, pos + 1, [&](int p) {
-      return k_cache + (((int64_t)bt[p / PAGE_TOK] * G + g) * PAGE_TOK + (p % PAGE_TOK)) * d;
-    });
-    for (int p = a0; p < a1; p += 8) {  // 8 keys of one page per step
-      const AT* vq = v_cache + ((int64_t)bt[p / PAGE_TOK] * Gv + gv) * dv * PAGE_TOK + (p % PAGE_TOK);
+  // tokens [p0, p1), tiles aligned to 8 keys
+  auto tokens = [&](int p0, int p1) {
+    for (int a0 = p0 & ~7; a0 < p1; a0 += TILE, ++tile) {
+      if (tile % WATT_WAVES != wave) continue;
+      const int a1 = min(a0 + TILE, (p1 + 7) & ~7);
+      weigh(a0, a1 - a0, p0, p1, [&](int p) {
+        return k_cache + (((int64_t)bt[p / PAGE_TOK] * G + g) * PAGE_TOK + (p % PAGE_TOK)) * d;
+      });
+      for (int p = a0; p < a1; p += 8) {  // 8 keys of one page per step
+        const AT* vq = v_cache + ((int64_t)bt[p / PAGE_TOK] * Gv + gv) * dv * PAGE_TOK + (p % PAGE_TOK);
 #pragma unroll
-      for (int c = 0; c < 4; ++c) {
-        const int i = lane + 64 * c;
-        if (i < dv) {
-          float vv[8];
-          ld8(vq + (int64_t)i * PAGE_TOK, vv);
+        for (int c = 0; c < 4; ++c) {
+          const int i = lane + 64 * c;
+          if (i < dv) {
+            float vv[8];
+            ld8(vq + (int64_t)i * PAGE_TOK, vv);
 #pragma unroll
-          for (int r = 0; r < REP; ++r)
+            for (int r = 0; r < REP; ++r)
 #pragma unroll
-            for (int e = 0; e < 8; ++e) {
-              const float w = ws[r * TILE + p - a0 + e];
-              acc[r][c] += w != 0.0f ? w * vv[e] : 0.0f;  // (a slot no token has written yet may hold anything)
-            }
+              for (int e = 0; e < 8; ++e) {
+                const float w = ws[r * TILE + p - a0 + e];
+                acc[r][c] += w != 0.0f ? w * vv[e] : 0.0f;  // (a slot no token has written yet may hold anything)
+              }
+          }
         }
       }
     }
-  }
+  };
+  if (keep > 0 && lo > 0) tokens(0, min(keep, lo));  // kept first tokens before the window
+  tokens(lo, pos + 1);
   // merge the waves: M = max m_w, out = sum_w acc_w e^(m_w - M) / sum_w l_w e^(m_w - M)
   const int ms = 2 + dv;
 #pragma unroll
@@ -538,7 +547,8 @@ __global__ __launch_bounds__(256) void attn_window_pool_mfma_k(
     const uint16_t* __restrict__ q, const uint16_t* __restrict__ k_cache, const uint16_t* __restrict__ v_cache,
     const uint16_t* __restrict__ kp, const uint16_t* __restrict__ vp, const int* __restrict__ block_tables, int width,
     const int* __restrict__ cu_q, const int* __restrict__ ctx_lens, const float* __restrict__ sink, float scale, int window,
-    int pool, int per, OT* __restrict__ out, int ldo, int H, int G, int Gv, int chunk, int d_rt, int dv_rt) {
+    int pool, int per, OT* __restrict__ out, int ldo, int H, int G, int Gv, int chunk, int d_rt, int dv_rt, int keep,
+    float softcap) {
   // key size D = 32 NK, value size DV = 32 NV (pooled blocks: NK == NV, not RAG); G / Gv neighbouring key heads share a value head
   constexpr int D = NK * 32, DV = NV * 32, ND = NV * 2, QT = 2;
   constexpr int KT = (D > 192 || DV > 192) ? 32 : 64;  // keys per tile (a page holds a whole number of tiles)
@@ -581,6 +591,7 @@ __global__ __launch_bounds__(256) void attn_window_pool_mfma_k(
 #pragma unroll
     for (int db = 0; db < ND; ++db) o[qt][db] = f32x4{0.f, 0.f, 0.f, 0.f};
   const float sc2 = scale * L2E;
+  const float cap_l2 = softcap * L2E, inv_cap2 = softcap > 0.0f ? 2.0f / softcap : 0.0f;
   const int* bt = block_tables + (int64_t)b * width;
   const int wlast = ctx - qlen + wq0 + min(128, qlen - wq0) - 1;  // the workgroup's last query
   const int wpos0 = ctx - qlen + wq0;
@@ -601,7 +612,7 @@ __global__ __launch_bounds__(256) void attn_window_pool_mfma_k(
         if (!active || kb >= blocks_seen(last)) continue;  // (wave-uniform) none of these blocks is seen by this wave
         full = kb + 32 <= blocks_seen(pos0);
       } else {
-        if (!active || kb > last || kb + 31 < k_first) continue;
+        if (!active || kb > last || (kb + 31 < k_first && kb >= keep)) continue;
         full = kb + 31 <= pos0 && kb >= k_last;
       }
       f32x4 s[2][QT];
@@ -626,9 +637,10 @@ __global__ __launch_bounds__(256) void attn_window_pool_mfma_k(
 #pragma unroll
           for (int r = 0; r < 4; ++r) {
             float t = s[kt][qt][r] * sc2;
+            if (softcap > 0.0f) t = capped_l2(t, inv_cap2, cap_l2);
             if (!full) {
               const int kpos = kb + kt * 16 + 4 * g4 + r;
-              const bool vis = pooled ? kpos < qnb[qt] : (kpos <= qpos[qt] && kpos >= qlo[qt]);
+              const bool vis = pooled ? kpos < qnb[qt] : (kpos <= qpos[qt] && (kpos >= qlo[qt] || kpos < keep));
               t = vis ? t : -INFINITY;
             }
             s[kt][qt][r] = t;
@@ -709,8 +721,12 @@ __global__ __launch_bounds__(256) void attn_window_pool_mfma_k(
       rv[j] = !RAG || vrow < dv ? ld16(v_cache + (pgv * dv + vrow) * PAGE_TOK + koff + vc * 8) : s16x8{0, 0, 0, 0, 0, 0, 0, 0};
     }
   };
-  fetch(t_lo);
-  for (int tb = t_lo; tb <= wlast; tb += KT) {
+  // tiles of kept first tokens before the window, then the tiles from t_lo on
+  const int nkt = (min(keep, t_lo) + KT - 1) / KT, ntile = nkt + (wlast - t_lo) / KT + 1;
+  auto tile_at = [&](int i) { return i < nkt ? i * KT : t_lo + (i - nkt) * KT; };
+  fetch(tile_at(0));
+  for (int it = 0; it < ntile; ++it) {
+    const int tb = tile_at(it);
     __syncthreads();  // the previous tile has been consumed
 #pragma unroll
     for (int j = 0; j < NCH; ++j) {
@@ -727,7 +743,7 @@ __global__ __launch_bounds__(256) void attn_window_pool_mfma_k(
       st16(&sV[vrow][vc * 8], rv[j]);
     }
     __syncthreads();
-    if (tb + KT <= wlast) fetch(tb + KT);  // in flight while this tile is consumed
+    if (it + 1 < ntile) fetch(tile_at(it + 1));  // in flight while this tile is consumed
     consume(tb, false);
   }
 #pragma unroll
@@ -1129,12 +1145,12 @@ template <int NK, int NV, typename OT, bool RAG>
 void launch_wattn_mfma(dim3 grid, const at::Tensor& q, const at::Tensor& k_cache, const at::Tensor& v_cache, const uint16_t* kp,
                        const uint16_t* vp, const at::Tensor& block_tables, const at::Tensor& cu_q, const at::Tensor& ctx_lens,
                        const float* sink, float scale, int window, int pool, int per, at::Tensor& out, int ldo, int H, int G,
-                       int chunk) {
+                       int chunk, int keep, float softcap) {
   attn_window_pool_mfma_k<NK, NV, OT, RAG><<<grid, 256, 0, stream()>>>(
       (const uint16_t*)q.data_ptr(), (const uint16_t*)k_cache.data_ptr(), (const uint16_t*)v_cache.data_ptr(), kp, vp,
       block_tables.data_ptr<int>(), (int)block_tables.size(1), cu_q.data_ptr<int>(), ctx_lens.data_ptr<int>(), sink, scale,
       window, pool, per, (OT*)out.data_ptr(), ldo, H, G, (int)v_cache.size(1), chunk, (int)k_cache.size(3),
-      (int)v_cache.size(2));
+      (int)v_cache.size(2), keep, softcap);
 }
 
 // max_qlen: the longest run of new tokens of one sequence in this step (below 16: single decoded tokens and short
@@ -1142,7 +1158,8 @@ void launch_wattn_mfma(dim3 grid, const at::Tensor& q, const at::Tensor& k_cache
 void attn_window_pool(const at::Tensor& q, const at::Tensor& k_cache, const at::Tensor& v_cache,
                       const c10::optional<at::Tensor>& kp, const c10::optional<at::Tensor>& vp, const at::Tensor& block_tables,
                       const at::Tensor& cu_q, const at::Tensor& ctx_lens, const c10::optional<at::Tensor>& sink, double scale,
-                      int64_t window, int64_t pool, at::Tensor& out, int64_t max_qlen, int64_t chunk) {
+                      int64_t window, int64_t pool, at::Tensor& out, int64_t max_qlen, int64_t chunk, int64_t keep,
+                      double softcap) {
   MCHECK(q.is_cuda() && is_act(q) && q.is_contiguous() && q.dim() == 3, "q must be contiguous [T, H, d]");
   const int64_t T = q.size(0), H = q.size(1), d = q.size(2), B = ctx_lens.numel();
   if (T == 0 || B == 0) return;
@@ -1151,6 +1168,7 @@ void attn_window_pool(const at::Tensor& q, const at::Tensor& k_cache, const at::
   check_kv(k_cache, v_cache, q.scalar_type(), G, d, dv);
   MCHECK(G > 0 && H % G == 0 && d <= 256 && dv <= 256, "head counts / sizes (at most 256)");
   MCHECK(window >= 0 && pool >= 0 && chunk >= 0 && (pool == 0 || chunk == 0), "window / pool / chunk must not be negative (and no pool beside a chunk)");
+  MCHECK(keep >= 0 && softcap >= 0 && (keep == 0 || pool == 0), "kept tokens / softcap must not be negative (and no pool beside kept tokens)");
   int per = 0;
   const bool pooled = pool > 0 && window > 0;
   if (pooled) {
@@ -1173,7 +1191,8 @@ void attn_window_pool(const at::Tensor& q, const at::Tensor& k_cache, const at::
   const int ldo = act_ld(out, T, H * dv, "out");
   const bool o32 = out.scalar_type() == at::kFloat;
   if (q.scalar_type() == at::kBFloat16 && !pooled && WATT_MFMA &&
-      window_attention(q, k_cache, v_cache, block_tables, cu_q, ctx_lens, sp, scale, window, chunk, out, ldo, max_qlen))
+      window_attention(q, k_cache, v_cache, block_tables, cu_q, ctx_lens, sp, scale, window, chunk, keep, softcap, out, ldo,
+                       max_qlen))
     return;
   // the MFMA kernel: bf16 caches, runs of 16 tokens or more, value size = key size in {32, 64, 96, 128} (bf16 or fp32 output)
   // or twice the key size in {32, 64} with fp32 output (differential attention's maps), or (bf16 output, no pooled blocks)
@@ -1189,7 +1208,7 @@ void attn_window_pool(const at::Tensor& q, const at::Tensor& k_cache, const at::
     const int64_t big = (std::max(d, dv) + 31) / 32;
 #define WATT_MFMA_GO(NK, NV, OT, ...)                                                                                       \
   launch_wattn_mfma<NK, NV, OT, ##__VA_ARGS__>(grid, q, k_cache, v_cache, kpp, vpp, block_tables, cu_q, ctx_lens, sp, (float)scale,       \
-                                (int)window, pl, per, out, ldo, (int)H, (int)G, (int)chunk)
+                                (int)window, pl, per, out, ldo, (int)H, (int)G, (int)chunk, (int)keep, (float)softcap)
     if (ragged && big == 1) WATT_MFMA_GO(1, 1, uint16_t, true);
     else if (ragged && big == 2) WATT_MFMA_GO(2, 2, uint16_t, true);
     else if (ragged && big == 3) WATT_MFMA_GO(3, 3, uint16_t, true);
@@ -1222,7 +1241,7 @@ void attn_window_pool(const at::Tensor& q, const at::Tensor& k_cache, const at::
       pooled ? (const AT*)kp->data_ptr() : nullptr, pooled ? (const AT*)vp->data_ptr() : nullptr,                          \
       block_tables.data_ptr<int>(), (int)block_tables.size(1), cu_q.data_ptr<int>(), ctx_lens.data_ptr<int>(), (int)B, sp, \
       (float)scale, (int)window, pooled ? (int)pool : 0, per, (OT*)out.data_ptr(), ldo, (int)H, (int)G, (int)d, (int)dv,  \
-      (int)Gv, (int)chunk)
+      (int)Gv, (int)chunk, (int)keep, (float)softcap)
 #define WATT_REP(AT, OT)                   \
   switch (rep) {                           \
     case 8: WATT_GO(AT, OT, 8); break;     \
@@ -1284,14 +1303,14 @@ void ssd_prep(const at::Tensor& P, int64_t x_off, int64_t dt_off, const at::Tens
 void ssd_gate_norm(const at::Tensor& o, const at::Tensor& xbc, const at::Tensor& skip_d, const at::Tensor& P, int64_t z_off,
                    const at::Tensor& w, int64_t groups, double eps, at::Tensor& out) {
   f32c(o, "o");
-  f32c(xbc, "xbc");
   f32c(skip_d, "skip_d");
   f32c(w, "w");
   const int ldp = ld_of(P, "P");
-  MCHECK(o.dim() == 2 && xbc.dim() == 2, "o [T, inner], xbc [T, C]");
-  const int64_t T = o.size(0), inner = o.size(1), C = xbc.size(1), H = skip_d.numel();
+  const int64_t C = ld_of(xbc, "xbc");  // (the row stride: xbc may be the last columns of wider rows)
+  MCHECK(o.dim() == 2, "o must be [T, inner]");
+  const int64_t T = o.size(0), inner = o.size(1), H = skip_d.numel();
   if (T == 0) return;
-  MCHECK(P.size(0) == T && xbc.size(0) == T && C >= inner && H > 0 && inner % H == 0 && w.numel() == inner && groups >= 1 &&
+  MCHECK(P.size(0) == T && xbc.size(0) == T && xbc.size(1) >= inner && H > 0 && inner % H == 0 && w.numel() == inner && groups >= 1 &&
              inner % groups == 0,
          "ssd_gate_norm: shape mismatch");
   cols_ok(P, z_off, inner, "gate");

@@ -55,20 +55,20 @@ __global__ __launch_bounds__(256) void sandwich_add_norm_k(float* __restrict__ x
                                                            const float* __restrict__ wb, const float* __restrict__ bb,
                                                            const float* __restrict__ wn, const float* __restrict__ bn,
                                                            const float* __restrict__ yb, float mult, float eps,
-                                                           AT* __restrict__ out, int ldo, int D, int S, int64_t ss) {
+                                                           AT* __restrict__ out, int ldo, int D, int S, int64_t ss, int layer) {
   __shared__ float red[8];
   const int64_t t = blockIdx.x;
   float* xr = x + t * D;
   if (y) {
     const float* yr = y + t * ldy;
     float mu, r;
-    row_norm_stats(yr, S, ss, yb, D, bb != nullptr, eps, red, &mu, &r);
+    row_norm_stats(yr, S, ss, yb, D, layer || bb, eps, red, &mu, &r);
     for (int i = threadIdx.x; i < D; i += blockDim.x) 
       xr[i] += mult * ((slab1(yr + i, S, ss) + (yb ? yb[i] : 0.0f) - mu) * r * wb[i] + (bb ? bb[i] : 0.0f));
   }
   if (wn) {  // (a thread re-reads the elements it wrote itself)
     float mu, r;
-    row_norm_stats(xr, 1, 0, nullptr, D, bn != nullptr, eps, red, &mu, &r);
+    row_norm_stats(xr, 1, 0, nullptr, D, layer || bn, eps, red, &mu, &r);
     for (int i = threadIdx.x; i < D; i += blockDim.x) stf(out + t * ldo + i, (xr[i] - mu) * r * wn[i] + (bn ? bn[i] : 0.0f));
   } else if (out) {
     for (int i = threadIdx.x; i < D; i += blockDim.x) stf(out + t * ldo + i, xr[i]);
@@ -574,7 +574,8 @@ __global__ __launch_bounds__(256) void sandwich_add_norm_reg_k(float* __restrict
                                                                const float* __restrict__ wb, const float* __restrict__ bb,
                                                                const float* __restrict__ wn, const float* __restrict__ bn,
                                                                const float* __restrict__ yb, float mult, float eps,
-                                                               AT* __restrict__ out, int ldo, int D, int S, int64_t ss_) {
+                                                               AT* __restrict__ out, int ldo, int D, int S, int64_t ss_,
+                                                               int layer) {
   __shared__ float red[8];
   const int64_t t = blockIdx.x;
   float* xr = x + t * D;
@@ -622,7 +623,7 @@ __global__ __launch_bounds__(256) void sandwich_add_norm_reg_k(float* __restrict
       }
     }
     float mu, rs;
-    stats(yv, bb != nullptr, &mu, &rs);
+    stats(yv, layer || bb, &mu, &rs);
 #pragma unroll
     for (int r = 0; r < R; ++r) {
       const int i = 4 * (threadIdx.x + 256 * r);
@@ -636,7 +637,7 @@ __global__ __launch_bounds__(256) void sandwich_add_norm_reg_k(float* __restrict
   }
   if (wn) {
     float mu, rs;
-    stats(xv, bn != nullptr, &mu, &rs);
+    stats(xv, layer || bn, &mu, &rs);
 #pragma unroll
     for (int r = 0; r < R; ++r) {
       const int i = 4 * (threadIdx.x + 256 * r);
@@ -662,7 +663,7 @@ const bool LATT_MFMA = []() { const char* e = getenv("XOT_LATT_MFMA"); return !(
 void sandwich_add_norm(at::Tensor& x, const c10::optional<at::Tensor>& y, const c10::optional<at::Tensor>& wb,
                        const c10::optional<at::Tensor>& wn, double eps, const c10::optional<at::Tensor>& out,
                        const c10::optional<at::Tensor>& bb, const c10::optional<at::Tensor>& bn, double mult,
-                       const c10::optional<at::Tensor>& yb) {
+                       const c10::optional<at::Tensor>& yb, bool layer) {
   f32c(x, "x");
   MCHECK(x.dim() == 2, "x must be [T, D]");
   const int64_t T = x.size(0), D = x.size(1);
@@ -716,7 +717,7 @@ void sandwich_add_norm(at::Tensor& x, const c10::optional<at::Tensor>& y, const 
   for (const float* p : {(const float*)x.data_ptr<float>(), bp, np, bbp, bnp, ybp, (const float*)op}) al(p);
 #define SAN_GO(KERNEL, AT)                                                                                              \
   KERNEL<<<T, 256, 0, stream()>>>(x.data_ptr<float>(), yp, ldy, bp, bbp, np, bnp, ybp, (float)mult, (float)eps, (AT*)op, ldo, \
-                                  (int)D, S, ss)
+                                  (int)D, S, ss, (int)layer)
 #define SAN_PICK(AT)                                                     \
   if (vec && D <= 1024) SAN_GO((sandwich_add_norm_reg_k<AT, 1>), AT);      \
   else if (vec && D <= 2048) SAN_GO((sandwich_add_norm_reg_k<AT, 2>), AT); \

@@ -19,6 +19,12 @@ __device__ __forceinline__ float siluf_(float x) { return x / (1.0f + expf(-x));
 __device__ __forceinline__ float softplusf_(float x) { return log1pf(expf(-fabsf(x))) + fmaxf(x, 0.0f); }
 __device__ __forceinline__ float logsigmoidf_(float x) { return fminf(x, 0.0f) - log1pf(expf(-fabsf(x))); }
 
+// a score s scaled by log2 e -> cap tanh(s / cap) scaled likewise (inv_cap2 = 2 / cap, cap_l2 = cap log2 e), with the base-2
+// exponential and the reciprocal of the hardware: tanh(x) = 1 - 2 / (e^2x + 1)
+__device__ __forceinline__ float capped_l2(float s_l2, float inv_cap2, float cap_l2) {
+  return cap_l2 - 2.0f * cap_l2 * __builtin_amdgcn_rcpf(__builtin_amdgcn_exp2f(s_l2 * inv_cap2) + 1.0f);
+}
+
 // sum over the workgroup; red: at least (threads / 64) floats of LDS
 __device__ __forceinline__ float block_sum(float v, float* red) {
   v = wave_sum(v);

@@ -588,7 +588,9 @@ __global__ void gla_prep_k(const float* __restrict__ P, int ldp, int a1_off, int
 // (a decay per key channel).   MODE 2: S = g S + k v^T; o = S^T q (one decay per head: the state-space-duality form
 // with k = B, q = C, v = dt x).   MODE 3: MODE 2 with an input scale b per head and token and a normaliser: the state has
 // one value channel more than v (dvin + 1), fed with ones, S = g S + k (b [v | 1])^T, so the last channel is n = g n + b k
-// and the last output n . q (the stabilised matrix memory of xLSTM, g and b computed by its gate kernel).
+// and the last output n . q (the stabilised matrix memory of xLSTM, g and b computed by its gate kernel).   MODE 4: the delta
+// rule with a decay per key channel, S = diag(a) S, then as MODE 1.   MODE 5: MODE 2 with an input scale per head and token,
+// S = g S + k (b v)^T (SSD with v = x, b = dt).
 template <int CTRL>
 __device__ __forceinline__ float dpp_add(float v) {
   const int m = __builtin_amdgcn_update_dpp(0, __float_as_int(v), CTRL, 0xf, 0xf, false);
@@ -612,7 +614,8 @@ __global__ __launch_bounds__(256) void linear_recurrence_k(
     const int* __restrict__ state_slots, const int* __restrict__ cu_q, int H, int G, int d, int dv, int dvin, int dstride,
     float* __restrict__ out) {
   constexpr int DP = KR * RS;  // padded key dim
-  constexpr bool DELTA = MODE == 1, SCALAR = MODE != 0, NORMCH = MODE == 3;
+  constexpr bool DELTA = MODE == 1 || MODE == 4, SCALAR = MODE != 0 && MODE != 4, NORMCH = MODE == 3;
+  constexpr bool INSCALE = MODE == 3 || MODE == 5, BETA = DELTA || INSCALE;
   constexpr int COLS = 256 / RS;
   constexpr int TB = DP >= 256 ? 8 : 16;
   constexpr int NQ = TB * DP / 256, NV = (TB * COLS + 255) / 256;
@@ -661,9 +664,9 @@ __global__ __launch_bounds__(256) void linear_recurrence_k(
       pv[j] = (e < TB * COLS && c < dvin && tb + tt < n) ? v[(int64_t)(t0 + tb + tt) * ldv + h * dvin + c] : 0.0f;
       if (NORMCH && e < TB * COLS && c == dvin && tb + tt < n) pv[j] = 1.0f;
     }
-    if (SCALAR && tid < TB && tb + tid < n) {
-      pg0 = decay[(int64_t)(t0 + tb + tid) * dstride + h];  // (dstride 0: one fixed decay per head, decay [H])
-      if (DELTA || NORMCH) pg1 = beta[(int64_t)(t0 + tb + tid) * H + h];
+    if (tid < TB && tb + tid < n) {
+      if (SCALAR) pg0 = decay[(int64_t)(t0 + tb + tid) * dstride + h];  // (dstride 0: one fixed decay per head, decay [H])
+      if (BETA) pg1 = beta[(int64_t)(t0 + tb + tid) * H + h];
     }
   };
   auto stage = [&](int buf) {  // registers -> LDS
@@ -679,7 +682,7 @@ __global__ __launch_bounds__(256) void linear_recurrence_k(
       const int e = tid + 256 * j;
       if (e < TB * COLS) sv[buf][e / COLS][e % COLS] = pv[j];
     }
-    if (SCALAR && tid < TB) {
+    if ((SCALAR || BETA) && tid < TB) {
       sg[buf][tid][0] = pg0;
       sg[buf][tid][1] = pg1;
     }
@@ -694,7 +697,7 @@ __global__ __launch_bounds__(256) void linear_recurrence_k(
     if (more) fetch(tb + TB);
 #pragma unroll 2
     for (int tt = 0; tt < nt; ++tt) {
-      const float vc = NORMCH ? sv[buf][tt][cl] * sg[buf][tt][1] : sv[buf][tt][cl];
+      const float vc = INSCALE ? sv[buf][tt][cl] * sg[buf][tt][1] : sv[buf][tt][cl];
       float kk[KR], qq[KR];
 #pragma unroll
       for (int m = 0; m < KR; ++m) {
@@ -707,7 +710,7 @@ __global__ __launch_bounds__(256) void linear_recurrence_k(
         float d0 = 0.0f, d1 = 0.0f, d2 = 0.0f, d3 = 0.0f;
 #pragma unroll
         for (int m = 0; m < KR; ++m) {
-          s[m] *= g;
+          s[m] *= SCALAR ? g : sa[buf][tt][rg * KR + m];
           const float p = s[m] * kk[m];
           if ((m & 3) == 0) d0 += p; else if ((m & 3) == 1) d1 += p; else if ((m & 3) == 2) d2 += p; else d3 += p;
         }
@@ -1069,12 +1072,12 @@ void launch_rec(int KR, dim3 grid, const float* q, int ldq, const float* k, int 
 
 // q / k [T, G d], v [T, H dv]: fp32 rows of unit inner stride (column slices allowed).  decay [T, H] (delta rule, or
 // without beta: one decay per head and a plain outer-product write; a 1-D [H]: the same decay at every token) or [T, H d]
-// (per key channel); beta [T, H] (delta
-// only; an input scale for a state with a normaliser channel: then v is [T, H (dv - 1)]).  state [slots, H, dv, d] (S^T: key
+// (per key channel; with beta: the delta rule on such a decay); beta [T, H] (delta
+// only; with `plain`, or for a state with a normaliser channel, an input scale; in the latter case v is [T, H (dv - 1)]).  state [slots, H, dv, d] (S^T: key
 // rows contiguous).
 void linear_recurrence(const at::Tensor& q, const at::Tensor& k, const at::Tensor& v, const at::Tensor& decay,
                        const c10::optional<at::Tensor>& beta, double q_scale, at::Tensor& state, const at::Tensor& state_slots,
-                       const at::Tensor& cu_q, at::Tensor& out) {
+                       const at::Tensor& cu_q, at::Tensor& out, bool plain) {
   const int ldq = ld_of(q, "q"), ldk = ld_of(k, "k"), ldv = ld_of(v, "v");
   f32c(decay, "decay");
   f32c(state, "state");
@@ -1092,16 +1095,17 @@ void linear_recurrence(const at::Tensor& q, const at::Tensor& k, const at::Tenso
          "linear_recurrence: shape mismatch");
   MCHECK(cu_q.numel() == B + 1, "cu_q must hold B + 1 offsets");
   MCHECK(!normch || beta.has_value(), "a state with a normaliser channel needs the input scales");
-  const bool delta = beta.has_value() && !normch;
+  const bool delta = beta.has_value() && !normch && !plain, inscale = beta.has_value() && !normch && plain;
+  const bool chan = delta && d > 1 && decay.numel() == T * H * d;  // a decay per key channel under the delta rule
   if (beta.has_value()) {
     f32c(*beta, "beta");
-    MCHECK(beta->numel() == T * H && decay.numel() == T * H, "delta rule: beta / decay must be [T, H]");
+    MCHECK(beta->numel() == T * H && (chan || decay.numel() == T * H), "beta must be [T, H], the decay [T, H] (delta rule: or [T, H d])");
   } else if (decay.numel() != T * H && !(decay.dim() == 1 && decay.numel() == H)) {
     MCHECK(decay.numel() == T * H * d && G == H, "per-channel decay must be [T, H d] with one q / k head per value head");
   }
   // one decay per head (and token: [T, H]; or fixed: a 1-D [H]), q / k shared by H / G heads
-  const bool fixed = !delta && !normch && decay.dim() == 1 && decay.numel() == H;
-  const bool scalar = !delta && !normch && (fixed || decay.numel() == T * H);
+  const bool fixed = !beta.has_value() && decay.dim() == 1 && decay.numel() == H;
+  const bool scalar = !beta.has_value() && (fixed || decay.numel() == T * H);
   int DP = 16;
   while (DP < d) DP *= 2;
   MCHECK(DP <= 256, "linear_recurrence: key dim above 256");
@@ -1116,7 +1120,7 @@ void linear_recurrence(const at::Tensor& q, const at::Tensor& k, const at::Tenso
                    decay.data_ptr<float>(), bp, (float)q_scale, state.data_ptr<float>(), state_slots.data_ptr<int>(),        \
                    cu_q.data_ptr<int>(), (int)H, (int)G, (int)d, (int)dv, (int)dvin, fixed ? 0 : (int)H,         \
                    out.data_ptr<float>())
-  if (delta) REC_GO(16, 1); else if (normch) REC_GO(16, 3); else if (scalar) REC_GO(16, 2); else REC_GO(16, 0);
+  if (chan) REC_GO(16, 4); else if (inscale) REC_GO(16, 5); else if (delta) REC_GO(16, 1); else if (normch) REC_GO(16, 3); else if (scalar) REC_GO(16, 2); else REC_GO(16, 0);
 #undef REC_GO
 }
 

@@ -25,6 +25,9 @@ __device__ __forceinline__ int first_seen(int pos, int window, int chunk) {
   return chunk > 0 ? max(lo, pos - pos % chunk) : lo;
 }
 
+// key `key` is seen by the query at `pos` whose window / chunk starts at lo; the first `keep` tokens stay visible
+__device__ __forceinline__ bool seen(int key, int pos, int lo, int keep) { return key <= pos && (key >= lo || key < keep); }
+
 // two probabilities in one dword of bf16
 __device__ __forceinline__ uint32_t pack2(float a, float b) {
   typedef __bf16 bf16x2_w __attribute__((ext_vector_type(2)));
@@ -45,12 +48,12 @@ __device__ __forceinline__ int k_swz(int r) {
 // 8 waves, two 16-row blocks each.  Pages arrive by LDS-DMA in a three-deep ring (two in flight), swizzled through the
 // per-lane source addresses.  Waves skip pages none of their rows sees; the latest rows' workgroups start first, those of
 // one (sequence, kv head) on one XCD.
-template <int DK, int DV, typename OT>
+template <int DK, int DV, typename OT, bool CAP>
 __global__ __launch_bounds__(512, 1) void window_prefill_k(
     const uint16_t* __restrict__ q, const uint16_t* __restrict__ kc, const uint16_t* __restrict__ vc,
     const int* __restrict__ block_tables, int width, const int* __restrict__ cu_q, const int* __restrict__ ctx_lens,
     const float* __restrict__ sink, float scale_l2, int window, int chunk, OT* __restrict__ out, int ldo, int H, int G, int Gv,
-    int num_pages) {
+    int num_pages, int keep, float inv_cap2, float cap_l2) {
   constexpr int KS = DK / 32, NDT = DV / 16;
   constexpr int KGPR = DK / 8;                                     // 16-byte granules of a K row
   constexpr int KEL = PAGE_TOK * DK, VEL = PAGE_TOK * DV;          // elements of a page's images
@@ -100,6 +103,9 @@ __global__ __launch_bounds__(512, 1) void window_prefill_k(
   const int last_row = min(nrows, row0 + 256) - 1;
   const int p_first = first_seen(pos0 + row0 / rep, window, chunk) / PAGE_TOK;
   const int p_end = (pos0 + last_row / rep) / PAGE_TOK + 1;
+  // pages in order: those of kept first tokens before the window, then p_first on
+  const int nkp = min((keep + PAGE_TOK - 1) / PAGE_TOK, p_first), nit = nkp + p_end - p_first;
+  auto page_at = [&](int i) { return i < nkp ? i : p_first + i - nkp; };
   // the wave's rows: the last key any of them sees, the first row's position, the first key of the first / last row
   const int wr0 = row0 + 32 * wave, wr1 = min(nrows - 1, wr0 + 31);
   const bool live = wr1 >= wr0;
@@ -162,6 +168,15 @@ __global__ __launch_bounds__(512, 1) void window_prefill_k(
       st[1][j] = mfma16(ka[t % KPF], qf[1][s], st[1][j]);
       __builtin_amdgcn_sched_barrier(0);
     }
+    if constexpr (CAP) {
+#pragma unroll
+      for (int blk = 0; blk < 2; ++blk)
+#pragma unroll
+        for (int j = 0; j < 4; ++j)
+#pragma unroll
+          for (int r = 0; r < 4; ++r) st[blk][j][r] = capped_l2(st[blk][j][r] * scale_l2, inv_cap2, cap_l2);
+    }
+    const float sc = CAP ? 1.0f : scale_l2;
     const bool masked = key0 + PAGE_TOK - 1 > wmin || key0 < wlo_last;  // (wave-uniform)
 #pragma unroll
     for (int blk = 0; blk < 2; ++blk) {
@@ -171,13 +186,13 @@ __global__ __launch_bounds__(512, 1) void window_prefill_k(
 #pragma unroll
           for (int r = 0; r < 4; ++r) {
             const int key = key0 + 32 * (j >> 1) + 8 * g + 4 * (j & 1) + r;
-            st[blk][j][r] = key <= qpos[blk] && key >= qlo[blk] ? st[blk][j][r] * scale_l2 : -INFINITY;
+            st[blk][j][r] = seen(key, qpos[blk], qlo[blk], keep) ? st[blk][j][r] * sc : -INFINITY;
           }
-      } else {
+      } else if constexpr (!CAP) {
 #pragma unroll
         for (int j = 0; j < 4; ++j)
 #pragma unroll
-          for (int r = 0; r < 4; ++r) st[blk][j][r] *= scale_l2;
+          for (int r = 0; r < 4; ++r) st[blk][j][r] *= sc;
       }
       float mt = NEG_W;
 #pragma unroll
@@ -236,21 +251,21 @@ __global__ __launch_bounds__(512, 1) void window_prefill_k(
     }
   };
 
-  // ring: page p + 2 is issued once every wave is past page p - 1
-  issue(p_first, 0);
-  if (p_first + 1 < p_end) issue(p_first + 1, 1);
-  for (int p = p_first; p < p_end; ++p) {
-    const int buf = (p - p_first) % 3;
-    if (p + 1 < p_end)
-      asm volatile("s_waitcnt vmcnt(%0)" ::"n"(CPW) : "memory");  // this wave's share of page p has landed
+  // ring: page i + 2 is issued once every wave is past page i - 1
+  issue(page_at(0), 0);
+  if (nit > 1) issue(page_at(1), 1);
+  for (int i = 0; i < nit; ++i) {
+    const int buf = i % 3;
+    if (i + 1 < nit)
+      asm volatile("s_waitcnt vmcnt(%0)" ::"n"(CPW) : "memory");  // this wave's share of page i has landed
     else
       asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
     asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
     __builtin_amdgcn_s_barrier();
     asm volatile("" ::: "memory");
-    if (p + 2 < p_end) issue(p + 2, (p - p_first + 2) % 3);
-    const int key0 = p * PAGE_TOK;
-    if (key0 > wmax || key0 + PAGE_TOK <= wlo_first) continue;  // (wave-uniform) no row of this wave sees the page
+    if (i + 2 < nit) issue(page_at(i + 2), (i + 2) % 3);
+    const int key0 = page_at(i) * PAGE_TOK;
+    if (key0 > wmax || (key0 + PAGE_TOK <= wlo_first && key0 >= keep)) continue;  // (wave-uniform) no row of this wave sees the page
     const uint16_t* Ks = smem + buf * (KEL + VEL);
     s16x8 pf[2][2];
     float alpha[2];
@@ -289,12 +304,12 @@ __global__ __launch_bounds__(512, 1) void window_prefill_k(
 // sums and (maximum, denominator) into part [T][G][nsplit][rep][dv + 2].
 constexpr int WDW = 8;
 
-template <int NK, bool RAG, typename OT>
+template <int NK, bool RAG, typename OT, bool CAP>
 __global__ __launch_bounds__(64 * WDW, 1) void window_decode_k(
     const uint16_t* __restrict__ q, const uint16_t* __restrict__ kc, const uint16_t* __restrict__ vc,
     const int* __restrict__ block_tables, int width, const int* __restrict__ ctx_lens, const float* __restrict__ sink,
     float scale_l2, int window, int chunk, OT* __restrict__ out, int ldo, int H, int G, int Gv, int d_rt, int dv_rt,
-    int num_pages, float* __restrict__ part, int nsplit) {
+    int num_pages, float* __restrict__ part, int nsplit, int keep, float inv_cap2, float cap_l2) {
   constexpr int NDT = NK * 2;
   const int d = RAG ? d_rt : NK * 32, dv = RAG ? dv_rt : NK * 32;
   extern __shared__ float sm[];  // merge: [WDW][rep][dv + 2]
@@ -309,9 +324,11 @@ __global__ __launch_bounds__(64 * WDW, 1) void window_decode_k(
     return;
   }
   const int pos = ctx - 1, lo = first_seen(pos, window, chunk);
-  const int pa = lo / PAGE_TOK, np = pos / PAGE_TOK + 1 - pa;
+  // visible pages in order: those of kept first tokens before the window, then the window's or chunk's own
+  const int pa = lo / PAGE_TOK, nkp = min((keep + PAGE_TOK - 1) / PAGE_TOK, pa), np = nkp + pos / PAGE_TOK + 1 - pa;
+  auto page_at = [&](int i) { return i < nkp ? i : pa + i - nkp; };
   // this share's pages [s0, s1) of the np visible ones
-  const int s0 = pa + (int)((int64_t)np * sp / nsplit), s1 = pa + (int)((int64_t)np * (sp + 1) / nsplit);
+  const int s0 = (int)((int64_t)np * sp / nsplit), s1 = (int)((int64_t)np * (sp + 1) / nsplit);
   const s16x8 zero = {0, 0, 0, 0, 0, 0, 0, 0};
   s16x8 qf[NK];
   {
@@ -327,8 +344,8 @@ __global__ __launch_bounds__(64 * WDW, 1) void window_decode_k(
   for (int dt = 0; dt < NDT; ++dt) o[dt] = f32x4{0.f, 0.f, 0.f, 0.f};
   const int* bt = block_tables + (int64_t)b * width;
   s16x8 kf[4][NK];
-  auto load_k = [&](int p) {
-    const uint16_t* kb = kc + ((int64_t)min(max(bt[p], 0), num_pages - 1) * G + kvh) * PAGE_TOK * d + 8 * g;
+  auto load_k = [&](int i) {
+    const uint16_t* kb = kc + ((int64_t)min(max(bt[page_at(i)], 0), num_pages - 1) * G + kvh) * PAGE_TOK * d + 8 * g;
 #pragma unroll
     for (int j = 0; j < 4; ++j) {
       const int r = 32 * (j >> 1) + 8 * (c >> 2) + 4 * (j & 1) + (c & 3);
@@ -339,7 +356,7 @@ __global__ __launch_bounds__(64 * WDW, 1) void window_decode_k(
   int p = s0 + wave;
   if (p < s1) load_k(p);
   for (; p < s1; p += WDW) {
-    const uint16_t* vb = vc + ((int64_t)min(max(bt[p], 0), num_pages - 1) * Gv + gv) * PAGE_TOK * dv + 8 * g;
+    const uint16_t* vb = vc + ((int64_t)min(max(bt[page_at(p)], 0), num_pages - 1) * Gv + gv) * PAGE_TOK * dv + 8 * g;
     s16x8 vf[NDT][2];
 #pragma unroll
     for (int dt = 0; dt < NDT; ++dt)
@@ -354,14 +371,15 @@ __global__ __launch_bounds__(64 * WDW, 1) void window_decode_k(
       for (int s = 0; s < NK; ++s) st[j] = mfma16(kf[j][s], qf[s], st[j]);
     }
     if (p + WDW < s1) load_k(p + WDW);
-    const int key0 = p * PAGE_TOK;
+    const int key0 = page_at(p) * PAGE_TOK;
     float mt = NEG_W;
 #pragma unroll
     for (int j = 0; j < 4; ++j)
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
         const int key = key0 + 32 * (j >> 1) + 8 * g + 4 * (j & 1) + r;
-        st[j][r] = key <= pos && key >= lo ? st[j][r] * scale_l2 : -INFINITY;
+        const float t = CAP ? capped_l2(st[j][r] * scale_l2, inv_cap2, cap_l2) : st[j][r] * scale_l2;
+        st[j][r] = seen(key, pos, lo, keep) ? t : -INFINITY;
         mt = fmaxf(mt, st[j][r]);
       }
     mt = fmaxf(mt, __shfl_xor(mt, 16, 64));
@@ -459,35 +477,36 @@ struct WinArgs {
   const at::Tensor &q, &k, &v, &bt, &cu, &ctx;
   const float* sink;
   float scale_l2;
-  int window, chunk, ldo;
+  int window, chunk, ldo, keep;
+  float inv_cap2, cap_l2;  // softcap (0: none)
 };
 
-template <int DK, int DV, typename OT>
+template <int DK, int DV, typename OT, bool CAP>
 void go_prefill(const WinArgs& a, at::Tensor& out, int64_t max_qlen) {
   const int H = (int)a.q.size(1), G = (int)a.k.size(1), Gv = (int)a.v.size(1);
   constexpr int SMEM = 3 * (DK + DV) * PAGE_TOK * 2;
-  auto kern = window_prefill_k<DK, DV, OT>;
+  auto kern = window_prefill_k<DK, DV, OT, CAP>;
   static bool attr = hipFuncSetAttribute((const void*)kern, hipFuncAttributeMaxDynamicSharedMemorySize, SMEM) == hipSuccess;
   (void)attr;
   const dim3 grid((unsigned)((max_qlen * (H / G) + 255) / 256), (unsigned)G, (unsigned)a.ctx.numel());
   kern<<<grid, 512, SMEM, stream()>>>((const uint16_t*)a.q.data_ptr(), (const uint16_t*)a.k.data_ptr(),
                                       (const uint16_t*)a.v.data_ptr(), a.bt.data_ptr<int>(), (int)a.bt.size(1),
                                       a.cu.data_ptr<int>(), a.ctx.data_ptr<int>(), a.sink, a.scale_l2, a.window, a.chunk,
-                                      (OT*)out.data_ptr(), a.ldo, H, G, Gv, (int)a.k.size(0));
+                                      (OT*)out.data_ptr(), a.ldo, H, G, Gv, (int)a.k.size(0), a.keep, a.inv_cap2, a.cap_l2);
 }
 
-template <int NK, bool RAG, typename OT>
+template <int NK, bool RAG, typename OT, bool CAP>
 void go_decode(const WinArgs& a, at::Tensor& out, float* part, int nsplit) {
   const int H = (int)a.q.size(1), G = (int)a.k.size(1), Gv = (int)a.v.size(1), dv = (int)a.v.size(2), B = (int)a.ctx.numel();
   const int smem = WDW * (H / G) * (dv + 2) * 4;
-  auto kern = window_decode_k<NK, RAG, OT>;
+  auto kern = window_decode_k<NK, RAG, OT, CAP>;
   static bool attr = hipFuncSetAttribute((const void*)kern, hipFuncAttributeMaxDynamicSharedMemorySize,
                                          WDW * 16 * (32 * NK + 2) * 4) == hipSuccess;
   (void)attr;
   kern<<<dim3(B, G, nsplit), 64 * WDW, smem, stream()>>>(
       (const uint16_t*)a.q.data_ptr(), (const uint16_t*)a.k.data_ptr(), (const uint16_t*)a.v.data_ptr(), a.bt.data_ptr<int>(),
       (int)a.bt.size(1), a.ctx.data_ptr<int>(), a.sink, a.scale_l2, a.window, a.chunk, (OT*)out.data_ptr(), a.ldo, H, G, Gv,
-      (int)a.q.size(2), dv, (int)a.k.size(0), part, nsplit);
+      (int)a.q.size(2), dv, (int)a.k.size(0), part, nsplit, a.keep, a.inv_cap2, a.cap_l2);
   if (nsplit > 1)
     window_merge_k<OT><<<dim3(B, G), 256, 0, stream()>>>(part, a.ctx.data_ptr<int>(), (OT*)out.data_ptr(), a.ldo, H / G, dv,
                                                          nsplit, G);
@@ -499,25 +518,29 @@ void go_decode(const WinArgs& a, at::Tensor& out, float* part, int nsplit) {
 // no pooled blocks.  Returns false when these kernels do not take the step.
 bool window_attention(const at::Tensor& q, const at::Tensor& k_cache, const at::Tensor& v_cache, const at::Tensor& block_tables,
                       const at::Tensor& cu_q, const at::Tensor& ctx_lens, const float* sink, double scale, int64_t window,
-                      int64_t chunk, at::Tensor& out, int64_t ldo, int64_t max_qlen) {
+                      int64_t chunk, int64_t keep, double softcap, at::Tensor& out, int64_t ldo, int64_t max_qlen) {
   const int64_t T = q.size(0), H = q.size(1), d = q.size(2), G = k_cache.size(1), dv = v_cache.size(2), B = ctx_lens.numel();
   const int64_t rep = H / G, width = block_tables.size(1);
   const bool o32 = out.scalar_type() == at::kFloat;
-  const WinArgs a{q, k_cache, v_cache, block_tables, cu_q, ctx_lens, sink, (float)(scale * L2E_W), (int)window, (int)chunk, (int)ldo};
+  const WinArgs a{q, k_cache, v_cache, block_tables, cu_q, ctx_lens, sink, (float)(scale * L2E_W), (int)window, (int)chunk, (int)ldo,
+                  (int)keep, (float)(softcap > 0 ? 2.0 / softcap : 0.0), (float)(softcap * L2E_W)};
+  const bool cap = softcap > 0;
   if (max_qlen == 1 && T == B && rep <= 16 && d % 8 == 0 && dv % 8 == 0 && d <= 128 && dv <= 128) {
     // shares of the visible pages: enough workgroups for the 256 CUs, at least two pages per wave of a share
     int64_t pages = width;
     if (chunk > 0) pages = std::min(pages, (chunk + 63) / 64 + 1);
     if (window > 0) pages = std::min(pages, (window + 63) / 64 + 1);
+    pages = std::min(width, pages + (keep + 63) / 64);
     const int64_t nsplit = std::max<int64_t>(1, std::min<int64_t>((256 + B * G - 1) / (B * G), pages / (2 * WDW)));
     at::Tensor part;
     if (nsplit > 1) part = at::empty({B * G * nsplit * rep * (dv + 2)}, q.options().dtype(at::kFloat));
     float* pp = nsplit > 1 ? part.data_ptr<float>() : nullptr;
     const int64_t n = (std::max(d, dv) + 31) / 32;
     const bool rag = d != 32 * n || dv != 32 * n;
-#define WD_OT(NK, RAG)                                     \
-  (o32 ? go_decode<NK, RAG, float>(a, out, pp, (int)nsplit) \
-       : go_decode<NK, RAG, uint16_t>(a, out, pp, (int)nsplit))
+#define WD_CAP(NK, RAG, OT)                                                \
+  (cap ? go_decode<NK, RAG, OT, true>(a, out, pp, (int)nsplit)              \
+       : go_decode<NK, RAG, OT, false>(a, out, pp, (int)nsplit))
+#define WD_OT(NK, RAG) (o32 ? WD_CAP(NK, RAG, float) : WD_CAP(NK, RAG, uint16_t))
 #define WD_GO(NK) (rag ? WD_OT(NK, true) : WD_OT(NK, false))
     switch (n) {
       case 1: WD_GO(1); break;
@@ -527,13 +550,16 @@ bool window_attention(const at::Tensor& q, const at::Tensor& k_cache, const at::
     }
 #undef WD_GO
 #undef WD_OT
+#undef WD_CAP
     return true;
   }
   if (max_qlen >= 16 && ldo % 4 == 0) {
 #define WP_GO(DK, DV)                                            \
   if (d == DK && dv == DV) {                                     \
-    if (o32) go_prefill<DK, DV, float>(a, out, max_qlen);        \
-    else go_prefill<DK, DV, uint16_t>(a, out, max_qlen);         \
+    if (o32 && cap) go_prefill<DK, DV, float, true>(a, out, max_qlen); \
+    else if (o32) go_prefill<DK, DV, float, false>(a, out, max_qlen);  \
+    else if (cap) go_prefill<DK, DV, uint16_t, true>(a, out, max_qlen); \
+    else go_prefill<DK, DV, uint16_t, false>(a, out, max_qlen);  \
     return true;                                                 \
   }
     WP_GO(64, 64)

@@ -8,6 +8,7 @@ layer count comes from config.json and is validated against the model card.
 from __future__ import annotations
 
 import json
+import math
 from dataclasses import asdict, dataclass, field, replace
 from pathlib import Path
 from typing import Optional
@@ -38,20 +39,24 @@ class LinearRecurrenceSpec:
     q / k shared by heads / kv_heads value heads, short causal convolutions (conv taps) + SiLU on q, k, v,
     unit-norm q and k, q scaled by dim^-1/2.
   rule "gla": decay per key channel sigmoid(z)^(1/tau) with a low-rank z, write k v^T, q scaled by dim^-1/2.
+  rule "channel_delta": the delta rule with one decay per head and key channel, g = exp(-exp(A_log[head]) softplus(W_a2 (W_a1
+    h) + dt_bias)) acting on the state's key rows, and a low-rank sigmoid output gate W_g2 (W_g1 h) (rank, gate_rank: from the
+    tensors' shapes).
   rule "lightning": one fixed decay per head (`decays`), SiLU on q, k, v, write k v^T, no scale; the heads' outputs are
     RMS-normed together, weighted and gated by a sigmoid.
   rule "mlstm": the matrix memory of xLSTM.  Log input gate i = cap tanh(z_i / cap), log forget gate f = logsigmoid(cap
     tanh(z_f / cap)) per head (gate_cap), a running maximum m_t = max(f + m_(t-1), i) that starts at 0, S <- e^(f + m_(t-1) -
     m_t) S + e^(i - m_t) k v^T and a normaliser n likewise from k alone, o = S^T q / (max(|n . q|, e^(-m_t)) + 1e-6), q
     scaled by dim^-1/2.  The normaliser travels as one more value channel of the state (value = 1), the maximum beside it."""
-  rule: str  # delta | gla | lightning | mlstm
+  rule: str  # delta | channel_delta | gla | lightning | mlstm
   heads: int
   kv_heads: int
   dim: int
   vdim: int
-  conv: int = 0  # taps of the short convolutions (delta)
+  conv: int = 0  # taps of the short convolutions (delta, channel_delta)
   tau: float = 1.0  # decay temperature (gla)
-  rank: int = 0  # rank of the decay projection (gla; from the tensor's shape)
+  rank: int = 0  # rank of the decay projection (gla, channel_delta; from the tensor's shape)
+  gate_rank: int = 0  # rank of the output gate (channel_delta; from the tensor's shape)
   decays: tuple = ()  # lightning: one per head
   gate_cap: float = 0.0  # mlstm
 
@@ -73,7 +78,11 @@ class WindowAttnSpec:
   by element.  chunk > 0: a query sees only tokens of its own block of `chunk` positions, counted from the sequence's
   start.  proj_norm: one weighted RMS norm over the whole query projection (and one over the whole key projection) before
   the rotation.  rot_interleaved: rotation pairs (2i, 2i + 1) instead of (i, i + rot_dims / 2).  sink_one: one is added to
-  the softmax's denominator (a sink whose logit is zero).  out_bias: the output projection has a bias."""
+  the softmax's denominator (a sink whose logit is zero).  out_bias: the output projection has a bias.  keep_first > 0: the
+  sequence's first tokens stay visible outside the window.  rot_scaling may also be ("yarn", factor, original, fast, slow):
+  YaRN frequencies, cos and sin times 0.1 ln(factor) + 1.  conv > 0: causal convolutions of that many taps over time on
+  every q / k / v channel, before norms and rotation (their last inputs are per-request state).  head_norm: weighted RMS norm
+  of every query / key head before the rotation.  softcap > 0: scores <- softcap * tanh(score / softcap)."""
   heads: int
   kv_heads: int
   dim: int
@@ -94,6 +103,25 @@ class WindowAttnSpec:
   rot_interleaved: bool = False
   sink_one: bool = False
   out_bias: bool = False
+  keep_first: int = 0
+  conv: int = 0
+  head_norm: bool = False
+  softcap: float = 0.0
+
+  @property
+  def conv_channels(self) -> int:
+    return self.heads * self.dim + self.kv_heads * (self.dim + self.vdim) if self.conv else 0
+
+  def rope_scaling(self) -> Optional[dict]:
+    """rot_scaling in the words of the rotary table builder (ops.rope)."""
+    r = self.rot_scaling
+    if not r:
+      return None
+    if r[0] == "yarn":
+      return dict(rope_type="yarn", factor=r[1], original_max_position_embeddings=r[2], beta_fast=r[3], beta_slow=r[4],
+                  attention_factor=0.1 * math.log(r[1]) + 1.0)
+    return dict(rope_type="llama3", factor=r[0], low_freq_factor=r[1], high_freq_factor=r[2],
+                original_max_position_embeddings=r[3])
 
 
 @dataclass(frozen=True)
@@ -210,8 +238,9 @@ class MixedLayerSpec:
   ssd: Optional[SSDSpec] = None
   ffn: Optional[FeedForwardSpec] = None
   lattn: Optional[LatentAttnSpec] = None  # sandwich blocks
-  dattn: Optional[DiffAttnSpec] = None  # sandwich blocks; a "parallel" layer there is wattn beside rec
+  dattn: Optional[DiffAttnSpec] = None  # sandwich blocks; a "parallel" layer there is wattn beside rec or ssd
   side: int = 0  # size of the layer's per-token side input (a slice of a second embedding table), 0: none
+  weights_of: int = -1  # >= 0: the layer has no tensors of its own and uses that layer's (its caches and states are its own)
 
   @property
   def kv_dims(self) -> Optional[tuple]:
@@ -231,20 +260,24 @@ class MixedLayerSpec:
   @property
   def state_dims(self) -> Optional[tuple]:
     """(heads, value channels, key dim, convolution taps, convolution channels, scalars per head) of the layer's
-    recurrent state."""
+    recurrent state (heads 0: convolutions only).  Convolutions of two mixers side by side share one state: the channels
+    of both, the longer one's taps."""
     if self.rec is not None:
       r = self.rec
       return r.heads, r.state_vdim, r.dim, r.conv, (2 * r.kv_heads * r.dim + r.heads * r.vdim) if r.conv > 0 else 0, \
         1 if r.rule == "mlstm" else 0
+    wc, wt = (self.wattn.conv_channels, self.wattn.conv) if self.wattn is not None else (0, 0)
     if self.ssd is not None:
       m = self.ssd
-      return m.heads, m.vdim, m.state, m.conv, m.conv_channels if m.conv > 0 else 0, 0
+      return m.heads, m.vdim, m.state, max(m.conv, wt), (m.conv_channels if m.conv > 0 else 0) + wc, 0
+    if wc:
+      return 0, 0, 0, wt, wc, 0
     return None
 
 
 @dataclass(frozen=True)
 class ModelConfig:
-  model_type: str  # llama | qwen2 | mistral | mixtral | ... | tarepel | mogelix | nenizen | kopalorn | torinex
+  model_type: str  # llama | qwen2 | mistral | mixtral | ... | tarepel | mogelix | nenizen | kopalorn | torinex | zepalorn
   vocab_size: int
   hidden_size: int
   intermediate_size: int
@@ -310,6 +343,15 @@ class ModelConfig:
   loop_input: str = "linear"  # linear | add
   # sandwich blocks without the norms in front (Torinex): the sublayers read the stream itself, x += norm_b(sublayer(x))
   input_norm: bool = True
+  norm_bias: bool = True  # layer norms carry a bias (Zepalorn: a weight only)
+
+  def weights_owner(self, i: int) -> int:
+    """The layer whose tensors layer i uses (itself unless it shares another's)."""
+    seen = set()
+    while self.layer_specs and self.layer_specs[i].weights_of >= 0 and i not in seen:
+      seen.add(i)
+      i = self.layer_specs[i].weights_of
+    return i
 
   @property
   def side_dim(self) -> int:
@@ -417,7 +459,8 @@ class ModelConfig:
 
   def num_params(self) -> int:
     emb = self.vocab_size * self.hidden_size
-    layers = sum(self.params_per_layer(i) for i in range(self.num_layers)) + self.vocab_size * self.side_dim * self.num_layers
+    own = [i for i in range(self.num_layers) if self.weights_owner(i) == i]  # (shared tensors count once)
+    layers = sum(self.params_per_layer(i) for i in own) + self.vocab_size * self.side_dim * self.num_layers
     return layers + emb * (1 if self.tie_word_embeddings else 2) + self.hidden_size
 
   def to_dict(self) -> dict:
@@ -428,6 +471,7 @@ class ModelConfig:
   def with_layers(self, n: int) -> "ModelConfig":
     if self.layer_specs is not None and n != len(self.layer_specs):
       specs = tuple(self.layer_specs[i % len(self.layer_specs)] for i in range(n))
+      specs = tuple(replace(s, weights_of=-1) if s.weights_of >= n else s for s in specs)
       loop = self.loop if self.loop and self.loop[1] <= n else None  # (a loop that no longer fits is dropped)
       return replace(self, num_layers=n, layer_specs=specs, loop=loop)
     return replace(self, num_layers=n)
@@ -461,7 +505,26 @@ def _outnorm_params(D: int, s: MixedLayerSpec) -> int:
   return n + (2 * D * s.side + D if s.side else 0)
 
 
+def _conv_sandwich_params(D: int, s: MixedLayerSpec) -> int:
+  """Layers of bias-free layer-norm sandwich blocks: channel-decay delta rule, window attention, or convolved attention
+  beside a Mamba-2 mixer; clamped gated feed-forward."""
+  a, r, m, f = s.wattn, s.rec, s.ssd, s.ffn
+  n = 2 * D + (2 * D + 3 * D * f.ff if f is not None else 0)
+  if r is not None:
+    qk, hv, ra, rg = 2 * r.kv_heads * r.dim, r.heads * r.vdim, r.rank or 8, r.gate_rank or 8
+    n += (D + r.conv) * (qk + hv) + (D + 1) * r.heads + ra * (D + r.heads * r.dim) + r.heads * r.dim + rg * (D + hv) + r.vdim + hv * D
+  if a is not None:
+    n += D * (a.heads * a.dim + a.kv_heads * (a.dim + a.vdim)) + a.heads * a.vdim * D + a.conv * a.conv_channels + \
+      (2 * a.dim if a.head_norm else 0)
+  if m is not None:
+    n += D * (2 * m.inner + 2 * m.groups * m.state + m.heads) + m.conv_channels * (m.conv + 1) + 3 * m.heads + m.inner + m.inner * D
+    n += 2 * D if a is not None else 0
+  return n
+
+
 def mixed_layer_params(D: int, s: MixedLayerSpec) -> int:
+  if s.kind == "channel_delta" or (s.wattn is not None and not s.wattn.bias):
+    return _conv_sandwich_params(D, s)
   if s.wattn is not None and s.wattn.proj_norm:
     return _outnorm_params(D, s)
   if s.dattn is not None or (s.rec is not None and s.rec.rule in ("lightning", "mlstm")):
@@ -803,7 +866,91 @@ def _torinex_config(cfg: dict) -> ModelConfig:
     layer_specs=tuple(specs), block="sandwich", input_norm=False)
 
 
+def _rot_fields(i: int, m: dict) -> tuple:
+  """(dims, base, scaling tuple or None) of a mixer's "rot" entry with YaRN scaling."""
+  rot = m.get("rot") or {}
+  dims, sc = int(rot.get("dims", 0)), rot.get("scaling")
+  if dims % 2 or dims > int(m["dim"]):
+    raise ValueError(f"layer {i}: {dims} rotary dims do not fit heads of {m['dim']}")
+  scaling = ("yarn", float(sc["factor"]), float(sc["original"]), float(sc["fast"]), float(sc["slow"])) if sc else None
+  return dims, float(rot.get("base", 10000.0)), scaling
+
+
+def _zepalorn_config(cfg: dict) -> ModelConfig:
+  """Zepalorn config.json: {"architecture", "vocab", "width", "norm": {"eps"}, "embedding": {"scale"}, "layers": [{"type":
+  "channel_delta" | "attention" | "parallel", "mixer": {...}, "mlp": {"kind": "dense", "ff", "limit"} | null,
+  "weights_of": j}]}.  "channel_delta": {"heads", "kv_heads", "dim", "vdim", "conv"}; "attention": {"heads", "kv_heads", "dim",
+  "vdim", "scale", "mask": {"size", "keep_first"}, "rot": {"base", "dims", "scaling": {"factor", "original", "fast", "slow"}}};
+  "parallel": {"left": the attention's keys (a mask without "keep_first" counts chunks) and "conv", "softcap"; "right":
+  {"heads", "vdim", "state", "groups", "conv", "norm_groups"}}.  Without "mask" every earlier token is seen, without "rot"
+  nothing is rotated; "weights_of": j shares layer j's tensors.  Projection ranks come from the checkpoint."""
+  specs, L = [], cfg["layers"]
+
+  def entry(i):  # a layer that shares tensors may leave the rest of its entry to the other one
+    e, seen = L[i], {i}
+    while "mixer" not in e and e.get("weights_of") is not None and int(e["weights_of"]) not in seen:
+      seen.add(int(e["weights_of"]))
+      e = L[int(e["weights_of"])]
+    return e
+  for i in range(len(L)):
+    e = entry(i)
+    m, mlp, kind = e["mixer"], e.get("mlp"), e["type"]
+    ffn = None
+    if mlp is not None:
+      if mlp.get("kind", "dense") != "dense":
+        raise ValueError(f"layer {i}: unsupported feed-forward kind {mlp.get('kind')!r}")
+      ffn = FeedForwardSpec("clamped_glu", int(mlp["ff"]), limit=float(mlp["limit"]))
+    wo = L[i].get("weights_of")
+    wo = -1 if wo is None else int(wo)
+    if kind == "channel_delta":
+      r = LinearRecurrenceSpec("channel_delta", int(m["heads"]), int(m["kv_heads"]), int(m["dim"]), int(m["vdim"]), conv=int(m["conv"]),
+                               rank=int(m.get("rank", 0)), gate_rank=int(m.get("gate_rank", 0)))
+      if r.heads % r.kv_heads or r.conv < 1:
+        raise ValueError(f"layer {i}: heads {r.heads} / kv_heads {r.kv_heads} / taps {r.conv} do not fit")
+      specs.append(MixedLayerSpec(kind, rec=r, ffn=ffn, weights_of=wo))
+      continue
+    if kind not in ("attention", "parallel"):
+      raise ValueError(f"layer {i}: unknown layer type {kind!r}")
+    par = kind == "parallel"
+    a = m["left"] if par else m
+    dims, base, scaling = _rot_fields(i, a)
+    mask = a.get("mask") or {}
+    w = WindowAttnSpec(int(a["heads"]), int(a["kv_heads"]), int(a["dim"]), int(a["vdim"]), 0 if par else int(mask.get("size", 0)), 0,
+                       dims, base, scaling, float(a["scale"]), qk_norm=False, bias=False, sink=False,
+                       chunk=int(mask.get("size", 0)) if par else 0, rot_interleaved=par, keep_first=int(mask.get("keep_first", 0)),
+                       conv=int(a["conv"]) if par else 0, head_norm=par, softcap=float(a.get("softcap") or 0.0) if par else 0.0)
+    if w.heads % w.kv_heads or (par and w.conv < 1):
+      raise ValueError(f"layer {i}: heads {w.heads} / kv_heads {w.kv_heads} / taps {w.conv} do not fit")
+    ssd = None
+    if par:
+      b = m["right"]
+      ssd = SSDSpec(int(b["heads"]), int(b["vdim"]), int(b["state"]), int(b["groups"]), int(b["conv"]), int(b["norm_groups"]))
+      if ssd.heads % ssd.groups or ssd.inner % ssd.norm_groups or ssd.conv < 1:
+        raise ValueError(f"layer {i}: heads {ssd.heads} / groups {ssd.groups} / norm_groups {ssd.norm_groups} do not fit")
+    specs.append(MixedLayerSpec(kind, wattn=w, ssd=ssd, ffn=ffn, weights_of=wo))
+  for i, s in enumerate(specs):
+    if s.weights_of >= 0:
+      if s.weights_of >= len(specs) or replace(specs[s.weights_of], weights_of=-1) != replace(s, weights_of=-1):
+        raise ValueError(f"layer {i}: weights_of {s.weights_of} must name a layer of the same kind and sizes")
+      j, hops = i, 0
+      while specs[j].weights_of >= 0:
+        j, hops = specs[j].weights_of, hops + 1
+        if hops > len(specs):
+          raise ValueError(f"layer {i}: weights_of runs in a circle")
+  first = next((s.wattn or s.rec for s in specs), None)
+  return ModelConfig(
+    model_type="zepalorn", vocab_size=int(cfg["vocab"]), hidden_size=int(cfg["width"]),
+    intermediate_size=max([s.ffn.ff for s in specs if s.ffn is not None] + [0]), num_layers=len(specs),
+    num_heads=first.heads, num_kv_heads=first.kv_heads, head_dim=first.dim, rms_norm_eps=float(cfg["norm"]["eps"]),
+    rope_theta=getattr(first, "rot_base", 10000.0), max_position_embeddings=int(cfg.get("max_positions", 1 << 20)),
+    tie_word_embeddings=True, bos_token_id=int(cfg.get("bos_token_id", 0)), eos_token_ids=tuple(cfg.get("eos_token_ids", ())),
+    layer_specs=tuple(specs), block="sandwich", embed_scale=float((cfg.get("embedding") or {}).get("scale", 1.0)),
+    norm_kind="layer", norm_bias=False)
+
+
 def from_hf_config(cfg: dict) -> ModelConfig:
+  if cfg.get("architecture") == "Zepalorn":
+    return _zepalorn_config(cfg)
   if cfg.get("architecture") == "Torinex":
     return _torinex_config(cfg)
   if cfg.get("architecture") == "Kopalorn":
@@ -1117,6 +1264,22 @@ TINY_TORINEX = {
                "rot": {"base": 500.0, "dims": 16}, "scale": 0.3}},
   ]}
 PRESETS["tiny-torinex"] = _torinex_config(TINY_TORINEX)
+_TINY_YARN = {"factor": 4.0, "original": 128, "fast": 16.0, "slow": 1.0}
+_TINY_DELTA = {"heads": 4, "kv_heads": 2, "dim": 24, "vdim": 16, "conv": 3}
+TINY_ZEPALORN = {
+  "architecture": "Zepalorn", "vocab": 296, "width": 88, "norm": {"eps": 1e-5}, "embedding": {"scale": 5.0},
+  "layers": [
+    {"type": "channel_delta", "mlp": {"kind": "dense", "ff": 144, "limit": 1.5}, "mixer": _TINY_DELTA},
+    {"type": "attention", "mlp": None,
+     "mixer": {"heads": 6, "kv_heads": 2, "dim": 16, "vdim": 24, "mask": {"size": 21, "keep_first": 3},
+               "rot": {"base": 20000.0, "dims": 12, "scaling": _TINY_YARN}, "scale": 0.3}},
+    {"type": "channel_delta", "mlp": {"kind": "dense", "ff": 144, "limit": 1.5}, "mixer": _TINY_DELTA, "weights_of": 0},
+    {"type": "parallel", "mlp": {"kind": "dense", "ff": 96, "limit": 3.0},
+     "mixer": {"left": {"heads": 4, "kv_heads": 1, "dim": 24, "vdim": 16, "conv": 2, "mask": {"size": 37}, "softcap": 8.0,
+                        "rot": {"base": 5000.0, "dims": 16, "scaling": _TINY_YARN}, "scale": 0.25},
+               "right": {"heads": 6, "vdim": 8, "state": 20, "groups": 3, "conv": 4, "norm_groups": 2}}},
+  ]}
+PRESETS["tiny-zepalorn"] = _zepalorn_config(TINY_ZEPALORN)
 # aliases of the reference's model cards that share an architecture
 for _alias, _base in {"llama-3.1-70b-bf16": "llama-3.1-70b", "nemotron-70b": "llama-3.1-70b",
                       "deepseek-r1-distill-llama-70b": "llama-3.1-70b", "deepseek-r1-distill-llama-8b": "llama-3.1-8b",

@@ -70,6 +70,7 @@ _CARDS: List[tuple] = [
   ("tiny-nenizen", 5, "synthetic/tiny-nenizen", "Tiny Nenizen (synthetic)"),
   ("tiny-kopalorn", 4, "synthetic/tiny-kopalorn", "Tiny Kopalorn (synthetic)"),
   ("tiny-torinex", 4, "synthetic/tiny-torinex", "Tiny Torinex (synthetic)"),
+  ("tiny-zepalorn", 4, "synthetic/tiny-zepalorn", "Tiny Zepalorn (synthetic)"),
 ]
 
 model_cards: Dict[str, dict] = {mid: {"layers": n, "repo": {ENGINE: repo}} for mid, n, repo, _ in _CARDS}

@@ -42,6 +42,8 @@ MOE_BM = int(os.environ.get("XOT_MOE_BM", "0"))  # force the grouped gemm_big ti
 MOE_DN_SPLITS = int(os.environ.get("XOT_MOE_DN_SPLITS", "0"))  # force the grouped down GEMM's K split on gemm_big tiles
 MOE_PP2 = os.environ.get("XOT_MOE_PP2", "1") == "1"  # 256-row expert tiles on the two-phase ping-pong schedule
 PAGE = 64
+# tokens of a step from which the second projections of low-rank gates run as GEMMs (below: inside the gate kernel, in fp32)
+LOW_RANK_GEMM_ROWS = int(os.environ.get("XOT_LOW_RANK_GEMM_ROWS", "256"))
 
 
 def moe_tiles(rows: float, E: int) -> Tuple[int, int, int]:
@@ -184,10 +186,10 @@ class StatePool:
     self.aux: List[Optional[torch.Tensor]] = []
     for i, _ in c.layer_runs(layer_ids):  # (a looped layer: a state of its own in every pass)
       sd = c.layer_specs[i].state_dims  # (heads, value channels, key dim, taps, convolution channels, scalars per head)
-      self.S.append(None if sd is None else torch.zeros(slots, sd[0], sd[1], sd[2], device=device, dtype=torch.float32))
+      self.S.append(None if sd is None or not sd[0] else torch.zeros(slots, sd[0], sd[1], sd[2], device=device, dtype=torch.float32))
       self.conv.append(torch.zeros(slots, max(sd[3] - 1, 0), sd[4], device=device, dtype=torch.float32)
                        if sd is not None and sd[4] else None)
-      self.aux.append(torch.zeros(slots, sd[0], sd[5], device=device, dtype=torch.float32) if sd is not None and sd[5] else None)
+      self.aux.append(torch.zeros(slots, sd[0], sd[5], device=device, dtype=torch.float32) if sd is not None and sd[0] and sd[5] else None)
 
   def clear(self, slot: int) -> None:
     for t in self.S + self.conv + self.aux:
@@ -221,10 +223,8 @@ class ShardModel:
           self.rope_tabs[(a.rot_dims, a.rot_base)] = build_cos_sin(a.rot_dims, self.rope_rows, a.rot_base, None, self.device)
         a = c.layer_specs[i].wattn
         if a is not None and a.rot_dims and (a.rot_dims, a.rot_base, a.rot_scaling) not in self.rope_tabs:
-          sc = a.rot_scaling and dict(rope_type="llama3", factor=a.rot_scaling[0], low_freq_factor=a.rot_scaling[1],
-                                      high_freq_factor=a.rot_scaling[2], original_max_position_embeddings=a.rot_scaling[3])
           self.rope_tabs[(a.rot_dims, a.rot_base, a.rot_scaling)] = build_cos_sin(a.rot_dims, self.rope_rows, a.rot_base,
-                                                                                 sc, self.device)
+                                                                                 a.rope_scaling(), self.device)
         a = c.layer_specs[i].lattn or c.layer_specs[i].dattn
         if a is not None and a.rot_dims and (a.rot_dims, a.rot_base) not in self.rope_tabs:
           self.rope_tabs[(a.rot_dims, a.rot_base)] = build_cos_sin(a.rot_dims, self.rope_rows, a.rot_base, None, self.device)
@@ -581,7 +581,8 @@ class ShardModel:
   # ------------------------------------------------------------------ post-norm blocks (window attention / SSD, MoE)
   def _window_attn(self, P: torch.Tensor, lw, j: int, inp: StepInputs, mix: torch.Tensor) -> None:
     """Softmax attention over a sliding window or the query's chunk, pooled blocks and a sink: biases + norms + RoPE + paged
-    write, the pooled caches' update for blocks that this step completed, then the attention."""
+    write, the pooled caches' update for blocks that this step completed, then the attention.  (P of a layer whose
+    projections pass short convolutions: the convolved and normed rows, q | k | v in front.)"""
     a = lw.spec.wattn
     q = torch.empty(mix.shape[0], a.heads, a.dim, dtype=mix.dtype, device=P.device)
     tab = self.rope_tabs.get((a.rot_dims, a.rot_base, a.rot_scaling))
@@ -597,7 +598,8 @@ class ShardModel:
     pool = a.pool if self.kv.kp[j] is not None else 0
     o = mix[:, :a.heads * a.vdim]
     K.attn_window_pool(q, self.kv.k[j], self.kv.v[j], self.kv.kp[j], self.kv.vp[j], inp.block_tables, inp.cu_q,
-                       inp.ctx_lens, lw.sink, a.scale, a.window, pool, o, max_qlen=inp.max_qlen, chunk=a.chunk)
+                       inp.ctx_lens, lw.sink, a.scale, a.window, pool, o, max_qlen=inp.max_qlen, chunk=a.chunk,
+                       keep=a.keep_first, softcap=a.softcap)
     if a.gate != "none":  # one sigmoid gate per element, from the mixer's input, applied in place
       K.sigmoid_gate_mul(o, P, lw.cols["gate"][0], mix)
 
@@ -662,6 +664,51 @@ class ShardModel:
     K.linear_recurrence(xbc[:, inner + gn:], xbc[:, inner:inner + gn], v, decay, None, 1.0, st.S[j], inp.state_slots,
                         inp.cu_q, o)
     K.ssd_gate_norm(o, xbc, lw.skip_d, P, i0, lw.ssd_norm, m.norm_groups, self.c.rms_norm_eps, mix)
+
+  def _conv(self, P: torch.Tensor, off: int, lw, j: int, inp: StepInputs) -> torch.Tensor:
+    """The layer's short convolutions (every convolved channel of its mixers in one launch) with what follows them channel
+    by channel or head by head -> fp32 [T, channels]."""
+    out = torch.empty(P.shape[0], lw.conv_w.shape[0], dtype=torch.float32, device=P.device)
+    K.conv_prep(P, off, lw.conv_w, lw.conv_b, lw.conv_units, lw.conv_norm, self.state.conv[j], inp.state_slots, inp.cu_q,
+                self.c.rms_norm_eps, out, max_qlen=inp.max_qlen)
+    return out
+
+  def _low_rank(self, P: torch.Tensor, off: int, n: int, w: torch.Tensor) -> torch.Tensor:
+    """Second projection of a low-rank pair on the GEMM kernels: w (padded) times the operand copy of P[:, off : +n]."""
+    x = torch.zeros(P.shape[0], w.shape[1], dtype=w.dtype, device=P.device)
+    x[:, :n] = P[:, off:off + n].to(w.dtype)
+    return self._proj(x, w)
+
+  def _channel_delta(self, P: torch.Tensor, lw, j: int, inp: StepInputs, mix: torch.Tensor) -> None:
+    """Delta rule with a decay per key channel on the state slots: convolutions + SiLU + unit norms, step sizes and low-rank
+    decays and output gates (prompts: their second projections are GEMMs), the recurrence, the per-head gated norm."""
+    r, st, dev = lw.spec.rec, self.state, P.device
+    T, H, nk, nv = P.shape[0], r.heads, r.kv_heads * r.dim, r.heads * r.vdim
+    qkv = self._conv(P, lw.cols["rq"][0], lw, j, inp)
+    beta = torch.empty(T, H, dtype=torch.float32, device=dev)
+    decay = torch.empty(T, H * r.dim, dtype=torch.float32, device=dev)
+    (a0, an), (g0, gn) = lw.cols["ra1"], lw.cols["rg1"]
+    if P.is_cuda and lw.a2_p is not None and T >= LOW_RANK_GEMM_ROWS:
+      za, gate = self._low_rank(P, a0, an, lw.a2_p), self._low_rank(P, g0, gn, lw.g2_p)
+      K.recurrence_gates(P, lw.cols["rb"][0], beta, 0, None, lw.dt_bias, lw.A_log, decay, 0, None, None, za=za)
+    else:
+      gate = torch.empty(T, nv, dtype=torch.float32, device=dev)
+      K.recurrence_gates(P, lw.cols["rb"][0], beta, a0, lw.a2_w, lw.dt_bias, lw.A_log, decay, g0, lw.g2_w, gate)
+    o = torch.empty(T, nv, dtype=torch.float32, device=dev)
+    K.linear_recurrence(qkv[:, :nk], qkv[:, nk:2 * nk], qkv[:, 2 * nk:], decay, beta, 1.0, st.S[j], inp.state_slots, inp.cu_q, o)
+    K.gated_group_norm(o, None, lw.rec_norm, gate, 0, H, self.c.rms_norm_eps, mix)
+
+  def _ssd_conv(self, P: torch.Tensor, x: torch.Tensor, lw, j: int, inp: StepInputs, mix: torch.Tensor) -> None:
+    """Mamba-2 mixer whose convolved channels x = [x | B | C] are ready: step sizes and decays, the recurrence (input scale
+    dt), skip, gate, grouped norm."""
+    m, st, dev = lw.spec.ssd, self.state, P.device
+    T, inner, gn = P.shape[0], m.inner, m.groups * m.state
+    dt, decay = (torch.empty(T, m.heads, dtype=torch.float32, device=dev) for _ in range(2))
+    K.ssd_steps(P, lw.cols["dt"][0], lw.dt_bias, lw.A_log, dt, decay)
+    o = torch.empty(T, inner, dtype=torch.float32, device=dev)
+    K.linear_recurrence(x[:, inner + gn:inner + 2 * gn], x[:, inner:inner + gn], x[:, :inner], decay, dt, 1.0, st.S[j],
+                        inp.state_slots, inp.cu_q, o, plain=True)
+    K.ssd_gate_norm(o, x, lw.skip_d, P, lw.cols["z"][0], lw.ssd_norm, m.norm_groups, self.c.rms_norm_eps, mix)
 
   def _relu2_moe(self, hn: torch.Tensor, P: torch.Tensor, lw, rows) -> torch.Tensor:
     """Routed relu^2 experts + the gated shared expert -> fp32 [T, D].  Routing on the framework's top-k kernels (the
@@ -893,8 +940,9 @@ class ShardModel:
       P = hn @ ff_w^T                    gate | up, or router | shared expert's projections
       h += mult * norm2b(ff(P));  hn = the next run's norm1(h)
     The norms are RMS norms with a weight, or (norm_kind "layer") layer norms with weight and bias.  Mixers: latent
-    attention; differential attention; window / chunk attention; mlstm; gated attention beside lightning attention, each
-    projected to the width, RMS-normed with its own weight and averaged.
+    attention; differential attention; window / chunk attention; mlstm; the delta rule with channel decays; gated attention
+    beside lightning attention, or convolved attention beside Mamba-2, each projected to the width, RMS-normed with its own
+    weight and averaged.
     Without input norms (input_norm False) hn is the stream itself in the operand dtype.  A layer with a side input ends
     with h += norm(proj(gelu_tanh(hn @ gate^T) * its slice of the token's side-input row)).
     Returns h (non-last shard; with the token ids as one more column when the model has side inputs) or softcap(head(final_norm(h rows inp.last_idx)))."""
@@ -917,6 +965,7 @@ class ShardModel:
       x0 = h.clone()
     runs = self.runs
     eps, mult = c.rms_norm_eps, c.residual_mult
+    ln = c.norm_kind == "layer"
     fresh = True  # hn does not hold this run's normed input yet
     for j, (li, t) in enumerate(runs):
       lw = w.layers[li]
@@ -931,22 +980,29 @@ class ShardModel:
         h += w.loop_step[t]
         fresh = True
       if fresh:  # (no norm weight: the op copies the stream)
-        K.sandwich_add_norm(h, None, None, lw.norm1, eps, hn, bn=lw.norm1_b)
+        K.sandwich_add_norm(h, None, None, lw.norm1, eps, hn, bn=lw.norm1_b, layer=ln)
+      pair = s.wattn is not None and (s.rec is not None or s.ssd is not None)  # two mixers side by side
       # (window attention alone: the store kernel is the projection's only reader)
-      P = (self._proj_slabs if s.wattn is not None and s.wattn.gate == "none" and s.rec is None else self._proj)(hn, lw.in_w)
+      P = (self._proj_slabs if s.wattn is not None and s.wattn.gate == "none" and not pair else self._proj)(hn, lw.in_w)
       mix = rows("mix", lw.mix_cols["mix"][1], lw.out_w.shape[1])
       if s.lattn is not None:
         self._latent_attn(P, lw, j, inp, mix, rows)
       elif s.dattn is not None:
         self._diff_attn(P, lw, j, inp, mix)
       elif s.wattn is not None:
-        self._window_attn(P, lw, j, inp, mix)
+        X = self._conv(P, 0, lw, j, inp) if s.wattn.conv else P  # (also the convolved channels of a mixer beside it)
+        self._window_attn(X, lw, j, inp, mix)
+      elif s.rec.rule == "channel_delta":
+        self._channel_delta(P, lw, j, inp, mix)
       else:
         self._mlstm(P, lw, j, inp, mix)
-      y = (self._proj if s.wattn is not None and s.rec is not None else self._proj_slabs)(mix, lw.out_w)
-      if s.wattn is not None and s.rec is not None:  # the second mixer of a parallel layer, then the mean of the normed pair
+      y = (self._proj if pair else self._proj_slabs)(mix, lw.out_w)
+      if pair:  # the second mixer of a parallel layer, then the mean of the normed pair
         mix2 = rows("mix2", lw.mix_cols["mix2"][1], lw.out2_w.shape[1])
-        self._lightning(P, lw, j, inp, mix2)
+        if s.ssd is not None:
+          self._ssd_conv(P, X[:, s.wattn.conv_channels:], lw, j, inp, mix2)
+        else:
+          self._lightning(P, lw, j, inp, mix2)
         y2 = self._proj(mix2, lw.out2_w)
         y1, y = y, torch.empty(T, D, dtype=torch.float32, device=h.device)
         K.pair_norm_mean(y1, y2, lw.pair_w, eps, y)
@@ -958,10 +1014,16 @@ class ShardModel:
       after = (lw.side_norm is not None, f is not None)  # what still reads hn in this layer: the side input, the feed-forward
       if f is None:
         K.sandwich_add_norm(h, y, lw.norm1b, nxt, eps, hn if after[0] else hn_nxt, bb=lw.norm1b_b, bn=nxt_b, mult=mult,
-                            yb=lw.out_b)
+                            yb=lw.out_b, layer=ln)
       else:
-        K.sandwich_add_norm(h, y, lw.norm1b, lw.norm2, eps, hn, bb=lw.norm1b_b, bn=lw.norm2_b, mult=mult, yb=lw.out_b)
-        if f.kind == "clamped_glu":
+        K.sandwich_add_norm(h, y, lw.norm1b, lw.norm2, eps, hn, bb=lw.norm1b_b, bn=lw.norm2_b, mult=mult, yb=lw.out_b, layer=ln)
+        if f.kind == "clamped_glu" and lw.ff_cols is None:  # gate / up rows interleaved: the activation is the GEMM's epilogue
+          act = self._fused_act(hn, lw.ff_w, "clamp_glu", f.limit)
+          if act is None:
+            act = self._glu_tiles(self._proj(hn, lw.ff_w), True, f.limit,
+                                  torch.empty(T, lw.ff_w.shape[0] // 2, dtype=adt, device=h.device))
+          y = self._proj_slabs(act, lw.down_w)
+        elif f.kind == "clamped_glu":
           act = rows("act", f.ff, lw.down_w.shape[1])
           K.glu_act(self._proj(hn, lw.ff_w), lw.ff_cols["gate"][0], lw.ff_cols["up"][0], f.ff, True, f.limit, act)
           y = self._proj_slabs(act, lw.down_w)
@@ -975,7 +1037,8 @@ class ShardModel:
           y = self._relu2_moe(hn, self._proj(hn, lw.ff_w), lw, rows)
         else:
           y = self._glu_moe(hn, lw)
-        K.sandwich_add_norm(h, y, lw.norm2b, nxt, eps, hn if after[0] else hn_nxt, bb=lw.norm2b_b, bn=nxt_b, mult=mult)
+        K.sandwich_add_norm(h, y, lw.norm2b, nxt, eps, hn if after[0] else hn_nxt, bb=lw.norm2b_b, bn=nxt_b, mult=mult,
+                            layer=ln)
       if after[0]:
         K.sandwich_add_norm(h, self._side_input(hn, lw, li, ids, rows), lw.side_norm, nxt, eps, hn_nxt, bn=nxt_b)
       fresh = nl is None
@@ -983,7 +1046,7 @@ class ShardModel:
       return torch.cat([h, ids.to(torch.float32)[:, None]], 1) if c.side_dim else h
     hl = h.index_select(0, inp.last_idx)
     xn = torch.zeros(hl.shape[0], Dp, dtype=adt, device=h.device)
-    K.sandwich_add_norm(hl, None, None, w.norm, eps, xn, bn=w.norm_b)
+    K.sandwich_add_norm(hl, None, None, w.norm, eps, xn, bn=w.norm_b, layer=ln)
     logits = self._proj(xn, w.lm_head)[:, :c.vocab_size]
     if c.logit_softcap > 0:
       logits = torch.tanh(logits / c.logit_softcap) * c.logit_softcap

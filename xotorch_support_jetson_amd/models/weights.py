@@ -346,6 +346,7 @@ def prepare_for_decode(sw: "ShardWeights", keep_rowmajor: Iterable[str] = (), fp
       if lw.in_w.dtype == torch.bfloat16:
         lw.in_w, lw.out_w, lw.down_w, lw.ff_w = wide(lw.in_w), wide(lw.out_w), wide(lw.down_w), wide(lw.ff_w)
         lw.uq_w, lw.out2_w = wide(lw.uq_w), wide(lw.out2_w)
+        lw.a2_p, lw.g2_p = wide(lw.a2_p), wide(lw.g2_p)
         lw.side_gate_w, lw.side_proj_w, lw.sh_gu_w = wide(lw.side_gate_w), wide(lw.side_proj_w), wide(lw.sh_gu_w)
         lw.ex_up_w, lw.ex_down_w = conv(lw.ex_up_w), conv(lw.ex_down_w)  # experts: shuffled per expert
     if sw.lm_head is not None and sw.lm_head.dtype == torch.bfloat16:
@@ -561,6 +562,11 @@ def needed_files(model_dir: Path, c: ModelConfig, shard: Shard) -> set:
   """Safetensors files that hold this shard's tensors (for the downloader's allow patterns too)."""
   wm = {canonical_name(k): v for k, v in _weight_map(model_dir).items()}
   want = set()
+  if c.is_mixed:  # flat names: l<i>.* of the layers whose tensors this shard's layers use, and the ends
+    mine = {f"l{c.weights_owner(i)}" for i in shard.layers()}
+    ends = ({"embed", "loop", "side"} if shard.is_first_layer() else {"loop", "side"}) | \
+      ({"final", "head", "embed"} if shard.is_last_layer() else set())
+    return {f for name, f in wm.items() if name.split(".")[0] in mine | ends}
   for name, fname in wm.items():
     if (name.startswith("vision_tower.") or name.startswith("multi_modal_projector.")) and shard.is_first_layer():
       want.add(fname)
@@ -758,6 +764,16 @@ class MixedLayerWeights:
   side_proj_w: Optional[torch.Tensor] = None  # [Dn, side padded]
   side_norm: Optional[torch.Tensor] = None  # [D] fp32
   sh_gu_w: Optional[torch.Tensor] = None  # shared gated expert: gate / up rows interleaved by 16 [2 Fs, Dp]
+  # bias-free layer-norm sandwich blocks: `in_w` starts with the convolved channels (channel_delta: [q | k | v | decay rank |
+  # gate rank | beta]; attention beside Mamba-2: [q | k | v | x | B | C | z | dt], q / k rows in pair order), conv_units
+  # says what happens to each run of them behind the convolution (ops.reference.conv_units), conv_norm holds the head norms'
+  # weights; a2_w / g2_w are the second projections of the decay and the output gate, a2_p / g2_p the same padded for the
+  # GEMM kernels (prompts); ff_w of a dense clamped feed-forward has its gate / up rows interleaved by 16
+  conv_units: Optional[torch.Tensor] = None  # [units, 4] int32
+  conv_norm: Optional[torch.Tensor] = None  # fp32
+  g2_w: Optional[torch.Tensor] = None  # [H dv, gate rank]
+  a2_p: Optional[torch.Tensor] = None
+  g2_p: Optional[torch.Tensor] = None
 
   def tensors(self) -> Dict[str, torch.Tensor]:
     return {k: v for k, v in self.__dict__.items() if isinstance(v, torch.Tensor)}
@@ -1103,6 +1119,116 @@ def build_ln_sandwich_layer(spec, get, p: str, D: int, device, dtype) -> MixedLa
   return lw
 
 
+def build_conv_sandwich_layer(spec, get, p: str, D: int, device, dtype) -> MixedLayerWeights:
+  """One bias-free layer-norm sandwich layer (channel-decay delta rule, window attention with kept first tokens, or
+  convolved chunk attention beside a Mamba-2 mixer; clamped gated feed-forward) from `get(name)`."""
+  from ..ops.reference import CONV_RMS, CONV_SILU, CONV_UNIT, CONV_UNIT_SCALED, conv_units
+
+  def dev(t, dt=torch.float32):
+    return t.to(device=device, dtype=dt).contiguous()
+  m = p + "mix."
+  a, r, s, f = spec.wattn, spec.rec, spec.ssd, spec.ffn
+  out2, units, norms = None, [], []
+  if r is not None:
+    blocks = [("rq", get(m + "q")), ("rk", get(m + "k")), ("rv", get(m + "v")), ("ra1", get(m + "a1")), ("rg1", get(m + "g1")),
+              ("rb", get(m + "b"))]
+    conv, conv_b = torch.cat([get(m + n + ".conv") for n in ("q", "k", "v")], 0), None
+    units = [(r.dim, CONV_SILU | CONV_UNIT_SCALED)] * r.kv_heads + [(r.dim, CONV_SILU | CONV_UNIT)] * r.kv_heads + \
+      [(r.heads * r.vdim, CONV_SILU)]
+    out = get(m + "o")
+  else:
+    l = m + "left." if s is not None else m
+    order = _pair_order(a.dim, a.rot_dims) if a.rot_interleaved else torch.arange(a.dim)
+
+    def heads(t):  # rows of whole heads -> rotation pairs as the kernels have them
+      return t.reshape(-1, a.dim, *t.shape[1:])[:, order].reshape(t.shape)
+    blocks = [("q", heads(get(l + "q"))), ("k", heads(get(l + "k"))), ("v", get(l + "v"))]
+    out = get(l + "o")
+    if a.conv:
+      conv = torch.cat([heads(get(l + "q.conv")), heads(get(l + "k.conv")), get(l + "v.conv")], 0)
+      conv_b = torch.zeros(conv.shape[0])
+      norms = [heads(get(l + "q.norm")), heads(get(l + "k.norm"))] if a.head_norm else []
+      kind = CONV_RMS if a.head_norm else 0
+      units = [(a.dim, kind, 0)] * a.heads + [(a.dim, kind, a.dim)] * a.kv_heads + [(a.kv_heads * a.vdim, 0)]
+    if s is not None:
+      n = m + "right."
+      w, inner, C = get(n + "in"), s.inner, s.conv_channels
+      blocks += [("xbc", w[inner:inner + C]), ("z", w[:inner]), ("dt", w[inner + C:])]
+      taps = max(a.conv, s.conv)  # (the shorter filter starts with zeros)
+      conv = torch.cat([torch.nn.functional.pad(t, (taps - t.shape[1], 0)) for t in (conv, get(n + "conv"))], 0)
+      conv_b = torch.cat([conv_b, get(n + "conv.b")])
+      units = units + [(C, CONV_SILU)]
+      out2 = get(n + "o")
+  in_w, cols = _fused_rows(blocks, D)
+  lw = MixedLayerWeights(spec, dev(in_w, dtype), cols, dev(_pad2(out, _up(D, 64), _up(out.shape[1], 128)), dtype),
+                         {"mix": (0, out.shape[1])})
+  for n in ("norm1", "norm1b") + (("norm2", "norm2b") if f is not None else ()):
+    setattr(lw, n, dev(get(p + n)))
+  if units:
+    lw.conv_w, lw.conv_b = dev(conv), dev(conv_b) if conv_b is not None else None
+    lw.conv_units = conv_units(units, conv.shape[0]).to(device)
+    lw.conv_norm = dev(torch.cat(norms)) if norms else None
+  if r is not None:
+    lw.A_log, lw.dt_bias = dev(get(m + "A_log")), dev(get(m + "dt_bias"))
+    lw.rec_norm = dev(get(m + "norm").repeat(r.heads))
+    a2, g2 = get(m + "a2"), get(m + "g2")
+    lw.a2_w, lw.g2_w = dev(a2, dtype), dev(g2, dtype)
+    if dtype == torch.bfloat16:
+      lw.a2_p, lw.g2_p = (dev(_pad2(t, _up(t.shape[0], 64), _up(t.shape[1], 128)), dtype) for t in (a2, g2))
+  if s is not None:
+    lw.out2_w = dev(_pad2(out2, _up(D, 64), _up(out2.shape[1], 128)), dtype)
+    lw.mix_cols["mix2"] = (0, out2.shape[1])
+    lw.pair_w = dev(torch.stack([get(m + "left.out"), get(m + "right.out")]))
+    n = m + "right."
+    lw.A_log, lw.dt_bias, lw.skip_d, lw.ssd_norm = (dev(get(n + k)) for k in ("A_log", "dt_bias", "D", "norm"))
+  if f is not None:
+    q, Fp, Dp = p + "mlp.", _up(f.ff, 128), _up(D, 128)
+    lw.ff_w = dev(interleave_gate_up(_pad2(get(q + "gate"), Fp, Dp), _pad2(get(q + "up"), Fp, Dp)), dtype)
+    lw.down_w = dev(_pad2(get(q + "down"), _up(D, 64), Fp), dtype)
+  return lw
+
+
+def conv_sandwich_tensor_shapes(c: ModelConfig) -> Dict[str, tuple]:
+  """Name -> shape of every tensor of a bias-free layer-norm sandwich checkpoint (Zepalorn); layers that share another's
+  tensors have none, the LM head is the embedding table."""
+  D, out = c.hidden_size, {}
+  out["embed"] = (c.vocab_size, D)
+  for i, s in enumerate(c.layer_specs):
+    if c.weights_owner(i) != i:
+      continue
+    p, m, a, r, d, f = f"l{i}.", f"l{i}.mix.", s.wattn, s.rec, s.ssd, s.ffn
+    for n in ("norm1", "norm1b") + (("norm2", "norm2b") if f is not None else ()):
+      out[p + n] = (D,)
+    if r is not None:
+      for n, rows in (("q", r.kv_heads * r.dim), ("k", r.kv_heads * r.dim), ("v", r.heads * r.vdim)):
+        out[m + n], out[m + n + ".conv"] = (rows, D), (rows, r.conv)
+      out[m + "b"], out[m + "A_log"], out[m + "norm"] = (r.heads, D), (r.heads,), (r.vdim,)
+      ra, rg = r.rank or 8, r.gate_rank or 8
+      out[m + "a1"], out[m + "a2"], out[m + "dt_bias"] = (ra, D), (r.heads * r.dim, ra), (r.heads * r.dim,)
+      out[m + "g1"], out[m + "g2"], out[m + "o"] = (rg, D), (r.heads * r.vdim, rg), (D, r.heads * r.vdim)
+    if a is not None:
+      l = m + "left." if d is not None else m
+      for n, rows in (("q", a.heads * a.dim), ("k", a.kv_heads * a.dim), ("v", a.kv_heads * a.vdim)):
+        out[l + n] = (rows, D)
+        if a.head_norm and n != "v":
+          out[l + n + ".norm"] = (a.dim,)
+        if a.conv:
+          out[l + n + ".conv"] = (rows, a.conv)
+      out[l + "o"] = (D, a.heads * a.vdim)
+    if d is not None:
+      n = m + "right."
+      out[n + "in"] = (2 * d.inner + 2 * d.groups * d.state + d.heads, D)
+      out[n + "conv"], out[n + "conv.b"] = (d.conv_channels, d.conv), (d.conv_channels,)
+      out[n + "dt_bias"], out[n + "A_log"], out[n + "D"] = (d.heads,), (d.heads,), (d.heads,)
+      out[n + "norm"], out[n + "o"] = (d.inner,), (D, d.inner)
+      out[m + "left.out"], out[m + "right.out"] = (D,), (D,)
+    if f is not None:
+      q = p + "mlp."
+      out[q + "gate"], out[q + "up"], out[q + "down"] = (f.ff, D), (f.ff, D), (D, f.ff)
+  out["final.norm"] = (D,)
+  return out
+
+
 def ln_sandwich_tensor_shapes(c: ModelConfig) -> Dict[str, tuple]:
   """Name -> shape of every tensor of a layer-norm sandwich checkpoint (Kopalorn)."""
   D, out = c.hidden_size, {}
@@ -1225,6 +1351,8 @@ def mixed_tensor_shapes(c: ModelConfig) -> Dict[str, tuple]:
     return postln_tensor_shapes(c)
   if c.block == "sandwich" and not c.input_norm:
     return outnorm_tensor_shapes(c)
+  if c.block == "sandwich" and not c.norm_bias:
+    return conv_sandwich_tensor_shapes(c)
   if c.block == "sandwich":
     return ln_sandwich_tensor_shapes(c) if c.norm_kind == "layer" else sandwich_tensor_shapes(c)
   D, out = c.hidden_size, {}
@@ -1263,6 +1391,10 @@ def random_mixed_tensors(c: ModelConfig, seed: int = 0) -> Dict[str, torch.Tenso
     leaf = name.split(".")[-1]
     if name.endswith(".conv"):
       t = torch.randn(shape, generator=g) * 0.5
+    elif not c.norm_bias and leaf == "b" and len(shape) == 1:  # convolution bias
+      t = torch.randn(shape, generator=g) * 0.5
+    elif not c.norm_bias and leaf == "b":  # (a projection)
+      t = torch.randn(shape, generator=g) / shape[-1] ** 0.5
     elif c.norm_kind == "layer" and leaf in ("b", "correction", "out", "lq1", "lk1", "lq2", "lk2"):
       # norm biases, projection biases, gate biases (forget gates mostly open), the router's correction (large enough to
       # change the choice), the lambda vectors
@@ -1303,12 +1435,18 @@ def mixed_weights(c: ModelConfig, shard: Shard, get, device, dtype) -> ShardWeig
   sw = ShardWeights(c, shard)
   D = c.hidden_size
   build = {"postln": build_postln_layer, "sandwich": build_sandwich_layer}.get(c.block, build_mixed_layer)
-  if c.block == "sandwich" and c.norm_kind == "layer":
+  if c.block == "sandwich" and not c.norm_bias:
+    build = build_conv_sandwich_layer
+  elif c.block == "sandwich" and c.norm_kind == "layer":
     build = build_ln_sandwich_layer
   elif c.block == "sandwich" and not c.input_norm:
     build = build_outnorm_layer
+  owners: Dict[int, MixedLayerWeights] = {}  # (layers that share tensors share them on the device, too)
   for i in shard.layers():
-    sw.layers[i] = build(c.layer_specs[i], get, f"l{i}.", D, device, dtype)
+    o = c.weights_owner(i)
+    if o not in owners:
+      owners[o] = build(c.layer_specs[o], get, f"l{o}.", D, device, dtype)
+    sw.layers[i] = owners[o]
   if shard.is_first_layer():
     # gathered into the fp32 residual; a model that scales its embedding output gathers from the scaled table
     sw.embed = (get("embed") * c.embed_scale).to(device=device, dtype=torch.float32).contiguous()
@@ -1326,7 +1464,7 @@ def mixed_weights(c: ModelConfig, shard: Shard, get, device, dtype) -> ShardWeig
     sw.loop_step = get("loop.step").to(device=device, dtype=torch.float32).contiguous()
   if shard.is_last_layer():
     sw.norm = get("final.norm").reshape(-1).to(device=device, dtype=torch.float32)
-    if c.norm_kind == "layer":
+    if c.norm_kind == "layer" and c.norm_bias:
       sw.norm_b = get("final.norm.b").reshape(-1).to(device=device, dtype=torch.float32)
     head = torch.zeros(_up(c.vocab_size, 64), _up(D, 128))
     head[:c.vocab_size, :D] = get("embed" if c.tie_word_embeddings and c.is_mixed else "head")
@@ -1349,9 +1487,10 @@ def load_mixed_weights(model_dir: Path, c: ModelConfig, shard: Shard, device, dt
       handles[f] = safe_open(str(Path(model_dir) / f), framework="pt")
     return handles[f].get_tensor(name).float()
   want = mixed_tensor_shapes(c)
+  mine = {c.weights_owner(i) for i in shard.layers()}
   for name, shape in want.items():
-    if name.split(".")[0] in ("embed", "final", "head", "loop", "side") or int(name.split(".")[0][1:]) in shard.layers():
-      got = tuple(get(name).shape) if not name.endswith((".a1", ".a2")) else None
+    if name.split(".")[0] in ("embed", "final", "head", "loop", "side") or int(name.split(".")[0][1:]) in mine:
+      got = tuple(get(name).shape) if not name.endswith((".a1", ".a2", ".g1", ".g2")) else None
       if name == "loop.step" and got is not None and got[1:] == tuple(shape)[1:] and got[0] >= shape[0]:
         continue
       if got is not None and got != tuple(shape):

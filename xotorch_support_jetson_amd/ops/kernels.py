@@ -488,14 +488,39 @@ def gla_prep(P, a1_off: int, a2, a2_b, tau: float, decay) -> None:
   _mix("gla_prep", _gpu(P))(P, int(a1_off), a2, a2_b, float(tau), decay)
 
 
-def linear_recurrence(q, k, v, decay, beta, q_scale: float, state, state_slots, cu_q, out) -> None:
+conv_units = ref.conv_units
+
+
+def conv_prep(P, x_off: int, conv_w, conv_b, units, norm_w, conv_state, state_slots, cu_q, eps: float, out, max_qlen: int = 0) -> None:
+  """Causal convolutions over time of the channels P[:, x_off : +C] (conv_w [C, taps], last column the current token; conv_b
+  [C] or None) -> out [T, C] fp32, then per unit (conv_units) SiLU and a unit length or a weighted RMS norm (norm_w).  The
+  inputs before the step come from conv_state [slots, taps - 1, C], which takes the step's last ones.  max_qlen 1: every
+  sequence has one new token (the state is updated in the same launch)."""
+  _mix("conv_prep", _gpu(P))(P, int(x_off), conv_w, conv_b, units, norm_w, conv_state, state_slots, cu_q, float(eps), out,
+                             int(max_qlen))
+
+
+def recurrence_gates(P, b_off: int, beta, a1_off: int, a2, dt_bias, A_log, decay, g1_off: int, g2, gate, za=None) -> None:
+  """Gates of the channel-decay delta rule: beta [T, H] = sigmoid(P[:, b_off : +H]); decay [T, H d] = exp(-exp(A_log[head])
+  softplus(a2 P[:, a1_off : +rank] + dt_bias)) (za [T, >= H d]: that product, already made); gate [T, H dv] (or None) =
+  g2 P[:, g1_off : +rank], without its sigmoid."""
+  _mix("recurrence_gates", _gpu(P))(P, int(b_off), beta, int(a1_off), a2, dt_bias, A_log, decay, int(g1_off), g2, gate, za)
+
+
+def ssd_steps(P, dt_off: int, dt_bias, A_log, dt, decay) -> None:
+  """dt [T, H] = softplus(P[:, dt_off : +H] + dt_bias), decay [T, H] = exp(-exp(A_log) dt)."""
+  _mix("ssd_steps", _gpu(P))(P, int(dt_off), dt_bias, A_log, dt, decay)
+
+
+def linear_recurrence(q, k, v, decay, beta, q_scale: float, state, state_slots, cu_q, out, plain: bool = False) -> None:
   """Per sequence and value head, token by token on the fp32 state, stored S^T [slots, H, dv, d] (updated in place):
-  beta given (delta rule, decay [T, H]):  S *= g; u = beta (v - S^T k); S += k u^T; o = S^T q
+  beta given (delta rule, decay [T, H], or [T, H d] per key channel):  S *= g; u = beta (v - S^T k); S += k u^T; o = S^T q
+  (plain: beta scales the input of the plain write instead, S = g S + k (beta v)^T)
   else (decay [T, H d] per key channel, [T, H] per head, or a 1-D [H]: fixed per head):  S = diag(a) S + k v^T; o = S^T q.
   q is scaled by q_scale.
   A state with one value channel more than v has (decay [T, H], beta [T, H] an input scale): S = g S + k (beta [v | 1])^T,
   the last channel being a normaliser n = g n + beta k; out [T, H (dv + 1)] then ends each head with n . q."""
-  _mix("linear_recurrence", _gpu(q))(q, k, v, decay, beta, float(q_scale), state, state_slots, cu_q, out)
+  _mix("linear_recurrence", _gpu(q))(q, k, v, decay, beta, float(q_scale), state, state_slots, cu_q, out, bool(plain))
 
 
 def gated_rmsnorm(o, w, P, g_off: int, eps: float, out_scale: float, out) -> None:
@@ -532,12 +557,15 @@ def kv_pool_update(k_cache, v_cache, kp, vp, block_tables, cu_q, ctx_lens, pool:
 
 
 def attn_window_pool(q, k_cache, v_cache, kp, vp, block_tables, cu_q, ctx_lens, sink, scale: float, window: int,
-                     pool: int, out, max_qlen: int = 0, chunk: int = 0) -> None:
+                     pool: int, out, max_qlen: int = 0, chunk: int = 0, keep: int = 0, softcap: float = 0.0) -> None:
   """out [T, H dv] = softmax attention of each new token over the tokens at most window - 1 places back (window 0:
-  all) and, with chunk > 0, in its own block of `chunk` positions (counted from the sequence's start), the pooled blocks that end at or before position - window (pool 0: none), and the per-head sink logit.  Key
-  head g reads value head g / (G / Gv) (the caches' head counts); out may be fp32 beside bf16 caches."""
+  all) and, with chunk > 0, in its own block of `chunk` positions (counted from the sequence's start), the sequence's first
+  `keep` tokens wherever the query is (no pooled blocks then), the pooled blocks that end at or before position - window (pool 0: none), and the per-head sink logit.  Key
+  head g reads value head g / (G / Gv) (the caches' head counts); out may be fp32 beside bf16 caches.  softcap > 0:
+  scores are softcap * tanh(score / softcap)."""
   _mix("attn_window_pool", _gpu(q))(q, k_cache, v_cache, kp, vp, block_tables, cu_q, ctx_lens, sink, float(scale),
-                                    int(window), int(pool), out, int(max_qlen) or int(q.shape[0]), int(chunk))
+                                    int(window), int(pool), out, int(max_qlen) or int(q.shape[0]), int(chunk), int(keep),
+                                    float(softcap))
 
 
 def ssd_prep(P, x_off: int, dt_off: int, conv_w, conv_b, conv_state, state_slots, cu_q, A_log, dt_bias, H: int, dv: int,
@@ -571,12 +599,12 @@ def moe_weighted_sum(y, slot_of, topw, k: int, sh_y, P, shg_off: int, out, split
 
 
 # ------------------------------------------------------------------ sandwich blocks (csrc/latent.hip)
-def sandwich_add_norm(x, y, wb, wn, eps: float, out=None, bb=None, bn=None, mult: float = 1.0, yb=None) -> None:
+def sandwich_add_norm(x, y, wb, wn, eps: float, out=None, bb=None, bn=None, mult: float = 1.0, yb=None, layer: bool = False) -> None:
   """fp32 stream rows x [T, D] += mult * norm(y + yb) * wb in place (y None: nothing is added; yb: one fp32 number per
   column, or None); with wn, out[:, :D] = norm(x) * wn in out's dtype (the next GEMM's operand), with out alone out[:, :D] =
-  x.  norm = division by the RMS, or, with the biases bb / bn, the
-  layer norm (v - mean) / sqrt(var + eps) * w + b."""
-  _mix("sandwich_add_norm", _gpu(x))(x, y, wb, wn, float(eps), out, bb, bn, float(mult), yb)
+  x.  norm = division by the RMS, or, with the biases bb / bn or
+  with `layer`, the layer norm (v - mean) / sqrt(var + eps) * w (+ b)."""
+  _mix("sandwich_add_norm", _gpu(x))(x, y, wb, wn, float(eps), out, bb, bn, float(mult), yb, bool(layer))
 
 
 def latent_kv_store(P, ckv_off: int, R: int, dr: int, kv_norm, q_off: int, q_rank: int, q_norm, eps: float, rot_dims: int,

@@ -316,7 +316,73 @@ def gla_prep(P, a1_off, a2, a2_b, tau, decay):
   decay.copy_(torch.exp(F.logsigmoid(z) / tau))
 
 
-def linear_recurrence(q, k, v, decay, beta, q_scale, state, state_slots, cu_q, out):
+# what a unit of conv_units does behind its convolution: SiLU, then one of: division by sqrt(sum x^2 + 1e-6) (and times
+# n^-1/2), or a weighted RMS norm
+CONV_SILU, CONV_UNIT, CONV_UNIT_SCALED, CONV_RMS = 1, 2, 4, 8
+CONV_MAX = 256  # channels of a unit
+
+
+def conv_units(parts, C: int) -> torch.Tensor:
+  """[(channels, kind[, first norm weight])] over consecutive channels -> int32 [units, 4] (first channel, channels, kind,
+  first norm weight); runs without a norm are cut into pieces of CONV_MAX channels."""
+  rows, c0 = [], 0
+  for part in parts:
+    n, kind, off = int(part[0]), int(part[1]), int(part[2]) if len(part) > 2 else 0
+    if kind & ~CONV_SILU:
+      if n > CONV_MAX:
+        raise ValueError(f"a normed head of {n} channels (at most {CONV_MAX})")
+      rows.append((c0, n, kind, off))
+    else:
+      rows += [(c0 + i, min(CONV_MAX, n - i), kind, 0) for i in range(0, n, CONV_MAX)]
+    c0 += n
+  if c0 != C:
+    raise ValueError(f"the units cover {c0} of {C} channels")
+  return torch.tensor(rows, dtype=torch.int32)
+
+
+def conv_prep(P, x_off, conv_w, conv_b, units, norm_w, conv_state, state_slots, cu_q, eps, out, max_qlen=0):
+  C, taps = conv_w.shape
+  for b in range(state_slots.numel()):
+    t0, t1, slot = int(cu_q[b]), int(cu_q[b + 1]), int(state_slots[b])
+    if slot < 0 or t1 == t0:
+      continue
+    x = torch.cat([conv_state[slot], P[t0:t1, x_off:x_off + C].float()], 0)
+    y = sum(conv_w[:, j].float() * x[j:j + t1 - t0] for j in range(taps))
+    if conv_b is not None:
+      y = y + conv_b.float()
+    if taps > 1:
+      conv_state[slot] = x[x.shape[0] - (taps - 1):]
+    for c0, n, kind, off in units.tolist():
+      u = y[:, c0:c0 + n]
+      if kind & CONV_SILU:
+        u = F.silu(u)
+      if kind & (CONV_UNIT | CONV_UNIT_SCALED):
+        u = u / torch.sqrt(u.pow(2).sum(-1, keepdim=True) + 1e-6)
+        if kind & CONV_UNIT_SCALED:
+          u = u * n ** -0.5
+      elif kind & CONV_RMS:
+        u = u / torch.sqrt(u.pow(2).mean(-1, keepdim=True) + eps) * norm_w[off:off + n].float()
+      out[t0:t1, c0:c0 + n] = u
+
+
+def recurrence_gates(P, b_off, beta, a1_off, a2, dt_bias, A_log, decay, g1_off, g2, gate, za=None):
+  H = A_log.numel()
+  beta.copy_(torch.sigmoid(P[:, b_off:b_off + H].float()))
+  HD = dt_bias.numel()
+  z = za[:, :HD].float() if za is not None else P[:, a1_off:a1_off + a2.shape[1]].float() @ a2.float().t()
+  rate = torch.exp(A_log.float()).repeat_interleave(HD // H)
+  decay.copy_(torch.exp(-rate * F.softplus(z + dt_bias.float())))
+  if gate is not None:
+    gate.copy_(P[:, g1_off:g1_off + g2.shape[1]].float() @ g2.float().t())
+
+
+def ssd_steps(P, dt_off, dt_bias, A_log, dt, decay):
+  H = A_log.numel()
+  dt.copy_(F.softplus(P[:, dt_off:dt_off + H].float() + dt_bias.float()))
+  decay.copy_(torch.exp(-torch.exp(A_log.float()) * dt))
+
+
+def linear_recurrence(q, k, v, decay, beta, q_scale, state, state_slots, cu_q, out, plain=False):
   _, H, dv, d = state.shape  # stored transposed: S^T [dv, d] per head
   G = q.shape[1] // d
   rep = H // G
@@ -338,8 +404,11 @@ def linear_recurrence(q, k, v, decay, beta, q_scale, state, state_slots, cu_q, o
         vt = torch.cat([vt, torch.ones(H, 1)], 1) * beta[t].reshape(H, 1)
         S *= decay[t].reshape(H, 1, 1)
         S += kt[:, :, None] * vt[:, None, :]
-      elif beta is not None:
+      elif plain and beta is not None:  # one decay and one input scale per head
         S *= decay[t].reshape(H, 1, 1)
+        S += kt[:, :, None] * (beta[t].reshape(H, 1) * vt)[:, None, :]
+      elif beta is not None:
+        S *= decay[t].reshape(H, -1, 1)  # (one per head, or one per head and key channel)
         u = beta[t].reshape(H, 1) * (vt - torch.einsum("hdv,hd->hv", S, kt))
         S += kt[:, :, None] * u[:, None, :]
       elif decay.numel() == decay.shape[0] * H:  # one decay per head
@@ -432,7 +501,7 @@ def kv_pool_update(k_cache, v_cache, kp, vp, block_tables, cu_q, ctx_lens, pool,
 
 
 def attn_window_pool(q, k_cache, v_cache, kp, vp, block_tables, cu_q, ctx_lens, sink, scale, window, pool, out, max_qlen=0,
-                     chunk=0):
+                     chunk=0, keep=0, softcap=0.0):
   T, H, d = q.shape
   G, dv = k_cache.shape[1], v_cache.shape[2]
   rep = H // G
@@ -455,13 +524,15 @@ def attn_window_pool(q, k_cache, v_cache, kp, vp, block_tables, cu_q, ctx_lens, 
     kpos = torch.arange(n)[None, :]
     vis = kpos <= qpos
     if window:
-      vis = vis & (qpos - kpos < window)
+      vis = vis & ((qpos - kpos < window) | (kpos < keep))
     if chunk:
-      vis = vis & (qpos // chunk == kpos // chunk)
+      vis = vis & ((qpos // chunk == kpos // chunk) | (kpos < keep))
     if nb:
       last = torch.arange(nb)[None, :] * pool + pool - 1
       vis = torch.cat([vis, last <= qpos - window], 1)
     s = torch.einsum("shd,thd->hst", q[t0:t1].float(), k.repeat_interleave(rep, 1)) * scale
+    if softcap:
+      s = softcap * torch.tanh(s / softcap)
     s = s.masked_fill(~vis[None], float("-inf"))
     if sink is not None:
       s = torch.cat([s, sink.float()[:, None, None].expand(H, t1 - t0, 1)], -1)
@@ -522,16 +593,16 @@ def moe_weighted_sum(y, slot_of, topw, k, sh_y, P, shg_off, out, splits=1):
 
 # ------------------------------------------------------------------ sandwich blocks: latent attention, gated feed-forwards
 # Torch twins of csrc/latent.hip.
-def sandwich_add_norm(x, y, wb, wn, eps, out, bb=None, bn=None, mult=1.0, yb=None):
+def sandwich_add_norm(x, y, wb, wn, eps, out, bb=None, bn=None, mult=1.0, yb=None, layer=False):
   """x += mult * norm(y + yb) in place (y None: nothing is added); with wn, out[:, :D] = norm(x), with out alone = x.  norm(v) = v / rms(v) * w,
-  or with a bias (bb / bn) the layer norm (v - mean) / sqrt(var + eps) * w + b."""
+  or (layer, or with a bias bb / bn) the layer norm (v - mean) / sqrt(var + eps) * w (+ b)."""
   D = x.shape[1]
 
   def norm(v, w, b):
-    if b is None:
+    if b is None and not layer:
       return v / torch.sqrt(v.pow(2).mean(-1, keepdim=True) + eps) * w.float()
     c = v - v.mean(-1, keepdim=True)
-    return c / torch.sqrt(c.pow(2).mean(-1, keepdim=True) + eps) * w.float() + b.float()
+    return c / torch.sqrt(c.pow(2).mean(-1, keepdim=True) + eps) * w.float() + (b.float() if b is not None else 0.0)
   if y is not None:
     x += mult * norm(y[:, :D].float() + (yb.float() if yb is not None else 0.0), wb, bb)
   if out is not None:

@@ -52,9 +52,7 @@ def inv_frequencies(head_dim: int, theta: float, scaling: dict | None) -> torch.
     if scaling.get("truncate", True):
       lo, hi = math.floor(lo), math.ceil(hi)
     lo, hi = max(lo, 0), min(hi, dim - 1)
-    if lo == hi:
-      hi += 0.001
-    ramp = ((torch.arange(dim // 2, dtype=torch.float64) - lo) / (hi - lo)).clamp(0, 1)
+    ramp = ((torch.arange(dim // 2, dtype=torch.float64) - lo) / max(hi - lo, 0.001)).clamp(0, 1)
     extrap = 1.0 - ramp
     pos_freqs = base ** (torch.arange(0, dim, 2, dtype=torch.float64) / dim)
     return (1.0 / (factor * pos_freqs)) * (1 - extrap) + (1.0 / pos_freqs) * extrap
