@@ -237,11 +237,36 @@ def chunk_configs(name: str):
   return chunked, mixtral
 
 
+def delta_configs(name: str):
+  """(Zepalorn-design config, the closest existing model: the Tarepel-design stack of equal width, depth and feed-forward,
+  whose gated delta rule, chunk attention and dense gated feed-forward are its nearest kin).  Zepalorn layers in turn: delta
+  rule with channel decays (a head of the head size per attention head, decay and gate rank 128); sliding-window attention
+  with 4 kept tokens; convolved chunk attention with capped scores beside a Mamba-2 mixer of the width (heads of 64, state
+  128); the delta rule again.  No shared tensors (equal parameter reads on both sides)."""
+  from xotorch_support_jetson_amd.models.config import from_hf_config
+  z = MIXER_SIZES[name]
+  H, G, d, chunk, rot = z["attn"]
+  W = z["width"]
+  mlp = {"kind": "dense", "ff": z["ff"], "limit": 7.0}
+  yarn = {"base": 1e6, "dims": rot, "scaling": {"factor": 8.0, "original": 8192, "fast": 32.0, "slow": 1.0}}
+  att = {"heads": H, "kv_heads": G, "dim": d, "vdim": d, "scale": d ** -0.5, "rot": yarn}
+  kinds = [
+    {"type": "channel_delta", "mlp": mlp, "mixer": {"heads": H, "kv_heads": H, "dim": d, "vdim": d, "conv": 4, "rank": 128, "gate_rank": 128}},
+    {"type": "attention", "mlp": mlp, "mixer": dict(att, mask={"size": chunk, "keep_first": 4})},
+    {"type": "parallel", "mlp": mlp,
+     "mixer": {"left": dict(att, conv=4, mask={"size": chunk}, softcap=30.0),
+               "right": {"heads": W // 64, "vdim": 64, "state": 128, "groups": 8, "conv": 4, "norm_groups": 8}}},
+  ]
+  delta = from_hf_config({"architecture": "Zepalorn", "vocab": 32000, "width": W, "norm": {"eps": 1e-5}, "embedding": {"scale": W ** 0.5},
+                          "layers": [kinds[(0, 1, 2, 0)[i % 4]] for i in range(z["layers"])]})
+  return delta, mixer_configs(name)[0]
+
+
 def bench_mixers(args, sizes=None, kinds=("tarepel", "llama"), configs=mixer_configs,
                  what="Tarepel-design layers beside a Llama-style stack of equal size"):
   """Prefill and decode throughput of mixed-layer designs at sizes like a real model's (random weights), beside
   the closest existing model (--mixers: Tarepel beside a Llama-style stack of equal width, depth, heads and
-  feed-forward; --hybrid, --latent, --memory, --chunked: see their *_configs) on the same runner: one prefill step of --mixer-batch prompts of
+  feed-forward; --hybrid, --latent, --memory, --chunked, --delta: see their *_configs) on the same runner: one prefill step of --mixer-batch prompts of
   --prompt-len tokens, then HIP-graph decode steps at that context.  One JSON line; not the headline metric."""
   from xotorch_support_jetson_amd.inference.shard import Shard
   from xotorch_support_jetson_amd.runtime.runner import ShardRunner
@@ -325,8 +350,12 @@ def main():
   ap.add_argument("--chunked", default=None, metavar="SIZES",
                   help="instead of the headline: Torinex-design layers (chunk-local attention with projection norms, relu^2 "
                        "and clamped-expert feed-forwards, side inputs) beside a Mixtral-style stack at the named sizes; one GPU")
+  ap.add_argument("--delta", default=None, metavar="SIZES",
+                  help="instead of the headline: Zepalorn-design layers (delta rule with channel decays, window attention with "
+                       "kept tokens, convolved chunk attention beside Mamba-2) beside the Tarepel-design stack at the named sizes; "
+                       "one GPU")
   ap.add_argument("--mixer-batch", type=int, default=16,
-                  help="--mixers / --hybrid / --latent / --memory / --chunked: sequences per step")
+                  help="--mixers / --hybrid / --latent / --memory / --chunked / --delta: sequences per step")
   args = ap.parse_args()
   os.environ["XOT_WEIGHT_DTYPE"] = args.weight_dtype
   if args.mixers:
@@ -346,6 +375,10 @@ def main():
   if args.chunked:
     return bench_mixers(args, args.chunked, ("torinex", "mixtral"), chunk_configs,
                         "Torinex-design layers beside a Mixtral-style stack of equal size")
+
+  if args.delta:
+    return bench_mixers(args, args.delta, ("zepalorn", "tarepel"), delta_configs,
+                        "Zepalorn-design layers beside a Tarepel-design stack of equal size")
 
   from xotorch_support_jetson_amd.models.config import preset
   from xotorch_support_jetson_amd.parallel.comm import P2PTransport, init_distributed

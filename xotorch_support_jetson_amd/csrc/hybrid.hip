@@ -828,14 +828,14 @@ __global__ void conv_tail_store_k(const float* __restrict__ P, int ldp, int x_of
 // workgroup = (token, norm group)
 template <typename AT>
 __global__ void ssd_gate_norm_k(const float* __restrict__ o, const float* __restrict__ xbc, int C,
-                                const float* __restrict__ skip, const float* __restrict__ P, int ldp, int z_off,
-                                const float* __restrict__ w, float eps, AT* __restrict__ out, int ldo, int inner, int dv,
-                                int gs) {
+                                const float* __restrict__ skip, const float* __restrict__ P, int ldp, int S, int64_t ss_,
+                                int z_off, const float* __restrict__ w, float eps, AT* __restrict__ out, int ldo, int inner,
+                                int dv, int gs) {
   __shared__ float red[16];
   const int64_t t = blockIdx.x;
   const int c0 = blockIdx.y * gs;
   auto val = [&](int c) {
-    return (o[t * inner + c] + skip[c / dv] * xbc[t * C + c]) * siluf_(P[t * ldp + z_off + c]);
+    return (o[t * inner + c] + skip[c / dv] * xbc[t * C + c]) * siluf_(slab1(P + t * ldp + z_off + c, S, ss_));
   };
   float ss = 0.0f;
   for (int i = threadIdx.x; i < gs; i += blockDim.x) {
@@ -845,6 +845,43 @@ __global__ void ssd_gate_norm_k(const float* __restrict__ o, const float* __rest
   ss = block_sum(ss, red);
   const float k = 1.0f / sqrtf(ss / (float)gs + eps);
   for (int i = threadIdx.x; i < gs; i += blockDim.x) stf(out + t * ldo + c0 + i, val(c0 + i) * k * w[c0 + i]);
+}
+
+// Groups of at most 256 R values in whole vectors of four (as are heads and column offsets): a wave per (token, group), four
+// groups a workgroup, the group's values in registers between the sum and the write.
+template <typename AT, int R>
+__global__ __launch_bounds__(256) void ssd_gate_norm_wave_k(const float* __restrict__ o, const float* __restrict__ xbc, int C,
+                                                            const float* __restrict__ skip, const float* __restrict__ P, int ldp,
+                                                            int S, int64_t ss_, int z_off, const float* __restrict__ w, float eps,
+                                                            AT* __restrict__ out, int ldo, int inner, int dv, int gs,
+                                                            int64_t total) {
+  const int64_t id = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
+  if (id >= total) return;  // (wave-uniform; no workgroup barrier below)
+  const int groups = inner / gs, lane = threadIdx.x & 63;
+  const int64_t t = id / groups;
+  const int c0 = (int)(id - t * groups) * gs;
+  auto ld = [](const float* p) { return *reinterpret_cast<const f32x4*>(p); };
+  f32x4 y[R];
+  float ss = 0.0f;
+#pragma unroll
+  for (int r = 0; r < R; ++r) {
+    const int i = 4 * (lane + 64 * r), c = c0 + i;
+    y[r] = f32x4{0.f, 0.f, 0.f, 0.f};
+    if (i >= gs) continue;
+    const f32x4 z = slab4(P + t * ldp + z_off + c, S, ss_);
+    y[r] = ld(o + t * inner + c) + skip[c / dv] * ld(xbc + t * C + c);
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      y[r][e] *= siluf_(z[e]);
+      ss += y[r][e] * y[r][e];
+    }
+  }
+  const float k = 1.0f / sqrtf(wave_sum(ss) / (float)gs + eps);
+#pragma unroll
+  for (int r = 0; r < R; ++r) {
+    const int i = 4 * (lane + 64 * r);
+    if (i < gs) st4(out + t * ldo + c0 + i, y[r] * k * ld(w + c0 + i));
+  }
 }
 
 // ------------------------------------------------------------------ PolyNorm
@@ -1305,27 +1342,39 @@ void ssd_gate_norm(const at::Tensor& o, const at::Tensor& xbc, const at::Tensor&
   f32c(o, "o");
   f32c(skip_d, "skip_d");
   f32c(w, "w");
-  const int ldp = ld_of(P, "P");
+  const Slabs p = slabs_of(P, "P");
   const int64_t C = ld_of(xbc, "xbc");  // (the row stride: xbc may be the last columns of wider rows)
   MCHECK(o.dim() == 2, "o must be [T, inner]");
   const int64_t T = o.size(0), inner = o.size(1), H = skip_d.numel();
   if (T == 0) return;
-  MCHECK(P.size(0) == T && xbc.size(0) == T && xbc.size(1) >= inner && H > 0 && inner % H == 0 && w.numel() == inner && groups >= 1 &&
+  MCHECK(p.T == T && xbc.size(0) == T && xbc.size(1) >= inner && H > 0 && inner % H == 0 && w.numel() == inner && groups >= 1 &&
              inner % groups == 0,
          "ssd_gate_norm: shape mismatch");
-  cols_ok(P, z_off, inner, "gate");
+  cols_ok(p, z_off, inner, "gate");
   const int ldo = act_ld_min(out, T, inner, "out");
+  const int64_t gs = inner / groups, dv = inner / H;
+  auto al = [](const at::Tensor& t) { return (reinterpret_cast<uintptr_t>(t.data_ptr()) & 15) == 0; };
+  const bool bf = out.scalar_type() == at::kBFloat16;
+#define SGN_ARGS(AT)                                                                                                         \
+  o.data_ptr<float>(), xbc.data_ptr<float>(), (int)C, skip_d.data_ptr<float>(), p.p, p.ld, p.S, p.ss, (int)z_off,            \
+      w.data_ptr<float>(), (float)eps, (AT*)out.data_ptr(), ldo, (int)inner, (int)dv, (int)gs
+  if (p.vec && z_off % 4 == 0 && gs % 4 == 0 && dv % 4 == 0 && C % 4 == 0 && ldo % 4 == 0 && gs <= 1024 && al(o) && al(xbc) && al(w) &&
+      al(out)) {
+    const int64_t total = T * groups;
+    const unsigned grid = (unsigned)((total + 3) / 4);
+#define SGN_GO(AT, R) ssd_gate_norm_wave_k<AT, R><<<grid, 256, 0, stream()>>>(SGN_ARGS(AT), total)
+    if (gs <= 256) {
+      if (bf) SGN_GO(uint16_t, 1); else SGN_GO(float, 1);
+    } else {
+      if (bf) SGN_GO(uint16_t, 4); else SGN_GO(float, 4);
+    }
+#undef SGN_GO
+    return;
+  }
   const dim3 grid((unsigned)T, (unsigned)groups);
-  if (out.scalar_type() == at::kBFloat16)
-    ssd_gate_norm_k<uint16_t><<<grid, 256, 0, stream()>>>(o.data_ptr<float>(), xbc.data_ptr<float>(), (int)C,
-                                                          skip_d.data_ptr<float>(), P.data_ptr<float>(), ldp, (int)z_off,
-                                                          w.data_ptr<float>(), (float)eps, (uint16_t*)out.data_ptr(), ldo,
-                                                          (int)inner, (int)(inner / H), (int)(inner / groups));
-  else
-    ssd_gate_norm_k<float><<<grid, 256, 0, stream()>>>(o.data_ptr<float>(), xbc.data_ptr<float>(), (int)C,
-                                                       skip_d.data_ptr<float>(), P.data_ptr<float>(), ldp, (int)z_off,
-                                                       w.data_ptr<float>(), (float)eps, out.data_ptr<float>(), ldo, (int)inner,
-                                                       (int)(inner / H), (int)(inner / groups));
+  if (bf) ssd_gate_norm_k<uint16_t><<<grid, 256, 0, stream()>>>(SGN_ARGS(uint16_t));
+  else ssd_gate_norm_k<float><<<grid, 256, 0, stream()>>>(SGN_ARGS(float));
+#undef SGN_ARGS
 }
 
 void polynorm_act(const at::Tensor& P, int64_t up_off, int64_t F, const at::Tensor& coef, double eps, at::Tensor& out) {

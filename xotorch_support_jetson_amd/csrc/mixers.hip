@@ -578,8 +578,8 @@ __global__ void gla_prep_k(const float* __restrict__ P, int ldp, int a1_off, int
 
 // ------------------------------------------------------------------ the recurrence
 // State in memory: S^T [slots, H, dv, d] (a value channel's d key rows contiguous).
-// Workgroup = (sequence, value head, 256 / RS value channels); 256 threads = channels x RS row groups, the row group
-// in the low lane bits: the two dot products reduce inside DPP rows, register to register.  A thread keeps the KR
+// Workgroup = (sequence, value head, NC x 256 / RS value channels); 256 threads = channels x RS row groups, NC channels a
+// thread (their chains run side by side on the same LDS reads), the row group in the low lane bits: the two dot products reduce inside DPP rows, register to register.  A thread keeps the KR
 // consecutive key rows rg KR .. rg KR + KR - 1 of its channel in registers (d <= RS KR), so state loads and stores are
 // contiguous runs and a token's k / q slices are vector LDS reads.  The launcher uses RS = 16 (a whole DPP row per
 // value channel).  Tokens are staged through LDS TB at a time, double-buffered: the next block's global loads are in flight
@@ -607,7 +607,7 @@ __device__ __forceinline__ float group_sum(float v) {
   return v;
 }
 
-template <int KR, int RS, int MODE>
+template <int KR, int RS, int MODE, int NC>
 __global__ __launch_bounds__(256) void linear_recurrence_k(
     const float* __restrict__ q, int ldq, const float* __restrict__ k, int ldk, const float* __restrict__ v, int ldv,
     const float* __restrict__ decay, const float* __restrict__ beta, float q_scale, float* __restrict__ state,
@@ -616,76 +616,129 @@ __global__ __launch_bounds__(256) void linear_recurrence_k(
   constexpr int DP = KR * RS;  // padded key dim
   constexpr bool DELTA = MODE == 1 || MODE == 4, SCALAR = MODE != 0 && MODE != 4, NORMCH = MODE == 3;
   constexpr bool INSCALE = MODE == 3 || MODE == 5, BETA = DELTA || INSCALE;
-  constexpr int COLS = 256 / RS;
-  constexpr int TB = DP >= 256 ? 8 : 16;
-  constexpr int NQ = TB * DP / 256, NV = (TB * COLS + 255) / 256;
+  constexpr int CW = 256 / RS, COLS = CW * NC;
+  constexpr int TB = DP >= 256 || (DP == 128 && (NC > 1 || !SCALAR)) ? 8 : 16;
+  constexpr int NQ = (TB * DP + 255) / 256, NV = (TB * COLS + 255) / 256;
   __shared__ __attribute__((aligned(16))) float sq[2][TB][DP], sk[2][TB][DP], sa[2][TB][SCALAR ? 4 : DP];
   __shared__ float sv[2][TB][COLS], sg[2][TB][2];
   const int b = blockIdx.x, h = blockIdx.y, cb = blockIdx.z;
   const int slot = state_slots[b];
   const int t0 = cu_q[b], n = cu_q[b + 1] - t0;
   if (slot < 0 || n <= 0) return;
-  const int tid = threadIdx.x, rg = tid % RS, cl = tid / RS, col = cb * COLS + cl;
-  const bool live = col < dv;
+  const int tid = threadIdx.x, rg = tid % RS, cl = tid / RS;
   const int hk = h / (H / G);
-  float* S = state + (((int64_t)slot * H + h) * dv + (live ? col : 0)) * d + rg * KR;
-  float s[KR];
+  int col[NC];  // the thread's value channels
+  bool live[NC];
+  float* S[NC];
+  float s[NC][KR];
   // 16-byte state loads / stores where the thread's rows are whole float4s inside d (d and KR multiples of 4)
   const bool vec = KR % 4 == 0 && (d & 3) == 0;
 #pragma unroll
-  for (int m = 0; m < KR; m += (KR % 4 == 0 ? 4 : 1)) {
-    if (KR % 4 == 0 && vec) {
-      const bool in = live && rg * KR + m + 4 <= d;
-      const f32x4 x = in ? *reinterpret_cast<const f32x4*>(S + m) : f32x4{0.f, 0.f, 0.f, 0.f};
-      s[m] = x[0];
-      s[m + 1] = x[1];
-      s[m + 2] = x[2];
-      s[m + 3] = x[3];
-    } else {
+  for (int c = 0; c < NC; ++c) {
+    col[c] = cb * COLS + c * CW + cl;
+    live[c] = col[c] < dv;
+    S[c] = state + (((int64_t)slot * H + h) * dv + (live[c] ? col[c] : 0)) * d + rg * KR;
 #pragma unroll
-      for (int e = 0; e < (KR % 4 == 0 ? 4 : 1); ++e) s[m + e] = (live && rg * KR + m + e < d) ? S[m + e] : 0.0f;
+    for (int m = 0; m < KR; m += (KR % 4 == 0 ? 4 : 1)) {
+      if (KR % 4 == 0 && vec) {
+        const bool in = live[c] && rg * KR + m + 4 <= d;
+        const f32x4 x = in ? *reinterpret_cast<const f32x4*>(S[c] + m) : f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int e = 0; e < 4; ++e) s[c][m + (KR % 4 == 0 ? e : 0)] = x[e];
+      } else {
+#pragma unroll
+        for (int e = 0; e < (KR % 4 == 0 ? 4 : 1); ++e) s[c][m + e] = (live[c] && rg * KR + m + e < d) ? S[c][m + e] : 0.0f;
+      }
     }
   }
 
   float pq[NQ], pk[NQ], pa[SCALAR ? 1 : NQ], pv[NV], pg0 = 0.0f, pg1 = 0.0f;
-  auto fetch = [&](int tb) {  // global -> registers: tokens tb .. tb + TB - 1 of the sequence (zeros past its end)
+  // global -> registers: tokens tb .. tb + TB - 1 of the sequence.  Every load is issued without a branch (tokens past the end
+  // repeat the last one and are not consumed, key dims past d repeat the last one and are zeroed by stage), and nothing here
+  // waits for one.
+  auto fetch = [&](int tb) {
 #pragma unroll
     for (int j = 0; j < NQ; ++j) {
-      const int e = tid + 256 * j, tt = e / DP, i = e - tt * DP;
-      const int64_t t = t0 + tb + tt;
-      const bool in = i < d && tb + tt < n;
-      pq[j] = in ? q[t * ldq + hk * d + i] * q_scale : 0.0f;
-      pk[j] = in ? k[t * ldk + hk * d + i] : 0.0f;
-      if (!SCALAR) pa[j] = in ? decay[(t * H + h) * d + i] : 0.0f;
+      const int e = tid + 256 * j, tt = min(e / DP, TB - 1), i = min(e % DP, d - 1);
+      const int64_t t = t0 + min(tb + tt, n - 1);
+      pq[j] = q[t * ldq + hk * d + i];
+      pk[j] = k[t * ldk + hk * d + i];
+      if (!SCALAR) pa[j] = decay[(t * H + h) * d + i];
     }
 #pragma unroll
     for (int j = 0; j < NV; ++j) {
-      const int e = tid + 256 * j, tt = e / COLS, c = cb * COLS + e % COLS;
-      pv[j] = (e < TB * COLS && c < dvin && tb + tt < n) ? v[(int64_t)(t0 + tb + tt) * ldv + h * dvin + c] : 0.0f;
-      if (NORMCH && e < TB * COLS && c == dvin && tb + tt < n) pv[j] = 1.0f;
+      const int e = tid + 256 * j, tt = min(e / COLS, TB - 1), c = min(cb * COLS + e % COLS, dvin - 1);
+      pv[j] = v[(int64_t)(t0 + min(tb + tt, n - 1)) * ldv + h * dvin + c];
     }
-    if (tid < TB && tb + tid < n) {
-      if (SCALAR) pg0 = decay[(int64_t)(t0 + tb + tid) * dstride + h];  // (dstride 0: one fixed decay per head, decay [H])
-      if (BETA) pg1 = beta[(int64_t)(t0 + tb + tid) * H + h];
+    if (SCALAR || BETA) {
+      const int64_t t = t0 + min(tb + min(tid, TB - 1), n - 1);
+      if (SCALAR) pg0 = decay[t * dstride + h];  // (dstride 0: one fixed decay per head, decay [H])
+      if (BETA) pg1 = beta[t * H + h];
     }
   };
   auto stage = [&](int buf) {  // registers -> LDS
 #pragma unroll
     for (int j = 0; j < NQ; ++j) {
       const int e = tid + 256 * j, tt = e / DP, i = e - tt * DP;
-      sq[buf][tt][i] = pq[j];
-      sk[buf][tt][i] = pk[j];
-      if (!SCALAR) sa[buf][tt][i] = pa[j];
+      if (TB * DP % 256 != 0 && tt >= TB) continue;
+      sq[buf][tt][i] = i < d ? pq[j] * q_scale : 0.0f;
+      sk[buf][tt][i] = i < d ? pk[j] : 0.0f;
+      if (!SCALAR) sa[buf][tt][i] = i < d ? pa[j] : 0.0f;
     }
 #pragma unroll
     for (int j = 0; j < NV; ++j) {
       const int e = tid + 256 * j;
-      if (e < TB * COLS) sv[buf][e / COLS][e % COLS] = pv[j];
+      if (e < TB * COLS) sv[buf][e / COLS][e % COLS] = NORMCH && cb * COLS + e % COLS == dvin ? 1.0f : pv[j];
     }
     if ((SCALAR || BETA) && tid < TB) {
       sg[buf][tid][0] = pg0;
       sg[buf][tid][1] = pg1;
     }
+  };
+  struct Row {  // one token's share of a thread
+    float k[KR], q[KR], a[SCALAR ? 1 : KR], v[NC], g, b;
+  };
+  auto load = [&](int buf, int tt, Row& r) {
+#pragma unroll
+    for (int m = 0; m < KR; ++m) {
+      r.k[m] = sk[buf][tt][rg * KR + m];
+      r.q[m] = sq[buf][tt][rg * KR + m];
+      if (!SCALAR) r.a[m] = sa[buf][tt][rg * KR + m];
+    }
+#pragma unroll
+    for (int c = 0; c < NC; ++c) r.v[c] = sv[buf][tt][c * CW + cl];
+    r.g = SCALAR ? sg[buf][tt][0] : 0.0f;
+    r.b = BETA ? sg[buf][tt][1] : 0.0f;
+  };
+  float* op = out + (int64_t)t0 * H * dv + h * dv + cb * COLS + cl;
+  const int64_t ldo = (int64_t)H * dv;
+  auto step = [&](const Row& r) {
+#pragma unroll
+    for (int c = 0; c < NC; ++c) {
+      float u = r.v[c];
+      if (INSCALE) u *= r.b;
+      if (DELTA) {
+        float d0 = 0.0f, d1 = 0.0f, d2 = 0.0f, d3 = 0.0f;
+#pragma unroll
+        for (int m = 0; m < KR; ++m) {
+          s[c][m] *= SCALAR ? r.g : r.a[m];
+          const float p = s[c][m] * r.k[m];
+          if ((m & 3) == 0) d0 += p; else if ((m & 3) == 1) d1 += p; else if ((m & 3) == 2) d2 += p; else d3 += p;
+        }
+        u = r.b * (u - group_sum<RS>((d0 + d1) + (d2 + d3)));
+      }
+      float o0 = 0.0f, o1 = 0.0f, o2 = 0.0f, o3 = 0.0f;
+#pragma unroll
+      for (int m = 0; m < KR; ++m) {
+        if (DELTA) s[c][m] += r.k[m] * u;
+        else s[c][m] = (SCALAR ? r.g : r.a[m]) * s[c][m] + r.k[m] * u;
+        const float p = s[c][m] * r.q[m];
+        if ((m & 3) == 0) o0 += p; else if ((m & 3) == 1) o1 += p; else if ((m & 3) == 2) o2 += p; else o3 += p;
+      }
+      const float o = group_sum<RS>((o0 + o1) + (o2 + o3));
+      if (live[c] && rg == 0) op[c * CW] = o;
+    }
+    op += ldo;
   };
   fetch(0);
   stage(0);
@@ -695,63 +748,35 @@ __global__ __launch_bounds__(256) void linear_recurrence_k(
     const int nt = min(TB, n - tb);
     const bool more = tb + TB < n;
     if (more) fetch(tb + TB);
-#pragma unroll 2
-    for (int tt = 0; tt < nt; ++tt) {
-      const float vc = INSCALE ? sv[buf][tt][cl] * sg[buf][tt][1] : sv[buf][tt][cl];
-      float kk[KR], qq[KR];
-#pragma unroll
-      for (int m = 0; m < KR; ++m) {
-        kk[m] = sk[buf][tt][rg * KR + m];
-        qq[m] = sq[buf][tt][rg * KR + m];
+    Row ra, rb;  // a token's row is read while the one before it is worked on
+    load(buf, 0, ra);
+    for (int tt = 0; tt < nt; tt += 2) {
+      load(buf, min(tt + 1, TB - 1), rb);
+      step(ra);
+      if (tt + 1 < nt) {
+        load(buf, min(tt + 2, TB - 1), ra);
+        step(rb);
       }
-      float o0 = 0.0f, o1 = 0.0f, o2 = 0.0f, o3 = 0.0f;
-      if (DELTA) {
-        const float g = sg[buf][tt][0], bt = sg[buf][tt][1];
-        float d0 = 0.0f, d1 = 0.0f, d2 = 0.0f, d3 = 0.0f;
-#pragma unroll
-        for (int m = 0; m < KR; ++m) {
-          s[m] *= SCALAR ? g : sa[buf][tt][rg * KR + m];
-          const float p = s[m] * kk[m];
-          if ((m & 3) == 0) d0 += p; else if ((m & 3) == 1) d1 += p; else if ((m & 3) == 2) d2 += p; else d3 += p;
-        }
-        const float u = bt * (vc - group_sum<RS>((d0 + d1) + (d2 + d3)));
-#pragma unroll
-        for (int m = 0; m < KR; ++m) {
-          s[m] += kk[m] * u;
-          const float p = s[m] * qq[m];
-          if ((m & 3) == 0) o0 += p; else if ((m & 3) == 1) o1 += p; else if ((m & 3) == 2) o2 += p; else o3 += p;
-        }
-      } else if (SCALAR) {
-        const float g = sg[buf][tt][0];
-#pragma unroll
-        for (int m = 0; m < KR; ++m) {
-          s[m] = g * s[m] + kk[m] * vc;
-          const float p = s[m] * qq[m];
-          if ((m & 3) == 0) o0 += p; else if ((m & 3) == 1) o1 += p; else if ((m & 3) == 2) o2 += p; else o3 += p;
-        }
-      } else {
-#pragma unroll
-        for (int m = 0; m < KR; ++m) {
-          s[m] = sa[buf][tt][rg * KR + m] * s[m] + kk[m] * vc;
-          const float p = s[m] * qq[m];
-          if ((m & 3) == 0) o0 += p; else if ((m & 3) == 1) o1 += p; else if ((m & 3) == 2) o2 += p; else o3 += p;
-        }
-      }
-      const float o = group_sum<RS>((o0 + o1) + (o2 + o3));
-      if (live && rg == 0) out[(int64_t)(t0 + tb + tt) * H * dv + h * dv + col] = o;
     }
     if (more) stage(buf ^ 1);  // (its last readers passed the barrier that ended the previous block)
     __syncthreads();
   }
-  if (live) {
+#pragma unroll
+  for (int c = 0; c < NC; ++c) {
+    if (!live[c]) continue;
 #pragma unroll
     for (int m = 0; m < KR; m += (KR % 4 == 0 ? 4 : 1)) {
       if (KR % 4 == 0 && vec) {
-        if (rg * KR + m + 4 <= d) *reinterpret_cast<f32x4*>(S + m) = f32x4{s[m], s[m + 1], s[m + 2], s[m + 3]};
+        if (rg * KR + m + 4 <= d) {
+          f32x4 x;
+#pragma unroll
+          for (int e = 0; e < 4; ++e) x[e] = s[c][m + (KR % 4 == 0 ? e : 0)];
+          *reinterpret_cast<f32x4*>(S[c] + m) = x;
+        }
       } else {
 #pragma unroll
         for (int e = 0; e < (KR % 4 == 0 ? 4 : 1); ++e)
-          if (rg * KR + m + e < d) S[m + e] = s[m + e];
+          if (rg * KR + m + e < d) S[c][m + e] = s[c][m + e];
       }
     }
   }
@@ -1049,13 +1074,16 @@ void gla_prep(const at::Tensor& P, int64_t a1_off, const at::Tensor& a2, const a
                                                          decay.data_ptr<float>());
 }
 
-template <int RS, int MODE>
+// XOT_REC_COLS=1 / 2 forces the recurrences' channels per thread (A/B runs)
+const int REC_COLS = []() { const char* e = getenv("XOT_REC_COLS"); return e ? atoi(e) : 0; }();
+
+template <int RS, int MODE, int NC>
 void launch_rec(int KR, dim3 grid, const float* q, int ldq, const float* k, int ldk, const float* v, int ldv, const float* decay,
                 const float* beta, float q_scale, float* state, const int* slots, const int* cu, int H, int G, int d, int dv,
                 int dvin, int dstride, float* out) {
 #define REC_CASE(DPAD)                                                                                                 \
   case DPAD:                                                                                                           \
-    linear_recurrence_k<DPAD / RS, RS, MODE><<<grid, 256, 0, stream()>>>(q, ldq, k, ldk, v, ldv, decay, beta, q_scale, \
+    linear_recurrence_k<DPAD / RS, RS, MODE, NC><<<grid, 256, 0, stream()>>>(q, ldq, k, ldk, v, ldv, decay, beta, q_scale, \
                                                                           state, slots, cu, H, G, d, dv, dvin, dstride, out); \
     break;
   switch (KR * RS) {  // padded key dim
@@ -1112,15 +1140,24 @@ void linear_recurrence(const at::Tensor& q, const at::Tensor& k, const at::Tenso
   // 16 row groups per value channel (4 and 8, with more rows per thread, measured slower at 8 x 2048 tokens and 16
   // heads: d 64 / dv 128 0.89 / 0.75 / 0.70 ms with 4 / 8 / 16, d 128 / dv 128 1.57 / 1.28 / 1.23)
   const int RS = 16;
-  const int cols = 256 / RS;
+  // two channels a thread for prompts whose (sequence, head, 32 channels) workgroups still put two on every CU
+  const bool two = (chan || inscale) && dv > 16 && REC_COLS != 1 && (REC_COLS == 2 || (T >= 16 * B && B * H * ((dv + 31) / 32) >= 512));
+  const int cols = 256 / RS * (two ? 2 : 1);
   const dim3 grid((unsigned)B, (unsigned)H, (unsigned)((dv + cols - 1) / cols));
   const float* bp = beta.has_value() ? beta->data_ptr<float>() : nullptr;
-#define REC_GO(R, D)                                                                                                          \
-  launch_rec<R, D>(DP / R, grid, q.data_ptr<float>(), ldq, k.data_ptr<float>(), ldk, v.data_ptr<float>(), ldv,              \
+#define REC_GO(R, D, N)                                                                                                       \
+  launch_rec<R, D, N>(DP / R, grid, q.data_ptr<float>(), ldq, k.data_ptr<float>(), ldk, v.data_ptr<float>(), ldv,              \
                    decay.data_ptr<float>(), bp, (float)q_scale, state.data_ptr<float>(), state_slots.data_ptr<int>(),        \
                    cu_q.data_ptr<int>(), (int)H, (int)G, (int)d, (int)dv, (int)dvin, fixed ? 0 : (int)H,         \
                    out.data_ptr<float>())
-  if (chan) REC_GO(16, 4); else if (inscale) REC_GO(16, 5); else if (delta) REC_GO(16, 1); else if (normch) REC_GO(16, 3); else if (scalar) REC_GO(16, 2); else REC_GO(16, 0);
+  if (chan && two) REC_GO(16, 4, 2);
+  else if (chan) REC_GO(16, 4, 1);
+  else if (inscale && two) REC_GO(16, 5, 2);
+  else if (inscale) REC_GO(16, 5, 1);
+  else if (delta) REC_GO(16, 1, 1);
+  else if (normch) REC_GO(16, 3, 1);
+  else if (scalar) REC_GO(16, 2, 1);
+  else REC_GO(16, 0, 1);
 #undef REC_GO
 }
 

@@ -150,21 +150,56 @@ __global__ __launch_bounds__(256) void gated_group_norm_wave_k(const float* __re
 }
 
 // ------------------------------------------------------------------ mean of two normed rows
+// (y2 may be S split-K slabs)
 __global__ __launch_bounds__(256) void pair_norm_mean_k(const float* __restrict__ y1, int ld1, const float* __restrict__ y2,
-                                                        int ld2, const float* __restrict__ w, float eps,
+                                                        int ld2, int S, int64_t ss, const float* __restrict__ w, float eps,
                                                         float* __restrict__ out, int D) {
   __shared__ float red[16];
   const int64_t t = blockIdx.x;
   const float *a = y1 + t * ld1, *b = y2 + t * ld2;
   float sa = 0.0f, sb = 0.0f;
   for (int i = threadIdx.x; i < D; i += blockDim.x) {
+    const float vb = slab1(b + i, S, ss);
     sa += a[i] * a[i];
-    sb += b[i] * b[i];
+    sb += vb * vb;
   }
   sa = block_sum(sa, red);
   sb = block_sum(sb, red);
   const float ka = 0.5f / sqrtf(sa / (float)D + eps), kb = 0.5f / sqrtf(sb / (float)D + eps);
-  for (int i = threadIdx.x; i < D; i += blockDim.x) out[t * D + i] = a[i] * ka * w[i] + b[i] * kb * w[D + i];
+  for (int i = threadIdx.x; i < D; i += blockDim.x) out[t * D + i] = a[i] * ka * w[i] + slab1(b + i, S, ss) * kb * w[D + i];
+}
+
+// Rows of at most 1024 R numbers in whole vectors of four: both rows stay in registers between the sums and the write.
+template <int R>
+__global__ __launch_bounds__(256) void pair_norm_mean_reg_k(const float* __restrict__ y1, int ld1, const float* __restrict__ y2,
+                                                            int ld2, int S, int64_t ss, const float* __restrict__ w, float eps,
+                                                            float* __restrict__ out, int D) {
+  __shared__ float red[16];
+  const int64_t t = blockIdx.x;
+  auto ld = [](const float* p) { return *reinterpret_cast<const f32x4*>(p); };
+  f32x4 a[R], b[R];
+  float sa = 0.0f, sb = 0.0f;
+#pragma unroll
+  for (int r = 0; r < R; ++r) {
+    const int i = 4 * (threadIdx.x + 256 * r);
+    a[r] = b[r] = f32x4{0.f, 0.f, 0.f, 0.f};
+    if (i >= D) continue;
+    a[r] = ld(y1 + t * ld1 + i);
+    b[r] = slab4(y2 + t * ld2 + i, S, ss);
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      sa += a[r][e] * a[r][e];
+      sb += b[r][e] * b[r][e];
+    }
+  }
+  sa = block_sum(sa, red);
+  sb = block_sum(sb, red);
+  const float ka = 0.5f / sqrtf(sa / (float)D + eps), kb = 0.5f / sqrtf(sb / (float)D + eps);
+#pragma unroll
+  for (int r = 0; r < R; ++r) {
+    const int i = 4 * (threadIdx.x + 256 * r);
+    if (i < D) *reinterpret_cast<f32x4*>(out + t * D + i) = a[r] * ka * ld(w + i) + b[r] * kb * ld(w + D + i);
+  }
 }
 
 // ------------------------------------------------------------------ host side
@@ -294,16 +329,23 @@ void gated_group_norm(const at::Tensor& o, const c10::optional<at::Tensor>& m, c
 }
 
 void pair_norm_mean(const at::Tensor& y1, const at::Tensor& y2, const at::Tensor& w, double eps, at::Tensor& out) {
-  const int ld1 = ld_of(y1, "y1"), ld2 = ld_of(y2, "y2");
+  const int ld1 = ld_of(y1, "y1");
+  const Slabs p2 = slabs_of(y2, "y2");
   f32c(w, "w");
   f32c(out, "out");
   MCHECK(out.dim() == 2, "out must be [T, D]");
   const int64_t T = out.size(0), D = out.size(1);
   if (T == 0) return;
-  MCHECK(y1.size(0) == T && y2.size(0) == T && y1.size(1) >= D && y2.size(1) >= D && w.numel() == 2 * D,
-         "pair_norm_mean: shape mismatch");
-  pair_norm_mean_k<<<T, 256, 0, stream()>>>(y1.data_ptr<float>(), ld1, y2.data_ptr<float>(), ld2, w.data_ptr<float>(), (float)eps,
-                                            out.data_ptr<float>(), (int)D);
+  MCHECK(y1.size(0) == T && p2.T == T && y1.size(1) >= D && p2.n >= D && w.numel() == 2 * D, "pair_norm_mean: shape mismatch");
+  auto al = [](const at::Tensor& t) { return (reinterpret_cast<uintptr_t>(t.data_ptr()) & 15) == 0; };
+#define PNM_GO(KERNEL)                                                                                                  \
+  KERNEL<<<T, 256, 0, stream()>>>(y1.data_ptr<float>(), ld1, p2.p, p2.ld, p2.S, p2.ss, w.data_ptr<float>(), (float)eps, \
+                                  out.data_ptr<float>(), (int)D)
+  const bool vec = p2.vec && D % 4 == 0 && ld1 % 4 == 0 && al(y1) && al(w) && al(out);
+  if (vec && D <= 2048) PNM_GO(pair_norm_mean_reg_k<2>);
+  else if (vec && D <= 4096) PNM_GO(pair_norm_mean_reg_k<4>);
+  else PNM_GO(pair_norm_mean_k);
+#undef PNM_GO
 }
 
 }  // namespace

@@ -668,9 +668,9 @@ class ShardModel:
   def _conv(self, P: torch.Tensor, off: int, lw, j: int, inp: StepInputs) -> torch.Tensor:
     """The layer's short convolutions (every convolved channel of its mixers in one launch) with what follows them channel
     by channel or head by head -> fp32 [T, channels]."""
-    out = torch.empty(P.shape[0], lw.conv_w.shape[0], dtype=torch.float32, device=P.device)
+    out = torch.empty(P.shape[-2], lw.conv_w.shape[0], dtype=torch.float32, device=P.device)
     K.conv_prep(P, off, lw.conv_w, lw.conv_b, lw.conv_units, lw.conv_norm, self.state.conv[j], inp.state_slots, inp.cu_q,
-                self.c.rms_norm_eps, out, max_qlen=inp.max_qlen)
+                self.c.rms_norm_eps, out, max_qlen=inp.max_qlen, width=lw.conv_width)
     return out
 
   def _low_rank(self, P: torch.Tensor, off: int, n: int, w: torch.Tensor) -> torch.Tensor:
@@ -683,12 +683,12 @@ class ShardModel:
     """Delta rule with a decay per key channel on the state slots: convolutions + SiLU + unit norms, step sizes and low-rank
     decays and output gates (prompts: their second projections are GEMMs), the recurrence, the per-head gated norm."""
     r, st, dev = lw.spec.rec, self.state, P.device
-    T, H, nk, nv = P.shape[0], r.heads, r.kv_heads * r.dim, r.heads * r.vdim
+    T, H, nk, nv = mix.shape[0], r.heads, r.kv_heads * r.dim, r.heads * r.vdim
     qkv = self._conv(P, lw.cols["rq"][0], lw, j, inp)
     beta = torch.empty(T, H, dtype=torch.float32, device=dev)
     decay = torch.empty(T, H * r.dim, dtype=torch.float32, device=dev)
     (a0, an), (g0, gn) = lw.cols["ra1"], lw.cols["rg1"]
-    if P.is_cuda and lw.a2_p is not None and T >= LOW_RANK_GEMM_ROWS:
+    if P.is_cuda and P.dim() == 2 and lw.a2_p is not None and T >= LOW_RANK_GEMM_ROWS:
       za, gate = self._low_rank(P, a0, an, lw.a2_p), self._low_rank(P, g0, gn, lw.g2_p)
       K.recurrence_gates(P, lw.cols["rb"][0], beta, 0, None, lw.dt_bias, lw.A_log, decay, 0, None, None, za=za)
     else:
@@ -702,7 +702,7 @@ class ShardModel:
     """Mamba-2 mixer whose convolved channels x = [x | B | C] are ready: step sizes and decays, the recurrence (input scale
     dt), skip, gate, grouped norm."""
     m, st, dev = lw.spec.ssd, self.state, P.device
-    T, inner, gn = P.shape[0], m.inner, m.groups * m.state
+    T, inner, gn = mix.shape[0], m.inner, m.groups * m.state
     dt, decay = (torch.empty(T, m.heads, dtype=torch.float32, device=dev) for _ in range(2))
     K.ssd_steps(P, lw.cols["dt"][0], lw.dt_bias, lw.A_log, dt, decay)
     o = torch.empty(T, inner, dtype=torch.float32, device=dev)
@@ -982,8 +982,10 @@ class ShardModel:
       if fresh:  # (no norm weight: the op copies the stream)
         K.sandwich_add_norm(h, None, None, lw.norm1, eps, hn, bn=lw.norm1_b, layer=ln)
       pair = s.wattn is not None and (s.rec is not None or s.ssd is not None)  # two mixers side by side
-      # (window attention alone: the store kernel is the projection's only reader)
-      P = (self._proj_slabs if s.wattn is not None and s.wattn.gate == "none" and not pair else self._proj)(hn, lw.in_w)
+      # (projections whose readers sum split-K slabs themselves, all of them before the next GEMM: window attention alone,
+      # and everything behind short convolutions)
+      sums = s.wattn is not None and s.wattn.gate == "none" and not pair or lw.conv_units is not None
+      P = (self._proj_slabs if sums else self._proj)(hn, lw.in_w)
       mix = rows("mix", lw.mix_cols["mix"][1], lw.out_w.shape[1])
       if s.lattn is not None:
         self._latent_attn(P, lw, j, inp, mix, rows)
@@ -996,14 +998,15 @@ class ShardModel:
         self._channel_delta(P, lw, j, inp, mix)
       else:
         self._mlstm(P, lw, j, inp, mix)
-      y = (self._proj if pair else self._proj_slabs)(mix, lw.out_w)
       if pair:  # the second mixer of a parallel layer, then the mean of the normed pair
         mix2 = rows("mix2", lw.mix_cols["mix2"][1], lw.out2_w.shape[1])
         if s.ssd is not None:
           self._ssd_conv(P, X[:, s.wattn.conv_channels:], lw, j, inp, mix2)
         else:
           self._lightning(P, lw, j, inp, mix2)
-        y2 = self._proj(mix2, lw.out2_w)
+      y = (self._proj if pair else self._proj_slabs)(mix, lw.out_w)
+      if pair:
+        y2 = self._proj_slabs(mix2, lw.out2_w)
         y1, y = y, torch.empty(T, D, dtype=torch.float32, device=h.device)
         K.pair_norm_mean(y1, y2, lw.pair_w, eps, y)
       f = s.ffn

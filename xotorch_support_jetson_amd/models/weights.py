@@ -770,6 +770,7 @@ class MixedLayerWeights:
   # weights; a2_w / g2_w are the second projections of the decay and the output gate, a2_p / g2_p the same padded for the
   # GEMM kernels (prompts); ff_w of a dense clamped feed-forward has its gate / up rows interleaved by 16
   conv_units: Optional[torch.Tensor] = None  # [units, 4] int32
+  conv_width: int = 0  # the most channels of a unit
   conv_norm: Optional[torch.Tensor] = None  # fp32
   g2_w: Optional[torch.Tensor] = None  # [H dv, gate rank]
   a2_p: Optional[torch.Tensor] = None
@@ -1166,7 +1167,8 @@ def build_conv_sandwich_layer(spec, get, p: str, D: int, device, dtype) -> Mixed
     setattr(lw, n, dev(get(p + n)))
   if units:
     lw.conv_w, lw.conv_b = dev(conv), dev(conv_b) if conv_b is not None else None
-    lw.conv_units = conv_units(units, conv.shape[0]).to(device)
+    u, lw.conv_width = conv_units(units, conv.shape[0])
+    lw.conv_units = u.to(device)
     lw.conv_norm = dev(torch.cat(norms)) if norms else None
   if r is not None:
     lw.A_log, lw.dt_bias = dev(get(m + "A_log")), dev(get(m + "dt_bias"))

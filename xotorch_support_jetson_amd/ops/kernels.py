@@ -491,13 +491,15 @@ def gla_prep(P, a1_off: int, a2, a2_b, tau: float, decay) -> None:
 conv_units = ref.conv_units
 
 
-def conv_prep(P, x_off: int, conv_w, conv_b, units, norm_w, conv_state, state_slots, cu_q, eps: float, out, max_qlen: int = 0) -> None:
+def conv_prep(P, x_off: int, conv_w, conv_b, units, norm_w, conv_state, state_slots, cu_q, eps: float, out, max_qlen: int = 0,
+              width: int = 256) -> None:
   """Causal convolutions over time of the channels P[:, x_off : +C] (conv_w [C, taps], last column the current token; conv_b
   [C] or None) -> out [T, C] fp32, then per unit (conv_units) SiLU and a unit length or a weighted RMS norm (norm_w).  The
   inputs before the step come from conv_state [slots, taps - 1, C], which takes the step's last ones.  max_qlen 1: every
-  sequence has one new token (the state is updated in the same launch)."""
+  sequence has one new token (the state is updated in the same launch).  width: the most channels of a unit.  P may be [T, n]
+  or unreduced split-K slabs [S, T, n] (also below)."""
   _mix("conv_prep", _gpu(P))(P, int(x_off), conv_w, conv_b, units, norm_w, conv_state, state_slots, cu_q, float(eps), out,
-                             int(max_qlen))
+                             int(max_qlen), int(width))
 
 
 def recurrence_gates(P, b_off: int, beta, a1_off: int, a2, dt_bias, A_log, decay, g1_off: int, g2, gate, za=None) -> None:

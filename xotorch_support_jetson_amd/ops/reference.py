@@ -322,25 +322,28 @@ CONV_SILU, CONV_UNIT, CONV_UNIT_SCALED, CONV_RMS = 1, 2, 4, 8
 CONV_MAX = 256  # channels of a unit
 
 
-def conv_units(parts, C: int) -> torch.Tensor:
-  """[(channels, kind[, first norm weight])] over consecutive channels -> int32 [units, 4] (first channel, channels, kind,
-  first norm weight); runs without a norm are cut into pieces of CONV_MAX channels."""
+def conv_units(parts, C: int):
+  """[(channels, kind[, first norm weight])] over consecutive channels -> (int32 [units, 4]: first channel, channels, kind,
+  first norm weight; the most channels of a unit).  Runs without a norm are cut into pieces as wide as the widest normed
+  head asks a wave to be (64, 128 or CONV_MAX channels)."""
+  heads = [int(p[0]) for p in parts if int(p[1]) & ~CONV_SILU]
+  if heads and max(heads) > CONV_MAX:
+    raise ValueError(f"a normed head of {max(heads)} channels (at most {CONV_MAX})")
+  width = next(w for w in (64, 128, CONV_MAX) if w >= max(heads)) if heads else CONV_MAX
   rows, c0 = [], 0
   for part in parts:
     n, kind, off = int(part[0]), int(part[1]), int(part[2]) if len(part) > 2 else 0
     if kind & ~CONV_SILU:
-      if n > CONV_MAX:
-        raise ValueError(f"a normed head of {n} channels (at most {CONV_MAX})")
       rows.append((c0, n, kind, off))
     else:
-      rows += [(c0 + i, min(CONV_MAX, n - i), kind, 0) for i in range(0, n, CONV_MAX)]
+      rows += [(c0 + i, min(width, n - i), kind, 0) for i in range(0, n, width)]
     c0 += n
   if c0 != C:
     raise ValueError(f"the units cover {c0} of {C} channels")
-  return torch.tensor(rows, dtype=torch.int32)
+  return torch.tensor(rows, dtype=torch.int32), width
 
 
-def conv_prep(P, x_off, conv_w, conv_b, units, norm_w, conv_state, state_slots, cu_q, eps, out, max_qlen=0):
+def conv_prep(P, x_off, conv_w, conv_b, units, norm_w, conv_state, state_slots, cu_q, eps, out, max_qlen=0, width=CONV_MAX):
   C, taps = conv_w.shape
   for b in range(state_slots.numel()):
     t0, t1, slot = int(cu_q[b]), int(cu_q[b + 1]), int(state_slots[b])
