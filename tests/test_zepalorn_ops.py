@@ -175,6 +175,41 @@ def test_gates_of_the_channel_delta_rule(dev, dtype, H, d, dv, ra, rg, T):
   close(decay2, want, 1e-5, "decay of a finished product")
 
 
+@pytest.mark.parametrize("dev,dtype", RUNS)
+@pytest.mark.parametrize("kind", ["gates", "steps"])
+@pytest.mark.parametrize("taps", [1, 3, 4, 7])
+def test_single_tokens_do_convolutions_and_gates_at_once(dev, dtype, kind, taps):
+  """One call for convolutions and gates (or step sizes) gives what the separate ones give, states included; a padding row
+  (slot -1) keeps its hands off the states."""
+  T, H, d, dv, ra, rg, C = 11, 3, 20, 24, 40, 12, 2 * 20 + 90
+  parts = [(20, CONV_SILU | CONV_UNIT), (20, CONV_RMS, 3), (90, CONV_SILU)]
+  units, width = conv_units(parts, C)
+  n = C + ra + rg + 2 * H
+  P, w, nw = rnd(T, n, seed=1).to(dev), rnd(C, taps, seed=2).to(dev), rnd(30, seed=3).to(dev)
+  if dev != "cpu":
+    P = torch.stack([P * 0.5, P * 0.25, P * 0.25])
+  slots = torch.tensor([3, 0, 7, 1, -1, 2, 9, 8, 4, 10, 5], dtype=torch.int32, device=dev)
+  state = rnd(12, taps - 1, C, seed=4).to(dev)
+  dt_bias, A_log = rnd(H * d if kind == "gates" else H, seed=5).to(dev), rnd(H, seed=6).to(dev)
+  a2, g2 = rnd(H * d, ra, seed=7).to(dev, dtype), rnd(H * dv, rg, seed=8).to(dev, dtype)
+
+  def outs():
+    s = {"out": torch.full((T, C), 2.0, device=dev), "state": state.clone(), "decay": torch.zeros(T, dt_bias.numel(), device=dev),
+         "first": torch.zeros(T, H, device=dev), "gate": torch.zeros(T, H * dv, device=dev)}
+    args = (C, s["first"], C + H, a2, dt_bias, A_log, s["decay"], C + H + ra, g2, s["gate"]) if kind == "gates" else \
+      (C, dt_bias, A_log, s["first"], s["decay"])
+    return s, args
+  both, args = outs()
+  conv = (0, w, None, units.to(dev), nw)
+  K.conv_prep(P, *conv, both["state"], slots, cuts([1] * T, dev), 1e-5, both["out"], max_qlen=1, width=width, **{kind: args})
+  apart, args = outs()
+  K.conv_prep(P, *conv, apart["state"], slots, cuts([1] * T, dev), 1e-5, apart["out"], max_qlen=1, width=width)
+  (K.recurrence_gates if kind == "gates" else K.ssd_steps)(P, *args)
+  for k in both:
+    assert torch.equal(both[k], apart[k]), k
+  assert torch.equal(both["state"][[6, 11]], state[[6, 11]]) and float(both["out"][4].min()) == 2.0
+
+
 @pytest.mark.parametrize("dev", DEVS)
 def test_ssd_steps(dev):
   T, H = 7, 5

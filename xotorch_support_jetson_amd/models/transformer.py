@@ -665,12 +665,12 @@ class ShardModel:
                         inp.cu_q, o)
     K.ssd_gate_norm(o, xbc, lw.skip_d, P, i0, lw.ssd_norm, m.norm_groups, self.c.rms_norm_eps, mix)
 
-  def _conv(self, P: torch.Tensor, off: int, lw, j: int, inp: StepInputs) -> torch.Tensor:
+  def _conv(self, P: torch.Tensor, off: int, lw, j: int, inp: StepInputs, **gates) -> torch.Tensor:
     """The layer's short convolutions (every convolved channel of its mixers in one launch) with what follows them channel
-    by channel or head by head -> fp32 [T, channels]."""
+    by channel or head by head -> fp32 [T, channels]; gates: the recurrence's gates or step sizes, made along with them."""
     out = torch.empty(P.shape[-2], lw.conv_w.shape[0], dtype=torch.float32, device=P.device)
     K.conv_prep(P, off, lw.conv_w, lw.conv_b, lw.conv_units, lw.conv_norm, self.state.conv[j], inp.state_slots, inp.cu_q,
-                self.c.rms_norm_eps, out, max_qlen=inp.max_qlen, width=lw.conv_width)
+                self.c.rms_norm_eps, out, max_qlen=inp.max_qlen, width=lw.conv_width, **gates)
     return out
 
   def _low_rank(self, P: torch.Tensor, off: int, n: int, w: torch.Tensor) -> torch.Tensor:
@@ -684,27 +684,27 @@ class ShardModel:
     decays and output gates (prompts: their second projections are GEMMs), the recurrence, the per-head gated norm."""
     r, st, dev = lw.spec.rec, self.state, P.device
     T, H, nk, nv = mix.shape[0], r.heads, r.kv_heads * r.dim, r.heads * r.vdim
-    qkv = self._conv(P, lw.cols["rq"][0], lw, j, inp)
     beta = torch.empty(T, H, dtype=torch.float32, device=dev)
     decay = torch.empty(T, H * r.dim, dtype=torch.float32, device=dev)
     (a0, an), (g0, gn) = lw.cols["ra1"], lw.cols["rg1"]
     if P.is_cuda and P.dim() == 2 and lw.a2_p is not None and T >= LOW_RANK_GEMM_ROWS:
+      qkv = self._conv(P, lw.cols["rq"][0], lw, j, inp)
       za, gate = self._low_rank(P, a0, an, lw.a2_p), self._low_rank(P, g0, gn, lw.g2_p)
       K.recurrence_gates(P, lw.cols["rb"][0], beta, 0, None, lw.dt_bias, lw.A_log, decay, 0, None, None, za=za)
     else:
       gate = torch.empty(T, nv, dtype=torch.float32, device=dev)
-      K.recurrence_gates(P, lw.cols["rb"][0], beta, a0, lw.a2_w, lw.dt_bias, lw.A_log, decay, g0, lw.g2_w, gate)
+      qkv = self._conv(P, lw.cols["rq"][0], lw, j, inp,
+                       gates=(lw.cols["rb"][0], beta, a0, lw.a2_w, lw.dt_bias, lw.A_log, decay, g0, lw.g2_w, gate))
     o = torch.empty(T, nv, dtype=torch.float32, device=dev)
     K.linear_recurrence(qkv[:, :nk], qkv[:, nk:2 * nk], qkv[:, 2 * nk:], decay, beta, 1.0, st.S[j], inp.state_slots, inp.cu_q, o)
     K.gated_group_norm(o, None, lw.rec_norm, gate, 0, H, self.c.rms_norm_eps, mix)
 
-  def _ssd_conv(self, P: torch.Tensor, x: torch.Tensor, lw, j: int, inp: StepInputs, mix: torch.Tensor) -> None:
-    """Mamba-2 mixer whose convolved channels x = [x | B | C] are ready: step sizes and decays, the recurrence (input scale
+  def _ssd_conv(self, P: torch.Tensor, x: torch.Tensor, dt: torch.Tensor, decay: torch.Tensor, lw, j: int, inp: StepInputs,
+                mix: torch.Tensor) -> None:
+    """Mamba-2 mixer whose convolved channels x = [x | B | C], step sizes and decays are ready: the recurrence (input scale
     dt), skip, gate, grouped norm."""
     m, st, dev = lw.spec.ssd, self.state, P.device
     T, inner, gn = mix.shape[0], m.inner, m.groups * m.state
-    dt, decay = (torch.empty(T, m.heads, dtype=torch.float32, device=dev) for _ in range(2))
-    K.ssd_steps(P, lw.cols["dt"][0], lw.dt_bias, lw.A_log, dt, decay)
     o = torch.empty(T, inner, dtype=torch.float32, device=dev)
     K.linear_recurrence(x[:, inner + gn:inner + 2 * gn], x[:, inner:inner + gn], x[:, :inner], decay, dt, 1.0, st.S[j],
                         inp.state_slots, inp.cu_q, o, plain=True)
@@ -992,7 +992,10 @@ class ShardModel:
       elif s.dattn is not None:
         self._diff_attn(P, lw, j, inp, mix)
       elif s.wattn is not None:
-        X = self._conv(P, 0, lw, j, inp) if s.wattn.conv else P  # (also the convolved channels of a mixer beside it)
+        X = P
+        if s.wattn.conv:  # (also the convolved channels of a mixer beside it, and its step sizes)
+          dts = [torch.empty(T, s.ssd.heads, dtype=torch.float32, device=h.device) for _ in range(2)] if s.ssd is not None else None
+          X = self._conv(P, 0, lw, j, inp, **({"steps": (lw.cols["dt"][0], lw.dt_bias, lw.A_log, *dts)} if dts else {}))
         self._window_attn(X, lw, j, inp, mix)
       elif s.rec.rule == "channel_delta":
         self._channel_delta(P, lw, j, inp, mix)
@@ -1001,7 +1004,7 @@ class ShardModel:
       if pair:  # the second mixer of a parallel layer, then the mean of the normed pair
         mix2 = rows("mix2", lw.mix_cols["mix2"][1], lw.out2_w.shape[1])
         if s.ssd is not None:
-          self._ssd_conv(P, X[:, s.wattn.conv_channels:], lw, j, inp, mix2)
+          self._ssd_conv(P, X[:, s.wattn.conv_channels:], *dts, lw, j, inp, mix2)
         else:
           self._lightning(P, lw, j, inp, mix2)
       y = (self._proj if pair else self._proj_slabs)(mix, lw.out_w)

@@ -492,14 +492,30 @@ conv_units = ref.conv_units
 
 
 def conv_prep(P, x_off: int, conv_w, conv_b, units, norm_w, conv_state, state_slots, cu_q, eps: float, out, max_qlen: int = 0,
-              width: int = 256) -> None:
+              width: int = 256, gates: tuple | None = None, steps: tuple | None = None) -> None:
   """Causal convolutions over time of the channels P[:, x_off : +C] (conv_w [C, taps], last column the current token; conv_b
   [C] or None) -> out [T, C] fp32, then per unit (conv_units) SiLU and a unit length or a weighted RMS norm (norm_w).  The
   inputs before the step come from conv_state [slots, taps - 1, C], which takes the step's last ones.  max_qlen 1: every
   sequence has one new token (the state is updated in the same launch).  width: the most channels of a unit.  P may be [T, n]
-  or unreduced split-K slabs [S, T, n] (also below)."""
+  or unreduced split-K slabs [S, T, n] (also below).  gates / steps: the arguments behind P of recurrence_gates or ssd_steps,
+  which read the same projection: done as well, for single tokens in the same launch."""
+  if _gpu(P) and max_qlen == 1 and P.shape[-2] == state_slots.numel() and (gates is not None) != (steps is not None):
+    if gates is not None:
+      b_off, beta, a1_off, a2, dt_bias, A_log, decay, g1_off, g2, gate = gates
+      dt_off, dt = 0, None
+    else:
+      dt_off, dt_bias, A_log, dt, decay = steps
+      b_off = a1_off = g1_off = 0
+      beta = a2 = g2 = gate = None
+    require().conv_prep_gates(P, int(x_off), conv_w, conv_b, units, norm_w, conv_state, state_slots, cu_q, float(eps), out, int(width),
+                              int(b_off), beta, int(a1_off), a2, dt_bias, A_log, decay, int(g1_off), g2, gate, int(dt_off), dt)
+    return
   _mix("conv_prep", _gpu(P))(P, int(x_off), conv_w, conv_b, units, norm_w, conv_state, state_slots, cu_q, float(eps), out,
                              int(max_qlen), int(width))
+  if gates is not None:
+    recurrence_gates(P, *gates)
+  if steps is not None:
+    ssd_steps(P, *steps)
 
 
 def recurrence_gates(P, b_off: int, beta, a1_off: int, a2, dt_bias, A_log, decay, g1_off: int, g2, gate, za=None) -> None:
