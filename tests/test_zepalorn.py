@@ -346,7 +346,7 @@ def _marked_window(window, keep):
 
 
 @pytest.mark.parametrize("dev,dtype", RUNS)
-@pytest.mark.parametrize("window,keep", [(16, 4), (64, 1), (65, 64), (9, 70), (100, 0), (40, 130)])
+@pytest.mark.parametrize("window,keep", [(16, 4), (64, 1), (65, 64), (9, 70), (100, 0), (44, 130)])
 def test_window_and_kept_token_edges(dev, dtype, window, keep):
   """B as the last kept token and as the first that is not kept, B just inside and just outside the window: in a prompt, in
   portions that end on and straddle the edges, and decoded one by one."""

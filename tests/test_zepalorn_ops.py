@@ -307,7 +307,7 @@ def test_ssd_skip_gate_and_grouped_norm(dev, dtype, H, dv, groups, S):
 
 # ------------------------------------------------------------------ rotation, attention
 @pytest.mark.parametrize("rot", [
-  {"base": 10000.0, "dims": 32, "scaling": {"factor": 8.0, "original": 2048, "fast": 32.0, "slow": 1.0}},
+  {"base": 20000.0, "dims": 32, "scaling": {"factor": 6.0, "original": 4096, "fast": 24.0, "slow": 1.0}},
   {"base": 500.0, "dims": 6, "scaling": {"factor": 3.0, "original": 64, "fast": 4.0, "slow": 2.0}},
   {"base": 1e6, "dims": 64, "scaling": {"factor": 1.0, "original": 4096, "fast": 32.0, "slow": 1.0}},
   {"base": 100.0, "dims": 4, "scaling": {"factor": 4.0, "original": 1000000, "fast": 1.0, "slow": 0.5}},  # (hi below lo)
@@ -324,9 +324,9 @@ def test_yarn_table(rot):
 
 
 CASES = [  # H, G, d, dv, window, chunk, keep, softcap, context lengths, new tokens
-  (4, 2, 64, 64, 40, 0, 4, 0.0, [150, 131], [100, 1]), (4, 2, 64, 64, 40, 0, 70, 0.0, [250, 90], [1, 1]),
+  (6, 2, 64, 64, 37, 0, 5, 0.0, [150, 131], [100, 1]), (6, 2, 64, 64, 37, 0, 70, 0.0, [250, 90], [1, 1]),
   (8, 2, 16, 24, 21, 0, 3, 0.0, [150, 40], [60, 1]), (6, 3, 72, 40, 65, 0, 1, 4.0, [180, 66], [80, 30]),
-  (4, 1, 128, 128, 0, 96, 0, 3.0, [200, 97], [110, 97]), (4, 1, 128, 128, 0, 96, 0, 3.0, [200, 97, 192], [1, 1, 1]),
+  (4, 1, 128, 128, 0, 90, 0, 3.0, [200, 91], [110, 91]), (4, 1, 128, 128, 0, 90, 0, 3.0, [200, 91, 180], [1, 1, 1]),
   (5, 5, 12, 20, 9, 0, 130, 0.0, [300, 64], [70, 3]), (2, 1, 128, 64, 64, 0, 64, 0.0, [400, 65], [150, 20]),
   (16, 1, 96, 96, 100, 0, 5, 2.0, [700, 260], [1, 1]), (3, 1, 40, 40, 1, 0, 2, 0.0, [70, 3], [70, 3]),
   (1, 1, 8, 8, 0, 5, 0, 1.5, [33, 70], [2, 5]), (4, 4, 32, 32, 200, 0, 10, 0.0, [150, 5], [150, 5]), (2, 2, 64, 64, 0, 64, 0, 30.0, [640, 1], [1, 1]),
